@@ -509,12 +509,9 @@ LCC_DEVICE void gemm_big_body(
 
   auto issue = [&](int kt, int stage) {
     u32x4* sbase = dsmem + stage * STAGE;
-    if (SCHED != 5) {      // (SCHED 4 / 5: timing diagnostics, only the activation / only the W half of the DMA ring)
 #pragma unroll
     for (int q = 0; q < A_PER_WAVE; ++q)
       glds16((asrc[q] + kt * BK), lds_addr(sbase + (wave * A_PER_WAVE + q) * 64));
-    }
-    if (SCHED != 4)
 #pragma unroll
     for (int q = 0; q < B_PER_WAVE; ++q)
       glds16((bsrc[q] + (size_t)kt * (W8 ? 512 : 1024)), lds_addr(sbase + A_UNITS + (wave * B_PER_WAVE + q) * 64));
@@ -551,12 +548,12 @@ LCC_DEVICE void gemm_big_body(
     __builtin_amdgcn_s_barrier();   // tile kt complete in LDS; every wave is done reading tile kt-1
     // SCHED 6 issues the same pieces one at a time between the row tiles of MFMAs below (a burst of 8 DMA instructions right after the
     // barrier holds the wave's issue port for ~60-100 cycles each while BOTH waves of the SIMD are at the same point)
-    if (SCHED != 2 && SCHED != 6 && kt + NSTAGE - 1 < nkt) issue(kt + NSTAGE - 1, (kt + NSTAGE - 1 - kt0) % NSTAGE);   // SCHED 2: timing diagnostic, no DMA
+    if (SCHED != 6 && kt + NSTAGE - 1 < nkt) issue(kt + NSTAGE - 1, (kt + NSTAGE - 1 - kt0) % NSTAGE);
     const u32x4* s = dsmem + ((kt - kt0) % NSTAGE) * STAGE;
     // ragged last row tile (e.g. M = 386 = 3 x 128 + 2): a wave whose WM rows are all past M skips the multiply and only keeps
     // feeding the DMA ring and the barriers (wave-uniform branch around the whole k-tile body; a finer per-16-row predicate
     // made hipcc if-convert the accumulators and spill)
-    if (!wave_has_rows || (SCHED >= 3 && SCHED <= 5)) {      // SCHED 3-5: timing diagnostics, DMA ring (or half of it) + barriers only
+    if (!wave_has_rows) {
       if (SCHED == 6 && kt + NSTAGE - 1 < nkt) issue(kt + NSTAGE - 1, (kt + NSTAGE - 1 - kt0) % NSTAGE);   // no MFMA stream to spread them over
     } else if (SCHED == 0) {
 #pragma unroll
@@ -1083,14 +1080,6 @@ static void launch_vh(const GemmArgs& a, hipStream_t st) {
 }
 template <int BM, int EPI>
 static void launch_big(const GemmArgs& a, hipStream_t st) {
-  if constexpr (BM == 256 && EPI == EPI_SWIGLU) {
-    // LCC_GEMM_DIAG (tools/bench_gemm_diag.py; results are WRONG by construction): 2 = no DMA after the prologue, 3 = no MFMAs
-    static const int diag = [] { const char* v = getenv("LCC_GEMM_DIAG"); return v ? atoi(v) : 0; }();
-    if (diag == 2 && !a.w_fp8) return launch_big_s<BM, EPI, 2, false>(a, st);
-    if (diag == 3 && !a.w_fp8) return launch_big_s<BM, EPI, 3, false>(a, st);
-    if (diag == 4 && !a.w_fp8) return launch_big_s<BM, EPI, 4, false>(a, st);
-    if (diag == 5 && !a.w_fp8) return launch_big_s<BM, EPI, 5, false>(a, st);
-  }
   // pinned fragment-read pipeline with the LDS-DMA pieces spread between the row-tile steps (SCHED 6, default since round 3:
   // bit-identical to the burst-behind-the-barrier order SCHED 1 -- tools/gemm_checksum.py -- and 1.6-3.3 % faster on the prefill
   // GEMMs, +0.6 / +0.8 % tokens/s at 1 / 8 streams, profiles/r03/gemm_sched_spread_dma.txt); LCC_GEMM_SCHED=1 restores SCHED 1

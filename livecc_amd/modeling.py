@@ -276,7 +276,7 @@ class LiveCCForConditionalGeneration:
         Each request: input_ids (1-D, full history like the reference's cat(past_ids, new_ids)), optional
         pixel_values_videos+video_grid_thw or uint8 frames, and `state` (StreamState or None).
         `prefetch`: clips ({'frames': uint8 GPU tensor, 'frames_layout': ...}) that a LATER call will pass as `frames`: their vision
-        tower (compute-bound) is launched on a low-priority side stream right after this call's prefill and runs under its decode
+        tower (compute-bound) is launched on a side stream right after this call's prefill and runs under its decode
         steps (HBM-bound weight streaming); the later call picks the embeddings up by the clip's storage (pointer, shape, layout).
         The frames must not be modified in between.  Results are bit-identical to the un-prefetched call.
         Thread-safe: the whole call (ViT, prefill, every decode step, the token read-back) runs under the model's engine lock."""
@@ -419,12 +419,8 @@ class LiveCCForConditionalGeneration:
         if self._side is None:
             # (A CU-masked stream -- hipExtStreamCreateWithCUMask, 48..176 CUs for the ViT -- was measured much slower: 150-182
             # tokens/s instead of 256: the decode kernels on the main stream slowed to 150 us per layer for every mask size.)
-            prio = 0
-            try:   # numerically greatest = lowest priority: decode kernels win the arbitration for CUs
-                prio = max(torch.cuda.Stream.priority_range())
-            except Exception:
-                pass
-            self._side = torch.cuda.Stream(device=self.device, priority=prio)
+            # Default priority, like every stream of the process.
+            self._side = torch.cuda.Stream(device=self.device)
         return self._side
 
     def _prefetch_vit(self, prefetch: Sequence[dict]) -> None:

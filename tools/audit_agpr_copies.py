@@ -19,7 +19,7 @@ CSRC = os.path.join(ROOT, "livecc_amd", "csrc")
 
 
 def asm_of(src, out):
-    subprocess.run(["/opt/rocm/bin/hipcc", "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", f"-I{ROOT}/include", f"-I{CSRC}", "-S",
+    subprocess.run(["/opt/rocm/bin/hipcc", "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", f"-I{ROOT}/include", f"-I{CSRC}", "-S",
                     "--cuda-device-only", src, "-o", out], check=True, capture_output=True)
     return open(out).read()
 
