@@ -299,6 +299,42 @@ int lcc_sample_topk_topp(const void* logits, int ld, int B, int V, uint32_t* see
                          int hist_ld, int32_t* hist_col, float* scores_out, float temperature, int top_k, float top_p,
                          uint64_t seed, uint32_t* rng_ctr, void* stream);
 
+/* ---- layer-list decoders: row operators and latent attention (no reference counterpart).  Channel counts are padded to multiples of 64 with
+ * zero weights; the residual stream x is fp32.
+ * Dynamic Tanh: y = tanh(alpha x) w + b, alpha one bf16 value, w / b bf16 [dim]: no row statistic. */
+/* x [rows,dim] = embedding rows, h = bf16(norm(x)); the id of row i is ids[i], or ids[indirect[i]] */
+int lcc_embed_dyt(const int32_t* ids, const int32_t* indirect, const void* table, const void* norm_w, const void* norm_b, const void* alpha, float* x,
+                  void* h, int rows, int dim, void* stream);
+/* x += sum of the nsplit slabs [nsplit][rows][dim]; h = bf16(norm(x)) */
+int lcc_resid_dyt(float* x, const float* partial, int nsplit, const void* norm_w, const void* norm_b, const void* alpha, void* h, int rows, int dim,
+                  void* stream);
+/* z = sum of the slabs [nsplit][rows][ld], capped: cap * tanh(z / cap) (cap <= 0: off).  out [rows][ld] (-inf from column vocab on) and / or
+ * dense [rows][vocab] */
+int lcc_logits_cap(const float* partial, int nsplit, int rows, int ld, int vocab, float cap, float* out, float* dense, void* stream);
+/* behind the fused input projection (slabs [nsplit][rows][ldn], columns: query latent | cache latent | one gate per head): RMS norms over the
+ * real ranks, the normed cache latent appended to the slot's arena at tok_pos[row] (NULL: kv_len[slot]), gates through the sigmoid.
+ * kv_rank_pad 0: the layer keeps no latent of its own.  kv_offset: elements from the arena's start to the layer's [Lmax][kv_rank_pad]. */
+int lcc_latent_norm_append(const float* partial, int nsplit, int rows, int ldn, int q_rank, int q_rank_pad, const void* q_norm, int kv_rank,
+                           int kv_rank_pad, const void* kv_norm, int heads, float eps, const int32_t* tok_stream, const int32_t* tok_pos,
+                           const int32_t* kv_len, void* const* kv_base, int64_t kv_offset, void* cq_out, float* gate_out, void* stream);
+/* cached latents of 16-row tiles (slot, first key, keys of the stream) back to back, zero past the stream's keys: row-major and MFMA-packed */
+int lcc_latent_gather(void* const* kv_base, int64_t kv_offset, int kv_rank_pad, const int32_t* tile_slot, const int32_t* tile_key0,
+                      const int32_t* tile_nkeys, int n_tiles, void* rows_out, void* packed_out, void* stream);
+/* causal multi-head attention: q [rows][heads*dim], k [keys][heads*dim], vt [heads*vdim][ldv], groups of <= 256 rows of one stream (first row,
+ * rows, position of the first row, first key row; the stream's keys are stored in whole, finite 32-row tiles); out [rows][ldo] bf16,
+ * scaled per head by gate [rows][heads] (optional).  dim, vdim in {64, 128}: MFMA kernel, else a plain one (dim % 8 == 0, vdim <= 1024) */
+int lcc_attn_mha(const void* q, const void* k, const void* vt, int ldv, const float* gate, void* out, int ldo, const int32_t* grp_q0,
+                 const int32_t* grp_nq, const int32_t* grp_pos0, const int32_t* grp_key0, int n_groups, int rows, int heads, int dim, int vdim, float scale,
+                 void* stream);
+/* out [rows][heads][kv_rank_pad] = Uk_h^T q_h; q as slabs [nsplit][rows][heads*dim]; ukt = packed [heads*kv_rank_pad, dim] */
+int lcc_latent_absorb(const float* q_partial, int nsplit, int rows, int heads, int dim, const void* ukt_packed, int kv_rank_pad, void* out, void* stream);
+/* one token per row: attention of the absorbed queries over kv_len[slot] + 1 cached latents, split over nsplit <= 128 blocks per row (scratch
+ * ws_o [rows*heads*nsplit*kv_rank_pad], ws_ml [rows*heads*nsplit*2]), then out[row][h*vdim ..] = gate * Uv_h (weighted latent); uv row-major.
+ * The slot's latents are readable in whole 64-row tiles.  kv_rank_pad / 64 in {1, 2, 3, 4, 6, 8, 12, 16} */
+int lcc_latent_attn_decode(const void* q_latent, const int32_t* slots, const int32_t* kv_len, void* const* kv_base, int64_t kv_offset, int rows, int heads,
+                           int kv_rank_pad, float scale, int nsplit, float* ws_o, float* ws_ml, const void* uv, int vdim, const float* gate, void* out,
+                           int ldo, void* stream);
+
 /* ------------------------------------------------------------------------------------------------
  * Model level -- what `model.generate(**inputs, past_key_values=...)` (ref:demo/infer.py:165-172) executes:
  * ViT (Q2VL:700-729) -> embed+scatter -> 28x decoder layer -> lm_head -> processors -> sample, with the
@@ -324,6 +360,25 @@ typedef struct {
 } lcc_engine_limits;
 
 lcc_engine* lcc_engine_create(const lcc_model_config* cfg, const lcc_engine_limits* lim);
+
+/* Second model family: decoders given as a list of layers.  The engine object, its buffers, slots, lcc_llm_prefill / lcc_llm_decode, the samplers
+ * and the slot calls are the same; there is no vision tower and prefill takes no positions (pos3 may be NULL).  A slot's arena holds one
+ * [max_kv_len][kv_rank_pad] bf16 block per layer that owns a latent.  Sizes named *_pad are the stored ones (zero rows / columns). */
+enum { LCC_FAMILY_QWEN2VL = 0, LCC_FAMILY_DECODER = 1 };
+enum { LCC_MIXER_LATENT = 1 };
+typedef struct {
+  int mixer;                                    /* LCC_MIXER_* */
+  int heads, q_rank, kv_rank;                   /* the model's: norms divide by the real ranks */
+  int dim_pad, vdim_pad, q_rank_pad, kv_rank_pad;
+  int kv_from;                                  /* -1: the layer has a latent of its own; else the earlier layer whose cache it reads */
+  float scale;                                  /* of the scores */
+  int ff_pad;                                   /* 0: no feed-forward */
+} lcc_decoder_layer;
+typedef struct {
+  int vocab_size, vocab_pad, width_pad, n_layers;
+  float norm_eps, logit_softcap;                /* logit_softcap <= 0: none */
+} lcc_decoder_config;
+lcc_engine* lcc_engine_create_decoder(const lcc_decoder_config* cfg, const lcc_decoder_layer* layers, const lcc_engine_limits* lim);
 void lcc_engine_destroy(lcc_engine* e);
 /* bytes the caller must provide (allocated by PyTorch so that torch.distributed can broadcast into them) */
 size_t lcc_engine_workspace_bytes(const lcc_engine* e);
@@ -373,6 +428,7 @@ int lcc_engine_profile_read_step_index(lcc_engine* e, int32_t* idx_out, int max_
  * max_rows fails with LCC_ERR_STATE.  lcc_debug_set_vit_taps: the same for the vision tower (Q2VL:700-729): taps bf16
  * [vit_depth + 1][max_rows][vit_embed] (0 = PatchEmbed output, l+1 = output of block l), overrides [vit_depth + 1][max_rows][vit_embed]
  * (input of block l; [vit_depth] = input of the PatchMerger). */
+/* Decoder family: taps = fp32 [n_layers + 1][max_rows][width_pad] (0 = embeddings, l+1 = residual after layer l); no overrides. */
 int lcc_debug_set_llm_taps(lcc_engine* e, void* taps, const void* overrides, int max_rows);
 int lcc_debug_set_vit_taps(lcc_engine* e, void* taps, const void* overrides, int max_rows);
 /* Teacher forcing (tests only; what the HF oracle does with a forcing LogitsProcessor): while bound, the token the sampler chose at
@@ -385,6 +441,8 @@ int lcc_debug_set_forced_tokens(lcc_engine* e, const int32_t* dev_tokens, int n_
 /* stream (slot) state */
 int lcc_slot_reset(lcc_engine* e, int slot, void* stream);                 /* new video stream: empty KV, empty history */
 int lcc_slot_set_length(lcc_engine* e, int slot, int kv_len, int next_pos, void* stream);  /* truncate after EOS */
+/* the token each slot consumes in its next decode step, instead of the one sampled last (replaying given ids); a frozen slot runs again */
+int lcc_slot_set_tokens(lcc_engine* e, int n_streams, const int32_t* slots, const int32_t* tokens, void* stream);
 int lcc_slot_get_length(const lcc_engine* e, int slot, int* kv_len, int* next_pos);
 
 typedef struct {
@@ -403,13 +461,16 @@ typedef struct {
   int eos_token;             /* <|im_end|>: a slot that samples it is frozen for the rest of the call (HF stopping criteria) */
   int suppress_eos;          /* 1 = MinNewTokensLength active for the whole call (min_new_tokens == max_new_tokens) */
   float* scores_out;         /* optional device fp32 [n_streams, V] of processed scores of the LAST step */
-  void* logits_out;          /* optional device bf16 [steps, n_streams, V] raw logits of every step (parity tests) */
+  void* logits_out;          /* optional device bf16 [steps, n_streams, V] raw logits of every step (parity tests); decoder family: fp32
+                                [steps, n_streams, vocab_size], after the cap (scores_out there has row pitch vocab_pad) */
   int eos_token2;            /* second EOS id of generation_config.json (<|endoftext|>) or -1 */
   int do_sample;             /* 0: argmax (lcc_sample_greedy); 1: lcc_sample_topk_topp with the fields below */
   float temperature;         /* > 0 */
   int top_k;                 /* 0 = off */
   float top_p;               /* (0, 1]; 1 = off */
   uint64_t seed;             /* Philox key; the per-slot draw counters live in the engine state (reset by lcc_slot_reset) */
+  /* decoder family, prefill: fp32 logits [n_prompt_rows, vocab] of these packed rows of the call (host array; 0 = none) */
+  int n_prompt_rows; const int32_t* prompt_rows; float* prompt_logits_out;
 } lcc_sampling;
 
 /* Prefill of n_streams streams: host arrays are copied through the engine's pinned meta ring.

@@ -46,7 +46,20 @@ class Sampling(C.Structure):
     _fields_ = [("repetition_penalty", C.c_float), ("thr_token", C.c_int), ("use_thr", C.c_int),
                 ("thr_base", C.c_float), ("thr_step", C.c_float), ("eos_token", C.c_int), ("suppress_eos", C.c_int),
                 ("scores_out", C.c_void_p), ("logits_out", C.c_void_p), ("eos_token2", C.c_int), ("do_sample", C.c_int),
-                ("temperature", C.c_float), ("top_k", C.c_int), ("top_p", C.c_float), ("seed", C.c_uint64)]
+                ("temperature", C.c_float), ("top_k", C.c_int), ("top_p", C.c_float), ("seed", C.c_uint64),
+                ("n_prompt_rows", C.c_int), ("prompt_rows", C.c_void_p), ("prompt_logits_out", C.c_void_p)]
+
+
+class DecoderLayer(C.Structure):
+    _fields_ = [(n, C.c_int) for n in ("mixer", "heads", "q_rank", "kv_rank", "dim_pad", "vdim_pad", "q_rank_pad", "kv_rank_pad", "kv_from")] + \
+               [("scale", C.c_float), ("ff_pad", C.c_int)]
+
+
+class DecoderConfigC(C.Structure):
+    _fields_ = [(n, C.c_int) for n in ("vocab_size", "vocab_pad", "width_pad", "n_layers")] + [("norm_eps", C.c_float), ("logit_softcap", C.c_float)]
+
+
+MIXER_LATENT = 1            # LCC_MIXER_LATENT
 
 
 def declared_symbols() -> List[str]:
@@ -134,6 +147,16 @@ def load():
                                     vp, vp, vp]),
         "lcc_sample_topk_topp": (i32, [vp, i32, i32, i32, vp, i32, vp, f32, i32, i32, f32, i32, i32, i32, vp, vp, vp, i32, vp,
                                        vp, f32, i32, f32, C.c_uint64, vp, vp]),
+        "lcc_embed_dyt": (i32, [vp, vp, vp, vp, vp, vp, vp, vp, i32, i32, vp]),
+        "lcc_resid_dyt": (i32, [vp, vp, i32, vp, vp, vp, vp, i32, i32, vp]),
+        "lcc_logits_cap": (i32, [vp, i32, i32, i32, i32, f32, vp, vp, vp]),
+        "lcc_latent_norm_append": (i32, [vp, i32, i32, i32, i32, i32, vp, i32, i32, vp, i32, f32, vp, vp, vp, vp, i64, vp, vp, vp]),
+        "lcc_latent_gather": (i32, [vp, i64, i32, vp, vp, vp, i32, vp, vp, vp]),
+        "lcc_attn_mha": (i32, [vp, vp, vp, i32, vp, vp, i32, vp, vp, vp, vp, i32, i32, i32, i32, i32, f32, vp]),
+        "lcc_latent_absorb": (i32, [vp, i32, i32, i32, i32, vp, i32, vp, vp]),
+        "lcc_latent_attn_decode": (i32, [vp, vp, vp, vp, i64, i32, i32, i32, f32, i32, vp, vp, vp, i32, vp, vp, i32, vp]),
+        "lcc_engine_create_decoder": (vp, [C.POINTER(DecoderConfigC), C.POINTER(DecoderLayer), C.POINTER(EngineLimits)]),
+        "lcc_slot_set_tokens": (i32, [vp, i32, vp, vp, vp]),
         "lcc_engine_create": (vp, [C.POINTER(ModelConfig), C.POINTER(EngineLimits)]),
         "lcc_engine_destroy": (None, [vp]),
         "lcc_engine_workspace_bytes": (sz, [vp]),

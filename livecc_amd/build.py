@@ -9,9 +9,20 @@ import sys
 HERE = os.path.dirname(os.path.abspath(__file__))
 
 
-def build(verbose: bool = True, force: bool = False) -> str:
+def build_engine(verbose: bool = True, force: bool = False) -> str:
+    """The HIP library alone (what serving a model needs); one build at a time per checkout."""
+    import fcntl
+    out = os.path.join(HERE, "_C")
+    os.makedirs(out, exist_ok=True)
+    with open(os.path.join(out, ".lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        return _make(verbose, force)
+
+
+def _make(verbose: bool, force: bool) -> str:
     csrc = os.path.join(HERE, "csrc")
-    cmd = ["make", "-C", csrc, "-j", str(min(8, os.cpu_count() or 1))]
+    jobs = int(os.environ.get("MAX_JOBS") or 8)
+    cmd = ["make", "-C", csrc, "-j", str(max(1, min(16, jobs, os.cpu_count() or 1)))]
     if force:
         subprocess.run(["make", "-C", csrc, "clean"], check=True, capture_output=not verbose)
     r = subprocess.run(cmd, capture_output=True, text=True)
@@ -22,6 +33,11 @@ def build(verbose: bool = True, force: bool = False) -> str:
         print(r.stdout.strip().splitlines()[-1])
     so = os.path.join(HERE, "_C", "liblivecc_amd.so")
     assert os.path.exists(so), so
+    return so
+
+
+def build(verbose: bool = True, force: bool = False) -> str:
+    so = build_engine(verbose=verbose, force=force)
     build_torch_ops(verbose=verbose, force=force)
     return so
 

@@ -1,4 +1,4 @@
-"""Model-shape description for the LiveCC / Qwen2-VL hot path.
+"""Model-shape descriptions: the LiveCC / Qwen2-VL hot path, and decoders given as a list of layers (`DebunexConfig`).
 
 The reference never defines shapes itself: `demo/infer.py:43-47` calls
 `Qwen2VLForConditionalGeneration.from_pretrained(model_path, ...)` and the shapes come
@@ -11,7 +11,7 @@ from __future__ import annotations
 import dataclasses
 import json
 import os
-from typing import List
+from typing import List, Optional
 
 
 @dataclasses.dataclass
@@ -206,13 +206,203 @@ def small() -> LiveCCConfig:
     )
 
 
+# ---- layer-list decoders ----
+def _up(n: int, m: int = 64) -> int:
+    return (n + m - 1) // m * m
+
+
+def pad_head_dim(d: int) -> int:
+    """Stored channels per head: 64 or 128 (the MFMA attention kernels), else the next multiple of 64."""
+    return _up(d)
+
+
+KV_RANK_TILES = (1, 2, 3, 4, 6, 8, 12, 16)       # 64-channel tiles the latent decode attention is built for
+
+
+def pad_kv_rank(r: int) -> int:
+    for t in KV_RANK_TILES:
+        if r <= 64 * t:
+            return 64 * t
+    raise ValueError(f"latent rank {r} exceeds {64 * KV_RANK_TILES[-1]}, the largest the latent attention kernels are built for")
+
+
+@dataclasses.dataclass
+class LatentMixerSpec:
+    """Latent attention without positions: queries and keys / values through normed low-rank vectors, a sigmoid gate per head."""
+    heads: int
+    dim: int                      # query / key channels per head
+    vdim: int                     # value channels per head
+    q_rank: int
+    kv_rank: int
+    scale: float
+    kv_from: Optional[int] = None  # the layer whose cached latent this one reads (None: its own)
+
+    @property
+    def dim_pad(self) -> int:
+        return pad_head_dim(self.dim)
+
+    @property
+    def vdim_pad(self) -> int:
+        return pad_head_dim(self.vdim)
+
+    @property
+    def q_rank_pad(self) -> int:
+        return _up(self.q_rank)
+
+    @property
+    def kv_rank_pad(self) -> int:
+        return pad_kv_rank(self.kv_rank)
+
+    @property
+    def in_rows(self) -> int:
+        """Rows of the fused input projection: query latent | own cache latent | gates."""
+        return self.q_rank_pad + (self.kv_rank_pad if self.kv_from is None else 0) + _up(self.heads, 16)
+
+
+@dataclasses.dataclass
+class DecoderLayerSpec:
+    mixer: LatentMixerSpec
+    ff: int = 0                   # width of the gated feed-forward; 0: none
+
+    @property
+    def ff_pad(self) -> int:
+        return _up(self.ff)
+
+
+@dataclasses.dataclass
+class DebunexConfig:
+    """A decoder-only language model given as a list of layers; both sublayers of a layer run in parallel behind one Dynamic-Tanh norm."""
+    vocab_size: int
+    hidden_size: int
+    layers: List[DecoderLayerSpec]
+    norm_eps: float = 1e-5
+    logit_softcap: Optional[float] = None
+    max_position_embeddings: int = 32768          # default KV capacity of a stream; the model itself has no positions
+    eos_token_id: Optional[int] = None
+    name: str = "debunex"
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def width_pad(self) -> int:
+        return _up(self.hidden_size)
+
+    @property
+    def vocab_pad(self) -> int:
+        return _up(self.vocab_size)
+
+    @property
+    def kv_bytes_per_token(self) -> int:
+        return sum(2 * l.mixer.kv_rank_pad for l in self.layers if l.mixer.kv_from is None)
+
+    def decode_weight_bytes(self) -> int:
+        """bf16 weight bytes one decode step reads (stored sizes)."""
+        n = self.vocab_pad * self.width_pad
+        for l in self.layers:
+            m = l.mixer
+            n += m.in_rows * self.width_pad + m.heads * m.dim_pad * (m.q_rank_pad + m.kv_rank_pad) + m.heads * m.vdim_pad * m.kv_rank_pad
+            n += self.width_pad * (m.heads * m.vdim_pad + 3 * l.ff_pad)
+        return 2 * n
+
+    def validate(self) -> None:
+        if not self.layers:
+            raise ValueError("a decoder needs at least one layer")
+        for i, l in enumerate(self.layers):
+            m = l.mixer
+            if min(m.heads, m.dim, m.vdim, m.q_rank, m.kv_rank) < 1 or l.ff < 0:
+                raise ValueError(f"layer {i}: sizes must be positive")
+            if max(m.dim_pad, m.vdim_pad) > 1024:
+                raise ValueError(f"layer {i}: head sizes above 1024 are not supported")
+            pad_kv_rank(m.kv_rank)
+            if m.kv_from is not None:
+                if not 0 <= m.kv_from < i:
+                    raise ValueError(f"layer {i}: kv_from {m.kv_from} is not an earlier layer")
+                o = self.layers[m.kv_from].mixer
+                if o.kv_from is not None or o.kv_rank != m.kv_rank:
+                    raise ValueError(f"layer {i}: layer {m.kv_from} has no latent of rank {m.kv_rank} of its own")
+
+    @classmethod
+    def from_dict(cls, raw: dict, name: str = "debunex") -> "DebunexConfig":
+        layers = []
+        for i, e in enumerate(raw["layers"]):
+            if e["type"] != "latent_attention":
+                raise ValueError(f"layer {i}: unknown layer type {e['type']!r}")
+            m = e["mixer"]
+            mlp = e.get("mlp")
+            if mlp is not None and mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward {mlp['kind']!r}")
+            kf = m.get("kv_from")
+            layers.append(DecoderLayerSpec(
+                LatentMixerSpec(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]), q_rank=int(m["q_rank"]), kv_rank=int(m["kv_rank"]),
+                                scale=float(m["scale"]), kv_from=None if kf is None else int(kf)), 0 if mlp is None else int(mlp["ff"])))
+        cap, eos = raw.get("logit_softcap"), raw.get("eos_token_id")
+        cfg = cls(vocab_size=int(raw["vocab"]), hidden_size=int(raw["width"]), layers=layers, norm_eps=float(raw["norm"]["eps"]),
+                  logit_softcap=None if cap is None else float(cap), eos_token_id=None if eos is None else int(eos), name=name)
+        cfg.validate()
+        return cfg
+
+    def to_dict(self) -> dict:
+        """The config.json form."""
+        out = {"architecture": "Debunex", "vocab": self.vocab_size, "width": self.hidden_size, "norm": {"eps": self.norm_eps}, "layers": []}
+        if self.logit_softcap is not None:
+            out["logit_softcap"] = self.logit_softcap
+        if self.eos_token_id is not None:
+            out["eos_token_id"] = self.eos_token_id
+        for l in self.layers:
+            m = {k: v for k, v in dataclasses.asdict(l.mixer).items() if v is not None}
+            out["layers"].append({"type": "latent_attention", "mixer": m, "mlp": {"kind": "dense", "ff": l.ff} if l.ff else None})
+        return out
+
+    @classmethod
+    def from_pretrained(cls, path: str) -> "DebunexConfig":
+        with open(os.path.join(path, "config.json")) as f:
+            return cls.from_dict(json.load(f), name=os.path.basename(os.path.normpath(path)))
+
+
+def _debunex(width, vocab, n_layers, ff, heads, dim, vdim, q_rank, kv_rank, share, name, cap=30.0, eps=1e-5) -> DebunexConfig:
+    """`share`: layers per cached latent (1: every layer its own)."""
+    layers = [DecoderLayerSpec(LatentMixerSpec(heads, dim, vdim, q_rank, kv_rank, dim ** -0.5, None if i % share == 0 else i - i % share), ff)
+              for i in range(n_layers)]
+    return DebunexConfig(vocab, width, layers, eps, cap, name=name)
+
+
+def debunex_tiny() -> DebunexConfig:
+    return _debunex(192, 320, 3, 256, 3, 24, 40, 48, 56, 2, "debunex-tiny")
+
+
+def debunex_2b() -> DebunexConfig:
+    """Qwen2-VL-2B's width, feed-forward, heads, depth and vocabulary with latent attention."""
+    return _debunex(1536, 151936, 28, 8960, 12, 128, 128, 768, 512, 2, "debunex-2b")
+
+
+def debunex_7b() -> DebunexConfig:
+    """LiveCC-7B's width, feed-forward, heads, depth and vocabulary with latent attention."""
+    return _debunex(3584, 152064, 28, 18944, 28, 128, 128, 1536, 512, 2, "debunex-7b")
+
+
+# config.json "architecture" -> configuration class; checkpoints without the key are Qwen2-VL ones
+ARCHITECTURES = {"Debunex": DebunexConfig}
+
+
 PRESETS = {"livecc-7b": livecc_7b, "qwen2vl-2b": qwen2vl_2b, "qwen2vl-2b-untied": qwen2vl_2b_untied, "qwen2vl-72b": qwen2vl_72b,
-           "tiny": tiny, "small": small}
+           "tiny": tiny, "small": small, "debunex-tiny": debunex_tiny, "debunex-2b": debunex_2b, "debunex-7b": debunex_7b}
 
 
-def get_config(name: str) -> LiveCCConfig:
+def architecture_of(path: str) -> Optional[str]:
+    """The "architecture" of a checkpoint directory's config.json, None for a Qwen2-VL one."""
+    with open(os.path.join(path, "config.json")) as f:
+        arch = json.load(f).get("architecture")
+    if arch is not None and arch not in ARCHITECTURES:
+        raise KeyError(f"unknown architecture {arch!r} in {path}; known: {sorted(ARCHITECTURES)}")
+    return arch
+
+
+def get_config(name: str):
     if name in PRESETS:
         return PRESETS[name]()
     if os.path.isdir(name):
-        return LiveCCConfig.from_pretrained(name)
+        arch = architecture_of(name)
+        return (LiveCCConfig if arch is None else ARCHITECTURES[arch]).from_pretrained(name)
     raise KeyError(f"unknown config {name!r}; presets: {sorted(PRESETS)}")

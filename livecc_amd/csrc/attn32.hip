@@ -86,10 +86,11 @@ __device__ unsigned int lcc_attn32_ones_page[256] = {[0 ... 255] = 0x3F803F80u};
 // LM (round 6, the tower kernel only): the softmax denominator comes out of the P . V MFMAs -- the V^T rows 80..95 of the third d-tile do not
 // exist at d = 80 and are fed with ONES, so O^T rows 80..95 accumulate sum_k bf16(P) under the same lazy rescale as O -- instead of 16 v_add +
 // the l_run update per region.  l then sums the ROUNDED probabilities the numerator uses (fp32 accumulation either way).
-template <int D, int PW, bool LM, class Issue>
+// D = channels of q / k, DV = channels of v.
+template <int D, int DV, int PW, bool LM, class Issue>
 LCC_DEVICE void attn32_key_loop(const u32x4* alds, Issue issue, const u32x4 (&qf)[D / 16], int tb, int te, int mlim, int lim, float scale_log2e,
-                                bool active, int lane, int hh, f32x16 (&o)[(D + 31) / 32], float& m_run, float& l_run) {
-  constexpr int KP = D / 16, DT = (D + 31) / 32, VP = 2 * DT, NP = KP + VP, NSTAGE = 10;
+                                bool active, int lane, int hh, f32x16 (&o)[(DV + 31) / 32], float& m_run, float& l_run) {
+  constexpr int KP = D / 16, DT = (DV + 31) / 32, VP = 2 * DT, NP = KP + VP, NSTAGE = 10;
   auto stage_of = [&](int t) { return alds + ((t - tb) % NSTAGE) * (NP * 64); };
   bf16x8 p_prev[2];                                     // P of the previous tile, its P . V still pending
   p_prev[0] = as_bf16x8((u32x4){0u, 0u, 0u, 0u});
@@ -168,7 +169,8 @@ LCC_DEVICE void attn32_key_loop(const u32x4* alds, Issue issue, const u32x4 (&qf
 
   issue(tb); issue(tb + 1); issue(tb + 2); issue(tb + 3); issue(tb + 4); issue(tb + 5);
   for (int t = tb; t < te; t += 2) {
-    if (PW == 2) asm volatile("s_waitcnt vmcnt(4)" ::: "memory");
+    if (PW == 1) asm volatile("s_waitcnt vmcnt(2)" ::: "memory");
+    else if (PW == 2) asm volatile("s_waitcnt vmcnt(4)" ::: "memory");
     else if (PW == 3) asm volatile("s_waitcnt vmcnt(6)" ::: "memory");
     else if (PW == 4) asm volatile("s_waitcnt vmcnt(8)" ::: "memory");
     else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
@@ -290,7 +292,7 @@ __global__ __launch_bounds__(NWAVE * 64, 2) void attn_gqa32_kernel(
   int min_limit = key_limit;                             // wave-wide minimum of the key limits: tiles entirely below it need no mask
 #pragma unroll
   for (int off = 32; off > 0; off >>= 1) min_limit = min(min_limit, __shfl_xor(min_limit, off, 64));
-  attn32_key_loop<D, PW, false>(alds, issue, qf, tb, te, min(min_limit, te * 32), min(key_limit, te * 32), scale_log2e, active, lane, hh, o, m_run, l_run);
+  attn32_key_loop<D, D, PW, false>(alds, issue, qf, tb, te, min(min_limit, te * 32), min(key_limit, te * 32), scale_log2e, active, lane, hh, o, m_run, l_run);
   if (!active) return;
 
   float l = xor32_sum(l_run);
@@ -400,7 +402,7 @@ __global__ __launch_bounds__(NWAVE * 64, 2) void attn_vit32_kernel(
 #pragma unroll
     for (int r = 0; r < 16; ++r) o[dt][r] = 0.f;
   float m_run = -INFINITY, l_run = 0.f;
-  attn32_key_loop<D, PW, LM>(alds, issue, qf, 0, ntile, sl, sl, scale_log2e, active, lane, hh, o, m_run, l_run);
+  attn32_key_loop<D, D, PW, LM>(alds, issue, qf, 0, ntile, sl, sl, scale_log2e, active, lane, hh, o, m_run, l_run);
   const float l = LM ? o[2][8] : xor32_sum(l_run);       // LM: row 80 + 4 hh of O^T, every one of rows 80..95 holds the sum over ALL keys
   if (active && col < nq) {
     const float inv = 1.f / l;
@@ -525,6 +527,101 @@ int attn_prefill32_launch(const bf16_t* q, bf16_t* out, const int32_t* tile_stre
   else
     attn_gqa32_kernel<8><<<grid, dim3(512), lds, st>>>(q, out, tile_stream, tile_q0, tile_nq, tile_pos0, kv_base, lay, layer, n_q_heads,
                                                        scale_log2e, S, ws_o, ws_ml, n_tiles, xcd, pack);
+  return 0;
+}
+
+// ------------------------------------------------------------------------------------------------------------------------------
+// Causal multi-head attention (one KV head per query head) over freshly formed keys and transposed values -- the prefill form of latent
+// attention (latent.hip).  Work item = (head, group of up to 256 rows of one stream), wave w owns rows 32 w ..; the eight waves share the
+// head's K / V^T tiles through the ring.  A wave whose rows end before the group's last key tile runs that tile fully masked.  Items are
+// dealt to the XCDs in contiguous chunks, groups fastest (and from the back: the long ones first), so the groups that read the same keys share
+// an L2.  The per-head output factor `gate` is applied before the one rounding to bf16.
+// ------------------------------------------------------------------------------------------------------------------------------
+template <int DK, int DV>
+__global__ __launch_bounds__(512, 2) void attn_mha32_kernel(MhaArgs a) {
+  constexpr int NWAVE = 8, KP = DK / 16, DT = DV / 32, VP = 2 * DT, NP = KP + VP, NSTAGE = 10, PW = (NP + NWAVE - 1) / NWAVE;
+  extern __shared__ __attribute__((aligned(16))) u32x4 alds[];
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int col = lane & 31, hh = lane >> 5;
+  const int n_items = a.n_groups * a.heads;
+  const int item = (int)(blockIdx.x & 7) * ((n_items + 7) >> 3) + (int)(blockIdx.x >> 3);
+  if ((int)(blockIdx.x >> 3) >= ((n_items + 7) >> 3) || item >= n_items) return;      // the whole block leaves before any barrier
+  const int h = item / a.n_groups, grp = a.n_groups - 1 - (item - h * a.n_groups);
+  const int q0 = a.grp_q0[grp], nq = a.grp_nq[grp], pos0 = a.grp_pos0[grp], key0 = a.grp_key0[grp];
+  const int ldq = a.heads * DK;
+  const bool active = wave * 32 < nq;
+  const int qr = min(wave * 32 + col, nq - 1);           // clamped: surplus columns compute a valid row and are not stored
+  const bool valid = wave * 32 + col < nq;
+  const int ntile = (pos0 + nq + 31) / 32;               // the keys are stored in whole 32-key tiles (zero-filled)
+  const bf16_t* kbase = a.k + (size_t)key0 * ldq + h * DK;
+  const bf16_t* vbase = a.vt + (size_t)h * DV * a.ldv + key0;
+
+  u32x4 qf[KP];
+  {
+    const bf16_t* qp = a.q + (size_t)(q0 + qr) * ldq + h * DK + hh * 8;
+#pragma unroll
+    for (int ks = 0; ks < KP; ++ks) qf[ks] = ld16(qp + ks * 16);
+#pragma unroll
+    for (int ks = 0; ks < KP; ++ks) settle_load(qf[ks]);     // before the first LDS-DMA piece (common.h: glds16)
+  }
+  const bf16_t* pbase[PW];
+  size_t pstride[PW];
+#pragma unroll
+  for (int j = 0; j < PW; ++j) {
+    const int p = min(j * NWAVE + wave, NP - 1);         // surplus slots re-fetch the last piece (same bytes, same place)
+    if (p < KP) {
+      pbase[j] = kbase + (size_t)swap23(col) * ldq + p * 16 + hh * 8;
+      pstride[j] = (size_t)32 * ldq;
+    } else {
+      const int dt = (p - KP) >> 1, s = (p - KP) & 1;
+      pbase[j] = vbase + (size_t)(dt * 32 + col) * a.ldv + s * 16 + hh * 8;
+      pstride[j] = 32;
+    }
+  }
+  int tb = 0;
+  asm volatile("" : "+s"(tb));      // opaque: with a known first tile hipcc splits the ring's index arithmetic into registers it then spills
+  auto issue = [&](int t) {
+    const int tc = min(t, ntile - 1);
+    u32x4* sbase = alds + ((t - tb) % NSTAGE) * (NP * 64);
+#pragma unroll
+    for (int j = 0; j < PW; ++j) glds16(pbase[j] + (size_t)tc * pstride[j], lds_addr(sbase + min(j * NWAVE + wave, NP - 1) * 64));
+  };
+  f32x16 o[DT];
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+    for (int r = 0; r < 16; ++r) o[dt][r] = 0.f;
+  float m_run = -INFINITY, l_run = 0.f;
+  const int key_limit = pos0 + qr + 1;
+  int min_limit = pos0 + min(wave * 32, nq - 1) + 1;            // of the wave's first row
+  asm volatile("" : "+v"(min_limit));
+  attn32_key_loop<DK, DV, PW, false>(alds, issue, qf, tb, ntile, min_limit, key_limit, a.scale_log2e, active, lane, hh, o, m_run, l_run);
+  if (!active) return;
+  const float l = xor32_sum(l_run);
+  if (valid) {
+    const float f = (a.gate ? a.gate[(size_t)(q0 + qr) * a.heads + h] : 1.f) / l;
+    bf16_t* op = a.out + (size_t)(q0 + qr) * a.ldo + h * DV;
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+      for (int r4 = 0; r4 < 4; ++r4)
+        st8(op + dt * 32 + 8 * r4 + 4 * hh, (u32x2){pack2(o[dt][4 * r4] * f, o[dt][4 * r4 + 1] * f), pack2(o[dt][4 * r4 + 2] * f, o[dt][4 * r4 + 3] * f)});
+  }
+}
+template <int DK, int DV>
+static void mha32_go(const MhaArgs& a, hipStream_t st) {
+  constexpr size_t lds = (size_t)10 * (DK / 16 + 2 * (DV / 32)) * 1024;
+  static DeviceOnce once;   // per instantiation
+  if (once.first()) (void)hipFuncSetAttribute((const void*)attn_mha32_kernel<DK, DV>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+  const long n_items = (long)a.n_groups * a.heads;
+  attn_mha32_kernel<DK, DV><<<dim3((unsigned)((n_items + 7) / 8 * 8)), dim3(512), lds, st>>>(a);
+}
+int attn_mha32_launch(const MhaArgs& a, hipStream_t st) {
+  if (a.dim == 128 && a.vdim == 128) mha32_go<128, 128>(a, st);
+  else if (a.dim == 64 && a.vdim == 64) mha32_go<64, 64>(a, st);
+  else if (a.dim == 64 && a.vdim == 128) mha32_go<64, 128>(a, st);
+  else if (a.dim == 128 && a.vdim == 64) mha32_go<128, 64>(a, st);
+  else return LCC_ERR_SHAPE;
   return 0;
 }
 

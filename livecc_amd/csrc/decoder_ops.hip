@@ -1,0 +1,119 @@
+// Row operators of the layer-list decoders (engine_decoder.hip): embedding, residual add and norm, logits.
+//
+// The residual stream is fp32 from the embedding to the last norm.  The norm is Dynamic Tanh, y = tanh(alpha x) w + b: it needs no row
+// statistic, so it runs in the pass that writes the residual -- the consumer GEMM reads ready bf16 activations and no launch exists for the
+// norm alone.  Rows are padded to a multiple of 64 channels with zero weights, so a padding channel stays 0 through the norm (w = b = 0).
+#include "common.h"
+#include "kernels.h"
+
+namespace lcc {
+
+LCC_DEVICE float dyt(float x, float alpha, float w, float b) { return fmaf(tanhf(alpha * x), w, b); }
+LCC_DEVICE u32x4 dyt8(const float (&x)[8], float alpha, const bf16_t* w, const bf16_t* b) {
+  const u32x4 wv = ld16(w), bv = ld16(b);
+  u32x4 o;
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+    o[e] = pack2(dyt(x[2 * e], alpha, lo2f(wv[e]), lo2f(bv[e])), dyt(x[2 * e + 1], alpha, hi2f(wv[e]), hi2f(bv[e])));
+  return o;
+}
+
+// x = embedding row (fp32), h = norm(x).  ids[i], or -- decode -- the slot's current token ids[indirect[i]].
+__global__ __launch_bounds__(256) void embed_dyt_kernel(const int32_t* __restrict__ ids, const int32_t* __restrict__ indirect,
+                                                        const bf16_t* __restrict__ table, DytNorm nm, float* __restrict__ x,
+                                                        bf16_t* __restrict__ h, int rows, int dim) {
+  const int cpr = dim >> 3;
+  const float alpha = bf2f(nm.alpha[0]);
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < (int64_t)rows * cpr; i += (int64_t)gridDim.x * 256) {
+    const int r = (int)(i / cpr), c = (int)(i - (int64_t)r * cpr) * 8;
+    const int id = indirect ? ids[indirect[r]] : ids[r];
+    const u32x4 q = ld16(table + (size_t)id * dim + c);
+    float v[8];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) { v[2 * e] = lo2f(q[e]); v[2 * e + 1] = hi2f(q[e]); }
+    float* xp = x + (size_t)r * dim + c;
+    *reinterpret_cast<f32x4*>(xp) = (f32x4){v[0], v[1], v[2], v[3]};
+    *reinterpret_cast<f32x4*>(xp + 4) = (f32x4){v[4], v[5], v[6], v[7]};
+    st16(h + (size_t)r * dim + c, dyt8(v, alpha, nm.w + c, nm.b + c));
+  }
+}
+
+// x += sum of the nsplit fp32 slabs of the layer's output product, h = norm(x) of the NEXT norm
+__global__ __launch_bounds__(256) void resid_dyt_kernel(float* __restrict__ x, const float* __restrict__ part, int nsplit, DytNorm nm,
+                                                        bf16_t* __restrict__ h, int rows, int dim) {
+  const int cpr = dim >> 3;
+  const float alpha = bf2f(nm.alpha[0]);
+  const size_t slab = (size_t)rows * dim;
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < (int64_t)rows * cpr; i += (int64_t)gridDim.x * 256) {
+    const int c = (int)(i % cpr) * 8;
+    const size_t off = (size_t)i * 8;
+    f32x4 a = *reinterpret_cast<const f32x4*>(x + off), b = *reinterpret_cast<const f32x4*>(x + off + 4);
+    f32x4 sa = {0.f, 0.f, 0.f, 0.f}, sb = {0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < nsplit; ++s) {
+      sa += *reinterpret_cast<const f32x4*>(part + s * slab + off);
+      sb += *reinterpret_cast<const f32x4*>(part + s * slab + off + 4);
+    }
+    a += sa; b += sb;
+    *reinterpret_cast<f32x4*>(x + off) = a;
+    *reinterpret_cast<f32x4*>(x + off + 4) = b;
+    const float v[8] = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+    st16(h + off, dyt8(v, alpha, nm.w + c, nm.b + c));
+  }
+}
+
+// logits = cap * tanh(z / cap) (cap <= 0: z) of the fp32 slabs z [nsplit][rows][ld]; ids past the vocabulary are -inf.  `out` [rows][ld]
+// feeds the sampler, `dense` [rows][vocab] (optional) is the caller's copy.
+__global__ __launch_bounds__(256) void logits_cap_kernel(const float* __restrict__ part, int nsplit, int rows, int ld, int vocab, float cap,
+                                                         float* __restrict__ out, float* __restrict__ dense) {
+  const size_t slab = (size_t)rows * ld;
+  const float inv = cap > 0.f ? 1.f / cap : 0.f;
+  for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < slab; i += (size_t)gridDim.x * 256) {
+    const int r = (int)(i / ld), n = (int)(i - (size_t)r * ld);
+    float z = 0.f;
+    for (int s = 0; s < nsplit; ++s) z += part[s * slab + i];
+    if (cap > 0.f) z = cap * tanhf(z * inv);
+    if (out) out[i] = n < vocab ? z : -INFINITY;
+    if (dense && n < vocab) dense[(size_t)r * vocab + n] = z;
+  }
+}
+
+// the caller's own continuation: the token a slot consumes in its next decode step; its generate counters restart as after a prefill
+__global__ void set_tokens_kernel(const int32_t* __restrict__ slots, const int32_t* __restrict__ toks, int n, int32_t* __restrict__ cur_tok,
+                                  int32_t* __restrict__ done, int32_t* __restrict__ hist_col) {
+  const int i = blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= n) return;
+  const int s = slots[i];
+  cur_tok[s] = toks[i]; done[s] = 0; hist_col[s] = 0;
+}
+
+static unsigned grid_for(int64_t items) { return (unsigned)((items + 255) / 256 < 4096 ? (items + 255) / 256 : 4096); }
+
+static bool dyt_ok(const DytNorm& n) { return n.w && n.b && n.alpha && ((((uintptr_t)n.w) | ((uintptr_t)n.b)) & 15) == 0; }
+int embed_dyt(const int32_t* ids, const int32_t* indirect, const bf16_t* table, const DytNorm& nm, float* x, bf16_t* h, int rows, int dim, hipStream_t st) {
+  if (rows <= 0) return 0;
+  if (dim <= 0 || (dim & 7)) return LCC_ERR_SHAPE;
+  if (!ids || !table || !x || !h || !dyt_ok(nm)) return LCC_ERR_ARG;
+  embed_dyt_kernel<<<dim3(grid_for((int64_t)rows * (dim >> 3))), dim3(256), 0, st>>>(ids, indirect, table, nm, x, h, rows, dim);
+  return 0;
+}
+int resid_dyt(float* x, const float* part, int nsplit, const DytNorm& nm, bf16_t* h, int rows, int dim, hipStream_t st) {
+  if (rows <= 0) return 0;
+  if (dim <= 0 || (dim & 7) || nsplit < 0) return LCC_ERR_SHAPE;
+  if (!x || !h || (nsplit > 0 && !part) || !dyt_ok(nm)) return LCC_ERR_ARG;
+  resid_dyt_kernel<<<dim3(grid_for((int64_t)rows * (dim >> 3))), dim3(256), 0, st>>>(x, part, nsplit, nm, h, rows, dim);
+  return 0;
+}
+int logits_cap(const float* part, int nsplit, int rows, int ld, int vocab, float cap, float* out, float* dense, hipStream_t st) {
+  if (rows <= 0) return 0;
+  if (nsplit < 1 || vocab < 1 || ld < vocab) return LCC_ERR_SHAPE;
+  if (!part || (!out && !dense)) return LCC_ERR_ARG;
+  logits_cap_kernel<<<dim3(grid_for((int64_t)rows * ld)), dim3(256), 0, st>>>(part, nsplit, rows, ld, vocab, cap, out, dense);
+  return 0;
+}
+int set_tokens(const int32_t* slots, const int32_t* toks, int n, int32_t* cur_tok, int32_t* done, int32_t* hist_col, hipStream_t st) {
+  if (n <= 0) return 0;
+  set_tokens_kernel<<<dim3((n + 63) / 64), dim3(64), 0, st>>>(slots, toks, n, cur_tok, done, hist_col);
+  return 0;
+}
+
+}  // namespace lcc

@@ -157,13 +157,16 @@ extern "C" int lcc_engine_profile_read_step_index(lcc_engine* e, int32_t* idx_ou
   *n_out = n;
   return 0;
 }
-extern "C" size_t lcc_engine_workspace_bytes(const lcc_engine* e) { return std::max(e->llm_ws_bytes(), e->vit_ws_bytes()); }
+extern "C" size_t lcc_engine_workspace_bytes(const lcc_engine* e) {
+  return e->family == LCC_FAMILY_DECODER ? lcc_decoder_ws_bytes(e) : std::max(e->llm_ws_bytes(), e->vit_ws_bytes());
+}
 extern "C" size_t lcc_engine_state_bytes(const lcc_engine* e) {
   const size_t B = e->lim.max_slots;
   return align_up(B * 4) * 6 + 256 + align_up(B * 8) + align_up(B * (size_t)e->lim.max_history * 4) + align_up(B * (size_t)e->words * 4) + 4096 + 1024 + 1024;
 }
-extern "C" size_t lcc_engine_kv_bytes_per_slot(const lcc_engine* e) { return e->lay.total() * 2; }
+extern "C" size_t lcc_engine_kv_bytes_per_slot(const lcc_engine* e) { return (e->family == LCC_FAMILY_DECODER ? e->dec_kv_total : e->lay.total()) * 2; }
 extern "C" size_t lcc_engine_meta_bytes(const lcc_engine* e) {
+  if (e->family == LCC_FAMILY_DECODER) return align_up(lcc_decoder_meta_bytes(e) + 4096, 4096) * META_RING;
   const size_t S = e->lim.max_new_rows, P = e->lim.max_patches, B = e->lim.max_slots;
   const size_t llm = (7 * S + 4 * (S / 16 + B + 1) + 4 * B + 64) * 4;
   const size_t vit = (P + P / 4 + 8 * (P / 16 + 64) + 128) * 4;     // + P / 4: grp_off of the fused q|k|v projection
@@ -230,6 +233,11 @@ extern "C" int lcc_engine_set_weight(lcc_engine* e, const char* name, const void
 }
 
 static int resolve_weights(lcc_engine* e, std::string* missing) {
+  if (e->family == LCC_FAMILY_DECODER) {
+    const int r = lcc_decoder_resolve_weights(e, missing);
+    e->weights_resolved = r == 0;
+    return r;
+  }
   auto get = [&](const std::string& n) -> const bf16_t* {
     auto it = e->w.find(n);
     if (it == e->w.end()) { if (missing) { *missing += n; *missing += ' '; } return nullptr; }

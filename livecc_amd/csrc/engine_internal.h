@@ -56,6 +56,12 @@ struct LlmLayerW {
   const float* qkv_s_dec;                          // scales of the row-permuted decode copy (fp8 arenas with decode copies)
 };
 
+struct DecLayerW {     // a layer of a layer-list decoder (engine_decoder.hip)
+  DytNorm norm;
+  const bf16_t *in_w = nullptr, *q_norm = nullptr, *kv_norm = nullptr, *uq_w = nullptr, *uk_w = nullptr, *ukt_w = nullptr, *uv_w = nullptr,
+               *gate_up_w = nullptr, *out_w = nullptr;
+};
+
 struct Carver {  // bump allocator over a caller-provided region
   char* base = nullptr;
   size_t off = 0;
@@ -72,8 +78,17 @@ constexpr int MAX_SPLIT = 8;
 
 
 struct lcc_engine {
-  lcc_model_config c;
+  int family = LCC_FAMILY_QWEN2VL;
+  lcc_model_config c;          // decoder family: vocabulary / width hold the padded sizes, the rest is unused
   lcc_engine_limits lim;
+  // family LCC_FAMILY_DECODER
+  lcc_decoder_config dc = {};
+  std::vector<lcc_decoder_layer> dl;
+  std::vector<DecLayerW> dw;
+  DytNorm dec_final_norm;
+  std::vector<size_t> dec_kv_off;      // element offset of a layer's latents inside a slot's arena (layers that own one)
+  size_t dec_kv_total = 0;
+  static int dec_in_rows(const lcc_decoder_layer& L);      // output rows of the fused input projection
   int qd, kvd, qkvd, words, E, vit_hd;
   int cu_count = 256;          // compute units of the device current at lcc_engine_create
   KvLayout lay;
@@ -167,4 +182,13 @@ struct MetaWriter {
 };
 int meta_begin(lcc_engine* e, MetaWriter* mw);
 int meta_commit(MetaWriter* mw, hipStream_t st);
+// logits -> processors -> sampler for `n` rows of a call of B streams starting at row r0 (engine_llm.hip); f32: fp32 logits, else bf16
+int lcc_sample_rows(lcc_engine* e, const void* logits, bool f32, int n, int B, int r0, const int32_t* d_slots, const lcc_sampling* sp, int step_index,
+                    float* ws, hipStream_t st);
+// engine_decoder.hip
+size_t lcc_decoder_ws_bytes(const lcc_engine* e);
+size_t lcc_decoder_meta_bytes(const lcc_engine* e);
+int lcc_decoder_resolve_weights(lcc_engine* e, std::string* missing);
+int lcc_decoder_prefill(lcc_engine* e, int n_streams, const int32_t* slots, const int32_t* n_new, const int32_t* ids, int S, const lcc_sampling* sp, hipStream_t st);
+int lcc_decoder_decode(lcc_engine* e, int n_streams, const int32_t* d_slots, int max_len, int n_steps, int first_step_index, const lcc_sampling* sp, hipStream_t st);
 extern int g_decode_chain;        // engine_llm.hip; lcc_slot_read_tokens turns it off after a failed hand-off

@@ -257,6 +257,13 @@ int head_and_sample(lcc_engine* e, const LlmBuffers& b, const bf16_t* xn_rows, i
     if (e->lm_head_s != nullptr) { g.w_fp8 = 1; g.wscale = e->lm_head_s; }
     LCC_TRY(gemm_bf16(g, st));
   }
+  return lcc_sample_rows(e, logits, false, B, B, 0, d_slots, sp, step_index, b.ws_ml, st);
+}
+}  // namespace
+
+int lcc_sample_rows(lcc_engine* e, const void* logits, bool f32, int n, int B, int r0, const int32_t* d_slots, const lcc_sampling* sp, int step_index,
+                    float* ws, hipStream_t st) {
+  const int V = e->c.vocab_size;
   const float pen = sp ? sp->repetition_penalty : 1.0f;
   const int thr_tok = sp ? sp->thr_token : -1;
   const int use_thr = sp ? sp->use_thr : 0;
@@ -269,26 +276,25 @@ int head_and_sample(lcc_engine* e, const LlmBuffers& b, const bf16_t* xn_rows, i
   // processed scores keep the oracle's definition (EOS unmasked unless the caller asked)
   const int sup_eos = ((sp && sp->suppress_eos) ? 1 : 0) | (forcing ? 2 : 0);
   if (sp && sp->do_sample && sp->top_k != 1) {
-    LCC_TRY(sample_topk_topp(logits, V, B, V, e->d_seen, e->words, d_slots, pen <= 0.f ? 1.0f : pen, thr_tok, use_thr, thr, sp->eos_token,
+    LCC_TRY(sample_topk_topp(logits, f32, V, n, V, e->d_seen, e->words, d_slots, pen <= 0.f ? 1.0f : pen, thr_tok, use_thr, thr, sp->eos_token,
                              eos2, sup_eos, e->d_done, e->d_cur_tok, e->d_history, e->lim.max_history, e->d_hist_col,
                              sp->scores_out, sp->temperature, sp->top_k, sp->top_p, sp->seed, e->d_rng_ctr, st));
     if (forcing)
-      LCC_TRY(force_tokens(d_slots, e->forced + (size_t)step_index * B, B, e->d_cur_tok, e->d_history, e->lim.max_history, e->d_hist_col, e->d_done,
+      LCC_TRY(force_tokens(d_slots, e->forced + (size_t)step_index * B + r0, n, e->d_cur_tok, e->d_history, e->lim.max_history, e->d_hist_col, e->d_done,
                            sp->suppress_eos ? -1 : sp->eos_token, sp->suppress_eos ? -1 : eos2, st));
     return 0;
   }
   // top_k == 1 (the released generation_config): the top-k warper leaves one finite score -> the draw IS the argmax
-  LCC_TRY(sample_greedy(logits, V, B, V, e->d_seen, e->words, d_slots, pen <= 0.f ? 1.0f : pen, thr_tok, use_thr, thr,
+  LCC_TRY(sample_greedy(logits, f32, V, n, V, e->d_seen, e->words, d_slots, pen <= 0.f ? 1.0f : pen, thr_tok, use_thr, thr,
                         sp ? sp->eos_token : -1, eos2, sup_eos, e->d_done, e->d_cur_tok, e->d_history, e->lim.max_history,
-                        e->d_hist_col, sp ? sp->scores_out : nullptr, b.ws_ml, st));
+                        e->d_hist_col, sp ? sp->scores_out : nullptr, ws, st));
   if (forcing) {
     const bool keep_going = sp && sp->suppress_eos;      // force_length: a forced EOS does not end the slot either
-    LCC_TRY(force_tokens(d_slots, e->forced + (size_t)step_index * B, B, e->d_cur_tok, e->d_history, e->lim.max_history, e->d_hist_col, e->d_done,
+    LCC_TRY(force_tokens(d_slots, e->forced + (size_t)step_index * B + r0, n, e->d_cur_tok, e->d_history, e->lim.max_history, e->d_hist_col, e->d_done,
                          keep_going || !sp ? -1 : sp->eos_token, keep_going || !sp ? -1 : eos2, st));
   }
   return 0;
 }
-}  // namespace
 
 extern "C" int lcc_llm_prefill(lcc_engine* e, int n_streams, const int32_t* slots, const int32_t* n_new, const int32_t* ids,
                                const int32_t* vit_index, const void* vit_embeds, const int32_t* pos3, const lcc_sampling* sp,
@@ -296,7 +302,9 @@ extern "C" int lcc_llm_prefill(lcc_engine* e, int n_streams, const int32_t* slot
   LCC_TRY(ensure_ready(e));
   CallScope in_flight;
   std::lock_guard<std::mutex> lk(e->mu_llm);
-  if (n_streams <= 0 || !slots || !n_new || !ids || !pos3) return fail(LCC_ERR_ARG, "null argument");
+  const bool decoder = e->family == LCC_FAMILY_DECODER;
+  if (n_streams <= 0 || !slots || !n_new || !ids || (!pos3 && !decoder)) return fail(LCC_ERR_ARG, "null argument");
+  if (!decoder && sp && sp->n_prompt_rows > 0) return fail(LCC_ERR_ARG, "prompt_rows: logits of prompt positions are available for decoder models only");
   if (n_streams > e->lim.max_slots) return fail(LCC_ERR_STATE, "too many streams");
   hipStream_t st = (hipStream_t)stream;
   int S = 0;
@@ -310,9 +318,10 @@ extern "C" int lcc_llm_prefill(lcc_engine* e, int n_streams, const int32_t* slot
   }
   if (S > e->lim.max_new_rows) return fail(LCC_ERR_STATE, "%d new rows > max_new_rows %d", S, e->lim.max_new_rows);
   for (int i = 0; i < S; ++i) {
-    if (ids[i] < 0 || ids[i] >= e->c.vocab_size) return fail(LCC_ERR_ARG, "token id %d out of range at %d", ids[i], i);
+    if (ids[i] < 0 || ids[i] >= (decoder ? e->dc.vocab_size : e->c.vocab_size)) return fail(LCC_ERR_ARG, "token id %d out of range at %d", ids[i], i);
     if (vit_index && vit_index[i] >= 0 && !vit_embeds) return fail(LCC_ERR_ARG, "vit_index set but vit_embeds is null");
   }
+  if (decoder) return lcc_decoder_prefill(e, n_streams, slots, n_new, ids, S, sp, st);
   LlmBuffers bf; LCC_TRY(carve_llm(e, &bf));
 
   // host tables
@@ -439,11 +448,16 @@ extern "C" int lcc_llm_decode(lcc_engine* e, int n_streams, const int32_t* slots
     max_len = std::max(max_len, e->h_kv_len[s] + n_steps);
   }
   if (first_step_index + n_steps > e->lim.max_history) return fail(LCC_ERR_STATE, "history capacity %d exceeded", e->lim.max_history);
-  LlmBuffers bf; LCC_TRY(carve_llm(e, &bf));
   MetaWriter mw; LCC_TRY(meta_begin(e, &mw));
   int32_t* d_slots;
   if (!mw.put(slots, n_streams, &d_slots)) return fail(LCC_ERR_STATE, "meta ring slot too small");
   LCC_TRY(meta_commit(&mw, st));
+  if (e->family == LCC_FAMILY_DECODER) {
+    LCC_TRY(lcc_decoder_decode(e, n_streams, d_slots, max_len, n_steps, first_step_index, sp, st));
+    for (int b = 0; b < n_streams; ++b) { e->h_kv_len[slots[b]] += n_steps; e->h_pos[slots[b]] += n_steps; }
+    return 0;
+  }
+  LlmBuffers bf; LCC_TRY(carve_llm(e, &bf));
   const int ntile = (max_len + 31) / 32;
   // key tiles per split of the per-wave decode attention (tuning knob LCC_ATTN_TPS, default 4) and the split cap (LCC_ATTN_MAXSPLIT, 64)
   static const int tps = [] { const char* v = getenv("LCC_ATTN_TPS"); return v ? std::max(1, atoi(v)) : 4; }();

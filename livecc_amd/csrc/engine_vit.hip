@@ -31,6 +31,7 @@ extern "C" int lcc_vit_encode(lcc_engine* e, int n_clips, const lcc_clip* clips,
   CallScope in_flight;
   std::lock_guard<std::mutex> lk(e->mu_vit);
   GridCapScope cap_scope(e->vit_grid_cap);
+  if (e->family != LCC_FAMILY_QWEN2VL) return fail(LCC_ERR_STATE, "this model has no vision tower");
   if (n_clips <= 0 || !clips || !rope_cos || !rope_sin || !out_embeds) return fail(LCC_ERR_ARG, "null argument");
   hipStream_t st = (hipStream_t)stream;
   const int E = e->E, heads = e->c.vit_heads, MLP = e->c.vit_mlp, H = e->c.hidden_size, PD = e->c.patch_dim;

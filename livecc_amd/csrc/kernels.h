@@ -161,15 +161,15 @@ int attn_decode_fused_bf16(const float* qkv_part, int ns_qkv, const bf16_t* bias
                            const int32_t* slots, const int32_t* kv_len, bf16_t* const* kv_base, KvLayout lay, int layer, int B,
                            int n_q_heads, int nsplit, float* ws_o, float* ws_ml, int32_t* counters, bf16_t* out, hipStream_t st);
 
-// ---- sampler (sampler.hip) ----
+// ---- sampler (sampler.hip) ----  logits bf16, or fp32 (f32)
 int seen_set(uint32_t* seen, int words_per_stream, const int32_t* ids, const int32_t* slot_of_id, int n, int indirect,
              const int32_t* done, hipStream_t st);
-int sample_greedy(const bf16_t* logits, int ld, int B, int V, uint32_t* seen, int words_per_stream,
+int sample_greedy(const void* logits, bool f32, int ld, int B, int V, uint32_t* seen, int words_per_stream,
                   const int32_t* stream_slot, float repetition_penalty, int thr_token, int use_thr, float thr_value,
                   int eos_token, int eos_token2, int suppress_eos, int32_t* done, int32_t* out_tokens, int32_t* history, int hist_ld,
                   int32_t* hist_col, float* scores_out, float* ws, hipStream_t st);
 // do_sample: temperature -> top-k -> top-p -> multinomial (Philox stream per slot); top_k 0 = off, top_p 1 = off
-int sample_topk_topp(const bf16_t* logits, int ld, int B, int V, uint32_t* seen, int words_per_stream, const int32_t* stream_slot,
+int sample_topk_topp(const void* logits, bool f32, int ld, int B, int V, uint32_t* seen, int words_per_stream, const int32_t* stream_slot,
                      float repetition_penalty, int thr_token, int use_thr, float thr_value, int eos_token, int eos_token2,
                      int suppress_eos, int32_t* done, int32_t* out_tokens, int32_t* history, int hist_ld, int32_t* hist_col,
                      float* scores_out, float temperature, int top_k, float top_p, uint64_t seed, uint32_t* rng_ctr, hipStream_t st);
@@ -218,5 +218,46 @@ void dgemv_attach_events_to_next_swiglu(hipEvent_t start, hipEvent_t stop);
 int dgemv_chain_capacity();
 int dgemv_down_qkv(const DgArgs& down, const DgArgs& qkv, unsigned* flag, unsigned target, unsigned* err, hipStream_t st);
 int dgemv_norm_bf16(const DgArgs& a, hipStream_t st);     // [final RMSNorm] lm_head
+
+// ---- layer-list decoders: row operators (decoder_ops.hip) ----
+struct DytNorm { const bf16_t* w = nullptr; const bf16_t* b = nullptr; const bf16_t* alpha = nullptr; };   // y = tanh(alpha x) w + b; alpha: one value
+int embed_dyt(const int32_t* ids, const int32_t* indirect, const bf16_t* table, const DytNorm& nm, float* x, bf16_t* h, int rows, int dim, hipStream_t st);
+int resid_dyt(float* x, const float* part, int nsplit, const DytNorm& nm, bf16_t* h, int rows, int dim, hipStream_t st);
+int logits_cap(const float* part, int nsplit, int rows, int ld, int vocab, float cap, float* out, float* dense, hipStream_t st);
+int set_tokens(const int32_t* slots, const int32_t* toks, int n, int32_t* cur_tok, int32_t* done, int32_t* hist_col, hipStream_t st);
+
+// ---- latent attention (latent.hip, attn32.hip) ----
+struct LatentInArgs {            // behind the fused input projection: norms, cache append, gates
+  const float* part = nullptr; int nsplit = 1, rows = 0, ldn = 0;     // fp32 slabs [nsplit][rows][ldn]: query latent | cache latent | gate per head
+  int qp = 0, rp = 0, q_rank = 0, kv_rank = 0, heads = 0; float eps = 0.f;   // padded widths (rp = 0: no latent of its own) and real ranks
+  const bf16_t* q_norm = nullptr; const bf16_t* kv_norm = nullptr;
+  bf16_t* cq = nullptr; float* gate = nullptr;
+  const int32_t* tok_stream = nullptr; const int32_t* tok_pos = nullptr; const int32_t* kv_len = nullptr;   // tok_pos null: kv_len[slot]
+  bf16_t* const* kv_base = nullptr; size_t kv_off = 0;
+};
+int latent_norm_append(const LatentInArgs& a, hipStream_t st);
+int latent_gather(bf16_t* const* kv_base, size_t kv_off, int rp, const int32_t* tile_slot, const int32_t* tile_key0, const int32_t* tile_nkeys,
+                  int n_tiles, bf16_t* rows_out, bf16_t* frag_out, hipStream_t st);
+struct MhaArgs {                 // causal multi-head attention of packed rows over keys [keys][heads dim] and transposed values [heads vdim][ldv]
+  const bf16_t* q = nullptr; const bf16_t* k = nullptr; const bf16_t* vt = nullptr; int ldv = 0;
+  const float* gate = nullptr;   // optional fp32 [rows][heads]: factor of a head's output
+  bf16_t* out = nullptr; int ldo = 0;
+  // groups of up to MHA_GROUP_ROWS consecutive rows of one stream, rows ascending: first row, rows, position of the first row, first key row of the stream
+  const int32_t* grp_q0 = nullptr; const int32_t* grp_nq = nullptr; const int32_t* grp_pos0 = nullptr; const int32_t* grp_key0 = nullptr;
+  int n_groups = 0, rows = 0, heads = 0, dim = 0, vdim = 0; float scale_log2e = 0.f;
+};
+constexpr int MHA_GROUP_ROWS = 256;
+int attn_mha(const MhaArgs& a, hipStream_t st);
+int attn_mha32_launch(const MhaArgs& a, hipStream_t st);      // dim, vdim in {64, 128}
+int latent_absorb(const float* q_part, int nsplit, int rows, int heads, int dim, const bf16_t* ukt, int rp, bf16_t* out, hipStream_t st);
+constexpr int LATENT_MAX_SPLIT = 128;
+struct LatentDecodeArgs {
+  const bf16_t* q = nullptr;     // [rows][heads][rp] absorbed queries
+  int rows = 0, heads = 0, rp = 0, nsplit = 1; float scale_log2e = 0.f;
+  const int32_t* slots = nullptr; const int32_t* kv_len = nullptr; bf16_t* const* kv_base = nullptr; size_t kv_off = 0;
+  float* ws_o = nullptr; float* ws_ml = nullptr;               // [rows][heads][nsplit][rp], [rows][heads][nsplit][2]
+};
+int latent_attn_decode(const LatentDecodeArgs& a, hipStream_t st);
+int latent_merge_uv(const LatentDecodeArgs& a, const bf16_t* uv, int vdim, const float* gate, bf16_t* out, int ldo, hipStream_t st);
 
 }  // namespace lcc

@@ -1,0 +1,429 @@
+// Latent attention without positions (gfx950).  Per token and owning layer the cache holds ONE normed vector c of `rank` values
+// ([Lmax][rank] bf16 per slot, rank padded to a multiple of 64 with zeros); every head's keys and values are linear maps of it:
+//     k_h = Uk_h c,  v_h = Uv_h c,  score = (q_h . k_h) scale
+// Two evaluations of the same sums:
+//   * prefill: k and v of every visible key are formed by two GEMMs per layer and the attention is an ordinary multi-head one
+//     (attn32.hip: attn_mha32_kernel; attn_mha_rows_kernel here for head sizes above 128) -- per (query, key, head) dim + vdim products;
+//   * decode: the key map moves to the query, a_h = Uk_h^T q_h, so that score = (a_h . c) scale and all heads share the cached vector; the
+//     weighted sum of c is mapped through Uv_h once per token -- 2 rank products per (key, head), and the only HBM traffic per key is c.
+// The query and key norms, the scores, the softmax and the gates are fp32; matrix operands are bf16 with fp32 accumulation.
+#include <algorithm>
+#include <cstdlib>
+
+#include "common.h"
+#include "kernels.h"
+
+namespace lcc {
+
+// ------------------------------------------------------------------------------------------------------------------------------
+// One block per new row behind the fused input projection: part = fp32 slabs [nsplit][rows][ldn] with the columns
+//   [0, qp) query latent | [qp, qp + rp) cache latent (rp = 0: the layer reads another layer's cache) | then one gate value per head.
+// Writes the normed query latent (bf16 [rows][qp]), the normed cache latent straight into the slot's arena, and the sigmoid gates (fp32).
+// The padding columns are exact zeros (zero weight rows), so the sums of squares run over the padded widths and divide by the real ones.
+// ------------------------------------------------------------------------------------------------------------------------------
+__global__ __launch_bounds__(256) void latent_norm_append_kernel(LatentInArgs a) {
+  __shared__ float red[2][4];
+  const int row = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const size_t slab = (size_t)a.rows * a.ldn;
+  const float* src = a.part + (size_t)row * a.ldn;
+  auto at = [&](int c) {
+    f32x4 v = *reinterpret_cast<const f32x4*>(src + c);
+    for (int s = 1; s < a.nsplit; ++s) v += *reinterpret_cast<const f32x4*>(src + s * slab + c);
+    return v;
+  };
+  float sq = 0.f, sk = 0.f;
+  for (int c = tid * 4; c < a.qp; c += 1024) { const f32x4 v = at(c); sq += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
+  for (int c = tid * 4; c < a.rp; c += 1024) { const f32x4 v = at(a.qp + c); sk += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
+  sq = wave_sum(sq); sk = wave_sum(sk);
+  if (lane == 0) { red[0][wave] = sq; red[1][wave] = sk; }
+  __syncthreads();
+  sq = (red[0][0] + red[0][1]) + (red[0][2] + red[0][3]);
+  sk = (red[1][0] + red[1][1]) + (red[1][2] + red[1][3]);
+  const float iq = 1.f / sqrtf(sq / (float)a.q_rank + a.eps);
+  for (int c = tid * 4; c < a.qp; c += 1024) {
+    const f32x4 v = at(c);
+    const u32x2 w = ld8(a.q_norm + c);
+    st8(a.cq + (size_t)row * a.qp + c, (u32x2){pack2(v[0] * iq * lo2f(w.x), v[1] * iq * hi2f(w.x)), pack2(v[2] * iq * lo2f(w.y), v[3] * iq * hi2f(w.y))});
+  }
+  if (a.rp > 0) {
+    const float ik = 1.f / sqrtf(sk / (float)a.kv_rank + a.eps);
+    const int slot = a.tok_stream[row];
+    const int pos = a.tok_pos ? a.tok_pos[row] : a.kv_len[slot];
+    bf16_t* dst = a.kv_base[slot] + a.kv_off + (size_t)pos * a.rp;
+    for (int c = tid * 4; c < a.rp; c += 1024) {
+      const f32x4 v = at(a.qp + c);
+      const u32x2 w = ld8(a.kv_norm + c);
+      st8(dst + c, (u32x2){pack2(v[0] * ik * lo2f(w.x), v[1] * ik * hi2f(w.x)), pack2(v[2] * ik * lo2f(w.y), v[3] * ik * hi2f(w.y))});
+    }
+  }
+  for (int h = tid; h < a.heads; h += 256) {
+    float z = src[a.qp + a.rp + h];
+    for (int s = 1; s < a.nsplit; ++s) z += src[s * slab + a.qp + a.rp + h];
+    a.gate[(size_t)row * a.heads + h] = 1.f / (1.f + expf(-z));
+  }
+}
+int latent_norm_append(const LatentInArgs& a, hipStream_t st) {
+  if (a.rows <= 0) return 0;
+  if ((a.qp & 63) || a.qp <= 0 || (a.rp & 63) || a.rp < 0 || a.nsplit < 1 || (a.ldn & 3) || a.ldn < a.qp + a.rp + a.heads) return LCC_ERR_SHAPE;
+  if (!a.part || !a.q_norm || !a.cq || !a.gate || a.q_rank < 1) return LCC_ERR_ARG;
+  if (a.rp > 0 && (!a.kv_norm || !a.tok_stream || (!a.tok_pos && !a.kv_len) || !a.kv_base || a.kv_rank < 1)) return LCC_ERR_ARG;
+  latent_norm_append_kernel<<<dim3(a.rows), dim3(256), 0, st>>>(a);
+  return 0;
+}
+
+// ------------------------------------------------------------------------------------------------------------------------------
+// Prefill: the visible latents of the call's streams, back to back.  16-row tiles (slot, first key, keys of the stream): every stream starts
+// at a multiple of 32 rows and is zero-filled up to the next one.  Written twice: row-major [rows][rp] (A operand of the key GEMM) and in
+// MFMA fragment order (the "weight" operand of the transposed value GEMM).
+// ------------------------------------------------------------------------------------------------------------------------------
+__global__ __launch_bounds__(256) void latent_gather_kernel(bf16_t* const* __restrict__ kv_base, size_t kv_off, int rp,
+                                                            const int32_t* __restrict__ tile_slot, const int32_t* __restrict__ tile_key0,
+                                                            const int32_t* __restrict__ tile_nkeys, bf16_t* __restrict__ rows_out,
+                                                            bf16_t* __restrict__ frag_out, int64_t pieces) {
+  const int per_tile = rp * 2;                 // 16-byte pieces of a 16-row tile
+  for (int64_t p = (int64_t)blockIdx.x * 256 + threadIdx.x; p < pieces; p += (int64_t)gridDim.x * 256) {
+    const int rt = (int)(p / per_tile), q = (int)(p - (int64_t)rt * per_tile);
+    const int kb = q >> 6, g = (q >> 4) & 3, r = q & 15;
+    const int key = tile_key0[rt] + r, col = kb * 32 + g * 8;
+    u32x4 v = {0u, 0u, 0u, 0u};
+    if (key < tile_nkeys[rt]) v = ld16(kv_base[tile_slot[rt]] + kv_off + (size_t)key * rp + col);
+    st16(rows_out + ((size_t)rt * 16 + r) * rp + col, v);
+    st16(frag_out + (size_t)p * 8, v);
+  }
+}
+int latent_gather(bf16_t* const* kv_base, size_t kv_off, int rp, const int32_t* tile_slot, const int32_t* tile_key0, const int32_t* tile_nkeys,
+                  int n_tiles, bf16_t* rows_out, bf16_t* frag_out, hipStream_t st) {
+  if (n_tiles <= 0) return 0;
+  if (rp <= 0 || (rp & 63)) return LCC_ERR_SHAPE;
+  const int64_t pieces = (int64_t)n_tiles * rp * 2;
+  latent_gather_kernel<<<dim3((unsigned)std::min<int64_t>((pieces + 255) / 256, 8192)), dim3(256), 0, st>>>(kv_base, kv_off, rp, tile_slot, tile_key0, tile_nkeys,
+                                                                                                      rows_out, frag_out, pieces);
+  return 0;
+}
+
+// ------------------------------------------------------------------------------------------------------------------------------
+// Causal multi-head attention for head sizes the MFMA kernel does not serve: one block per (row, head), 256 keys at a time, one key per
+// thread for the scores and one channel per thread for the values.
+// ------------------------------------------------------------------------------------------------------------------------------
+__global__ __launch_bounds__(256) void attn_mha_rows_kernel(MhaArgs a) {
+  __shared__ float s_p[256], red[4];
+  extern __shared__ float s_qf[];
+  const int row = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  // the group of this row
+  int lo = 0, hi = a.n_groups - 1;
+  while (lo < hi) { const int mid = (lo + hi + 1) >> 1; if (a.grp_q0[mid] <= row) lo = mid; else hi = mid - 1; }
+  const int nkeys = a.grp_pos0[lo] + (row - a.grp_q0[lo]) + 1, kb = a.grp_key0[lo];
+  const int ldq = a.heads * a.dim;
+  for (int d = tid; d < a.dim; d += 256) s_qf[d] = bf2f(a.q[(size_t)row * ldq + h * a.dim + d]);
+  __syncthreads();
+  float m = -INFINITY, l = 0.f, o[4] = {0.f, 0.f, 0.f, 0.f};        // vdim <= 1024
+  for (int k0 = 0; k0 < nkeys; k0 += 256) {
+    const int key = k0 + tid;
+    float s = -INFINITY;
+    if (key < nkeys) {
+      const bf16_t* kp = a.k + (size_t)(kb + key) * ldq + h * a.dim;
+      float acc = 0.f;
+      for (int d = 0; d < a.dim; d += 8) {
+        const u32x4 v = ld16(kp + d);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc = fmaf(s_qf[d + 2 * e], lo2f(v[e]), fmaf(s_qf[d + 2 * e + 1], hi2f(v[e]), acc));
+      }
+      s = acc * a.scale_log2e;
+    }
+    const float wm = wave_max(s);
+    if (lane == 0) red[wave] = wm;
+    __syncthreads();
+    const float mn = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), m);
+    const float alpha = exp2f(m - mn), p = exp2f(s - mn);           // s = -inf -> 0
+    m = mn;
+    s_p[tid] = p;
+    __syncthreads();
+    const float ws = wave_sum(p);
+    if (lane == 0) red[wave] = ws;
+    __syncthreads();
+    l = l * alpha + (red[0] + red[1]) + (red[2] + red[3]);
+    const int n = min(256, nkeys - k0);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int d = tid + 256 * j;
+      if (d < a.vdim) {
+        const bf16_t* vp = a.vt + (size_t)(h * a.vdim + d) * a.ldv + kb + k0;
+        float acc = 0.f;
+        for (int i = 0; i < n; ++i) acc = fmaf(s_p[i], bf2f(vp[i]), acc);
+        o[j] = o[j] * alpha + acc;
+      }
+    }
+    __syncthreads();
+  }
+  const float f = (a.gate ? a.gate[(size_t)row * a.heads + h] : 1.f) / l;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int d = tid + 256 * j;
+    if (d < a.vdim) a.out[(size_t)row * a.ldo + h * a.vdim + d] = f2bf(o[j] * f);
+  }
+}
+static int mha_rows(const MhaArgs& a, hipStream_t st) {
+  attn_mha_rows_kernel<<<dim3(a.rows, a.heads), dim3(256), (size_t)a.dim * 4, st>>>(a);
+  return 0;
+}
+int attn_mha(const MhaArgs& a, hipStream_t st) {
+  if (a.rows <= 0 || a.n_groups <= 0) return 0;
+  if (a.heads < 1 || a.dim < 8 || (a.dim & 7) || a.dim > 8192 || a.vdim < 1 || a.vdim > 1024 || (a.ldv & 31) || (a.ldo & 3)) return LCC_ERR_SHAPE;
+  if (!a.q || !a.k || !a.vt || !a.out || !a.grp_q0 || !a.grp_nq || !a.grp_pos0 || !a.grp_key0) return LCC_ERR_ARG;
+  if ((a.dim == 64 || a.dim == 128) && (a.vdim == 64 || a.vdim == 128)) return attn_mha32_launch(a, st);
+  return mha_rows(a, st);
+}
+
+// ------------------------------------------------------------------------------------------------------------------------------
+// Decode, step 1: a_h = Uk_h^T q_h for every head and row.  q arrives as the fp32 slabs of the query up-projection; the block's 16 rows are
+// summed and rounded once.  grid (rank / 64, heads, row groups); wave w owns 16 rank rows; D'[r][row]: a lane stores 4 consecutive r.
+// ------------------------------------------------------------------------------------------------------------------------------
+__global__ __launch_bounds__(256) void latent_absorb_kernel(const float* __restrict__ q_part, int nsplit, int rows, int heads, int dim,
+                                                            const bf16_t* __restrict__ ukt, int rp, bf16_t* __restrict__ out) {
+  extern __shared__ __attribute__((aligned(16))) bf16_t s_q[];       // [16][dim + 8]
+  const int h = blockIdx.y, b0 = blockIdx.z * 16, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, g = lane >> 4;
+  const int pitch = dim + 8, ldq = heads * dim, K32 = dim >> 5;
+  const size_t slab = (size_t)rows * ldq;
+  const int rt = h * (rp >> 4) + blockIdx.x * 4 + wave;              // 16-row tile of the stacked Uk^T
+  const bf16_t* wp = ukt + (size_t)rt * K32 * 512 + lane * 8;
+  u32x4 w0 = ld16(wp), w1 = ld16(wp + 512);                          // dim is a multiple of 64: in flight while q is summed
+  const int nrow = min(16, rows - b0);
+  for (int i = tid * 4; i < nrow * dim; i += 1024) {
+    const int r = i / dim, d = i - r * dim;
+    const float* p = q_part + (size_t)(b0 + r) * ldq + h * dim + d;
+    f32x4 v = *reinterpret_cast<const f32x4*>(p);
+    for (int s = 1; s < nsplit; ++s) v += *reinterpret_cast<const f32x4*>(p + s * slab);
+    st8(s_q + r * pitch + d, (u32x2){pack2(v[0], v[1]), pack2(v[2], v[3])});
+  }
+  __syncthreads();
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  const bf16_t* xq = s_q + min(li, nrow - 1) * pitch + g * 8;
+  for (int k = 0; k < K32; k += 2) {
+    acc = mfma16(as_bf16x8(w0), as_bf16x8(ld16(xq + k * 32)), acc);
+    acc = mfma16(as_bf16x8(w1), as_bf16x8(ld16(xq + k * 32 + 32)), acc);
+    if (k + 2 < K32) { w0 = ld16(wp + (size_t)(k + 2) * 512); w1 = ld16(wp + (size_t)(k + 3) * 512); }
+  }
+  if (li < nrow)
+    st8(out + ((size_t)(b0 + li) * heads + h) * rp + (blockIdx.x * 4 + wave) * 16 + g * 4, (u32x2){pack2(acc[0], acc[1]), pack2(acc[2], acc[3])});
+}
+int latent_absorb(const float* q_part, int nsplit, int rows, int heads, int dim, const bf16_t* ukt, int rp, bf16_t* out, hipStream_t st) {
+  if (rows <= 0) return 0;
+  if (nsplit < 1 || heads < 1 || (dim & 63) || dim < 64 || dim > 1024 || (rp & 63) || rp < 64) return LCC_ERR_SHAPE;
+  if (!q_part || !ukt || !out) return LCC_ERR_ARG;
+  latent_absorb_kernel<<<dim3(rp / 64, heads, (rows + 15) / 16), dim3(256), (size_t)16 * (dim + 8) * 2, st>>>(q_part, nsplit, rows, heads, dim, ukt, rp, out);
+  return 0;
+}
+
+// ------------------------------------------------------------------------------------------------------------------------------
+// Decode, step 2: attention over the cached latents, all heads of a row together.  rank = 64 RT.
+// Block = quads of 4 waves, one quad per 16 heads; 64 keys per iteration, staged once for all quads by LDS-DMA in MFMA fragment order
+// (1-KB pieces = 16 keys x 32 channels), double buffered.  Per iteration a wave multiplies its 16 keys with its quad's 16 queries
+// (S^T[key][head]: a lane owns 4 keys of one head), the quad agrees on the new maxima through LDS, and then each wave adds
+// C^T . P^T for its quarter of the channels (O^T[channel][head]: again one head per lane, so the rescale factor is lane-local).  The
+// C^T operand -- 8 keys of one channel per lane -- comes out of the same LDS image through ds_read_b64_tr_b16, which transposes 4 x 16
+// 16-bit blocks: in a group of 16 lanes, lane l supplies 4 consecutive channels of key l / 4 and receives channel l of 4 consecutive keys.
+// grid (splits, rows, head groups); partial (O, m, l) of every split as fp32.
+// ------------------------------------------------------------------------------------------------------------------------------
+typedef __attribute__((ext_vector_type(4))) short s16x4;
+LCC_DEVICE u32x2 lds_tr4x16(const void* p) {
+  return __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)(p)));
+}
+constexpr int LATENT_PP = 72;      // pitch of a head's 64 probabilities in LDS (16-byte aligned, spreads the banks)
+
+template <int RT, int NSTAGE>
+__global__ __launch_bounds__(RT >= 8 ? 512 : 1024) void latent_attn_decode_kernel(LatentDecodeArgs a) {
+  constexpr int RP = RT * 64, KB = RT * 2, NP = 4 * KB;              // channels, 32-channel blocks, pieces per 64-key tile
+  extern __shared__ __attribute__((aligned(16))) u32x4 lmem[];       // NSTAGE x NP pieces, then P, then the statistics
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), li = lane & 15, g = lane >> 4;
+  const int quad = wave >> 2, wq = wave & 3, nw = blockDim.x >> 6, nquad = nw >> 2;
+  bf16_t* s_p = reinterpret_cast<bf16_t*>(lmem + NSTAGE * NP * 64) + quad * 16 * LATENT_PP;
+  float* s_m = reinterpret_cast<float*>(reinterpret_cast<bf16_t*>(lmem + NSTAGE * NP * 64) + nquad * 16 * LATENT_PP) + quad * 64;
+  const int split = blockIdx.x, b = blockIdx.y;
+  const int head = (blockIdx.z * nquad + quad) * 16 + li;
+  const int slot = a.slots[b];
+  const int n = a.kv_len[slot] + 1;                                  // cached keys and the token of this step
+  const int ntile = (n + 63) >> 6, per = (ntile + a.nsplit - 1) / a.nsplit;
+  const int tb = split * per, te = min(ntile, tb + per);
+  if (tb >= te) return;                                              // the merge knows which splits exist
+  const bf16_t* cbase = a.kv_base[slot] + a.kv_off;
+
+  u32x4 qf[KB];                                                      // B operand: q[head][32 ks + 8 g ..]
+  {
+    const bf16_t* qp = a.q + ((size_t)b * a.heads + min(head, a.heads - 1)) * RP + g * 8;
+#pragma unroll
+    for (int ks = 0; ks < KB; ++ks) qf[ks] = ld16(qp + ks * 32);
+#pragma unroll
+    for (int ks = 0; ks < KB; ++ks) settle_load(qf[ks]);
+  }
+  auto issue = [&](int t, int stage) {
+    for (int p = wave; p < NP; p += nw) {
+      const int kt = p / KB, kb = p - kt * KB;
+      glds16(cbase + (size_t)(t * 64 + kt * 16 + li) * RP + kb * 32 + g * 8, lds_addr(lmem + (stage * NP + p) * 64));
+    }
+  };
+  f32x4 o[RT];
+#pragma unroll
+  for (int j = 0; j < RT; ++j) o[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  float m_run = -INFINITY, l_run = 0.f;
+
+  issue(tb, 0);
+  for (int t = tb; t < te; ++t) {
+    const int stage = NSTAGE == 2 ? ((t - tb) & 1) : 0;
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();                                                 // tile t is complete; everyone is done with tile t - 1
+    if (NSTAGE == 2 && t + 1 < te) issue(t + 1, stage ^ 1);
+    const u32x4* cs = lmem + stage * NP * 64;
+    f32x4 s = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < KB; ++ks) s = mfma16(as_bf16x8(cs[(wq * KB + ks) * 64 + lane]), as_bf16x8(qf[ks]), s);
+    const int k0 = t * 64 + wq * 16 + g * 4;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) s[r] = k0 + r < n ? s[r] * a.scale_log2e : -INFINITY;
+    float mx = fmaxf(fmaxf(s[0], s[1]), fmaxf(s[2], s[3]));
+    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    if (g == 0) s_m[wq * 16 + li] = mx;
+    __syncthreads();
+    const float m_new = fmaxf(fmaxf(fmaxf(s_m[li], s_m[16 + li]), fmaxf(s_m[32 + li], s_m[48 + li])), m_run);   // finite: a tile has >= 1 key
+    const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
+    m_run = m_new;
+    float p[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) p[r] = __builtin_amdgcn_exp2f(s[r] - m_new);
+    l_run = l_run * alpha + ((p[0] + p[1]) + (p[2] + p[3]));
+    st8(s_p + li * LATENT_PP + wq * 16 + g * 4, (u32x2){pack2(p[0], p[1]), pack2(p[2], p[3])});
+    __syncthreads();
+    const u32x4 pf0 = ld16(s_p + li * LATENT_PP + g * 8), pf1 = ld16(s_p + li * LATENT_PP + 32 + g * 8);
+#pragma unroll
+    for (int j = 0; j < RT; ++j) {
+      const int r = wq * (16 * RT) + j * 16 + (li & 3) * 4;          // this lane's source channels
+      const char* base = reinterpret_cast<const char*>(cs) + (r >> 5) * 1024 + ((r >> 3) & 3) * 256 + (r & 7) * 2;
+      f32x4 acc = o[j] * alpha;
+#pragma unroll
+      for (int ks = 0; ks < 2; ++ks) {
+        const int key = ks * 32 + g * 8 + (li >> 2);                 // and + 4 for the second half
+        const u32x2 lo = lds_tr4x16(base + (key >> 4) * (KB * 1024) + (key & 15) * 16);
+        const u32x2 hi = lds_tr4x16(base + (key >> 4) * (KB * 1024) + ((key & 15) + 4) * 16);
+        acc = mfma16(as_bf16x8((u32x4){lo.x, lo.y, hi.x, hi.y}), as_bf16x8(ks == 0 ? pf0 : pf1), acc);
+      }
+      o[j] = acc;
+    }
+    if (NSTAGE == 1 && t + 1 < te) { __syncthreads(); issue(t + 1, 0); }
+  }
+  // the quad's denominators: over the lane groups of a wave, then over its four waves
+  l_run += __shfl_xor(l_run, 16, 64);
+  l_run += __shfl_xor(l_run, 32, 64);
+  __syncthreads();
+  if (g == 0) s_m[wq * 16 + li] = l_run;
+  __syncthreads();
+  if (head >= a.heads) return;
+  const size_t pslot = ((size_t)b * a.heads + head) * a.nsplit + split;
+  if (wq == 0 && g == 0) {
+    a.ws_ml[pslot * 2] = m_run;
+    a.ws_ml[pslot * 2 + 1] = (s_m[li] + s_m[16 + li]) + (s_m[32 + li] + s_m[48 + li]);
+  }
+  float* op = a.ws_o + pslot * RP + wq * (16 * RT) + g * 4;
+#pragma unroll
+  for (int j = 0; j < RT; ++j) *reinterpret_cast<f32x4*>(op + j * 16) = o[j];
+}
+
+template <int RT>
+static void latent_decode_go(const LatentDecodeArgs& a, hipStream_t st) {
+  constexpr int NSTAGE = RT > 8 ? 1 : 2, MAXQ = RT >= 8 ? 2 : 4;
+  const int ht = (a.heads + 15) / 16, groups = (ht + MAXQ - 1) / MAXQ, quads = (ht + groups - 1) / groups;
+  const size_t lds = (size_t)NSTAGE * 8 * RT * 1024 + (size_t)quads * (16 * LATENT_PP * 2 + 256);
+  static DeviceOnce once;   // per instantiation
+  if (once.first())
+    (void)hipFuncSetAttribute((const void*)latent_attn_decode_kernel<RT, NSTAGE>, hipFuncAttributeMaxDynamicSharedMemorySize,
+                              (int)((size_t)NSTAGE * 8 * RT * 1024 + (size_t)MAXQ * (16 * LATENT_PP * 2 + 256)));
+  latent_attn_decode_kernel<RT, NSTAGE><<<dim3(a.nsplit, a.rows, groups), dim3(quads * 256), lds, st>>>(a);
+}
+int latent_attn_decode(const LatentDecodeArgs& a, hipStream_t st) {
+  if (a.rows <= 0) return 0;
+  if (a.heads < 1 || a.nsplit < 1 || a.nsplit > LATENT_MAX_SPLIT || a.rows > 65535) return LCC_ERR_SHAPE;
+  if (!a.q || !a.slots || !a.kv_len || !a.kv_base || !a.ws_o || !a.ws_ml) return LCC_ERR_ARG;
+  switch (a.rp) {      // the padded ranks (config.py: pad_kv_rank)
+    case 64: latent_decode_go<1>(a, st); break;
+    case 128: latent_decode_go<2>(a, st); break;
+    case 192: latent_decode_go<3>(a, st); break;
+    case 256: latent_decode_go<4>(a, st); break;
+    case 384: latent_decode_go<6>(a, st); break;
+    case 512: latent_decode_go<8>(a, st); break;
+    case 768: latent_decode_go<12>(a, st); break;
+    case 1024: latent_decode_go<16>(a, st); break;
+    default: return LCC_ERR_SHAPE;
+  }
+  return 0;
+}
+
+// ------------------------------------------------------------------------------------------------------------------------------
+// Decode, step 3: merge the splits, map the weighted latent through Uv_h, apply the head's gate.  grid (vdim / 64, heads, row groups).
+// ------------------------------------------------------------------------------------------------------------------------------
+// The wave's Uv fragments are requested before the merge, which hides their latency (rank <= 512; above, in two batches).
+template <int RT>
+__global__ __launch_bounds__(256) void latent_merge_uv_kernel(LatentDecodeArgs a, const bf16_t* __restrict__ uv, int vdim,
+                                                              const float* __restrict__ gate, bf16_t* __restrict__ out, int ldo) {
+  extern __shared__ __attribute__((aligned(16))) bf16_t s_o[];       // [16][rp + 8]
+  __shared__ float s_w[4][LATENT_MAX_SPLIT];
+  const int h = blockIdx.y, b0 = blockIdx.z * 16, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, g = lane >> 4;
+  constexpr int rp = RT * 64, pitch = rp + 8, KB = RT * 2, KW = KB > 16 ? KB / 2 : KB;
+  const int nrow = min(16, a.rows - b0);
+  const int v0 = (blockIdx.x * 4 + wave) * 16;
+  const bf16_t* wp = uv + (size_t)(h * vdim + v0 + li) * rp + g * 8;
+  u32x4 wf[KW];
+#pragma unroll
+  for (int k = 0; k < KW; ++k) wf[k] = ld16(wp + k * 32);
+  for (int r = wave; r < nrow; r += 4) {                             // a wave merges whole rows
+    const int b = b0 + r;
+    const int n = a.kv_len[a.slots[b]] + 1, ntile = (n + 63) >> 6, per = (ntile + a.nsplit - 1) / a.nsplit;
+    const int live = (ntile + per - 1) / per;                        // splits that ran
+    const size_t p0 = ((size_t)b * a.heads + h) * a.nsplit;
+    float m = -INFINITY;
+    for (int s = lane; s < live; s += 64) m = fmaxf(m, a.ws_ml[(p0 + s) * 2]);
+    m = wave_max(m);
+    float l = 0.f;
+    for (int s = lane; s < live; s += 64) {
+      const float e = __builtin_amdgcn_exp2f(a.ws_ml[(p0 + s) * 2] - m);
+      s_w[wave][s] = e;
+      l += e * a.ws_ml[(p0 + s) * 2 + 1];
+    }
+    const float inv = 1.f / wave_sum(l);
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");           // one wave, in-order LDS: the lanes' weights are visible to all lanes
+    __builtin_amdgcn_wave_barrier();
+    for (int c = lane * 4; c < rp; c += 256) {
+      f32x4 v = {0.f, 0.f, 0.f, 0.f};
+      for (int s = 0; s < live; ++s) v += *reinterpret_cast<const f32x4*>(a.ws_o + (p0 + s) * rp + c) * s_w[wave][s];
+      st8(s_o + r * pitch + c, (u32x2){pack2(v[0] * inv, v[1] * inv), pack2(v[2] * inv, v[3] * inv)});
+    }
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+  }
+  __syncthreads();
+  const bf16_t* xp = s_o + min(li, nrow - 1) * pitch + g * 8;
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int k = 0; k < KB; ++k) {
+    acc = mfma16(as_bf16x8(wf[k % KW]), as_bf16x8(ld16(xp + k * 32)), acc);
+    if (k + KW < KB) wf[k % KW] = ld16(wp + (k + KW) * 32);
+  }
+  if (li < nrow) {
+    const float f = gate ? gate[(size_t)(b0 + li) * a.heads + h] : 1.f;
+    st8(out + (size_t)(b0 + li) * ldo + h * vdim + v0 + g * 4, (u32x2){pack2(acc[0] * f, acc[1] * f), pack2(acc[2] * f, acc[3] * f)});
+  }
+}
+int latent_merge_uv(const LatentDecodeArgs& a, const bf16_t* uv, int vdim, const float* gate, bf16_t* out, int ldo, hipStream_t st) {
+  if (a.rows <= 0) return 0;
+  if ((vdim & 63) || vdim < 64 || (a.rp & 63) || a.rp < 64 || a.rp > 1024 || (ldo & 3) || a.nsplit > LATENT_MAX_SPLIT || a.nsplit < 1) return LCC_ERR_SHAPE;
+  if (!uv || !out || !a.ws_o || !a.ws_ml || !a.slots || !a.kv_len) return LCC_ERR_ARG;
+  const dim3 grid(vdim / 64, a.heads, (a.rows + 15) / 16);
+  const size_t lds = (size_t)16 * (a.rp + 8) * 2;
+#define LCC_MERGE(RT) case RT * 64: latent_merge_uv_kernel<RT><<<grid, dim3(256), lds, st>>>(a, uv, vdim, gate, out, ldo); break
+  switch (a.rp) {
+    LCC_MERGE(1); LCC_MERGE(2); LCC_MERGE(3); LCC_MERGE(4); LCC_MERGE(6); LCC_MERGE(8); LCC_MERGE(12); LCC_MERGE(16);
+    default: return LCC_ERR_SHAPE;
+  }
+#undef LCC_MERGE
+  return 0;
+}
+
+}  // namespace lcc

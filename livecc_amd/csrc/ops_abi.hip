@@ -360,7 +360,7 @@ extern "C" int lcc_sample_greedy(const void* logits, int ld, int B, int V, uint3
                                  int suppress_eos, int32_t* done, int32_t* out_tokens, int32_t* history, int hist_ld,
                                  int32_t* hist_col, float* scores_out, float* ws, void* stream) {
   if (!logits || !seen || !stream_slot || !out_tokens || (history && !hist_col)) return fail(LCC_ERR_ARG, "null pointer");
-  OP_RET(sample_greedy((const bf16_t*)logits, ld, B, V, seen, words_per_stream, stream_slot, repetition_penalty, thr_token, use_thr,
+  OP_RET(sample_greedy(logits, false, ld, B, V, seen, words_per_stream, stream_slot, repetition_penalty, thr_token, use_thr,
                        thr_value, eos_token, eos_token2, suppress_eos, done, out_tokens, history, hist_ld, hist_col, scores_out, ws,
                        (hipStream_t)stream), "lcc_sample_greedy");
 }
@@ -370,7 +370,57 @@ extern "C" int lcc_sample_topk_topp(const void* logits, int ld, int B, int V, ui
                                     int32_t* history, int hist_ld, int32_t* hist_col, float* scores_out, float temperature, int top_k,
                                     float top_p, uint64_t seed, uint32_t* rng_ctr, void* stream) {
   if (!logits || !seen || !stream_slot || !out_tokens || (history && !hist_col)) return fail(LCC_ERR_ARG, "null pointer");
-  OP_RET(sample_topk_topp((const bf16_t*)logits, ld, B, V, seen, words_per_stream, stream_slot, repetition_penalty, thr_token, use_thr,
+  OP_RET(sample_topk_topp(logits, false, ld, B, V, seen, words_per_stream, stream_slot, repetition_penalty, thr_token, use_thr,
                           thr_value, eos_token, eos_token2, suppress_eos, done, out_tokens, history, hist_ld, hist_col, scores_out,
                           temperature, top_k, top_p, seed, rng_ctr, (hipStream_t)stream), "lcc_sample_topk_topp");
+}
+
+// ---- layer-list decoders / latent attention ----
+extern "C" int lcc_embed_dyt(const int32_t* ids, const int32_t* indirect, const void* table, const void* norm_w, const void* norm_b, const void* alpha,
+                             float* x, void* h, int rows, int dim, void* stream) {
+  OP_RET(embed_dyt(ids, indirect, (const bf16_t*)table, DytNorm{(const bf16_t*)norm_w, (const bf16_t*)norm_b, (const bf16_t*)alpha}, x, (bf16_t*)h, rows, dim,
+                   (hipStream_t)stream), "lcc_embed_dyt");
+}
+extern "C" int lcc_resid_dyt(float* x, const float* partial, int nsplit, const void* norm_w, const void* norm_b, const void* alpha, void* h, int rows,
+                             int dim, void* stream) {
+  OP_RET(resid_dyt(x, partial, nsplit, DytNorm{(const bf16_t*)norm_w, (const bf16_t*)norm_b, (const bf16_t*)alpha}, (bf16_t*)h, rows, dim, (hipStream_t)stream),
+         "lcc_resid_dyt");
+}
+extern "C" int lcc_logits_cap(const float* partial, int nsplit, int rows, int ld, int vocab, float cap, float* out, float* dense, void* stream) {
+  OP_RET(logits_cap(partial, nsplit, rows, ld, vocab, cap, out, dense, (hipStream_t)stream), "lcc_logits_cap");
+}
+extern "C" int lcc_latent_norm_append(const float* partial, int nsplit, int rows, int ldn, int q_rank, int q_rank_pad, const void* q_norm, int kv_rank,
+                                      int kv_rank_pad, const void* kv_norm, int heads, float eps, const int32_t* tok_stream, const int32_t* tok_pos,
+                                      const int32_t* kv_len, void* const* kv_base, int64_t kv_offset, void* cq_out, float* gate_out, void* stream) {
+  LatentInArgs a; a.part = partial; a.nsplit = nsplit; a.rows = rows; a.ldn = ldn; a.qp = q_rank_pad; a.rp = kv_rank_pad; a.q_rank = q_rank; a.kv_rank = kv_rank;
+  a.heads = heads; a.eps = eps; a.q_norm = (const bf16_t*)q_norm; a.kv_norm = (const bf16_t*)kv_norm; a.cq = (bf16_t*)cq_out; a.gate = gate_out;
+  a.tok_stream = tok_stream; a.tok_pos = tok_pos; a.kv_len = kv_len; a.kv_base = (bf16_t* const*)kv_base; a.kv_off = (size_t)kv_offset;
+  OP_RET(latent_norm_append(a, (hipStream_t)stream), "lcc_latent_norm_append");
+}
+extern "C" int lcc_latent_gather(void* const* kv_base, int64_t kv_offset, int kv_rank_pad, const int32_t* tile_slot, const int32_t* tile_key0,
+                                 const int32_t* tile_nkeys, int n_tiles, void* rows_out, void* packed_out, void* stream) {
+  if (n_tiles > 0 && (!kv_base || !tile_slot || !tile_key0 || !tile_nkeys || !rows_out || !packed_out)) return fail(LCC_ERR_ARG, "lcc_latent_gather: null pointer");
+  OP_RET(latent_gather((bf16_t* const*)kv_base, (size_t)kv_offset, kv_rank_pad, tile_slot, tile_key0, tile_nkeys, n_tiles, (bf16_t*)rows_out,
+                       (bf16_t*)packed_out, (hipStream_t)stream), "lcc_latent_gather");
+}
+extern "C" int lcc_attn_mha(const void* q, const void* k, const void* vt, int ldv, const float* gate, void* out, int ldo, const int32_t* grp_q0,
+                            const int32_t* grp_nq, const int32_t* grp_pos0, const int32_t* grp_key0, int n_groups, int rows, int heads, int dim, int vdim,
+                            float scale, void* stream) {
+  MhaArgs a; a.q = (const bf16_t*)q; a.k = (const bf16_t*)k; a.vt = (const bf16_t*)vt; a.ldv = ldv; a.gate = gate; a.out = (bf16_t*)out; a.ldo = ldo;
+  a.grp_q0 = grp_q0; a.grp_nq = grp_nq; a.grp_pos0 = grp_pos0; a.grp_key0 = grp_key0; a.n_groups = n_groups; a.rows = rows; a.heads = heads; a.dim = dim;
+  a.vdim = vdim; a.scale_log2e = scale * 1.4426950408889634f;
+  OP_RET(attn_mha(a, (hipStream_t)stream), "lcc_attn_mha");
+}
+extern "C" int lcc_latent_absorb(const float* q_partial, int nsplit, int rows, int heads, int dim, const void* ukt_packed, int kv_rank_pad, void* out,
+                                 void* stream) {
+  OP_RET(latent_absorb(q_partial, nsplit, rows, heads, dim, (const bf16_t*)ukt_packed, kv_rank_pad, (bf16_t*)out, (hipStream_t)stream), "lcc_latent_absorb");
+}
+extern "C" int lcc_latent_attn_decode(const void* q_latent, const int32_t* slots, const int32_t* kv_len, void* const* kv_base, int64_t kv_offset, int rows,
+                                      int heads, int kv_rank_pad, float scale, int nsplit, float* ws_o, float* ws_ml, const void* uv, int vdim,
+                                      const float* gate, void* out, int ldo, void* stream) {
+  LatentDecodeArgs a; a.q = (const bf16_t*)q_latent; a.rows = rows; a.heads = heads; a.rp = kv_rank_pad; a.nsplit = nsplit;
+  a.scale_log2e = scale * 1.4426950408889634f; a.slots = slots; a.kv_len = kv_len; a.kv_base = (bf16_t* const*)kv_base; a.kv_off = (size_t)kv_offset;
+  a.ws_o = ws_o; a.ws_ml = ws_ml;
+  if (int r = latent_attn_decode(a, (hipStream_t)stream)) return fail(r, "lcc_latent_attn_decode: invalid arguments (%d)", r);
+  OP_RET(latent_merge_uv(a, (const bf16_t*)uv, vdim, gate, (bf16_t*)out, ldo, (hipStream_t)stream), "lcc_latent_attn_decode");
 }

@@ -36,12 +36,24 @@ int seen_set(uint32_t* seen, int words_per_stream, const int32_t* ids, const int
   return 0;
 }
 
+// 8 logits of chunk c: bf16 (one 16-byte load) or fp32
+LCC_DEVICE void load8_logits(const bf16_t* lg, int c, float (&v)[8]) {
+  const u32x4 q = ld16(lg + c * 8);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) { v[2 * e] = lo2f(q[e]); v[2 * e + 1] = hi2f(q[e]); }
+}
+LCC_DEVICE void load8_logits(const float* lg, int c, float (&v)[8]) {
+  const f32x4 a = *reinterpret_cast<const f32x4*>(lg + c * 8), b = *reinterpret_cast<const f32x4*>(lg + c * 8 + 4);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) { v[e] = a[e]; v[4 + e] = b[e]; }
+}
+
 struct Best { float v; int i; };
 LCC_DEVICE Best better(Best a, Best b) { return (b.v > a.v || (b.v == a.v && b.i < a.i)) ? b : a; }
 
-template <int NT>
+template <int NT, class LT>
 __global__ __launch_bounds__(NT) void sample_greedy_kernel(
-    const bf16_t* __restrict__ logits, int ld, int V, uint32_t* __restrict__ seen, int words,
+    const LT* __restrict__ logits, int ld, int V, uint32_t* __restrict__ seen, int words,
     const int32_t* __restrict__ stream_slot, float penalty, int thr_token, int use_thr, float thr_value,
     int eos_token, int eos_token2, int suppress_eos, int32_t* __restrict__ done,
     int32_t* __restrict__ out_tokens, int32_t* __restrict__ history, int hist_ld, int32_t* __restrict__ hist_col,
@@ -51,18 +63,16 @@ __global__ __launch_bounds__(NT) void sample_greedy_kernel(
   const int b = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int slot = stream_slot[b];
   if (done != nullptr && done[slot]) return;  // this stream already emitted EOS in this generate call
-  const bf16_t* lg = logits + (size_t)b * ld;
+  const LT* lg = logits + (size_t)b * ld;
   const uint32_t* sb = seen + (size_t)slot * words;
   float* so = scores_out ? scores_out + (size_t)b * V : nullptr;
 
   Best best = {-INFINITY, 0x7fffffff};
   float mx = -INFINITY, sum = 0.f, thr_score = -INFINITY;
   for (int c = tid; c * 8 < V; c += NT) {  // V % 8 == 0
-    const u32x4 q = ld16(lg + c * 8);
     const uint32_t bits = (sb[c >> 2] >> ((c & 3) * 8)) & 0xffu;
     float v[8];
-#pragma unroll
-    for (int e = 0; e < 4; ++e) { v[2 * e] = lo2f(q[e]); v[2 * e + 1] = hi2f(q[e]); }
+    load8_logits(lg, c, v);
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
       if (penalty != 1.0f && ((bits >> e) & 1u)) v[e] = v[e] < 0.f ? v[e] * penalty : v[e] / penalty;
@@ -122,8 +132,9 @@ __global__ __launch_bounds__(NT) void sample_greedy_kernel(
 // ---- two-stage variant: stage 1 spreads the V-wide pass over SAMPLE_NB blocks per stream, stage 2 merges the partials
 constexpr int SAMPLE_NB = 32;
 
+template <class LT>
 __global__ __launch_bounds__(256) void sample_partial_kernel(
-    const bf16_t* __restrict__ logits, int ld, int V, const uint32_t* __restrict__ seen, int words,
+    const LT* __restrict__ logits, int ld, int V, const uint32_t* __restrict__ seen, int words,
     const int32_t* __restrict__ stream_slot, float penalty, int thr_token, int eos_token, int eos_token2, int suppress_eos,
     const int32_t* __restrict__ done, float* __restrict__ part, float* __restrict__ scores_out) {
   __shared__ float s_max[4], s_sum[4], s_bv[4], s_thr[4];
@@ -131,7 +142,7 @@ __global__ __launch_bounds__(256) void sample_partial_kernel(
   const int b = blockIdx.y, blk = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int slot = stream_slot[b];
   if (done != nullptr && done[slot]) return;
-  const bf16_t* lg = logits + (size_t)b * ld;
+  const LT* lg = logits + (size_t)b * ld;
   const uint32_t* sb = seen + (size_t)slot * words;
   float* so = scores_out ? scores_out + (size_t)b * V : nullptr;
   const int nch = V / 8, per = (nch + SAMPLE_NB - 1) / SAMPLE_NB;
@@ -139,11 +150,9 @@ __global__ __launch_bounds__(256) void sample_partial_kernel(
   Best best = {-INFINITY, 0x7fffffff};
   float mx = -INFINITY, sum = 0.f, thr_score = -INFINITY;
   for (int c = c0 + tid; c < c1; c += 256) {
-    const u32x4 q = ld16(lg + c * 8);
     const uint32_t bits = (sb[c >> 2] >> ((c & 3) * 8)) & 0xffu;
     float v[8];
-#pragma unroll
-    for (int e = 0; e < 4; ++e) { v[2 * e] = lo2f(q[e]); v[2 * e + 1] = hi2f(q[e]); }
+    load8_logits(lg, c, v);
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
       if (penalty != 1.0f && ((bits >> e) & 1u)) v[e] = v[e] < 0.f ? v[e] * penalty : v[e] / penalty;
@@ -219,23 +228,34 @@ __global__ __launch_bounds__(64) void sample_final_kernel(
 
 // suppress_eos: bit 0 = both EOS ids are masked to -inf (MinNewTokensLengthLogitsProcessor); bit 1 = a picked EOS does not set done[slot]
 // (teacher forcing: the forced stream decides where a slot ends, and the processed scores keep HF's definition -- EOS unmasked)
-int sample_greedy(const bf16_t* logits, int ld, int B, int V, uint32_t* seen, int words_per_stream,
-                  const int32_t* stream_slot, float repetition_penalty, int thr_token, int use_thr, float thr_value,
-                  int eos_token, int eos_token2, int suppress_eos, int32_t* done, int32_t* out_tokens, int32_t* history, int hist_ld,
-                  int32_t* hist_col, float* scores_out, float* ws, hipStream_t st) {
+template <class LT>
+static int sample_greedy_t(const LT* logits, int ld, int B, int V, uint32_t* seen, int words_per_stream,
+                           const int32_t* stream_slot, float repetition_penalty, int thr_token, int use_thr, float thr_value,
+                           int eos_token, int eos_token2, int suppress_eos, int32_t* done, int32_t* out_tokens, int32_t* history, int hist_ld,
+                           int32_t* hist_col, float* scores_out, float* ws, hipStream_t st) {
   if (B <= 0) return 0;
   if ((V & 31) || (ld & 7) || words_per_stream * 32 < V) return LCC_ERR_SHAPE;
   if (ws != nullptr && V >= 8192) {   // ws: B * 32 * 8 floats of scratch
-    sample_partial_kernel<<<dim3(SAMPLE_NB, B), dim3(256), 0, st>>>(logits, ld, V, seen, words_per_stream, stream_slot, repetition_penalty,
+    sample_partial_kernel<LT><<<dim3(SAMPLE_NB, B), dim3(256), 0, st>>>(logits, ld, V, seen, words_per_stream, stream_slot, repetition_penalty,
                                                                    thr_token, eos_token, eos_token2, suppress_eos, done, ws, scores_out);
     sample_final_kernel<<<dim3(B), dim3(64), 0, st>>>(ws, V, stream_slot, thr_token, use_thr, thr_value, eos_token, eos_token2, suppress_eos & 2, done, out_tokens,
                                                       history, hist_ld, hist_col, scores_out);
     return 0;
   }
-  sample_greedy_kernel<1024><<<dim3(B), dim3(1024), 0, st>>>(logits, ld, V, seen, words_per_stream, stream_slot,
+  sample_greedy_kernel<1024, LT><<<dim3(B), dim3(1024), 0, st>>>(logits, ld, V, seen, words_per_stream, stream_slot,
                                                              repetition_penalty, thr_token, use_thr, thr_value, eos_token, eos_token2,
                                                              suppress_eos, done, out_tokens, history, hist_ld, hist_col, scores_out);
   return 0;
+}
+int sample_greedy(const void* logits, bool f32, int ld, int B, int V, uint32_t* seen, int words_per_stream,
+                  const int32_t* stream_slot, float repetition_penalty, int thr_token, int use_thr, float thr_value,
+                  int eos_token, int eos_token2, int suppress_eos, int32_t* done, int32_t* out_tokens, int32_t* history, int hist_ld,
+                  int32_t* hist_col, float* scores_out, float* ws, hipStream_t st) {
+  if (f32)
+    return sample_greedy_t((const float*)logits, ld, B, V, seen, words_per_stream, stream_slot, repetition_penalty, thr_token, use_thr, thr_value,
+                           eos_token, eos_token2, suppress_eos, done, out_tokens, history, hist_ld, hist_col, scores_out, ws, st);
+  return sample_greedy_t((const bf16_t*)logits, ld, B, V, seen, words_per_stream, stream_slot, repetition_penalty, thr_token, use_thr, thr_value,
+                         eos_token, eos_token2, suppress_eos, done, out_tokens, history, hist_ld, hist_col, scores_out, ws, st);
 }
 
 // ------------------------------------------------------------------------------------------------------------------------
@@ -275,7 +295,7 @@ LCC_DEVICE unsigned long long wave_sum_u64(unsigned long long v) {
 }
 
 struct SampleParams {
-  const bf16_t* logits; int ld, V; const uint32_t* seen; int words; const int32_t* stream_slot;
+  const void* logits; int ld, V; const uint32_t* seen; int words; const int32_t* stream_slot;
   float penalty; int thr_token, use_thr; float thr_value; int eos_token, eos_token2, suppress_eos;
   int32_t* done; int32_t* out_tokens; int32_t* history; int hist_ld; int32_t* hist_col; float* scores_out;
   float temperature; int top_k; float top_p; uint32_t seed_lo, seed_hi; uint32_t* rng_ctr;
@@ -284,6 +304,7 @@ struct SampleParams {
 constexpr int SNT = 1024;                       // threads per block
 constexpr double MASS_SCALE = 1099511627776.0;  // 2^40
 
+template <class LT>
 __global__ __launch_bounds__(SNT) void sample_topk_topp_kernel(SampleParams P) {
   __shared__ float s_f[SNT / 64][3];
   __shared__ unsigned long long s_hist[16][SNT];   // 128 KB: per-thread radix-16 histograms (the block may use all 160 KB of LDS)
@@ -294,7 +315,7 @@ __global__ __launch_bounds__(SNT) void sample_topk_topp_kernel(SampleParams P) {
   const int b = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int slot = P.stream_slot[b];
   if (P.done != nullptr && P.done[slot]) return;
-  const bf16_t* lg = P.logits + (size_t)b * P.ld;
+  const LT* lg = static_cast<const LT*>(P.logits) + (size_t)b * P.ld;
   const uint32_t* sb = P.seen + (size_t)slot * P.words;
   const int V = P.V, nch = V / 8;
   const float penalty = P.penalty;
@@ -302,10 +323,8 @@ __global__ __launch_bounds__(SNT) void sample_topk_topp_kernel(SampleParams P) {
 
   // processed scores BEFORE the warpers of the 8 ids of chunk c (penalty, EOS mask; `thr_dead` = threshold processor fired)
   auto load8 = [&](int c, int thr_dead, float (&v)[8]) {
-    const u32x4 q = ld16(lg + c * 8);
     const uint32_t bits = (sb[c >> 2] >> ((c & 3) * 8)) & 0xffu;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) { v[2 * e] = lo2f(q[e]); v[2 * e + 1] = hi2f(q[e]); }
+    load8_logits(lg, c, v);
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
       if (penalty != 1.0f && ((bits >> e) & 1u)) v[e] = v[e] < 0.f ? v[e] * penalty : v[e] / penalty;
@@ -516,7 +535,7 @@ __global__ __launch_bounds__(SNT) void sample_topk_topp_kernel(SampleParams P) {
   }
 }
 
-int sample_topk_topp(const bf16_t* logits, int ld, int B, int V, uint32_t* seen, int words_per_stream, const int32_t* stream_slot,
+int sample_topk_topp(const void* logits, bool f32, int ld, int B, int V, uint32_t* seen, int words_per_stream, const int32_t* stream_slot,
                      float repetition_penalty, int thr_token, int use_thr, float thr_value, int eos_token, int eos_token2,
                      int suppress_eos, int32_t* done, int32_t* out_tokens, int32_t* history, int hist_ld, int32_t* hist_col,
                      float* scores_out, float temperature, int top_k, float top_p, uint64_t seed, uint32_t* rng_ctr, hipStream_t st) {
@@ -526,7 +545,8 @@ int sample_topk_topp(const bf16_t* logits, int ld, int B, int V, uint32_t* seen,
   SampleParams P{logits, ld, V, seen, words_per_stream, stream_slot, repetition_penalty, thr_token, use_thr, thr_value, eos_token,
                  eos_token2, suppress_eos, done, out_tokens, history, hist_ld, hist_col, scores_out, temperature, top_k, top_p,
                  (uint32_t)(seed & 0xffffffffu), (uint32_t)(seed >> 32), rng_ctr};
-  sample_topk_topp_kernel<<<dim3(B), dim3(SNT), 0, st>>>(P);
+  if (f32) sample_topk_topp_kernel<float><<<dim3(B), dim3(SNT), 0, st>>>(P);
+  else sample_topk_topp_kernel<bf16_t><<<dim3(B), dim3(SNT), 0, st>>>(P);
   return 0;
 }
 

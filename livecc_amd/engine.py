@@ -10,7 +10,7 @@ import numpy as np
 import torch
 
 from . import _lib
-from .config import LiveCCConfig
+from .config import DebunexConfig, LiveCCConfig
 from .weights import WeightArena
 
 # HF image_processing_backends.py:307-311: mean*(1/rescale_factor), std*(1/rescale_factor) as fp32 tensors
@@ -52,7 +52,7 @@ class Sampling:
         self.thr_token, self.thr_base, self.thr_step = thr_token, thr_base, thr_step
         self.eos_token2, self.do_sample, self.temperature, self.top_k, self.top_p, self.seed = eos_token2, do_sample, temperature, top_k, top_p, seed
 
-    def to_c(self, scores_out=None, logits_out=None) -> _lib.Sampling:
+    def to_c(self, scores_out=None, logits_out=None, prompt_rows=None, prompt_logits_out=None) -> _lib.Sampling:
         s = _lib.Sampling()
         s.repetition_penalty = float(self.repetition_penalty)
         s.thr_token = int(self.thr_token) if self.thr_base is not None else -1
@@ -69,6 +69,10 @@ class Sampling:
         s.top_k = int(self.top_k or 0)
         s.top_p = float(self.top_p if self.top_p is not None else 1.0)
         s.seed = int(self.seed) & 0xFFFFFFFFFFFFFFFF
+        if prompt_rows is not None and len(prompt_rows):         # int32 numpy array: alive until the call returns
+            s.n_prompt_rows = len(prompt_rows)
+            s.prompt_rows = prompt_rows.ctypes.data
+            s.prompt_logits_out = prompt_logits_out.data_ptr()
         return s
 
 
@@ -87,16 +91,13 @@ class Engine:
         self.device = torch.device(device if device is not None else weights.device)
         assert self.device.type == "cuda"
         torch.cuda.set_device(self.device)
-        max_kv_len = (max_kv_len + 31) // 32 * 32
+        self.is_decoder = isinstance(cfg, DebunexConfig)
+        gran = 64 if self.is_decoder else 32
+        max_kv_len = (max_kv_len + gran - 1) // gran * gran
         self.max_slots, self.max_kv_len, self.max_history = max_slots, max_kv_len, max_history
         self.max_new_rows, self.max_patches = max_new_rows, max_patches
-        mc = _lib.ModelConfig(cfg.vocab_size, cfg.hidden_size, cfg.intermediate_size, cfg.num_hidden_layers,
-                              cfg.num_attention_heads, cfg.num_key_value_heads, cfg.head_dim, cfg.rms_norm_eps,
-                              cfg.mrope_section[0], cfg.mrope_section[1], cfg.mrope_section[2], cfg.vit_depth,
-                              cfg.vit_embed_dim, cfg.vit_num_heads, cfg.vit_mlp_dim, cfg.patch_dim, cfg.spatial_merge_size,
-                              1 if getattr(weights, "llm_fp8", False) else 0)
         lim = _lib.EngineLimits(max_slots, max_kv_len, max_new_rows, max_patches, max_history)
-        self.h = self.lib.lcc_engine_create(C.byref(mc), C.byref(lim))
+        self.h = self._create(cfg, lim)
         if not self.h:
             raise _lib.LccError("lcc_engine_create: " + self.lib.lcc_last_error().decode())
         lib, h = self.lib, self.h
@@ -108,6 +109,46 @@ class Engine:
         _lib.check(lib.lcc_engine_bind_buffers(h, self._ws.data_ptr(), self._ws.numel(), self._state.data_ptr(),
                                                self._state.numel(), self._meta_dev.data_ptr(), self._meta_host.data_ptr(), mb),
                    "lcc_engine_bind_buffers")
+        if not self.is_decoder:
+            self._bind_vit()
+        kvb = lib.lcc_engine_kv_bytes_per_slot(h)
+        self.kv_bytes_per_slot = kvb
+        # a decoder's arenas are bound when their slot is first used: short requests of many callers do not pay for max_slots windows
+        self._kv: List[Optional[torch.Tensor]] = [None] * max_slots
+        if not self.is_decoder:
+            for slot in range(max_slots):
+                self._bind_kv(slot)
+        for name in weights.names():
+            v = weights.view(name)
+            _lib.check(lib.lcc_engine_set_weight(h, name.encode(), v.data_ptr(), v.numel()), f"set_weight {name}")
+        if not self.is_decoder:
+            _lib.check(lib.lcc_engine_set_weight(h, b"inv_freq", weights.inv_freq.data_ptr(), weights.inv_freq.numel()), "inv_freq")
+        miss = C.create_string_buffer(512)
+        if not lib.lcc_engine_weights_ready(h, miss, 512):
+            raise _lib.LccError("missing weights: " + miss.value.decode())
+        m, s = fused_mean_std()
+        self._mean = (C.c_float * 3)(*m.tolist())
+        self._std = (C.c_float * 3)(*s.tolist())
+        self._rope_cache: Dict[tuple, Tuple[torch.Tensor, torch.Tensor]] = {}
+
+    def _create(self, cfg, lim):
+        if self.is_decoder:
+            layers = (_lib.DecoderLayer * cfg.num_hidden_layers)()
+            for i, l in enumerate(cfg.layers):
+                m = l.mixer
+                layers[i] = _lib.DecoderLayer(_lib.MIXER_LATENT, m.heads, m.q_rank, m.kv_rank, m.dim_pad, m.vdim_pad, m.q_rank_pad, m.kv_rank_pad,
+                                              -1 if m.kv_from is None else m.kv_from, m.scale, l.ff_pad)
+            dc = _lib.DecoderConfigC(cfg.vocab_size, cfg.vocab_pad, cfg.width_pad, cfg.num_hidden_layers, cfg.norm_eps, cfg.logit_softcap or 0.0)
+            return self.lib.lcc_engine_create_decoder(C.byref(dc), layers, C.byref(lim))
+        mc = _lib.ModelConfig(cfg.vocab_size, cfg.hidden_size, cfg.intermediate_size, cfg.num_hidden_layers,
+                              cfg.num_attention_heads, cfg.num_key_value_heads, cfg.head_dim, cfg.rms_norm_eps,
+                              cfg.mrope_section[0], cfg.mrope_section[1], cfg.mrope_section[2], cfg.vit_depth,
+                              cfg.vit_embed_dim, cfg.vit_num_heads, cfg.vit_mlp_dim, cfg.patch_dim, cfg.spatial_merge_size,
+                              1 if getattr(self.weights, "llm_fp8", False) else 0)
+        return self.lib.lcc_engine_create(C.byref(mc), C.byref(lim))
+
+    def _bind_vit(self) -> None:
+        lib, h = self.lib, self.h
         # private ViT workspace + meta ring: the vision tower of the NEXT turn's frames may then run on a second stream under the
         # current turn's decode steps (modeling.generate_batch(prefetch=...))
         self._ws_vit = torch.empty(lib.lcc_engine_vit_workspace_bytes(h), dtype=torch.uint8, device=self.device)
@@ -116,22 +157,12 @@ class Engine:
         self._vmeta_host = torch.empty(vmb, dtype=torch.uint8).pin_memory()
         _lib.check(lib.lcc_engine_bind_vit_buffers(h, self._ws_vit.data_ptr(), self._ws_vit.numel(), self._vmeta_dev.data_ptr(),
                                                    self._vmeta_host.data_ptr(), vmb), "lcc_engine_bind_vit_buffers")
-        kvb = lib.lcc_engine_kv_bytes_per_slot(h)
-        self.kv_bytes_per_slot = kvb
-        self._kv = [torch.zeros(kvb, dtype=torch.uint8, device=self.device) for _ in range(max_slots)]
-        for s, t in enumerate(self._kv):
-            _lib.check(lib.lcc_engine_bind_kv(h, s, t.data_ptr(), t.numel()), "lcc_engine_bind_kv")
-        for name in weights.names():
-            v = weights.view(name)
-            _lib.check(lib.lcc_engine_set_weight(h, name.encode(), v.data_ptr(), v.numel()), f"set_weight {name}")
-        _lib.check(lib.lcc_engine_set_weight(h, b"inv_freq", weights.inv_freq.data_ptr(), weights.inv_freq.numel()), "inv_freq")
-        miss = C.create_string_buffer(512)
-        if not lib.lcc_engine_weights_ready(h, miss, 512):
-            raise _lib.LccError("missing weights: " + miss.value.decode())
-        m, s = fused_mean_std()
-        self._mean = (C.c_float * 3)(*m.tolist())
-        self._std = (C.c_float * 3)(*s.tolist())
-        self._rope_cache: Dict[tuple, Tuple[torch.Tensor, torch.Tensor]] = {}
+
+    def _bind_kv(self, slot: int) -> None:
+        if self._kv[slot] is None:
+            t = torch.zeros(self.kv_bytes_per_slot, dtype=torch.uint8, device=self.device)
+            _lib.check(self.lib.lcc_engine_bind_kv(self.h, slot, t.data_ptr(), t.numel()), "lcc_engine_bind_kv")
+            self._kv[slot] = t
 
     def __del__(self):
         try:
@@ -147,6 +178,7 @@ class Engine:
         return torch.cuda.current_stream(self.device).cuda_stream
 
     def reset_slot(self, slot: int) -> None:
+        self._bind_kv(slot)
         _lib.check(self.lib.lcc_slot_reset(self.h, slot, self._stream()), "lcc_slot_reset")
 
     def slot_length(self, slot: int) -> Tuple[int, int]:
@@ -212,13 +244,21 @@ class Engine:
         return out
 
     def prefill(self, slots: Sequence[int], ids: Sequence[np.ndarray], pos3: Sequence[np.ndarray],
-                vit_embeds: Optional[torch.Tensor], sampling: Sampling, scores_out=None, logits_out=None) -> None:
+                vit_embeds: Optional[torch.Tensor], sampling: Sampling, scores_out=None, logits_out=None, prompt_rows=None,
+                prompt_logits_out=None) -> None:
         """ids[b]: int array of the new tokens of stream b; pos3[b]: [3, n_new] M-RoPE positions.  <|video_pad|> rows take
-        consecutive rows of `vit_embeds` (stream order)."""
+        consecutive rows of `vit_embeds` (stream order).  Decoders take neither positions nor embeddings; `prompt_rows` (int32, packed row
+        indices of the call) asks for the fp32 logits of those rows in `prompt_logits_out` [n, vocab]."""
         n = len(slots)
         ids_cat = np.concatenate([np.asarray(x, dtype=np.int32).reshape(-1) for x in ids])
         n_new = np.asarray([len(x) for x in ids], dtype=np.int32)
         S = int(n_new.sum())
+        if self.is_decoder:
+            slots_a = np.asarray(slots, dtype=np.int32)
+            sp = sampling.to_c(scores_out, logits_out, prompt_rows, prompt_logits_out)
+            _lib.check(self.lib.lcc_llm_prefill(self.h, n, slots_a.ctypes.data, n_new.ctypes.data, ids_cat.ctypes.data, None, None, None, C.byref(sp),
+                                                self._stream()), "lcc_llm_prefill")
+            return
         pos_cat = np.concatenate([np.asarray(p, dtype=np.int32).reshape(3, -1) for p in pos3], axis=1)
         assert pos_cat.shape == (3, S)
         pos_cat = np.ascontiguousarray(pos_cat)
@@ -245,6 +285,11 @@ class Engine:
         _lib.check(self.lib.lcc_llm_decode(self.h, len(slots), slots_a.ctypes.data, n_steps, first_step_index, C.byref(sp),
                                            self._stream()), "lcc_llm_decode")
 
+    def set_tokens(self, slots: Sequence[int], tokens: Sequence[int]) -> None:
+        """The ids the slots consume in their next decode step (instead of the sampled ones)."""
+        a, t = np.asarray(slots, dtype=np.int32), np.asarray(tokens, dtype=np.int32)
+        _lib.check(self.lib.lcc_slot_set_tokens(self.h, len(a), a.ctypes.data, t.ctypes.data, self._stream()), "lcc_slot_set_tokens")
+
     # ---- parity instrumentation (tests only): residual-stream taps / per-layer input overrides ----
     def set_llm_taps(self, max_rows: int, overrides: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
         """Bind (max_rows > 0) or unbind (0) the LLM taps; returns the tap tensor bf16 [2L+1, max_rows, H] that the following
@@ -254,7 +299,12 @@ class Engine:
             _lib.check(self.lib.lcc_debug_set_llm_taps(self.h, None, None, 0), "lcc_debug_set_llm_taps")
             self._llm_taps = self._llm_over = None
             return None
-        taps = torch.zeros(2 * cfg.num_hidden_layers + 1, max_rows, cfg.hidden_size, dtype=torch.bfloat16, device=self.device)
+        if self.is_decoder:        # the fp32 residual: [L+1, max_rows, padded width]
+            if overrides is not None:
+                raise ValueError("per-layer input overrides are not available for this model family")
+            taps = torch.zeros(cfg.num_hidden_layers + 1, max_rows, cfg.width_pad, dtype=torch.float32, device=self.device)
+        else:
+            taps = torch.zeros(2 * cfg.num_hidden_layers + 1, max_rows, cfg.hidden_size, dtype=torch.bfloat16, device=self.device)
         if overrides is not None:
             assert overrides.shape == (cfg.num_hidden_layers + 1, max_rows, cfg.hidden_size) and overrides.dtype == torch.bfloat16
             overrides = overrides.to(self.device).contiguous()

@@ -36,15 +36,15 @@ import numpy as np
 import torch
 
 from . import protocol
-from .config import LiveCCConfig, get_config
+from .config import DebunexConfig, LiveCCConfig, architecture_of, get_config
 from .engine import Engine, Sampling
-from .weights import WeightArena, from_hf_model as _arena_from_hf, from_pretrained as _arena_from_pretrained
+from .weights import WeightArena, from_hf_model as _arena_from_hf, from_pretrained as _arena_from_pretrained, make_arena
 
 
 class StreamState:
     """Opaque per-stream generation state (the `past_key_values` handle)."""
 
-    def __init__(self, model: "LiveCCForConditionalGeneration", slot: int):
+    def __init__(self, model: "EngineModel", slot: int):
         self.model, self.slot = model, slot
         self.rope_delta: Optional[int] = None
         self.released = False
@@ -106,29 +106,25 @@ def read_generation_config(model_path: str):
     return gen_cfg, eos_ids
 
 
-class LiveCCForConditionalGeneration:
-    main_input_name = "input_ids"
-    DECODE_GROUP = 64          # LCC_MAX_DECODE_BATCH of include/livecc_amd.h: streams decoded per weight pass
+def _check_load_args(torch_dtype, device_map):
+    """from_pretrained's dtype / device arguments -> device."""
+    if torch_dtype not in ("auto", torch.bfloat16, "bfloat16"):
+        raise ValueError("the MI355X engine computes in bf16 (torch_dtype='auto' of the released checkpoints)")
+    device = device_map if isinstance(device_map, (str, torch.device)) and device_map not in ("auto",) else "cuda"
+    if "cuda" not in str(device):
+        raise RuntimeError("livecc_amd has no CPU path; use device_map='cuda[:i]' (the oracle under oracle/ is the CPU path)")
+    return device
 
-    def __init__(self, cfg: LiveCCConfig, weights: WeightArena, device, max_streams: int = 1, max_kv_len: Optional[int] = None,
-                 max_new_rows: int = 4096, max_patches: int = 16384, max_history: int = 512,
-                 text_offset_rule: str = "hf4", eos_token_ids: Optional[Sequence[int]] = None):
-        """Capacity knobs (all served out of the box with the defaults, like the reference's flows):
-        max_history     = the largest max_new_tokens of one generate call (video_qa uses 512, ref demo/infer.py:236);
-        max_new_rows    = rows of ONE prefill launch sequence -- longer prompts (the one-shot 24k-token video_qa / MCQ prefill)
-                          are cut into pieces of at most this many rows over the carried KV (bit-identical to one pass);
-        max_patches     = ViT patches of ONE encode launch sequence -- longer clips are encoded in groups of temporal slices
-                          (slices never attend to each other, Q2VL vision_utils.py:60-65);
-        max_kv_len      = KV capacity per stream; default = the trained 32k window + max_history of generation headroom.
-        text_offset_rule: "hf4" = transformers-4.5x M-RoPE text offset after a vision block (what the released checkpoints
-        were trained with, ref README.md:30); "hf5" = the installed 5.15 oracle's rule.  Identical for every streaming chunk;
-        they differ for one-shot long clips (grid_t > max(h,w)/2).
-        PINNING STATUS: "hf5" is pinned to the EXECUTED transformers 5.15 (`get_rope_index`, tests/test_protocol.py + every one-shot GPU
-        fixture).  "hf4" is UNPINNED: it restates the 4.5x algorithm (`st_idx = llm_pos_ids_list[-1].max() + 1`) from memory of that
-        source -- no 4.5x wheel / sdist exists offline (searched the image and the pip cache, round 6) -- and is checked only against
-        that restatement (tests/test_protocol.py:137,177).  bench.py says so in `config.workload` whenever the hf4 rule is what ran."""
+
+class EngineModel:
+    """What every model family shares on one engine: stream slots, sampling parameters, batching (packed prefills, decode groups), the
+    generate loop.  A family adds its constructors and, where it has them, positions and embedding inputs."""
+    DECODE_GROUP = 64          # LCC_MAX_DECODE_BATCH of include/livecc_amd.h: streams decoded per weight pass
+    logits_dtype = torch.bfloat16          # of `output_logits`
+
+    def _init_engine(self, cfg, weights: WeightArena, device, max_streams: int, max_kv_len: Optional[int], max_new_rows: int, max_patches: int,
+                     max_history: int, eos_ids: Sequence[int]) -> None:
         self.cfg, self.weights = cfg, weights
-        self.config = _Cfg(cfg)
         self.device = torch.device(device)
         if max_kv_len is None:
             max_kv_len = cfg.max_position_embeddings + max_history
@@ -136,56 +132,31 @@ class LiveCCForConditionalGeneration:
                              max_new_rows=max_new_rows, max_patches=max_patches, max_history=max_history)
         self._free_slots = list(range(max_streams - 1, -1, -1))
         self._lock = threading.RLock()          # every engine entry point below holds it for the whole call (see the module docstring)
-        self.text_offset_rule = text_offset_rule
-        self.prepare_inputs_for_generation = None   # assignable, as ref demo/infer.py:50 does
         self.generation_config: dict = {}            # from_pretrained fills it from generation_config.json (do_sample / top_k ...)
-        # HF stops on ANY id of generation_config.eos_token_id ([<|im_end|>, <|endoftext|>] in the released checkpoints)
-        ids = [int(cfg.eos_token_id)] + [int(t) for t in (eos_token_ids or []) if int(t) != int(cfg.eos_token_id)]
-        if len(ids) > 2:
-            raise NotImplementedError(f"at most two EOS ids are supported, got {ids}")
-        self.eos_token_ids = ids
-        self.config.eos_token_id = ids[0] if len(ids) == 1 else list(ids)
-        # vision-tower prefetch (generate_batch(prefetch=...)): side stream, results keyed by the clip's storage
-        self._side: Optional[torch.cuda.Stream] = None
-        self._vit_cache: dict = {}
-        self._vit_last_event: Optional[torch.cuda.Event] = None
-        # CUs a prefetched vision tower may occupy while it runs under another turn's decode steps: -1 (default) = 128 for >= 4 clips (measured
-        # +1.5 % tokens/s at 8 streams, profiles/r05/prefetch_grid_cap_ab.txt; one stream's tower is too small to share: 276 -> 256-269 tokens/s
-        # under any cap), 0 = whole chip, n = n workgroups.  LCC_VIT_PREFETCH_CAP overrides.
-        self.prefetch_grid_cap = int(os.environ.get("LCC_VIT_PREFETCH_CAP", "-1"))
-
-    # ---- constructors ----
-    @classmethod
-    def from_pretrained(cls, model_path: str, torch_dtype="auto", device_map=None, attn_implementation=None, **kw):
-        """Same call as ref demo/infer.py:43-47.  bf16 only ('auto' resolves to bf16 for these checkpoints)."""
-        if torch_dtype not in ("auto", torch.bfloat16, "bfloat16"):
-            raise ValueError("the MI355X engine computes in bf16 (torch_dtype='auto' of the released checkpoints)")
-        device = device_map if isinstance(device_map, (str, torch.device)) and device_map not in ("auto",) else "cuda"
-        if "cuda" not in str(device):
-            raise RuntimeError("livecc_amd has no CPU path; use device_map='cuda[:i]' (the oracle under oracle/ is the CPU path)")
-        cfg = get_config(model_path)
-        gen_cfg, eos_ids = read_generation_config(model_path)
-        if eos_ids is not None and "eos_token_ids" not in kw:
-            kw["eos_token_ids"] = eos_ids
-        arena = _arena_from_pretrained(model_path, cfg, device, llm_fp8=bool(kw.pop("llm_fp8", False)))
-        model = cls(cfg, arena, device, **kw)
-        model.generation_config = gen_cfg
-        return model
-
-    @classmethod
-    def from_config(cls, cfg: LiveCCConfig, device="cuda", seed: int = 0, llm_fp8: bool = False, **kw):
-        """llm_fp8: quantise the LLM Linear weights to OCP e4m3 with per-output-row scales (the 72B single-GPU weight path)."""
-        return cls(cfg, WeightArena(cfg, device, llm_fp8=llm_fp8).fill_random(seed), device, **kw)
-
-    @classmethod
-    def from_hf_model(cls, hf_model, cfg: LiveCCConfig, device="cuda", llm_fp8: bool = False, **kw):
-        """Weights of an instantiated HF model (the oracle-parity constructor): positions follow the INSTALLED transformers
-        (5.x text-offset rule) unless told otherwise, so that one-shot long clips compare equal to that oracle."""
-        kw.setdefault("text_offset_rule", "hf5")
-        return cls(cfg, _arena_from_hf(hf_model, cfg, device, llm_fp8=llm_fp8), device, **kw)
+        if len(eos_ids) > 2:
+            raise NotImplementedError(f"at most two EOS ids are supported, got {list(eos_ids)}")
+        self.eos_token_ids = list(eos_ids)
 
     def eval(self):
         return self
+
+    # ---- what a family overrides ----
+    def _scores_width(self) -> int:
+        return self.cfg.vocab_size
+
+    def _embedding_rows(self, ids: np.ndarray) -> np.ndarray:
+        """Mask of the ids whose embedding row comes from the request (video tokens), not from the table."""
+        return np.zeros(len(ids), dtype=bool)
+
+    def _request_inputs(self, rq: dict, st: "StreamState", new: np.ndarray, past_len: int, clips: list):
+        """[3, n_new] positions of a request's new ids; appends the clips it brings."""
+        return np.zeros((3, len(new)), dtype=np.int64)
+
+    def _encode_clips(self, clips: list) -> Optional[torch.Tensor]:
+        return None
+
+    def _prefetch(self, prefetch) -> None:
+        raise NotImplementedError("this model takes no clips")
 
     # ---- stream slots ----
     def new_stream(self) -> StreamState:
@@ -209,15 +180,6 @@ class LiveCCForConditionalGeneration:
         # a reused object continues from its `count` (ref demo/infer.py:17: threshold = base + step * count)
         return int(p.token_id), float(p.base_threshold) + float(p.step) * int(getattr(p, "count", 0)), float(p.step)
 
-    def _positions(self, st: StreamState, ids_new: np.ndarray, grids, past_len: int) -> np.ndarray:
-        if past_len == 0:
-            pos, delta = protocol.rope_index_first_turn(ids_new, grids, self.cfg, self.text_offset_rule)
-            st.rope_delta = delta
-            return pos
-        if st.rope_delta is None:
-            st.rope_delta = 0
-        return protocol.positions_with_cache(past_len, len(ids_new), st.rope_delta)
-
     def _resolve_sampling(self, do_sample, kw) -> dict:
         """HF semantics (generation/utils.py `_prepare_generation_config`): explicit arguments override the checkpoint's
         generation_config.json, which overrides HF's defaults (do_sample False, temperature 1.0, top_k 50, top_p 1.0).
@@ -239,31 +201,6 @@ class LiveCCForConditionalGeneration:
             raise ValueError(f"top_k must be >= 0 and top_p in (0, 1], got {top_k}, {top_p}")
         seed = kw.get("seed", g.get("seed"))
         return dict(do_sample=True, temperature=float(temperature), top_k=top_k, top_p=float(top_p), seed=None if seed is None else int(seed))
-
-    @torch.inference_mode()
-    def generate(self, input_ids: torch.Tensor = None, pixel_values_videos: Optional[torch.Tensor] = None,
-                 video_grid_thw: Optional[torch.Tensor] = None, mm_token_type_ids=None,
-                 past_key_values: Optional[StreamState] = None, return_dict_in_generate: bool = True,
-                 do_sample: Optional[bool] = None, repetition_penalty: float = 1.0, logits_processor=None,
-                 max_new_tokens: int = 16, min_new_tokens: Optional[int] = None, pad_token_id: Optional[int] = None,
-                 eos_token_id: Optional[int] = None, frames: Optional[torch.Tensor] = None, frames_layout: str = "TCHW",
-                 output_logits: bool = False, output_scores: bool = False, attention_mask=None, teacher_tokens=None, **unused):
-        """`teacher_tokens` (tests): the generated tokens are forced to this sequence (what the HF oracle does with a forcing
-        LogitsProcessor) while `output_logits` keeps the model's own raw logits of every step."""
-        sampling_kw = self._resolve_sampling(do_sample, unused)
-        if attention_mask is not None and not bool(torch.as_tensor(attention_mask).all()):
-            raise NotImplementedError("padding masks are not supported (the reference passes none, infer.py:156)")
-        if input_ids.dim() != 2 or input_ids.shape[0] != 1:
-            raise ValueError("generate() is single-stream like the reference (batch 1); use generate_batch for many streams")
-        if min_new_tokens is not None and min_new_tokens not in (0, max_new_tokens):
-            raise NotImplementedError("min_new_tokens must be None/0 or equal to max_new_tokens")
-        r = self.generate_batch([dict(
-            input_ids=input_ids[0], pixel_values_videos=pixel_values_videos,
-            video_grid_thw=video_grid_thw, frames=frames, frames_layout=frames_layout, state=past_key_values)],
-            repetition_penalty=repetition_penalty, logits_processor=logits_processor, max_new_tokens=max_new_tokens,
-            force_length=bool(min_new_tokens), eos_token_id=eos_token_id, output_logits=output_logits,
-            output_scores=output_scores, teacher_tokens=None if teacher_tokens is None else [list(teacher_tokens)], **sampling_kw)[0]
-        return r if return_dict_in_generate else r.sequences
 
     @torch.inference_mode()
     def generate_batch(self, requests: Sequence[dict], repetition_penalty: float = 1.0, logits_processor=None,
@@ -302,7 +239,7 @@ class LiveCCForConditionalGeneration:
             eos_ids = [int(t) for t in (eos_token_id if isinstance(eos_token_id, (list, tuple)) else [eos_token_id])]
             if len(eos_ids) > 2:
                 raise NotImplementedError("at most two EOS ids are supported")
-        eos, eos2 = eos_ids[0], (eos_ids[1] if len(eos_ids) > 1 else -1)
+        eos, eos2 = (eos_ids + [-1, -1])[:2]          # -1: a model without an EOS id
         if max_new_tokens < 1 or max_new_tokens > eng.max_history:
             raise ValueError(f"max_new_tokens={max_new_tokens} exceeds this model's max_history={eng.max_history}: construct the model "
                              f"with max_history >= the largest max_new_tokens you generate (video_qa uses 512)")
@@ -332,37 +269,11 @@ class LiveCCForConditionalGeneration:
             if len(ids_full) <= past_len:
                 raise ValueError(f"input_ids ({len(ids_full)}) must extend the cached sequence ({past_len})")
             new = ids_full[past_len:]
-            grids = []
-            n_vid = int((new == cfg.video_token_id).sum())
-            if n_vid:
-                if rq.get("frames") is not None:
-                    f = rq["frames"]
-                    lay = rq.get("frames_layout", "TCHW")
-                    if not f.is_cuda:
-                        f = f.to(self.device, non_blocking=True)
-                    f = f.contiguous()
-                    T, H, W = (f.shape[0], f.shape[2], f.shape[3]) if lay == "TCHW" else (f.shape[0], f.shape[1], f.shape[2])
-                    grids = [protocol.grid_of(T, H, W, cfg)]
-                    clips.append(dict(frames=f, layout=lay, key=self._clip_key(f, lay)))
-                elif rq.get("pixel_values_videos") is not None:
-                    g = torch.as_tensor(rq["video_grid_thw"]).reshape(-1, 3).tolist()
-                    pv = rq["pixel_values_videos"].to(self.device, dtype=torch.float32).contiguous()
-                    off = 0
-                    for t, h, w in g:
-                        clips.append(dict(pixel_values=pv[off:off + t * h * w], grid=(t, h, w)))
-                        off += t * h * w
-                    grids = [tuple(x) for x in g]
-                else:
-                    raise ValueError("input_ids contain <|video_pad|> but no frames / pixel_values_videos were given")
-                if sum(protocol.num_video_tokens(g, cfg) for g in grids) != n_vid:
-                    raise ValueError(f"Video features and video tokens do not match, tokens: {n_vid}, features: "
-                                     f"{sum(protocol.num_video_tokens(g, cfg) for g in grids)}")
-            pos3.append(self._positions(st, new, grids, past_len))
+            pos3.append(self._request_inputs(rq, st, new, past_len, clips))
             states.append(st); ids_new.append(new); slots.append(st.slot); full_ids.append(ids_full)
-        vit = self._vit_for(clips) if clips else None
-        V = cfg.vocab_size
-        logits_buf = torch.empty(max_new_tokens, n, V, dtype=torch.bfloat16, device=self.device) if output_logits else None
-        scores_buf = torch.empty(n, V, dtype=torch.float32, device=self.device) if output_scores else None
+        vit = self._encode_clips(clips) if clips else None
+        logits_buf = torch.empty(max_new_tokens, n, cfg.vocab_size, dtype=self.logits_dtype, device=self.device) if output_logits else None
+        scores_buf = torch.empty(n, self._scores_width(), dtype=torch.float32, device=self.device) if output_scores else None
         sp = Sampling(repetition_penalty=repetition_penalty, eos_token=eos, suppress_eos=force_length,
                       thr_token=thr[0] if thr else -1, thr_base=thr[1] if thr else None, thr_step=thr[2] if thr else 0.0,
                       eos_token2=eos2, do_sample=do_sample, temperature=temperature, top_k=top_k, top_p=top_p, seed=seed)
@@ -383,7 +294,7 @@ class LiveCCForConditionalGeneration:
         eng = self.engine
         self._prefill(slots, ids_new, pos3, vit, sp, scores_buf, logits_buf)
         if prefetch:
-            self._prefetch_vit(prefetch)
+            self._prefetch(prefetch)
         # decode: the device loop needs no host round trip per token (EOS freezes a slot on the device); long generations
         # (video_qa: max_new_tokens=512, ref demo/infer.py:236) are cut into chunks of 32 steps so that the host can stop
         # early once every stream has emitted EOS.
@@ -407,8 +318,237 @@ class LiveCCForConditionalGeneration:
             seq = torch.from_numpy(np.concatenate([full_ids[b], np.asarray(toks, dtype=np.int64)])).view(1, -1).to(self.device)
             lg = logits_buf[:len(toks), b] if logits_buf is not None and n <= G else None
             outs.append(GenerateOutput(sequences=seq, past_key_values=st, logits=lg,
-                                       scores=scores_buf[b] if scores_buf is not None else None))
+                                       scores=scores_buf[b, :self.cfg.vocab_size] if scores_buf is not None else None))
         return outs
+
+    def _prefill(self, slots, ids_new, pos3, vit, sp, scores_buf, logits_buf, want=None, want_out=None) -> None:
+        """One packed prefill when everything fits `max_new_rows`; otherwise consecutive streams are packed into groups of at
+        most `max_new_rows` rows (one launch sequence per group), and a stream that is longer than that by itself is prefilled
+        alone in pieces over its carried KV (a prompt prefilled in one or in several calls gives bit-identical logits:
+        tests/test_gpu_fullsize.py; only the LAST piece's sampled token survives -- each prefill call restarts the history
+        column -- which is exactly the token of the un-split prefill)."""
+        eng = self.engine
+        cap = eng.max_new_rows
+        lens = [len(x) for x in ids_new]
+
+        def run(b, e, lo, hi, ids, pos, rows):
+            """Streams b .. e (or the piece lo .. hi of stream b) as one launch sequence, with the wanted prompt logits that fall into it."""
+            kw, parts, row = {}, [], 0
+            for i in range(b, e) if want is not None else ():
+                w = want[i]
+                sel = np.nonzero((w >= lo) & (w < hi))[0]
+                if len(sel):
+                    parts.append((i, sel, row + w[sel] - lo))
+                row += min(hi, lens[i]) - lo
+            if parts:
+                rows_w = np.concatenate([p[2] for p in parts]).astype(np.int32)
+                buf = torch.empty(len(rows_w), self.cfg.vocab_size, dtype=torch.float32, device=self.device)
+                kw = dict(prompt_rows=rows_w, prompt_logits_out=buf)
+            eng.prefill(slots[b:e], ids, pos, rows, sp, scores_out=sc(b, e), logits_out=lg(b, e), **kw)
+            off = 0
+            for i, sel, _ in parts:
+                want_out[i][torch.as_tensor(sel, device=self.device)] = buf[off:off + len(sel)]
+                off += len(sel)
+
+        sc = (lambda a, e: scores_buf[a:e]) if scores_buf is not None else (lambda a, e: None)
+        lg = (lambda a, e: logits_buf[0, a:e]) if logits_buf is not None else (lambda a, e: None)   # step 0 = the prefill's token
+        if sum(lens) <= cap:
+            run(0, len(slots), 0, cap, ids_new, pos3, vit)
+            return
+        is_vid = [self._embedding_rows(ids) for ids in ids_new]
+        n_vid = [int(m.sum()) for m in is_vid]
+        row0 = np.concatenate([[0], np.cumsum(n_vid)]).astype(np.int64)      # first ViT row of every stream
+        b, n = 0, len(slots)
+        while b < n:
+            if lens[b] > cap:                                   # one long prompt (one-shot video_qa / mcq): pieces over its own KV
+                ids, pos, nv_before = ids_new[b], pos3[b], 0
+                for a in range(0, lens[b], cap):
+                    e = min(lens[b], a + cap)
+                    k = int(is_vid[b][a:e].sum())
+                    rows = vit[row0[b] + nv_before:row0[b] + nv_before + k] if (vit is not None and k) else None
+                    nv_before += k
+                    run(b, b + 1, a, e, [ids[a:e]], [pos[:, a:e]], rows)
+                b += 1
+                continue
+            e, rows_sum = b, 0
+            while e < n and lens[e] <= cap and rows_sum + lens[e] <= cap:
+                rows_sum += lens[e]
+                e += 1
+            rows = vit[row0[b]:row0[e]] if (vit is not None and row0[e] > row0[b]) else None
+            run(b, e, 0, cap, ids_new[b:e], pos3[b:e], rows)
+            b = e
+
+    # ---- given ids instead of sampled ones ----
+    @torch.inference_mode()
+    def forward_step(self, entries: Sequence[tuple]) -> List[torch.Tensor]:
+        """One step of the engine over ids the caller supplies (replaying a trace, scoring a text): entries = (StreamState, new ids, places among
+        them whose logits are wanted), one batch; returns the fp32 logits [places, vocab] of every entry.  Streams that go on by one token run
+        the decode step, everything else one packed prefill -- the launch sequences `generate_batch` runs."""
+        if not self.engine.is_decoder:
+            raise NotImplementedError("forward_step serves decoder models")
+        with self._lock:
+            eng, V = self.engine, self.cfg.vocab_size
+            states = [e[0] for e in entries]
+            ids = [np.asarray(e[1], dtype=np.int64).reshape(-1) for e in entries]
+            want = [np.asarray(e[2], dtype=np.int64).reshape(-1) for e in entries]
+            if len(set(id(s) for s in states)) != len(states) or any(s.released or s.model is not self for s in states):
+                raise ValueError("every entry needs a live stream of its own")
+            for x, w in zip(ids, want):
+                if len(x) == 0 or (len(w) and (w.min() < 0 or w.max() >= len(x))):
+                    raise ValueError("an entry needs at least one id, and wanted places among its ids")
+            out = [torch.empty(len(w), V, dtype=torch.float32, device=self.device) for w in want]
+            sp = Sampling()
+            dec = [i for i, s in enumerate(states) if len(ids[i]) == 1 and s.get_seq_length() > 0]
+            pre = [i for i in range(len(states)) if i not in set(dec)]
+            G = min(self.DECODE_GROUP, eng.max_new_rows)
+            for b0 in range(0, len(dec), G):
+                grp = dec[b0:b0 + G]
+                slots = [states[i].slot for i in grp]
+                eng.set_tokens(slots, [int(ids[i][0]) for i in grp])
+                lg = torch.empty(1, len(grp), V, dtype=torch.float32, device=self.device)
+                eng.decode(slots, 1, 0, sp, logits_out=lg)
+                for k, i in enumerate(grp):
+                    out[i][:] = lg[0, k]
+            if pre:
+                self._prefill([states[i].slot for i in pre], [ids[i] for i in pre], [np.zeros((3, len(ids[i])), dtype=np.int64) for i in pre], None, sp,
+                              None, None, want=[want[i] for i in pre], want_out=[out[i] for i in pre])
+            return out
+
+
+class LiveCCForConditionalGeneration(EngineModel):
+    main_input_name = "input_ids"
+
+    def __init__(self, cfg: LiveCCConfig, weights: WeightArena, device, max_streams: int = 1, max_kv_len: Optional[int] = None,
+                 max_new_rows: int = 4096, max_patches: int = 16384, max_history: int = 512,
+                 text_offset_rule: str = "hf4", eos_token_ids: Optional[Sequence[int]] = None):
+        """Capacity knobs (all served out of the box with the defaults, like the reference's flows):
+        max_history     = the largest max_new_tokens of one generate call (video_qa uses 512, ref demo/infer.py:236);
+        max_new_rows    = rows of ONE prefill launch sequence -- longer prompts (the one-shot 24k-token video_qa / MCQ prefill)
+                          are cut into pieces of at most this many rows over the carried KV (bit-identical to one pass);
+        max_patches     = ViT patches of ONE encode launch sequence -- longer clips are encoded in groups of temporal slices
+                          (slices never attend to each other, Q2VL vision_utils.py:60-65);
+        max_kv_len      = KV capacity per stream; default = the trained 32k window + max_history of generation headroom.
+        text_offset_rule: "hf4" = transformers-4.5x M-RoPE text offset after a vision block (what the released checkpoints
+        were trained with, ref README.md:30); "hf5" = the installed 5.15 oracle's rule.  Identical for every streaming chunk;
+        they differ for one-shot long clips (grid_t > max(h,w)/2).
+        PINNING STATUS: "hf5" is pinned to the EXECUTED transformers 5.15 (`get_rope_index`, tests/test_protocol.py + every one-shot GPU
+        fixture).  "hf4" is UNPINNED: it restates the 4.5x algorithm (`st_idx = llm_pos_ids_list[-1].max() + 1`) from memory of that
+        source -- no 4.5x wheel / sdist exists offline (searched the image and the pip cache, round 6) -- and is checked only against
+        that restatement (tests/test_protocol.py:137,177).  bench.py says so in `config.workload` whenever the hf4 rule is what ran."""
+        # HF stops on ANY id of generation_config.eos_token_id ([<|im_end|>, <|endoftext|>] in the released checkpoints)
+        ids = [int(cfg.eos_token_id)] + [int(t) for t in (eos_token_ids or []) if int(t) != int(cfg.eos_token_id)]
+        self._init_engine(cfg, weights, device, max_streams, max_kv_len, max_new_rows, max_patches, max_history, ids)
+        self.config = _Cfg(cfg)
+        self.config.eos_token_id = ids[0] if len(ids) == 1 else list(ids)
+        self.text_offset_rule = text_offset_rule
+        self.prepare_inputs_for_generation = None   # assignable, as ref demo/infer.py:50 does
+        # vision-tower prefetch (generate_batch(prefetch=...)): side stream, results keyed by the clip's storage
+        self._side: Optional[torch.cuda.Stream] = None
+        self._vit_cache: dict = {}
+        self._vit_last_event: Optional[torch.cuda.Event] = None
+        # CUs a prefetched vision tower may occupy while it runs under another turn's decode steps: -1 (default) = 128 for >= 4 clips (measured
+        # +1.5 % tokens/s at 8 streams, profiles/r05/prefetch_grid_cap_ab.txt; one stream's tower is too small to share: 276 -> 256-269 tokens/s
+        # under any cap), 0 = whole chip, n = n workgroups.  LCC_VIT_PREFETCH_CAP overrides.
+        self.prefetch_grid_cap = int(os.environ.get("LCC_VIT_PREFETCH_CAP", "-1"))
+
+    # ---- constructors ----
+    @classmethod
+    def from_pretrained(cls, model_path: str, torch_dtype="auto", device_map=None, attn_implementation=None, **kw):
+        """Same call as ref demo/infer.py:43-47.  bf16 only ('auto' resolves to bf16 for these checkpoints)."""
+        device = _check_load_args(torch_dtype, device_map)
+        cfg = get_config(model_path)
+        gen_cfg, eos_ids = read_generation_config(model_path)
+        if eos_ids is not None and "eos_token_ids" not in kw:
+            kw["eos_token_ids"] = eos_ids
+        arena = _arena_from_pretrained(model_path, cfg, device, llm_fp8=bool(kw.pop("llm_fp8", False)))
+        model = cls(cfg, arena, device, **kw)
+        model.generation_config = gen_cfg
+        return model
+
+    @classmethod
+    def from_config(cls, cfg: LiveCCConfig, device="cuda", seed: int = 0, llm_fp8: bool = False, **kw):
+        """llm_fp8: quantise the LLM Linear weights to OCP e4m3 with per-output-row scales (the 72B single-GPU weight path)."""
+        return cls(cfg, WeightArena(cfg, device, llm_fp8=llm_fp8).fill_random(seed), device, **kw)
+
+    @classmethod
+    def from_hf_model(cls, hf_model, cfg: LiveCCConfig, device="cuda", llm_fp8: bool = False, **kw):
+        """Weights of an instantiated HF model (the oracle-parity constructor): positions follow the INSTALLED transformers
+        (5.x text-offset rule) unless told otherwise, so that one-shot long clips compare equal to that oracle."""
+        kw.setdefault("text_offset_rule", "hf5")
+        return cls(cfg, _arena_from_hf(hf_model, cfg, device, llm_fp8=llm_fp8), device, **kw)
+
+    # ---- family hooks of EngineModel ----
+    def _embedding_rows(self, ids: np.ndarray) -> np.ndarray:
+        return (ids == self.cfg.video_token_id) | (ids == self.cfg.image_token_id)
+
+    def _encode_clips(self, clips: list) -> torch.Tensor:
+        return self._vit_for(clips)
+
+    def _prefetch(self, prefetch) -> None:
+        self._prefetch_vit(prefetch)
+
+    def _request_inputs(self, rq: dict, st: StreamState, new: np.ndarray, past_len: int, clips: list) -> np.ndarray:
+        cfg = self.cfg
+        grids = []
+        n_vid = int((new == cfg.video_token_id).sum())
+        if n_vid:
+            if rq.get("frames") is not None:
+                f = rq["frames"]
+                lay = rq.get("frames_layout", "TCHW")
+                if not f.is_cuda:
+                    f = f.to(self.device, non_blocking=True)
+                f = f.contiguous()
+                T, H, W = (f.shape[0], f.shape[2], f.shape[3]) if lay == "TCHW" else (f.shape[0], f.shape[1], f.shape[2])
+                grids = [protocol.grid_of(T, H, W, cfg)]
+                clips.append(dict(frames=f, layout=lay, key=self._clip_key(f, lay)))
+            elif rq.get("pixel_values_videos") is not None:
+                g = torch.as_tensor(rq["video_grid_thw"]).reshape(-1, 3).tolist()
+                pv = rq["pixel_values_videos"].to(self.device, dtype=torch.float32).contiguous()
+                off = 0
+                for t, h, w in g:
+                    clips.append(dict(pixel_values=pv[off:off + t * h * w], grid=(t, h, w)))
+                    off += t * h * w
+                grids = [tuple(x) for x in g]
+            else:
+                raise ValueError("input_ids contain <|video_pad|> but no frames / pixel_values_videos were given")
+            if sum(protocol.num_video_tokens(g, cfg) for g in grids) != n_vid:
+                raise ValueError(f"Video features and video tokens do not match, tokens: {n_vid}, features: "
+                                 f"{sum(protocol.num_video_tokens(g, cfg) for g in grids)}")
+        return self._positions(st, new, grids, past_len)
+
+    def _positions(self, st: StreamState, ids_new: np.ndarray, grids, past_len: int) -> np.ndarray:
+        if past_len == 0:
+            pos, delta = protocol.rope_index_first_turn(ids_new, grids, self.cfg, self.text_offset_rule)
+            st.rope_delta = delta
+            return pos
+        if st.rope_delta is None:
+            st.rope_delta = 0
+        return protocol.positions_with_cache(past_len, len(ids_new), st.rope_delta)
+
+    @torch.inference_mode()
+    def generate(self, input_ids: torch.Tensor = None, pixel_values_videos: Optional[torch.Tensor] = None,
+                 video_grid_thw: Optional[torch.Tensor] = None, mm_token_type_ids=None,
+                 past_key_values: Optional[StreamState] = None, return_dict_in_generate: bool = True,
+                 do_sample: Optional[bool] = None, repetition_penalty: float = 1.0, logits_processor=None,
+                 max_new_tokens: int = 16, min_new_tokens: Optional[int] = None, pad_token_id: Optional[int] = None,
+                 eos_token_id: Optional[int] = None, frames: Optional[torch.Tensor] = None, frames_layout: str = "TCHW",
+                 output_logits: bool = False, output_scores: bool = False, attention_mask=None, teacher_tokens=None, **unused):
+        """`teacher_tokens` (tests): the generated tokens are forced to this sequence (what the HF oracle does with a forcing
+        LogitsProcessor) while `output_logits` keeps the model's own raw logits of every step."""
+        sampling_kw = self._resolve_sampling(do_sample, unused)
+        if attention_mask is not None and not bool(torch.as_tensor(attention_mask).all()):
+            raise NotImplementedError("padding masks are not supported (the reference passes none, infer.py:156)")
+        if input_ids.dim() != 2 or input_ids.shape[0] != 1:
+            raise ValueError("generate() is single-stream like the reference (batch 1); use generate_batch for many streams")
+        if min_new_tokens is not None and min_new_tokens not in (0, max_new_tokens):
+            raise NotImplementedError("min_new_tokens must be None/0 or equal to max_new_tokens")
+        r = self.generate_batch([dict(
+            input_ids=input_ids[0], pixel_values_videos=pixel_values_videos,
+            video_grid_thw=video_grid_thw, frames=frames, frames_layout=frames_layout, state=past_key_values)],
+            repetition_penalty=repetition_penalty, logits_processor=logits_processor, max_new_tokens=max_new_tokens,
+            force_length=bool(min_new_tokens), eos_token_id=eos_token_id, output_logits=output_logits,
+            output_scores=output_scores, teacher_tokens=None if teacher_tokens is None else [list(teacher_tokens)], **sampling_kw)[0]
+        return r if return_dict_in_generate else r.sequences
 
     # ---- vision-tower prefetch on a side stream ----
     @staticmethod
@@ -543,43 +683,6 @@ class LiveCCForConditionalGeneration:
         self._vit_last_event = ev
         return out
 
-    def _prefill(self, slots, ids_new, pos3, vit, sp, scores_buf, logits_buf) -> None:
-        """One packed prefill when everything fits `max_new_rows`; otherwise consecutive streams are packed into groups of at
-        most `max_new_rows` rows (one launch sequence per group), and a stream that is longer than that by itself is prefilled
-        alone in pieces over its carried KV (a prompt prefilled in one or in several calls gives bit-identical logits:
-        tests/test_gpu_fullsize.py; only the LAST piece's sampled token survives -- each prefill call restarts the history
-        column -- which is exactly the token of the un-split prefill)."""
-        cfg, eng = self.cfg, self.engine
-        cap = eng.max_new_rows
-        lens = [len(x) for x in ids_new]
-        if sum(lens) <= cap:
-            eng.prefill(slots, ids_new, pos3, vit, sp, scores_out=scores_buf, logits_out=logits_buf)
-            return
-        is_vid = [(ids == cfg.video_token_id) | (ids == cfg.image_token_id) for ids in ids_new]
-        n_vid = [int(m.sum()) for m in is_vid]
-        row0 = np.concatenate([[0], np.cumsum(n_vid)]).astype(np.int64)      # first ViT row of every stream
-        sc = (lambda a, e: scores_buf[a:e]) if scores_buf is not None else (lambda a, e: None)
-        lg = (lambda a, e: logits_buf[0, a:e]) if logits_buf is not None else (lambda a, e: None)   # step 0 = the prefill's token
-        b, n = 0, len(slots)
-        while b < n:
-            if lens[b] > cap:                                   # one long prompt (one-shot video_qa / mcq): pieces over its own KV
-                ids, pos, nv_before = ids_new[b], pos3[b], 0
-                for a in range(0, lens[b], cap):
-                    e = min(lens[b], a + cap)
-                    k = int(is_vid[b][a:e].sum())
-                    rows = vit[row0[b] + nv_before:row0[b] + nv_before + k] if (vit is not None and k) else None
-                    nv_before += k
-                    eng.prefill([slots[b]], [ids[a:e]], [pos[:, a:e]], rows, sp, scores_out=sc(b, b + 1), logits_out=lg(b, b + 1))
-                b += 1
-                continue
-            e, rows_sum = b, 0
-            while e < n and lens[e] <= cap and rows_sum + lens[e] <= cap:
-                rows_sum += lens[e]
-                e += 1
-            rows = vit[row0[b]:row0[e]] if (vit is not None and row0[e] > row0[b]) else None
-            eng.prefill(slots[b:e], ids_new[b:e], pos3[b:e], rows, sp, scores_out=sc(b, e), logits_out=lg(b, e))
-            b = e
-
     # ---- ViT only (frames/s benchmarks, parity tests) ----
     @torch.inference_mode()
     def get_video_features(self, pixel_values_videos: torch.Tensor = None, video_grid_thw=None, frames=None,
@@ -594,3 +697,60 @@ class LiveCCForConditionalGeneration:
                 clips.append(dict(pixel_values=pv[off:off + t * h * w], grid=(t, h, w)))
                 off += t * h * w
             return self._vit_encode(clips)
+
+
+class DebunexForCausalLM(EngineModel):
+    """Debunex on the engine: `from_pretrained(path)`, `generate(input_ids, past_key_values=...)`, `generate_batch([...])` with the sampling
+    arguments of the other family (greedy, repetition penalty, temperature / top-k / top-p), `forward_step` for given ids.  Text ids only;
+    raw logits are fp32.  bf16 weights and activations; no fp32 mode and no CPU path."""
+    main_input_name = "input_ids"
+    logits_dtype = torch.float32
+
+    def __init__(self, cfg: DebunexConfig, weights: WeightArena, device, max_streams: int = 1, max_kv_len: Optional[int] = None,
+                 max_new_rows: int = 4096, max_history: int = 512, eos_token_ids: Optional[Sequence[int]] = None):
+        ids = [] if cfg.eos_token_id is None else [int(cfg.eos_token_id)]
+        ids += [int(t) for t in (eos_token_ids or []) if int(t) not in ids]
+        self._init_engine(cfg, weights, device, max_streams, max_kv_len, max_new_rows, 0, max_history, ids)
+
+    @classmethod
+    def from_pretrained(cls, model_path: str, torch_dtype="auto", device_map=None, **kw):
+        device = _check_load_args(torch_dtype, device_map)
+        cfg = get_config(model_path)
+        if not isinstance(cfg, DebunexConfig):
+            raise ValueError(f"{model_path} is not a Debunex checkpoint")
+        gen_cfg, eos_ids = read_generation_config(model_path)
+        if eos_ids is not None and "eos_token_ids" not in kw:
+            kw["eos_token_ids"] = eos_ids
+        model = cls(cfg, _arena_from_pretrained(model_path, cfg, device), device, **kw)
+        model.generation_config = gen_cfg
+        return model
+
+    @classmethod
+    def from_config(cls, cfg: DebunexConfig, device="cuda", seed: int = 0, **kw):
+        return cls(cfg, make_arena(cfg, device).fill_random(seed), device, **kw)
+
+    def _scores_width(self) -> int:
+        return self.cfg.vocab_pad
+
+    @torch.inference_mode()
+    def generate(self, input_ids: torch.Tensor = None, past_key_values: Optional[StreamState] = None, return_dict_in_generate: bool = True,
+                 do_sample: Optional[bool] = None, repetition_penalty: float = 1.0, max_new_tokens: int = 16, min_new_tokens: Optional[int] = None,
+                 eos_token_id: Optional[int] = None, output_logits: bool = False, output_scores: bool = False, teacher_tokens=None, **unused):
+        sampling_kw = self._resolve_sampling(do_sample, unused)
+        if input_ids.dim() != 2 or input_ids.shape[0] != 1:
+            raise ValueError("generate() is single-stream (batch 1); use generate_batch for many streams")
+        if min_new_tokens is not None and min_new_tokens not in (0, max_new_tokens):
+            raise NotImplementedError("min_new_tokens must be None/0 or equal to max_new_tokens")
+        r = self.generate_batch([dict(input_ids=input_ids[0], state=past_key_values)], repetition_penalty=repetition_penalty,
+                                max_new_tokens=max_new_tokens, force_length=bool(min_new_tokens), eos_token_id=eos_token_id, output_logits=output_logits,
+                                output_scores=output_scores, teacher_tokens=None if teacher_tokens is None else [list(teacher_tokens)], **sampling_kw)[0]
+        return r if return_dict_in_generate else r.sequences
+
+
+# config.json "architecture" -> model class (None: a Qwen2-VL checkpoint)
+MODEL_CLASSES = {None: LiveCCForConditionalGeneration, "Debunex": DebunexForCausalLM}
+
+
+def load_model(model_path: str, **kw) -> EngineModel:
+    """The model class a checkpoint directory's config.json asks for, loaded with `from_pretrained(model_path, **kw)`."""
+    return MODEL_CLASSES[architecture_of(model_path)].from_pretrained(model_path, **kw)

@@ -24,7 +24,7 @@ from typing import Callable, Dict, Iterable, List, Tuple
 
 import torch
 
-from .config import LiveCCConfig
+from .config import DebunexConfig, LiveCCConfig
 
 
 def qkv_decode_row_permutation(cfg: LiveCCConfig) -> torch.Tensor:
@@ -143,12 +143,19 @@ def interleave_gate_up(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
 
 
 class WeightArena:
+    row_major = ROW_MAJOR
+
     def __init__(self, cfg: LiveCCConfig, device, llm_fp8: bool = False):
         """llm_fp8: the LLM Linear weights + lm_head are stored as OCP e4m3 bytes (PACKED8 order) followed by their fp32 row
         scales (`<name>.scale`) -- 1 byte per parameter instead of 2 (72B: 73 GB instead of 147 GB)."""
         self.cfg, self.device, self.llm_fp8 = cfg, torch.device(device), bool(llm_fp8)
-        self.shapes = weight_shapes(cfg, decode_copies=True)           # round 3: the fp8 arena carries the decode copies too (pipeline v2)
-        self.fp8 = set(fp8_weight_names(cfg)) if llm_fp8 else set()
+        self._allocate(weight_shapes(cfg, decode_copies=True), set(fp8_weight_names(cfg)) if llm_fp8 else set())   # fp8: the decode copies too
+        hd = cfg.head_dim
+        # HF Qwen2VLRotaryEmbedding.compute_default_rope_parameters (modeling_qwen2_vl.py:129-146), fp32 on CPU
+        self.inv_freq = (1.0 / (cfg.rope_theta ** (torch.arange(0, hd, 2, dtype=torch.float) / hd))).to(self.device)
+
+    def _allocate(self, shapes, fp8: set) -> None:
+        self.shapes, self.fp8 = shapes, fp8
         offs, total = {}, 0          # offsets / sizes in bf16 (2-byte) units
         for name, shp in self.shapes:
             n = 1
@@ -162,9 +169,6 @@ class WeightArena:
                 total += (2 * shp[0] + 127) // 128 * 128
         self.offsets, self.numel = offs, total
         self.flat = torch.empty(total, dtype=torch.bfloat16, device=self.device)
-        hd = cfg.head_dim
-        # HF Qwen2VLRotaryEmbedding.compute_default_rope_parameters (modeling_qwen2_vl.py:129-146), fp32 on CPU
-        self.inv_freq = (1.0 / (cfg.rope_theta ** (torch.arange(0, hd, 2, dtype=torch.float) / hd))).to(self.device)
 
     def is_fp8(self, name: str) -> bool:
         return name in self.fp8
@@ -180,7 +184,7 @@ class WeightArena:
         return self.flat[o:o + n].view(*shp)
 
     def is_packed(self, name: str) -> bool:
-        return len(self.offsets[name][2]) == 2 and name not in ROW_MAJOR
+        return len(self.offsets[name][2]) == 2 and name not in self.row_major
 
     def logical(self, name: str) -> torch.Tensor:
         """Row-major [N,K] values of a (possibly packed / fp8) weight (tests / export); fp8 weights come back dequantised (fp32)."""
@@ -303,6 +307,133 @@ class WeightArena:
         put("final_norm", sd_get("language_model.norm.weight"))
         put("lm_head", sd_get("language_model.embed_tokens.weight") if cfg.tie_word_embeddings else sd_get("lm_head.weight"))
         return self
+
+
+# ---- layer-list decoders ----
+def decoder_weight_shapes(cfg: DebunexConfig) -> List[Tuple[str, Tuple[int, ...]]]:
+    """Stored (zero-padded) shapes.  Per layer: norm; in_w = query latent | own cache latent | gate rows; uq_w; the key map twice (uk_w for
+    the prefill GEMM, ukt_w = per head [rank, dim] for the decode queries); uv_w row-major (an activation-side operand in prefill);
+    gate_up_w interleaved; out_w = [attention | feed-forward] columns side by side: the parallel sublayers are one product."""
+    W, V = cfg.width_pad, cfg.vocab_pad
+    norm = lambda p: [(p + "_w", (W,)), (p + "_b", (W,)), (p + "_alpha", (1,))]
+    out: List[Tuple[str, Tuple[int, ...]]] = [("embed", (cfg.vocab_size, W))]
+    for i, l in enumerate(cfg.layers):
+        m, p = l.mixer, f"dec.{i}."
+        R, Q = m.kv_rank_pad, m.q_rank_pad
+        out += norm(p + "norm") + [(p + "in_w", (m.in_rows, W)), (p + "q_norm", (Q,)), (p + "uq_w", (m.heads * m.dim_pad, Q)),
+                                   (p + "uk_w", (m.heads * m.dim_pad, R)), (p + "ukt_w", (m.heads * R, m.dim_pad)), (p + "uv_w", (m.heads * m.vdim_pad, R)),
+                                   (p + "out_w", (W, m.heads * m.vdim_pad + l.ff_pad))]
+        if m.kv_from is None:
+            out.append((p + "kv_norm", (R,)))
+        if l.ff:
+            out.append((p + "gate_up_w", (2 * l.ff_pad, W)))
+    return out + norm("final_norm") + [("lm_head", (V, W))]
+
+
+def decoder_param_shapes(cfg: DebunexConfig) -> Dict[str, Tuple[int, ...]]:
+    """Tensor names and shapes of a checkpoint."""
+    W = cfg.hidden_size
+    out: Dict[str, Tuple[int, ...]] = {"embed": (cfg.vocab_size, W), "head": (cfg.vocab_size, W)}
+    norms = ["final.norm"]
+    for i, l in enumerate(cfg.layers):
+        m, p = l.mixer, f"l{i}."
+        norms.append(p + "norm1")
+        out.update({p + "mix.dq": (m.q_rank, W), p + "mix.dq.norm": (m.q_rank,), p + "mix.uq": (m.heads * m.dim, m.q_rank),
+                    p + "mix.uk": (m.heads * m.dim, m.kv_rank), p + "mix.uv": (m.heads * m.vdim, m.kv_rank), p + "mix.g": (m.heads, W),
+                    p + "mix.o": (W, m.heads * m.vdim)})
+        if m.kv_from is None:
+            out.update({p + "mix.dkv": (m.kv_rank, W), p + "mix.dkv.norm": (m.kv_rank,)})
+        if l.ff:
+            out.update({p + "mlp.gate": (l.ff, W), p + "mlp.up": (l.ff, W), p + "mlp.down": (W, l.ff)})
+    for n in norms:
+        out.update({n: (W,), n + ".b": (W,), n + ".alpha": ()})
+    return out
+
+
+def _pad(t: torch.Tensor, shape: Tuple[int, ...]) -> torch.Tensor:
+    if tuple(t.shape) == tuple(shape):
+        return t
+    out = t.new_zeros(shape)
+    out[tuple(slice(0, n) for n in t.shape)] = t
+    return out
+
+
+class DecoderArena(WeightArena):
+    """The weights of a layer-list decoder in the engine's order; same flat arena, packing and views."""
+
+    def __init__(self, cfg: DebunexConfig, device):
+        self.cfg, self.device, self.llm_fp8 = cfg, torch.device(device), False
+        self._allocate(decoder_weight_shapes(cfg), set())
+        self.row_major = {"embed"} | {f"dec.{i}.uv_w" for i in range(cfg.num_hidden_layers)}
+
+    @torch.no_grad()
+    def load_state_dict(self, sd_get: Callable[[str], torch.Tensor]) -> "DecoderArena":
+        cfg = self.cfg
+        W = cfg.width_pad
+        shapes = decoder_param_shapes(cfg)
+
+        def get(name: str) -> torch.Tensor:
+            t = sd_get(name)
+            if tuple(t.shape) != shapes[name]:
+                raise ValueError(f"{name}: checkpoint shape {tuple(t.shape)}, the configuration says {shapes[name]}")
+            return t.to(torch.bfloat16)
+
+        def put_norm(dst: str, src: str) -> None:
+            self.store(dst + "_w", _pad(get(src), (W,)))
+            self.store(dst + "_b", _pad(get(src + ".b"), (W,)))
+            self.store(dst + "_alpha", get(src + ".alpha").reshape(1))
+
+        self.store("embed", _pad(get("embed"), (cfg.vocab_size, W)))
+        for i, l in enumerate(cfg.layers):
+            m, p, s = l.mixer, f"dec.{i}.", f"l{i}."
+            H, R, Q = m.heads, m.kv_rank_pad, m.q_rank_pad
+            put_norm(p + "norm", s + "norm1")
+            parts = [_pad(get(s + "mix.dq"), (Q, W))]
+            if m.kv_from is None:
+                parts.append(_pad(get(s + "mix.dkv"), (R, W)))
+                self.store(p + "kv_norm", _pad(get(s + "mix.dkv.norm"), (R,)))
+            parts.append(_pad(get(s + "mix.g"), (m.in_rows - sum(x.shape[0] for x in parts), W)))
+            self.store(p + "in_w", torch.cat(parts))
+            self.store(p + "q_norm", _pad(get(s + "mix.dq.norm"), (Q,)))
+            self.store(p + "uq_w", _pad(get(s + "mix.uq").view(H, m.dim, m.q_rank), (H, m.dim_pad, Q)).reshape(H * m.dim_pad, Q))
+            uk = _pad(get(s + "mix.uk").view(H, m.dim, m.kv_rank), (H, m.dim_pad, R))
+            self.store(p + "uk_w", uk.reshape(H * m.dim_pad, R))
+            self.store(p + "ukt_w", uk.transpose(1, 2).reshape(H * R, m.dim_pad))
+            self.store(p + "uv_w", _pad(get(s + "mix.uv").view(H, m.vdim, m.kv_rank), (H, m.vdim_pad, R)).reshape(H * m.vdim_pad, R))
+            cols = [_pad(get(s + "mix.o").view(cfg.hidden_size, H, m.vdim), (W, H, m.vdim_pad)).reshape(W, H * m.vdim_pad)]
+            if l.ff:
+                self.store(p + "gate_up_w", interleave_gate_up(_pad(get(s + "mlp.gate"), (l.ff_pad, W)), _pad(get(s + "mlp.up"), (l.ff_pad, W))))
+                cols.append(_pad(get(s + "mlp.down"), (W, l.ff_pad)))
+            self.store(p + "out_w", torch.cat(cols, dim=1))
+        put_norm("final_norm", "final.norm")
+        self.store("lm_head", _pad(get("head"), (cfg.vocab_pad, W)))
+        return self
+
+    @torch.no_grad()
+    def fill_random(self, seed: int = 0, std: float = 0.02) -> "DecoderArena":
+        """Random weights of the checkpoint's shapes, generated on the arena's device: N(0, std) matrices, latent norms around 1, Dynamic Tanh
+        with alpha 0.5 and a small bias."""
+        shapes = decoder_param_shapes(self.cfg)
+        g = torch.Generator(device=self.device).manual_seed(seed)
+
+        def make(name: str) -> torch.Tensor:
+            shp = shapes[name]
+            if name.endswith(".alpha"):
+                return torch.full((), 0.5, device=self.device)
+            x = torch.randn(shp, generator=g, device=self.device, dtype=torch.float32)
+            if len(shp) >= 2:
+                return x.mul_(std)
+            return x.mul_(0.05) if name.endswith(".b") else x.mul_(0.1).add_(1.0)
+        return self.load_state_dict(make)
+
+
+def make_arena(cfg, device, llm_fp8: bool = False) -> WeightArena:
+    """The weight arena of a configuration's model family."""
+    if isinstance(cfg, DebunexConfig):
+        if llm_fp8:
+            raise ValueError("fp8 weights are available for the Qwen2-VL family only")
+        return DecoderArena(cfg, device)
+    return WeightArena(cfg, device, llm_fp8=llm_fp8)
 
 
 TILE_PERIOD = 4194301      # prime: gcd with every row length is 1, so no two rows of any weight matrix are equal
@@ -451,4 +582,4 @@ def from_pretrained(path: str, cfg: LiveCCConfig, device, llm_fp8: bool = False)
         f, k = index[name]
         return handles[f].get_tensor(k)
 
-    return WeightArena(cfg, device, llm_fp8=llm_fp8).load_state_dict(get)
+    return make_arena(cfg, device, llm_fp8).load_state_dict(get)
