@@ -51,12 +51,18 @@ def parse(argv=None):
     ap.add_argument("--max-new-tokens", type=int, default=16)
     ap.add_argument("--fused-tails", type=int, default=None, choices=[0, 1],
                     help="debug A/B: fuse add+rmsnorm / rope+append into the decode GEMV tails (default: library default)")
-    ap.add_argument("--workload", choices=["stream60", "long480", "oneshot480"], default="stream60",
+    ap.add_argument("--workload", choices=["stream60", "long480", "oneshot480", "decoder"], default="stream60",
                     help="long480 = BASELINE.json configs[3]: one 480-frame 280x280 video (24k visual tokens), 12 tokens per turn, "
                          "KV growing to ~32k; oneshot480 = the OTHER half of configs[3]: the reference's video_qa / MCQ first turn "
                          "(ref demo/infer.py:182-242): all 480 frames in ONE generate call (ViT over 96,000 patches in 240 segments, "
                          "one 24k-row LLM prefill served in pieces, then 32 decode tokens at L ~ 24k); both override "
-                         "--frames/--height/--width/--max-new-tokens")
+                         "--frames/--height/--width/--max-new-tokens; decoder = prefill / decode throughput of the Debunex decoder beside the "
+                         "Qwen2-VL language model at equal size (tools/bench_decoder.py)")
+    ap.add_argument("--decoder-size", choices=["2b", "7b"], default=None, help="decoder: one size only")
+    ap.add_argument("--decoder-layers", type=int, default=28, help="decoder: layers of both models")
+    ap.add_argument("--decoder-prefill", default="512,2048,8192", help="decoder: prompt lengths")
+    ap.add_argument("--decoder-decode", default="1x1024,1x8192,8x4096,32x4096", help="decoder: streams x cached keys")
+    ap.add_argument("--decoder-only", action="store_true", help="decoder: without the model it is compared with")
     ap.add_argument("--time-budget-s", type=float, default=660.0,
                     help="target wall time of the whole run: the OPTIONAL blocks (live2fps history ladder, configs[3] / configs[4] children and their "
                          "fixture tests) are skipped -- with the reason in their block -- once the time left, after 130 s reserved for the CPU "
@@ -829,6 +835,10 @@ def main():
     t_bench0 = time.perf_counter()
     sections = {}            # wall seconds per block of this run (rank 0), reported as `sections_s`
     args = parse()
+    if args.workload == "decoder":
+        sys.path.insert(0, os.path.join(ROOT, "tools"))
+        import bench_decoder
+        return bench_decoder.main(args)
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
         sys.exit(self_launch(args))
     from livecc_amd import distributed as D, protocol

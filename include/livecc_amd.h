@@ -378,6 +378,9 @@ typedef struct {
   int vocab_size, vocab_pad, width_pad, n_layers;
   float norm_eps, logit_softcap;                /* logit_softcap <= 0: none */
 } lcc_decoder_config;
+/* 1 (default): decode steps of up to 16 streams run the fused launches (input + gate/up projections in one; query norm, up-projection, cache
+ * append and gates in one for up to 8 streams; output projection + residual + next norm in one); 0: separate launches.  Returns the old value */
+int lcc_debug_set_decoder_fused(int on);
 lcc_engine* lcc_engine_create_decoder(const lcc_decoder_config* cfg, const lcc_decoder_layer* layers, const lcc_engine_limits* lim);
 void lcc_engine_destroy(lcc_engine* e);
 /* bytes the caller must provide (allocated by PyTorch so that torch.distributed can broadcast into them) */

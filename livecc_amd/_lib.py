@@ -156,6 +156,7 @@ def load():
         "lcc_latent_absorb": (i32, [vp, i32, i32, i32, i32, vp, i32, vp, vp]),
         "lcc_latent_attn_decode": (i32, [vp, vp, vp, vp, i64, i32, i32, i32, f32, i32, vp, vp, vp, i32, vp, vp, i32, vp]),
         "lcc_engine_create_decoder": (vp, [C.POINTER(DecoderConfigC), C.POINTER(DecoderLayer), C.POINTER(EngineLimits)]),
+        "lcc_debug_set_decoder_fused": (i32, [i32]),
         "lcc_slot_set_tokens": (i32, [vp, i32, vp, vp, vp]),
         "lcc_engine_create": (vp, [C.POINTER(ModelConfig), C.POINTER(EngineLimits)]),
         "lcc_engine_destroy": (None, [vp]),

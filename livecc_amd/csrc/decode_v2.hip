@@ -29,13 +29,14 @@
 
 #include "common.h"
 #include "kernels.h"
+#include "latent_ops.h"
 
 namespace lcc {
 
 __device__ unsigned int lcc_zero_page_v2[64];  // 256 zero bytes: activation operand of absent K chunks
 
-enum { DG_PRO_PLAIN = 0, DG_PRO_NORM = 1 };
-enum { DG_EPI_BF16 = 0, DG_EPI_SWIGLU = 1, DG_EPI_RESID = 2, DG_EPI_ROPE = 3 };
+enum { DG_PRO_PLAIN = 0, DG_PRO_NORM = 1, DG_PRO_RMS32 = 2 };      // RMS32: fp32 rows, the wave that normalises a row forms its statistic
+enum { DG_EPI_BF16 = 0, DG_EPI_SWIGLU = 1, DG_EPI_RESID = 2, DG_EPI_ROPE = 3, DG_EPI_F32 = 4, DG_EPI_RESID_DYT = 5 };
 
 // ---- chained launches (round 3): two dependent GEMVs in ONE launch.  The consumer's blocks (q/k/v of layer l+1) are resident next to
 // the producer's (down_proj of layer l), request their weights -- which do not depend on the producer -- right away, and only then
@@ -195,6 +196,18 @@ LCC_DEVICE void dgemv_body(const DgArgs& a, const DgChain& ch, const int bid, f3
   const int kp = K >> 3, xpieces = PRO == DG_PRO_NORM ? M * kp : 0;
   f32x4 pv[PRO == DG_PRO_NORM ? MR : 1][2];
   u32x4 hv[PRO == DG_PRO_NORM ? XP : 1], nv[PRO == DG_PRO_NORM ? XP : 1];
+  // PRO_RMS32: wave m normalises row m (M <= NW, K <= 2048): 4-channel pieces lane, lane + 64, ..
+  constexpr int SP = PRO == DG_PRO_RMS32 ? 8 : 1;
+  f32x4 sv[SP];
+  u32x2 swv[SP];
+  if (PRO == DG_PRO_RMS32 && wave < M) {
+#pragma unroll
+    for (int u = 0; u < SP; ++u) {
+      const int c = min((lane + 64 * u) * 4, K - 4);
+      sv[u] = *reinterpret_cast<const f32x4*>(a.S32 + (size_t)wave * a.lds32 + c);
+      swv[u] = ld8(a.norm_w + c);
+    }
+  }
   if (PRO == DG_PRO_NORM) {
 #pragma unroll
     for (int m = 0; m < MR; ++m)
@@ -215,7 +228,15 @@ LCC_DEVICE void dgemv_body(const DgArgs& a, const DgChain& ch, const int bid, f3
   u32x2 e_h = {0u, 0u}, e_b = {0u, 0u}, e_c = {0u, 0u}, e_s = {0u, 0u};
   int e_pos = 0;
   bf16_t* e_base = nullptr;
+  f32x4 e_x = {0.f, 0.f, 0.f, 0.f};
+  float e_alpha = 0.f;
   if (wave == 0) {
+    if (EPI == DG_EPI_RESID_DYT) {
+      const int n = min(n0 + g * 4, N - 4);
+      e_x = *reinterpret_cast<const f32x4*>(a.X32 + (size_t)xm * N + n);
+      e_c = ld8(a.dyt.w + n); e_s = ld8(a.dyt.b + n);
+      e_alpha = bf2f(a.dyt.alpha[0]);
+    }
     if (EPI == DG_EPI_RESID) {
       const int n = n0 + g * 4;
       if (li < M && n < N) e_h = ld8(a.Hres + (size_t)li * N + n);
@@ -261,6 +282,23 @@ LCC_DEVICE void dgemv_body(const DgArgs& a, const DgChain& ch, const int bid, f3
                                                                  ld16(a.norm_w + (size_t)(p % kp) * 8), row_r(p / kp));
     __syncthreads();
   }
+  if (PRO == DG_PRO_RMS32) {
+    if (wave < M) {
+      float ss = 0.f;
+#pragma unroll
+      for (int u = 0; u < SP; ++u)
+        if ((lane + 64 * u) * 4 < K) ss += (sv[u][0] * sv[u][0] + sv[u][1] * sv[u][1]) + (sv[u][2] * sv[u][2] + sv[u][3] * sv[u][3]);
+      const float r = 1.f / sqrtf(wave_sum(ss) / (float)a.rank + a.eps);      // padding channels are zeros: the mean is over the real ones
+#pragma unroll
+      for (int u = 0; u < SP; ++u) {
+        const int c4 = (lane + 64 * u) * 4;
+        if (c4 < K)
+          st8(s_x + (size_t)wave * K + c4, (u32x2){pack2(sv[u][0] * r * lo2f(swv[u].x), sv[u][1] * r * hi2f(swv[u].x)),
+                                                   pack2(sv[u][2] * r * lo2f(swv[u].y), sv[u][3] * r * hi2f(swv[u].y))});
+      }
+    }
+    __syncthreads();
+  }
   for (; c < nchunk; c += 2 * STEP) {
     mma(sa, c);
     if (c + 2 * STEP < nchunk) { load_w(c + 2 * STEP, sa); load_x(c + 2 * STEP, sa); }   // wave-uniform: no loads past the last chunk
@@ -292,6 +330,16 @@ LCC_DEVICE void dgemv_body(const DgArgs& a, const DgChain& ch, const int bid, f3
       v[0] += lo2f(b.x); v[1] += hi2f(b.x); v[2] += lo2f(b.y); v[3] += hi2f(b.y);
     }
     st8(a.C + (size_t)li * a.ldc + n, (u32x2){pack2(v[0], v[1]), pack2(v[2], v[3])});
+  } else if (EPI == DG_EPI_F32) {
+    if (li < M && n0 + g * 4 < N) *reinterpret_cast<f32x4*>(a.C32 + (size_t)li * a.ldc + n0 + g * 4) = acc[0];
+  } else if (EPI == DG_EPI_RESID_DYT) {      // fp32 residual in place; the next norm has no row statistic and is finished here
+    const int n = n0 + g * 4;
+    if (li < M && n < N) {
+      const f32x4 v = e_x + acc[0];
+      *reinterpret_cast<f32x4*>(a.X32 + (size_t)li * N + n) = v;
+      st8(a.C + (size_t)li * N + n, (u32x2){pack2(dyt_value(v[0], e_alpha, lo2f(e_c.x), lo2f(e_s.x)), dyt_value(v[1], e_alpha, hi2f(e_c.x), hi2f(e_s.x))),
+                                            pack2(dyt_value(v[2], e_alpha, lo2f(e_c.y), lo2f(e_s.y)), dyt_value(v[3], e_alpha, hi2f(e_c.y), hi2f(e_s.y)))});
+    }
   } else if (EPI == DG_EPI_SWIGLU) {   // tile 0 = 16 gate rows, tile 1 = the 16 matching up rows (weights.py interleave_gate_up)
     if (li >= M || n0 >= N) return;
     float o[4];
@@ -379,6 +427,22 @@ __global__ __launch_bounds__(512, 4) void dgemv_down_qkv_kernel(DgArgs down, DgA
   else dgemv_body<1, DG_PRO_NORM, DG_EPI_ROPE, 8, 4, MR, DG_CHAIN_WAIT>(qkv, ch, (int)blockIdx.x - nb_down, red, s_x);
 }
 
+// ---- layer-list decoders (engine_decoder.hip): the same weight-streaming body behind a norm that is already applied ----
+// the fused input projection (fp32 out) and the gate/up projection (SwiGLU) of one layer in ONE launch: both read the normed row
+__global__ __launch_bounds__(256, 4) void dgemv_in_swiglu_kernel(DgArgs in, DgArgs sw, int nb_in) {
+  __shared__ f32x4 red[3][2][64];
+  const DgChain none{nullptr, 0u, nullptr, 0};
+  if ((int)blockIdx.x < nb_in) dgemv_body<1, DG_PRO_PLAIN, DG_EPI_F32, 4, 2, 2, DG_CHAIN_NONE>(in, none, blockIdx.x, reinterpret_cast<f32x4(*)[1][64]>(red), nullptr);
+  else dgemv_body<2, DG_PRO_PLAIN, DG_EPI_SWIGLU, 4, 1, 2, DG_CHAIN_NONE>(sw, none, (int)blockIdx.x - nb_in, red, nullptr);
+}
+// query up-projection of the normed query latent (norm as prologue, fp32 out); the M blocks behind it append the rows' cache latents and gates
+__global__ __launch_bounds__(512, 2) void dgemv_latent_q_kernel(DgArgs a, LatentInArgs row, int nb) {
+  __shared__ f32x4 red[7][1][64];
+  extern __shared__ __attribute__((aligned(16))) bf16_t s_x[];
+  if ((int)blockIdx.x < nb) dgemv_body<1, DG_PRO_RMS32, DG_EPI_F32, 8, 2, 2, DG_CHAIN_NONE>(a, DgChain{nullptr, 0u, nullptr, 0}, blockIdx.x, red, s_x);
+  else latent_row<512, false>(row, (int)blockIdx.x - nb, reinterpret_cast<float*>(red));
+}
+
 // ------------------------------------------------------------------------------------------------------------------------
 // step prologue: one block per stream does what were four launches (seen_set, embed_gather, mrope_table_decode, and the
 // first layer's RMSNorm statistic): marks the consumed token in the stream's seen-id bitmap (repetition penalty), gathers its
@@ -434,6 +498,32 @@ static int dg_check(const DgArgs& a, int pro, int epi) {
   if (epi == DG_EPI_ROPE && (a.bias == nullptr || a.cs == nullptr || a.sn == nullptr || a.tok_stream == nullptr || a.kv_len == nullptr ||
                              a.kv_base == nullptr || a.q_out == nullptr || a.lay.head_dim != 128 || (a.lay.lmax & 31) ||
                              a.N != (a.n_q_heads + 2 * a.lay.n_kv_heads) * 128)) return LCC_ERR_ARG;
+  return 0;
+}
+
+int dgemv_in_swiglu(const DgArgs& in, const DgArgs& sw, hipStream_t st) {
+  g_launch_counts[LC_DGEMV_V2]++;
+  if (in.M < 1 || in.M > 16 || sw.M != in.M || (in.N & 15) || (sw.N & 31) || (in.K & 31) || (sw.K & 31) || (in.ldx & 7) || (sw.ldx & 7) || (in.ldc & 3) || (sw.ldc & 3))
+    return LCC_ERR_SHAPE;
+  if (!in.W || !in.X || !in.C32 || in.wscale || (sw.N > 0 && (!sw.W || !sw.X || !sw.C || sw.wscale))) return LCC_ERR_ARG;
+  dgemv_in_swiglu_kernel<<<dim3(in.N / 16 + sw.N / 32), dim3(256), 0, st>>>(in, sw, in.N / 16);
+  return 0;
+}
+bool dgemv_latent_q_ok(int M, int K) { return M >= 1 && M <= 8 && K <= 2048 && (K & 31) == 0; }
+int dgemv_latent_q(const DgArgs& a, const LatentInArgs& row, hipStream_t st) {
+  g_launch_counts[LC_DGEMV_V2]++;
+  if (!dgemv_latent_q_ok(a.M, a.K) || (a.N & 15) || (a.lds32 & 3) || (a.ldc & 3) || a.rank < 1 || row.rows != a.M || row.nsplit != 1) return LCC_ERR_SHAPE;
+  if (!a.W || !a.S32 || !a.norm_w || !a.C32 || a.wscale) return LCC_ERR_ARG;
+  dgemv_latent_q_kernel<<<dim3(a.N / 16 + a.M), dim3(512), (size_t)a.M * a.K * 2, st>>>(a, row, a.N / 16);
+  return 0;
+}
+// fp32 residual += Linear(x), h = next norm
+int dgemv_resid_dyt(const DgArgs& a, hipStream_t st) {
+  g_launch_counts[LC_DGEMV_V2]++;
+  if (a.M < 1 || a.M > 16 || (a.N & 15) || (a.K & 31) || (a.ldx & 7)) return LCC_ERR_SHAPE;
+  if (!a.W || !a.X || !a.X32 || !a.C || !a.dyt.w || !a.dyt.b || !a.dyt.alpha || a.wscale) return LCC_ERR_ARG;
+  if (a.K >= 8192) dgemv_kernel<1, DG_PRO_PLAIN, DG_EPI_RESID_DYT, 16, 3><<<dim3(a.N / 16), dim3(1024), 0, st>>>(a);
+  else dgemv_kernel<1, DG_PRO_PLAIN, DG_EPI_RESID_DYT, 8, 4><<<dim3(a.N / 16), dim3(512), 0, st>>>(a);
   return 0;
 }
 

@@ -5,16 +5,16 @@
 // norm alone.  Rows are padded to a multiple of 64 channels with zero weights, so a padding channel stays 0 through the norm (w = b = 0).
 #include "common.h"
 #include "kernels.h"
+#include "latent_ops.h"
 
 namespace lcc {
 
-LCC_DEVICE float dyt(float x, float alpha, float w, float b) { return fmaf(tanhf(alpha * x), w, b); }
 LCC_DEVICE u32x4 dyt8(const float (&x)[8], float alpha, const bf16_t* w, const bf16_t* b) {
   const u32x4 wv = ld16(w), bv = ld16(b);
   u32x4 o;
 #pragma unroll
   for (int e = 0; e < 4; ++e)
-    o[e] = pack2(dyt(x[2 * e], alpha, lo2f(wv[e]), lo2f(bv[e])), dyt(x[2 * e + 1], alpha, hi2f(wv[e]), hi2f(bv[e])));
+    o[e] = pack2(dyt_value(x[2 * e], alpha, lo2f(wv[e]), lo2f(bv[e])), dyt_value(x[2 * e + 1], alpha, hi2f(wv[e]), hi2f(bv[e])));
   return o;
 }
 

@@ -4,6 +4,7 @@
 // engine's (engine.hip, engine_llm.hip); this file is the launch sequence of the layers and what they need in memory.
 //
 // A layer is
+// (decode steps of up to 16 rows fuse "in" with "ff", the norms with "query", and "out" with the residual and the next norm: decode_v2.hip)
 //   in      [Wdq | Wdkv | Wg] h           one GEMM, fp32 slabs
 //           norms -> query latent, c -> cache, gates          (latent_norm_append)
 //   query   Wuq cq                                            GEMM
@@ -61,7 +62,7 @@ size_t carve(const lcc_engine* e, DecBuffers* b, char* base) {
   Carver cv; cv.base = base;
   b->x = cv.take<float>(S * d.W); b->h = cv.take<bf16_t>(S * d.W);
   const size_t nmax = std::max(std::max(d.in_n, d.qd), d.W);
-  b->part_cap = std::max(std::max(S * nmax, (size_t)8 * 64 * nmax), std::max(LR * V, (size_t)16 << 20));
+  b->part_cap = std::max(std::max(S * nmax, (size_t)8 * 64 * nmax + 64), std::max(LR * V, (size_t)16 << 20));
   b->part = cv.take<float>(b->part_cap);
   b->gate = cv.take<float>(S * d.heads);
   b->cq = cv.take<bf16_t>(S * d.qp); b->q = cv.take<bf16_t>(S * d.qd); b->cat = cv.take<bf16_t>(S * d.cat);
@@ -110,8 +111,12 @@ int tap(lcc_engine* e, const DecBuffers& b, int index, int S, hipStream_t st) {
   return 0;
 }
 
+int g_fused_decode = 1;      // lcc_debug_set_decoder_fused: decode steps of up to 16 rows run the fused launches (6 per layer instead of 9)
+
 // S packed rows through every layer; pt null: a decode step over the streams `d_slots`.  On exit b.h holds the final norm of the residual.
-int run_decoder_layers(lcc_engine* e, const DecBuffers& b, int S, const PrefillTables* pt, const int32_t* d_slots, int nsplit_attn, hipStream_t st) {
+int run_decoder_layers(lcc_engine* e, const DecBuffers& b, int S, const PrefillTables* pt, const int32_t* d_slots, int nsplit_attn, const AttnDirect& direct,
+                       hipStream_t st) {
+  const bool fused = !pt && S <= 16 && g_fused_decode;
   const int W = e->c.hidden_size, NL = (int)e->dl.size();
   if (e->llm_over) return fail(LCC_ERR_STATE, "per-layer input overrides are not available for this model family");
   LCC_TRY(tap(e, b, 0, S, st));
@@ -123,11 +128,19 @@ int run_decoder_layers(lcc_engine* e, const DecBuffers& b, int S, const PrefillT
     const size_t kv_off = e->dec_kv_off[owner];
     const float scale_log2e = L.scale * 1.4426950408889634f;
     int ns = 1;
-    LCC_TRY(slab_gemm(b, b.h, W, w.in_w, S, in_n, W, &ns, st));
+    if (fused) {
+      DgArgs gi, gs;
+      gi.W = w.in_w; gi.M = S; gi.N = in_n; gi.K = W; gi.X = b.h; gi.ldx = W; gi.C32 = b.part; gi.ldc = in_n;
+      gs.W = w.gate_up_w; gs.M = S; gs.N = 2 * L.ff_pad; gs.K = W; gs.X = b.h; gs.ldx = W; gs.C = b.cat + L.heads * L.vdim_pad; gs.ldc = ldcat;
+      LCC_TRY(dgemv_in_swiglu(gi, gs, st));
+    } else {
+      LCC_TRY(slab_gemm(b, b.h, W, w.in_w, S, in_n, W, &ns, st));
+    }
     LatentInArgs in; in.part = b.part; in.nsplit = ns; in.rows = S; in.ldn = in_n; in.qp = L.q_rank_pad; in.rp = own ? rp : 0; in.q_rank = L.q_rank;
     in.kv_rank = L.kv_rank; in.heads = L.heads; in.eps = e->dc.norm_eps; in.q_norm = w.q_norm; in.kv_norm = w.kv_norm; in.cq = b.cq; in.gate = b.gate;
     in.tok_stream = pt ? pt->tok_stream : d_slots; in.tok_pos = pt ? pt->tok_pos : nullptr; in.kv_len = e->d_kv_len; in.kv_base = e->d_kv_base; in.kv_off = kv_off;
-    LCC_TRY(latent_norm_append(in, st));
+    const bool fused_q = fused && dgemv_latent_q_ok(S, L.q_rank_pad);
+    if (!fused_q) LCC_TRY(latent_norm_append(in, st));
     if (pt) {
       LCC_TRY(plain_gemm(b.cq, L.q_rank_pad, w.uq_w, b.q, L.heads * L.dim_pad, S, L.heads * L.dim_pad, L.q_rank_pad, LCC_EPI_NONE, st));
       for (const KeyGroup& kg : pt->groups) {
@@ -142,16 +155,31 @@ int run_decoder_layers(lcc_engine* e, const DecBuffers& b, int S, const PrefillT
         LCC_TRY(attn_mha(a, st));
       }
     } else {
-      LCC_TRY(slab_gemm(b, b.cq, L.q_rank_pad, w.uq_w, S, L.heads * L.dim_pad, L.q_rank_pad, &ns, st));
-      LCC_TRY(latent_absorb(b.part, ns, S, L.heads, L.dim_pad, w.ukt_w, rp, b.lat_q, st));
+      float* q32 = b.part;
+      if (fused_q) {
+        q32 = b.part + align_up((size_t)S * in_n, 64);      // beside the input projection it reads
+        DgArgs gq; gq.W = w.uq_w; gq.M = S; gq.N = L.heads * L.dim_pad; gq.K = L.q_rank_pad; gq.S32 = b.part; gq.lds32 = in_n; gq.rank = L.q_rank;
+        gq.norm_w = w.q_norm; gq.eps = e->dc.norm_eps; gq.C32 = q32; gq.ldc = gq.N;
+        LCC_TRY(dgemv_latent_q(gq, in, st));
+        ns = 1;
+      } else {
+        LCC_TRY(slab_gemm(b, b.cq, L.q_rank_pad, w.uq_w, S, L.heads * L.dim_pad, L.q_rank_pad, &ns, st));
+      }
+      LCC_TRY(latent_absorb(q32, ns, S, L.heads, L.dim_pad, w.ukt_w, rp, b.lat_q, st));
       LatentDecodeArgs a; a.q = b.lat_q; a.rows = S; a.heads = L.heads; a.rp = rp; a.nsplit = nsplit_attn; a.scale_log2e = scale_log2e; a.slots = d_slots;
-      a.kv_len = e->d_kv_len; a.kv_base = e->d_kv_base; a.kv_off = kv_off; a.ws_o = b.ws_o; a.ws_ml = b.ws_ml;
+      a.kv_len = e->d_kv_len; a.kv_base = e->d_kv_base; a.kv_off = kv_off; a.ws_o = b.ws_o; a.ws_ml = b.ws_ml; a.direct = direct;
       LCC_TRY(latent_attn_decode(a, st));
       LCC_TRY(latent_merge_uv(a, w.uv_w, L.vdim_pad, b.gate, b.cat, ldcat, st));
     }
-    if (L.ff_pad > 0) LCC_TRY(plain_gemm(b.h, W, w.gate_up_w, b.cat + L.heads * L.vdim_pad, ldcat, S, 2 * L.ff_pad, W, LCC_EPI_SWIGLU, st));
-    LCC_TRY(slab_gemm(b, b.cat, ldcat, w.out_w, S, W, ldcat, &ns, st));
-    LCC_TRY(resid_dyt(b.x, b.part, ns, l + 1 < NL ? e->dw[l + 1].norm : e->dec_final_norm, b.h, S, W, st));
+    if (!fused && L.ff_pad > 0) LCC_TRY(plain_gemm(b.h, W, w.gate_up_w, b.cat + L.heads * L.vdim_pad, ldcat, S, 2 * L.ff_pad, W, LCC_EPI_SWIGLU, st));
+    const DytNorm& next = l + 1 < NL ? e->dw[l + 1].norm : e->dec_final_norm;
+    if (fused) {
+      DgArgs go; go.W = w.out_w; go.M = S; go.N = W; go.K = ldcat; go.X = b.cat; go.ldx = ldcat; go.X32 = b.x; go.C = b.h; go.dyt = next;
+      LCC_TRY(dgemv_resid_dyt(go, st));
+    } else {
+      LCC_TRY(slab_gemm(b, b.cat, ldcat, w.out_w, S, W, ldcat, &ns, st));
+      LCC_TRY(resid_dyt(b.x, b.part, ns, next, b.h, S, W, st));
+    }
     LCC_TRY(tap(e, b, l + 1, S, st));
   }
   return 0;
@@ -291,7 +319,7 @@ int lcc_decoder_prefill(lcc_engine* e, int n_streams, const int32_t* slots, cons
   }
   LCC_TRY(seen_set(e->d_seen, e->words, d_ids, d_stream, S, 0, nullptr, st));
   LCC_TRY(embed_dyt(d_ids, nullptr, e->embed, e->dw[0].norm, bf.x, bf.h, S, e->c.hidden_size, st));
-  LCC_TRY(run_decoder_layers(e, bf, S, &pt, nullptr, 1, st));
+  LCC_TRY(run_decoder_layers(e, bf, S, &pt, nullptr, 1, AttnDirect(), st));
 
   const int LR = logit_rows_max(e), W = e->c.hidden_size;
   for (int r0 = 0; r0 < nw; r0 += LR) {
@@ -323,7 +351,7 @@ int lcc_decoder_prefill(lcc_engine* e, int n_streams, const int32_t* slots, cons
 }
 
 // the n_steps loop of lcc_llm_decode (engine_llm.hip) behind its checks
-int lcc_decoder_decode(lcc_engine* e, int n_streams, const int32_t* d_slots, int max_len, int n_steps, int first_step_index, const lcc_sampling* sp, hipStream_t st) {
+int lcc_decoder_decode(lcc_engine* e, int n_streams, const int32_t* slots, const int32_t* d_slots, int max_len, int n_steps, int first_step_index, const lcc_sampling* sp, hipStream_t st) {
   DecBuffers bf; LCC_TRY(carve_bound(e, &bf));
   const int nsplit = decode_splits(e, n_streams, max_len);
   for (int step = 0; step < n_steps; ++step) {
@@ -331,7 +359,12 @@ int lcc_decoder_decode(lcc_engine* e, int n_streams, const int32_t* d_slots, int
     if (prof_step) HIP_TRY(hipEventRecord(e->step_ev[2 * e->step_n], st));
     LCC_TRY(seen_set(e->d_seen, e->words, e->d_cur_tok, d_slots, n_streams, 1, e->d_done, st));
     LCC_TRY(embed_dyt(e->d_cur_tok, d_slots, e->embed, e->dw[0].norm, bf.x, bf.h, n_streams, e->c.hidden_size, st));
-    LCC_TRY(run_decoder_layers(e, bf, n_streams, nullptr, d_slots, nsplit, st));
+    AttnDirect dir;      // (a stream that EOS froze on the device has fewer keys than the host counts: its step is discarded, and the rows exist)
+    if (n_streams <= 4) {
+      for (int b = 0; b < n_streams; ++b) { dir.base[b] = (const bf16_t*)e->h_kv_base[slots[b]]; dir.n[b] = e->h_kv_len[slots[b]] + step + 1; }
+      dir.used = n_streams;
+    }
+    LCC_TRY(run_decoder_layers(e, bf, n_streams, nullptr, d_slots, nsplit, dir, st));
     LCC_TRY(advance_lengths(d_slots, e->d_kv_len, e->d_pos, n_streams, e->d_done, st));
     LCC_TRY(head_and_sample_decoder(e, bf, bf.h, n_streams, d_slots, sp, first_step_index + step, st));
     if (prof_step) {
@@ -358,4 +391,10 @@ extern "C" int lcc_slot_set_tokens(lcc_engine* e, int n_streams, const int32_t* 
   LCC_TRY(meta_commit(&mw, (hipStream_t)stream));
   LCC_TRY(set_tokens(d_slots, d_tok, n_streams, e->d_cur_tok, e->d_done, e->d_hist_col, (hipStream_t)stream));
   return check_launch("lcc_slot_set_tokens");
+}
+extern "C" int lcc_debug_set_decoder_fused(int on) {
+  if (lcc_knob_guard("lcc_debug_set_decoder_fused")) return -1;
+  const int old = g_fused_decode;
+  g_fused_decode = on ? 1 : 0;
+  return old;
 }

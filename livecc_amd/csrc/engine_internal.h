@@ -190,5 +190,5 @@ size_t lcc_decoder_ws_bytes(const lcc_engine* e);
 size_t lcc_decoder_meta_bytes(const lcc_engine* e);
 int lcc_decoder_resolve_weights(lcc_engine* e, std::string* missing);
 int lcc_decoder_prefill(lcc_engine* e, int n_streams, const int32_t* slots, const int32_t* n_new, const int32_t* ids, int S, const lcc_sampling* sp, hipStream_t st);
-int lcc_decoder_decode(lcc_engine* e, int n_streams, const int32_t* d_slots, int max_len, int n_steps, int first_step_index, const lcc_sampling* sp, hipStream_t st);
+int lcc_decoder_decode(lcc_engine* e, int n_streams, const int32_t* slots, const int32_t* d_slots, int max_len, int n_steps, int first_step_index, const lcc_sampling* sp, hipStream_t st);
 extern int g_decode_chain;        // engine_llm.hip; lcc_slot_read_tokens turns it off after a failed hand-off

@@ -453,7 +453,7 @@ extern "C" int lcc_llm_decode(lcc_engine* e, int n_streams, const int32_t* slots
   if (!mw.put(slots, n_streams, &d_slots)) return fail(LCC_ERR_STATE, "meta ring slot too small");
   LCC_TRY(meta_commit(&mw, st));
   if (e->family == LCC_FAMILY_DECODER) {
-    LCC_TRY(lcc_decoder_decode(e, n_streams, d_slots, max_len, n_steps, first_step_index, sp, st));
+    LCC_TRY(lcc_decoder_decode(e, n_streams, slots, d_slots, max_len, n_steps, first_step_index, sp, st));
     for (int b = 0; b < n_streams; ++b) { e->h_kv_len[slots[b]] += n_steps; e->h_pos[slots[b]] += n_steps; }
     return 0;
   }

@@ -193,6 +193,7 @@ int force_tokens(const int32_t* slots, const int32_t* forced, int B, int32_t* cu
                  int32_t* done, int eos, int eos2, hipStream_t st);
 
 // ---- decode layer pipeline v2 (decode_v2.hip): elementwise stages fused into the weight-streaming GEMVs ----
+struct DytNorm { const bf16_t* w = nullptr; const bf16_t* b = nullptr; const bf16_t* alpha = nullptr; };   // y = tanh(alpha x) w + b; alpha: one value
 struct DgArgs {
   const bf16_t* W = nullptr; int M = 0, N = 0, K = 0;
   const float* wscale = nullptr;   // non-null: W = OCP e4m3 bytes in the PACKED8 order [N/16][K/64][4 g][16 rows][16 k] + this fp32 scale per stored row
@@ -202,6 +203,9 @@ struct DgArgs {
   bf16_t* Hres = nullptr; float* stats_out = nullptr;                          // residual epilogue
   const bf16_t* cs = nullptr; const bf16_t* sn = nullptr; const int32_t* tok_stream = nullptr; const int32_t* kv_len = nullptr;
   bf16_t* const* kv_base = nullptr; KvLayout lay = {0, 0, 0, 0}; int layer = 0; bf16_t* q_out = nullptr; int n_q_heads = 0;   // rope epilogue
+  const float* S32 = nullptr; int lds32 = 0, rank = 0;                          // RMS prologue over fp32 rows [M][lds32], K stored and `rank` real channels (norm_w, eps)
+  float* C32 = nullptr;                                                         // fp32 epilogue, row pitch ldc
+  float* X32 = nullptr; DytNorm dyt;                                            // fp32 residual [M][N] in place, C = bf16 of the next norm
 };
 int decode_step_begin(const int32_t* slots, const int32_t* cur_tok, const int32_t* done, uint32_t* seen, int words, const bf16_t* table,
                       bf16_t* h, float* stats, int dim, const int32_t* pos, const float* inv_freq, bf16_t* cs, bf16_t* sn, int B,
@@ -220,7 +224,6 @@ int dgemv_down_qkv(const DgArgs& down, const DgArgs& qkv, unsigned* flag, unsign
 int dgemv_norm_bf16(const DgArgs& a, hipStream_t st);     // [final RMSNorm] lm_head
 
 // ---- layer-list decoders: row operators (decoder_ops.hip) ----
-struct DytNorm { const bf16_t* w = nullptr; const bf16_t* b = nullptr; const bf16_t* alpha = nullptr; };   // y = tanh(alpha x) w + b; alpha: one value
 int embed_dyt(const int32_t* ids, const int32_t* indirect, const bf16_t* table, const DytNorm& nm, float* x, bf16_t* h, int rows, int dim, hipStream_t st);
 int resid_dyt(float* x, const float* part, int nsplit, const DytNorm& nm, bf16_t* h, int rows, int dim, hipStream_t st);
 int logits_cap(const float* part, int nsplit, int rows, int ld, int vocab, float cap, float* out, float* dense, hipStream_t st);
@@ -236,6 +239,12 @@ struct LatentInArgs {            // behind the fused input projection: norms, ca
   bf16_t* const* kv_base = nullptr; size_t kv_off = 0;
 };
 int latent_norm_append(const LatentInArgs& a, hipStream_t st);
+// fused decode forms (decode_v2.hip; M <= 16): input projection + gate/up in one launch (sw.N = 0: none); query norm + up-projection with the rows'
+// cache appends and gates behind it (dgemv_latent_q_ok: M <= 8, query rank <= 2048); output projection + fp32 residual + next norm
+int dgemv_in_swiglu(const DgArgs& in, const DgArgs& sw, hipStream_t st);
+bool dgemv_latent_q_ok(int M, int K);
+int dgemv_latent_q(const DgArgs& a, const LatentInArgs& row, hipStream_t st);
+int dgemv_resid_dyt(const DgArgs& a, hipStream_t st);
 int latent_gather(bf16_t* const* kv_base, size_t kv_off, int rp, const int32_t* tile_slot, const int32_t* tile_key0, const int32_t* tile_nkeys,
                   int n_tiles, bf16_t* rows_out, bf16_t* frag_out, hipStream_t st);
 struct MhaArgs {                 // causal multi-head attention of packed rows over keys [keys][heads dim] and transposed values [heads vdim][ldv]
@@ -256,6 +265,7 @@ struct LatentDecodeArgs {
   int rows = 0, heads = 0, rp = 0, nsplit = 1; float scale_log2e = 0.f;
   const int32_t* slots = nullptr; const int32_t* kv_len = nullptr; bf16_t* const* kv_base = nullptr; size_t kv_off = 0;
   float* ws_o = nullptr; float* ws_ml = nullptr;               // [rows][heads][nsplit][rp], [rows][heads][nsplit][2]
+  AttnDirect direct;                                            // up to 4 rows: arena and key count by value
 };
 int latent_attn_decode(const LatentDecodeArgs& a, hipStream_t st);
 int latent_merge_uv(const LatentDecodeArgs& a, const bf16_t* uv, int vdim, const float* gate, bf16_t* out, int ldo, hipStream_t st);

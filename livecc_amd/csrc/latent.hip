@@ -12,6 +12,7 @@
 
 #include "common.h"
 #include "kernels.h"
+#include "latent_ops.h"
 
 namespace lcc {
 
@@ -22,45 +23,8 @@ namespace lcc {
 // The padding columns are exact zeros (zero weight rows), so the sums of squares run over the padded widths and divide by the real ones.
 // ------------------------------------------------------------------------------------------------------------------------------
 __global__ __launch_bounds__(256) void latent_norm_append_kernel(LatentInArgs a) {
-  __shared__ float red[2][4];
-  const int row = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const size_t slab = (size_t)a.rows * a.ldn;
-  const float* src = a.part + (size_t)row * a.ldn;
-  auto at = [&](int c) {
-    f32x4 v = *reinterpret_cast<const f32x4*>(src + c);
-    for (int s = 1; s < a.nsplit; ++s) v += *reinterpret_cast<const f32x4*>(src + s * slab + c);
-    return v;
-  };
-  float sq = 0.f, sk = 0.f;
-  for (int c = tid * 4; c < a.qp; c += 1024) { const f32x4 v = at(c); sq += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
-  for (int c = tid * 4; c < a.rp; c += 1024) { const f32x4 v = at(a.qp + c); sk += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
-  sq = wave_sum(sq); sk = wave_sum(sk);
-  if (lane == 0) { red[0][wave] = sq; red[1][wave] = sk; }
-  __syncthreads();
-  sq = (red[0][0] + red[0][1]) + (red[0][2] + red[0][3]);
-  sk = (red[1][0] + red[1][1]) + (red[1][2] + red[1][3]);
-  const float iq = 1.f / sqrtf(sq / (float)a.q_rank + a.eps);
-  for (int c = tid * 4; c < a.qp; c += 1024) {
-    const f32x4 v = at(c);
-    const u32x2 w = ld8(a.q_norm + c);
-    st8(a.cq + (size_t)row * a.qp + c, (u32x2){pack2(v[0] * iq * lo2f(w.x), v[1] * iq * hi2f(w.x)), pack2(v[2] * iq * lo2f(w.y), v[3] * iq * hi2f(w.y))});
-  }
-  if (a.rp > 0) {
-    const float ik = 1.f / sqrtf(sk / (float)a.kv_rank + a.eps);
-    const int slot = a.tok_stream[row];
-    const int pos = a.tok_pos ? a.tok_pos[row] : a.kv_len[slot];
-    bf16_t* dst = a.kv_base[slot] + a.kv_off + (size_t)pos * a.rp;
-    for (int c = tid * 4; c < a.rp; c += 1024) {
-      const f32x4 v = at(a.qp + c);
-      const u32x2 w = ld8(a.kv_norm + c);
-      st8(dst + c, (u32x2){pack2(v[0] * ik * lo2f(w.x), v[1] * ik * hi2f(w.x)), pack2(v[2] * ik * lo2f(w.y), v[3] * ik * hi2f(w.y))});
-    }
-  }
-  for (int h = tid; h < a.heads; h += 256) {
-    float z = src[a.qp + a.rp + h];
-    for (int s = 1; s < a.nsplit; ++s) z += src[s * slab + a.qp + a.rp + h];
-    a.gate[(size_t)row * a.heads + h] = 1.f / (1.f + expf(-z));
-  }
+  __shared__ float red[8];
+  latent_row<256, true>(a, blockIdx.x, red);
 }
 int latent_norm_append(const LatentInArgs& a, hipStream_t st) {
   if (a.rows <= 0) return 0;
@@ -216,8 +180,7 @@ int latent_absorb(const float* q_part, int nsplit, int rows, int heads, int dim,
 
 // ------------------------------------------------------------------------------------------------------------------------------
 // Decode, step 2: attention over the cached latents, all heads of a row together.  rank = 64 RT.
-// Block = quads of 4 waves, one quad per 16 heads; 64 keys per iteration, staged once for all quads by LDS-DMA in MFMA fragment order
-// (1-KB pieces = 16 keys x 32 channels), double buffered.  Per iteration a wave multiplies its 16 keys with its quad's 16 queries
+// Block = quads of 4 waves, one quad per 16 heads; 64 keys per iteration, staged once for all quads by LDS-DMA, double buffered.  Per iteration a wave multiplies its 16 keys with its quad's 16 queries
 // (S^T[key][head]: a lane owns 4 keys of one head), the quad agrees on the new maxima through LDS, and then each wave adds
 // C^T . P^T for its quarter of the channels (O^T[channel][head]: again one head per lane, so the rescale factor is lane-local).  The
 // C^T operand -- 8 keys of one channel per lane -- comes out of the same LDS image through ds_read_b64_tr_b16, which transposes 4 x 16
@@ -228,11 +191,16 @@ typedef __attribute__((ext_vector_type(4))) short s16x4;
 LCC_DEVICE u32x2 lds_tr4x16(const void* p) {
   return __builtin_bit_cast(u32x2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)(p)));
 }
+// LDS image of a key tile: rows of RT * 8 16-byte chunks, chunk c of key k at slot c ^ latent_swizzle(k).  The low three bits only: a DMA
+// instruction copies whole 128-byte lines (1 KB contiguous at rank 512).  Eight consecutive keys get eight different slots (score operand:
+// one chunk of 16 keys) and keys 4 i .. 4 i + 3 get disjoint slot PAIRS (value operand: two chunks of 4 keys), so both reads spread the banks.
+LCC_DEVICE int latent_swizzle(int key) { return ((key & 3) << 1) | ((key >> 2) & 1); }
 constexpr int LATENT_PP = 72;      // pitch of a head's 64 probabilities in LDS (16-byte aligned, spreads the banks)
 
 template <int RT, int NSTAGE>
-__global__ __launch_bounds__(RT >= 8 ? 512 : 1024) void latent_attn_decode_kernel(LatentDecodeArgs a) {
+__global__ __launch_bounds__(RT > 12 ? 256 : RT >= 6 ? 512 : 1024) void latent_attn_decode_kernel(LatentDecodeArgs a) {
   constexpr int RP = RT * 64, KB = RT * 2, NP = 4 * KB;              // channels, 32-channel blocks, pieces per 64-key tile
+  constexpr int PF = RT == 8 ? 8 : (KB < 4 || RT > 12 ? 2 : 4), PV = RT == 8 ? 6 : (KB < 4 || RT > 12 ? 2 : 4);      // fragments read ahead
   extern __shared__ __attribute__((aligned(16))) u32x4 lmem[];       // NSTAGE x NP pieces, then P, then the statistics
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), li = lane & 15, g = lane >> 4;
   const int quad = wave >> 2, wq = wave & 3, nw = blockDim.x >> 6, nquad = nw >> 2;
@@ -240,25 +208,20 @@ __global__ __launch_bounds__(RT >= 8 ? 512 : 1024) void latent_attn_decode_kerne
   float* s_m = reinterpret_cast<float*>(reinterpret_cast<bf16_t*>(lmem + NSTAGE * NP * 64) + nquad * 16 * LATENT_PP) + quad * 64;
   const int split = blockIdx.x, b = blockIdx.y;
   const int head = (blockIdx.z * nquad + quad) * 16 + li;
-  const int slot = a.slots[b];
-  const int n = a.kv_len[slot] + 1;                                  // cached keys and the token of this step
-  const int ntile = (n + 63) >> 6, per = (ntile + a.nsplit - 1) / a.nsplit;
-  const int tb = split * per, te = min(ntile, tb + per);
+  int n;                                                             // cached keys and the token of this step
+  const bf16_t* arena;
+  if (a.direct.used) { n = a.direct.n[b & 3]; arena = a.direct.base[b & 3]; }       // by value: no dependent loads in front of the first tile
+  else { const int slot = a.slots[b]; n = a.kv_len[slot] + 1; arena = a.kv_base[slot]; }
+  // split s takes the tiles s, s + nsplit, ..: the blocks of a row read neighbouring tiles at any time, so the memory channels share the load
+  const int ntile = (n + 63) >> 6, tb = split, te = ntile, step = a.nsplit;
   if (tb >= te) return;                                              // the merge knows which splits exist
-  const bf16_t* cbase = a.kv_base[slot] + a.kv_off;
+  const bf16_t* cbase = arena + a.kv_off;
 
-  u32x4 qf[KB];                                                      // B operand: q[head][32 ks + 8 g ..]
-  {
-    const bf16_t* qp = a.q + ((size_t)b * a.heads + min(head, a.heads - 1)) * RP + g * 8;
-#pragma unroll
-    for (int ks = 0; ks < KB; ++ks) qf[ks] = ld16(qp + ks * 32);
-#pragma unroll
-    for (int ks = 0; ks < KB; ++ks) settle_load(qf[ks]);
-  }
   auto issue = [&](int t, int stage) {
+    const bf16_t* src = cbase + (size_t)t * 64 * RP;
     for (int p = wave; p < NP; p += nw) {
-      const int kt = p / KB, kb = p - kt * KB;
-      glds16(cbase + (size_t)(t * 64 + kt * 16 + li) * RP + kb * 32 + g * 8, lds_addr(lmem + (stage * NP + p) * 64));
+      const int u = p * 64 + lane, key = u / (RT * 8), slot = u - key * (RT * 8);          // 16-byte units of the tile image
+      glds16(src + key * RP + (slot ^ latent_swizzle(key)) * 8, lds_addr(lmem + (stage * NP + p) * 64));
     }
   };
   f32x4 o[RT];
@@ -267,15 +230,55 @@ __global__ __launch_bounds__(RT >= 8 ? 512 : 1024) void latent_attn_decode_kerne
   float m_run = -INFINITY, l_run = 0.f;
 
   issue(tb, 0);
-  for (int t = tb; t < te; ++t) {
-    const int stage = NSTAGE == 2 ? ((t - tb) & 1) : 0;
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    __syncthreads();                                                 // tile t is complete; everyone is done with tile t - 1
-    if (NSTAGE == 2 && t + 1 < te) issue(t + 1, stage ^ 1);
-    const u32x4* cs = lmem + stage * NP * 64;
-    f32x4 s = {0.f, 0.f, 0.f, 0.f};
+  u32x4 qf[KB];                                                      // B operand: q[head][32 ks + 8 g ..]
+  if (NSTAGE == 2) {
+    // the quads' queries come through the second stage, copied like a key tile (fragment-shaped loads of 16 rows x 64 bytes by every wave
+    // took longer than the first key tile); the second tile is issued behind the first iteration's barrier
+    for (int p = wave; p < nquad * KB; p += nw) {
+      const int u = p * 64 + lane, r = u / (RT * 8), slot = u - r * (RT * 8);
+      const int hr = min((int)(blockIdx.z * nquad) * 16 + r, a.heads - 1);
+      glds16(a.q + ((size_t)b * a.heads + hr) * RP + (slot ^ latent_swizzle(r)) * 8, lds_addr(lmem + (NP + p) * 64));
+    }
+  } else {
+    const bf16_t* qp = a.q + ((size_t)b * a.heads + min(head, a.heads - 1)) * RP + g * 8;
 #pragma unroll
-    for (int ks = 0; ks < KB; ++ks) s = mfma16(as_bf16x8(cs[(wq * KB + ks) * 64 + lane]), as_bf16x8(qf[ks]), s);
+    for (int ks = 0; ks < KB; ++ks) qf[ks] = ld16(qp + ks * 32);
+  }
+  int stage = 0;
+  for (int t = tb; t < te; t += step, stage ^= NSTAGE - 1) {
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    if (NSTAGE == 1 && t == tb) {                                    // the queries have landed too (common.h: glds16)
+#pragma unroll
+      for (int ks = 0; ks < KB; ++ks) settle_load(qf[ks]);
+    }
+    __syncthreads();                                                 // tile t is complete; everyone is done with the tile before
+    if (NSTAGE == 2 && t == tb) {
+#pragma unroll
+      for (int ks = 0; ks < KB; ++ks) qf[ks] = lmem[NP * 64 + (quad * 16 + li) * (RT * 8) + ((ks * 4 + g) ^ latent_swizzle(li))];
+    }
+    if (NSTAGE == 2 && t != tb && t + step < te) issue(t + step, stage ^ 1);
+    const u32x4* cs = lmem + stage * NP * 64;
+    // fragment reads run PF steps ahead of their MFMAs (issue order pinned: hipcc otherwise waits for every read), two accumulator chains
+    f32x4 s = {0.f, 0.f, 0.f, 0.f}, s2 = {0.f, 0.f, 0.f, 0.f};
+    {
+      bf16x8 cf[PF];
+      const u32x4* krow = cs + (wq * 16 + li) * (RT * 8);
+      auto key_operand = [&](int ks) { return as_bf16x8(krow[(ks * 4 + g) ^ latent_swizzle(li)]); };
+#pragma unroll
+      for (int i = 0; i < PF; ++i) cf[i] = key_operand(i);
+#pragma unroll
+      for (int ks = 0; ks < KB; ++ks) {
+        if (ks & 1) s2 = mfma16(cf[ks % PF], as_bf16x8(qf[ks]), s2); else s = mfma16(cf[ks % PF], as_bf16x8(qf[ks]), s);
+        if (ks + PF < KB) cf[ks % PF] = key_operand(ks + PF);
+      }
+      __builtin_amdgcn_sched_group_barrier(0x100, PF, 0);
+#pragma unroll
+      for (int ks = 0; ks < KB; ++ks) {
+        __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);
+        if (ks + PF < KB) __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+      }
+    }
+    s += s2;
     const int k0 = t * 64 + wq * 16 + g * 4;
 #pragma unroll
     for (int r = 0; r < 4; ++r) s[r] = k0 + r < n ? s[r] * a.scale_log2e : -INFINITY;
@@ -284,6 +287,7 @@ __global__ __launch_bounds__(RT >= 8 ? 512 : 1024) void latent_attn_decode_kerne
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
     if (g == 0) s_m[wq * 16 + li] = mx;
     __syncthreads();
+    if (NSTAGE == 2 && t == tb && t + step < te) issue(t + step, 1);       // every wave holds its queries
     const float m_new = fmaxf(fmaxf(fmaxf(s_m[li], s_m[16 + li]), fmaxf(s_m[32 + li], s_m[48 + li])), m_run);   // finite: a tile has >= 1 key
     const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
     m_run = m_new;
@@ -293,22 +297,34 @@ __global__ __launch_bounds__(RT >= 8 ? 512 : 1024) void latent_attn_decode_kerne
     l_run = l_run * alpha + ((p[0] + p[1]) + (p[2] + p[3]));
     st8(s_p + li * LATENT_PP + wq * 16 + g * 4, (u32x2){pack2(p[0], p[1]), pack2(p[2], p[3])});
     __syncthreads();
-    const u32x4 pf0 = ld16(s_p + li * LATENT_PP + g * 8), pf1 = ld16(s_p + li * LATENT_PP + 32 + g * 8);
+    {
+      bf16x8 pf[2], cf[PV];
+      // C^T operand i = 2 j + ks: channels of step j, keys 32 ks ..; this lane supplies 4 channels of keys 8 g + li / 4 (+ 4) of the step
+      auto operand = [&](int i) {
+        const int j = i >> 1, ks = i & 1, r = wq * (16 * RT) + j * 16 + (li & 3) * 4, key = ks * 32 + g * 8 + (li >> 2);
+        const char* at = reinterpret_cast<const char*>(cs) + key * (RT * 128) + (r & 7) * 2;
+        const int sl = ((r >> 3) ^ latent_swizzle(key)) * 16;        // of key + 4: the low bit flips
+        const u32x2 lo = lds_tr4x16(at + sl), hi = lds_tr4x16(at + 4 * (RT * 128) + (sl ^ 16));
+        return as_bf16x8((u32x4){lo.x, lo.y, hi.x, hi.y});
+      };
+      pf[0] = as_bf16x8(ld16(s_p + li * LATENT_PP + g * 8)); pf[1] = as_bf16x8(ld16(s_p + li * LATENT_PP + 32 + g * 8));
 #pragma unroll
-    for (int j = 0; j < RT; ++j) {
-      const int r = wq * (16 * RT) + j * 16 + (li & 3) * 4;          // this lane's source channels
-      const char* base = reinterpret_cast<const char*>(cs) + (r >> 5) * 1024 + ((r >> 3) & 3) * 256 + (r & 7) * 2;
-      f32x4 acc = o[j] * alpha;
+      for (int i = 0; i < PV; ++i) cf[i] = operand(i);
 #pragma unroll
-      for (int ks = 0; ks < 2; ++ks) {
-        const int key = ks * 32 + g * 8 + (li >> 2);                 // and + 4 for the second half
-        const u32x2 lo = lds_tr4x16(base + (key >> 4) * (KB * 1024) + (key & 15) * 16);
-        const u32x2 hi = lds_tr4x16(base + (key >> 4) * (KB * 1024) + ((key & 15) + 4) * 16);
-        acc = mfma16(as_bf16x8((u32x4){lo.x, lo.y, hi.x, hi.y}), as_bf16x8(ks == 0 ? pf0 : pf1), acc);
+      for (int j = 0; j < RT; ++j) o[j] *= alpha;
+#pragma unroll
+      for (int i = 0; i < KB; ++i) {
+        o[i >> 1] = mfma16(cf[i % PV], pf[i & 1], o[i >> 1]);
+        if (i + PV < KB) cf[i % PV] = operand(i + PV);
       }
-      o[j] = acc;
+      __builtin_amdgcn_sched_group_barrier(0x100, 2 + 2 * PV, 1);
+#pragma unroll
+      for (int i = 0; i < KB; ++i) {
+        __builtin_amdgcn_sched_group_barrier(0x008, 1, 1);
+        if (i + PV < KB) __builtin_amdgcn_sched_group_barrier(0x100, 2, 1);
+      }
     }
-    if (NSTAGE == 1 && t + 1 < te) { __syncthreads(); issue(t + 1, 0); }
+    if (NSTAGE == 1 && t + step < te) { __syncthreads(); issue(t + step, 0); }
   }
   // the quad's denominators: over the lane groups of a wave, then over its four waves
   l_run += __shfl_xor(l_run, 16, 64);
@@ -329,7 +345,7 @@ __global__ __launch_bounds__(RT >= 8 ? 512 : 1024) void latent_attn_decode_kerne
 
 template <int RT>
 static void latent_decode_go(const LatentDecodeArgs& a, hipStream_t st) {
-  constexpr int NSTAGE = RT > 8 ? 1 : 2, MAXQ = RT >= 8 ? 2 : 4;
+  constexpr int NSTAGE = RT > 8 ? 1 : 2, MAXQ = RT > 12 ? 1 : RT >= 6 ? 2 : 4;
   const int ht = (a.heads + 15) / 16, groups = (ht + MAXQ - 1) / MAXQ, quads = (ht + groups - 1) / groups;
   const size_t lds = (size_t)NSTAGE * 8 * RT * 1024 + (size_t)quads * (16 * LATENT_PP * 2 + 256);
   static DeviceOnce once;   // per instantiation
@@ -359,53 +375,72 @@ int latent_attn_decode(const LatentDecodeArgs& a, hipStream_t st) {
 // ------------------------------------------------------------------------------------------------------------------------------
 // Decode, step 3: merge the splits, map the weighted latent through Uv_h, apply the head's gate.  grid (vdim / 64, heads, row groups).
 // ------------------------------------------------------------------------------------------------------------------------------
-// The wave's Uv fragments are requested before the merge, which hides their latency (rank <= 512; above, in two batches).
+// The Uv fragments of the first four waves are requested before the merge, which hides their latency (rank <= 512; above, in two batches).
 template <int RT>
-__global__ __launch_bounds__(256) void latent_merge_uv_kernel(LatentDecodeArgs a, const bf16_t* __restrict__ uv, int vdim,
-                                                              const float* __restrict__ gate, bf16_t* __restrict__ out, int ldo) {
-  extern __shared__ __attribute__((aligned(16))) bf16_t s_o[];       // [16][rp + 8]
-  __shared__ float s_w[4][LATENT_MAX_SPLIT];
-  const int h = blockIdx.y, b0 = blockIdx.z * 16, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, g = lane >> 4;
-  constexpr int rp = RT * 64, pitch = rp + 8, KB = RT * 2, KW = KB > 16 ? KB / 2 : KB;
-  const int nrow = min(16, a.rows - b0);
+__global__ __launch_bounds__(1024) void latent_merge_uv_kernel(LatentDecodeArgs a, const bf16_t* __restrict__ uv, int vdim,
+                                                               const float* __restrict__ gate, bf16_t* __restrict__ out, int ldo, int rpb) {
+  constexpr int rp = RT * 64, pitch = rp + 8, KB = RT * 2, KW = KB > 16 ? KB / 2 : KB, NC = rp / 4;
+  extern __shared__ __attribute__((aligned(16))) bf16_t s_o[];       // [rpb][rp + 8]
+  __shared__ float s_w[16][LATENT_MAX_SPLIT];
+  __shared__ f32x4 s_red[1024];
+  __shared__ int s_live[16];
+  const int h = blockIdx.y, b0 = blockIdx.z * rpb, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, g = lane >> 4;
+  const int nt = blockDim.x, nw = nt >> 6, nrow = min(rpb, a.rows - b0);
   const int v0 = (blockIdx.x * 4 + wave) * 16;
-  const bf16_t* wp = uv + (size_t)(h * vdim + v0 + li) * rp + g * 8;
+  const bf16_t* wp = uv + (size_t)(h * vdim + min(v0, vdim - 16) + li) * rp + g * 8;
   u32x4 wf[KW];
+  if (wave < 4) {
 #pragma unroll
-  for (int k = 0; k < KW; ++k) wf[k] = ld16(wp + k * 32);
-  for (int r = wave; r < nrow; r += 4) {                             // a wave merges whole rows
+    for (int k = 0; k < KW; ++k) wf[k] = ld16(wp + k * 32);
+  }
+  for (int r = wave; r < nrow; r += nw) {                            // the normalised weight of every split of a row
     const int b = b0 + r;
-    const int n = a.kv_len[a.slots[b]] + 1, ntile = (n + 63) >> 6, per = (ntile + a.nsplit - 1) / a.nsplit;
-    const int live = (ntile + per - 1) / per;                        // splits that ran
-    const size_t p0 = ((size_t)b * a.heads + h) * a.nsplit;
-    float m = -INFINITY;
-    for (int s = lane; s < live; s += 64) m = fmaxf(m, a.ws_ml[(p0 + s) * 2]);
-    m = wave_max(m);
-    float l = 0.f;
-    for (int s = lane; s < live; s += 64) {
-      const float e = __builtin_amdgcn_exp2f(a.ws_ml[(p0 + s) * 2] - m);
-      s_w[wave][s] = e;
-      l += e * a.ws_ml[(p0 + s) * 2 + 1];
-    }
-    const float inv = 1.f / wave_sum(l);
-    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");           // one wave, in-order LDS: the lanes' weights are visible to all lanes
-    __builtin_amdgcn_wave_barrier();
-    for (int c = lane * 4; c < rp; c += 256) {
-      f32x4 v = {0.f, 0.f, 0.f, 0.f};
-      for (int s = 0; s < live; ++s) v += *reinterpret_cast<const f32x4*>(a.ws_o + (p0 + s) * rp + c) * s_w[wave][s];
-      st8(s_o + r * pitch + c, (u32x2){pack2(v[0] * inv, v[1] * inv), pack2(v[2] * inv, v[3] * inv)});
-    }
-    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-    __builtin_amdgcn_wave_barrier();
+    const int n = a.direct.used ? a.direct.n[b & 3] : a.kv_len[a.slots[b]] + 1;
+    const int live = min(a.nsplit, (n + 63) >> 6);                   // splits that ran: one per key tile at most
+    const float* ml = a.ws_ml + ((size_t)b * a.heads + h) * a.nsplit * 2;
+    const bool h0 = lane < live, h1 = lane + 64 < live;              // LATENT_MAX_SPLIT = 128: two per lane
+    const float m0 = h0 ? ml[lane * 2] : -INFINITY, m1 = h1 ? ml[(lane + 64) * 2] : -INFINITY;
+    const float l0 = h0 ? ml[lane * 2 + 1] : 0.f, l1 = h1 ? ml[(lane + 64) * 2 + 1] : 0.f;
+    const float m = wave_max(fmaxf(m0, m1));
+    const float e0 = __builtin_amdgcn_exp2f(m0 - m), e1 = __builtin_amdgcn_exp2f(m1 - m);
+    const float inv = 1.f / wave_sum(e0 * l0 + e1 * l1);
+    s_w[r][lane] = e0 * inv;
+    s_w[r][lane + 64] = e1 * inv;
+    if (lane == 0) s_live[r] = live;
   }
   __syncthreads();
+  // weighted sum of the splits: one 4-channel piece per thread; with fewer pieces than threads several threads share a piece's splits
+  const int items = nrow * NC, share = max(1, nt / items), pieces = share > 1 ? items : nt;
+  for (int i0 = 0; i0 < items; i0 += pieces) {
+    const int part = share > 1 ? tid / items : 0, item = i0 + (share > 1 ? tid - part * items : tid);
+    const bool on = item < items && part < share;
+    const int r = on ? item / NC : 0, c = (on ? item - r * NC : 0) * 4;
+    f32x4 v = {0.f, 0.f, 0.f, 0.f};
+    if (on) {
+      const int live = s_live[r];
+      const float* op = a.ws_o + ((size_t)(b0 + r) * a.heads + h) * a.nsplit * rp + c;
+#pragma unroll 8
+      for (int s = part; s < live; s += share) v += *reinterpret_cast<const f32x4*>(op + (size_t)s * rp) * s_w[r][s];
+    }
+    if (share > 1) {
+      s_red[tid] = v;
+      __syncthreads();
+      if (on && part == 0)
+        for (int p = 1; p < share; ++p) v += s_red[p * items + item];
+    }
+    if (on && part == 0) st8(s_o + r * pitch + c, (u32x2){pack2(v[0], v[1]), pack2(v[2], v[3])});
+  }
+  __syncthreads();
+  if (wave >= 4) return;
   const bf16_t* xp = s_o + min(li, nrow - 1) * pitch + g * 8;
-  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f}, acc2 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int k = 0; k < KB; ++k) {
-    acc = mfma16(as_bf16x8(wf[k % KW]), as_bf16x8(ld16(xp + k * 32)), acc);
+    if (k & 1) acc2 = mfma16(as_bf16x8(wf[k % KW]), as_bf16x8(ld16(xp + k * 32)), acc2);
+    else acc = mfma16(as_bf16x8(wf[k % KW]), as_bf16x8(ld16(xp + k * 32)), acc);
     if (k + KW < KB) wf[k % KW] = ld16(wp + (k + KW) * 32);
   }
+  acc += acc2;
   if (li < nrow) {
     const float f = gate ? gate[(size_t)(b0 + li) * a.heads + h] : 1.f;
     st8(out + (size_t)(b0 + li) * ldo + h * vdim + v0 + g * 4, (u32x2){pack2(acc[0] * f, acc[1] * f), pack2(acc[2] * f, acc[3] * f)});
@@ -415,9 +450,12 @@ int latent_merge_uv(const LatentDecodeArgs& a, const bf16_t* uv, int vdim, const
   if (a.rows <= 0) return 0;
   if ((vdim & 63) || vdim < 64 || (a.rp & 63) || a.rp < 64 || a.rp > 1024 || (ldo & 3) || a.nsplit > LATENT_MAX_SPLIT || a.nsplit < 1) return LCC_ERR_SHAPE;
   if (!uv || !out || !a.ws_o || !a.ws_ml || !a.slots || !a.kv_len) return LCC_ERR_ARG;
-  const dim3 grid(vdim / 64, a.heads, (a.rows + 15) / 16);
-  const size_t lds = (size_t)16 * (a.rp + 8) * 2;
-#define LCC_MERGE(RT) case RT * 64: latent_merge_uv_kernel<RT><<<grid, dim3(256), lds, st>>>(a, uv, vdim, gate, out, ldo); break
+  int rpb = 16;                                                      // rows per block: as many as still give the chip a block per CU
+  while (rpb > 1 && (long)(vdim / 64) * a.heads * ((a.rows + rpb - 1) / rpb) < 256) rpb >>= 1;
+  const dim3 grid(vdim / 64, a.heads, (a.rows + rpb - 1) / rpb);
+  const size_t lds = (size_t)rpb * (a.rp + 8) * 2;
+  const int threads = rpb <= 4 ? 1024 : 512;
+#define LCC_MERGE(RT) case RT * 64: latent_merge_uv_kernel<RT><<<grid, dim3(threads), lds, st>>>(a, uv, vdim, gate, out, ldo, rpb); break
   switch (a.rp) {
     LCC_MERGE(1); LCC_MERGE(2); LCC_MERGE(3); LCC_MERGE(4); LCC_MERGE(6); LCC_MERGE(8); LCC_MERGE(12); LCC_MERGE(16);
     default: return LCC_ERR_SHAPE;

@@ -90,6 +90,8 @@ class Engine:
         self.cfg, self.weights = cfg, weights
         self.device = torch.device(device if device is not None else weights.device)
         assert self.device.type == "cuda"
+        if self.device.index is None:
+            self.device = torch.device("cuda", torch.cuda.current_device())
         torch.cuda.set_device(self.device)
         self.is_decoder = isinstance(cfg, DebunexConfig)
         gran = 64 if self.is_decoder else 32
