@@ -206,6 +206,8 @@ class Engine:
         """clips: dicts with either {'frames': uint8 device tensor, 'layout': 'THWC'|'TCHW'} or
         {'pixel_values': fp32 device [P,1176], 'grid': (t,h,w)}.  Returns bf16 [sum P/4, hidden].  `stream`: launch on that stream
         (the ViT has its own workspace; the caller orders consumers and later ViT calls with events)."""
+        if self.is_decoder:
+            raise _lib.LccError("vit_encode: this model has no vision tower")
         cfg = self.cfg
         arr = (_lib.Clip * len(clips))()
         grids, keep = [], []
