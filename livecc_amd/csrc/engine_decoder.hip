@@ -48,7 +48,7 @@ int decode_splits(const lcc_engine* e, int rows, int max_len) {
   const int ntile = (max_len + 63) / 64;
   if (forced > 0) return std::max(1, std::min(std::min(forced, LATENT_MAX_SPLIT), ntile));
   const int want = std::max(1, e->cu_count / std::max(1, rows));
-  return std::max(1, std::min(std::min(want, 64), ntile));
+  return std::max(1, std::min(std::min(want, ntile >= 256 ? LATENT_MAX_SPLIT : 64), ntile));      // (past 64 the merge costs what a tile saves, except on long caches)
 }
 size_t decode_slots(const lcc_engine* e) {     // (row, split) pairs of one decode launch, per head
   const int B = std::min(e->lim.max_slots, LCC_MAX_DECODE_BATCH);
