@@ -346,7 +346,11 @@ __global__ __launch_bounds__(RT > 12 ? 256 : RT >= 6 ? 512 : 1024) void latent_a
 template <int RT>
 static void latent_decode_go(const LatentDecodeArgs& a, hipStream_t st) {
   constexpr int NSTAGE = RT > 8 ? 1 : 2, MAXQ = RT > 12 ? 1 : RT >= 6 ? 2 : 4;
-  const int ht = (a.heads + 15) / 16, groups = (ht + MAXQ - 1) / MAXQ, quads = (ht + groups - 1) / groups;
+  const int ht = (a.heads + 15) / 16;
+  int groups = (ht + MAXQ - 1) / MAXQ;
+  // while compute units are idle, fewer heads per block (the tiles then come out of the L2 for all but the first of a row's head groups)
+  while (groups < ht && (long)a.nsplit * a.rows * std::min(2 * groups, ht) <= 256) groups = std::min(2 * groups, ht);
+  const int quads = (ht + groups - 1) / groups;
   const size_t lds = (size_t)NSTAGE * 8 * RT * 1024 + (size_t)quads * (16 * LATENT_PP * 2 + 256);
   static DeviceOnce once;   // per instantiation
   if (once.first())
@@ -373,12 +377,13 @@ int latent_attn_decode(const LatentDecodeArgs& a, hipStream_t st) {
 }
 
 // ------------------------------------------------------------------------------------------------------------------------------
-// Decode, step 3: merge the splits, map the weighted latent through Uv_h, apply the head's gate.  grid (vdim / 64, heads, row groups).
+// Decode, step 3: merge the splits, map the weighted latent through Uv_h, apply the head's gate.  One block per (head, group of rpb rows), a
+// wave per 16 value channels.
 // ------------------------------------------------------------------------------------------------------------------------------
-// The Uv fragments of the first four waves are requested before the merge, which hides their latency (rank <= 512; above, in two batches).
+// The Uv fragments are requested before the merge, which hides their latency (rank <= 512; above, in two batches).
 template <int RT>
 __global__ __launch_bounds__(1024) void latent_merge_uv_kernel(LatentDecodeArgs a, const bf16_t* __restrict__ uv, int vdim,
-                                                               const float* __restrict__ gate, bf16_t* __restrict__ out, int ldo, int rpb) {
+                                                               const float* __restrict__ gate, bf16_t* __restrict__ out, int ldo, int rpb, int vw) {
   constexpr int rp = RT * 64, pitch = rp + 8, KB = RT * 2, KW = KB > 16 ? KB / 2 : KB, NC = rp / 4;
   extern __shared__ __attribute__((aligned(16))) bf16_t s_o[];       // [rpb][rp + 8]
   __shared__ float s_w[16][LATENT_MAX_SPLIT];
@@ -386,10 +391,10 @@ __global__ __launch_bounds__(1024) void latent_merge_uv_kernel(LatentDecodeArgs 
   __shared__ int s_live[16];
   const int h = blockIdx.y, b0 = blockIdx.z * rpb, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, g = lane >> 4;
   const int nt = blockDim.x, nw = nt >> 6, nrow = min(rpb, a.rows - b0);
-  const int v0 = (blockIdx.x * 4 + wave) * 16;
+  const int v0 = wave < vw ? (int)(blockIdx.x * vw + wave) * 16 : vdim;      // this wave's value channels
   const bf16_t* wp = uv + (size_t)(h * vdim + min(v0, vdim - 16) + li) * rp + g * 8;
   u32x4 wf[KW];
-  if (wave < 4) {
+  if (v0 < vdim) {
 #pragma unroll
     for (int k = 0; k < KW; ++k) wf[k] = ld16(wp + k * 32);
   }
@@ -431,7 +436,7 @@ __global__ __launch_bounds__(1024) void latent_merge_uv_kernel(LatentDecodeArgs 
     if (on && part == 0) st8(s_o + r * pitch + c, (u32x2){pack2(v[0], v[1]), pack2(v[2], v[3])});
   }
   __syncthreads();
-  if (wave >= 4) return;
+  if (v0 >= vdim) return;
   const bf16_t* xp = s_o + min(li, nrow - 1) * pitch + g * 8;
   f32x4 acc = {0.f, 0.f, 0.f, 0.f}, acc2 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -451,11 +456,13 @@ int latent_merge_uv(const LatentDecodeArgs& a, const bf16_t* uv, int vdim, const
   if ((vdim & 63) || vdim < 64 || (a.rp & 63) || a.rp < 64 || a.rp > 1024 || (ldo & 3) || a.nsplit > LATENT_MAX_SPLIT || a.nsplit < 1) return LCC_ERR_SHAPE;
   if (!uv || !out || !a.ws_o || !a.ws_ml || !a.slots || !a.kv_len) return LCC_ERR_ARG;
   int rpb = 16;                                                      // rows per block: as many as still give the chip a block per CU
-  while (rpb > 1 && (long)(vdim / 64) * a.heads * ((a.rows + rpb - 1) / rpb) < 256) rpb >>= 1;
-  const dim3 grid(vdim / 64, a.heads, (a.rows + rpb - 1) / rpb);
+  while (rpb > 1 && (long)a.heads * ((a.rows + rpb - 1) / rpb) < 192) rpb >>= 1;
   const size_t lds = (size_t)rpb * (a.rp + 8) * 2;
   const int threads = rpb <= 4 ? 1024 : 512;
-#define LCC_MERGE(RT) case RT * 64: latent_merge_uv_kernel<RT><<<grid, dim3(threads), lds, st>>>(a, uv, vdim, gate, out, ldo, rpb); break
+  // value channels of a block: all its waves', or -- few blocks -- 64 (the blocks of a head then merge the same partial sums)
+  const int vw = a.heads * a.rows < 96 ? 4 : threads / 64;
+  const dim3 grid((vdim / 16 + vw - 1) / vw, a.heads, (a.rows + rpb - 1) / rpb);
+#define LCC_MERGE(RT) case RT * 64: latent_merge_uv_kernel<RT><<<grid, dim3(threads), lds, st>>>(a, uv, vdim, gate, out, ldo, rpb, vw); break
   switch (a.rp) {
     LCC_MERGE(1); LCC_MERGE(2); LCC_MERGE(3); LCC_MERGE(4); LCC_MERGE(6); LCC_MERGE(8); LCC_MERGE(12); LCC_MERGE(16);
     default: return LCC_ERR_SHAPE;
