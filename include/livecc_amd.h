@@ -363,9 +363,15 @@ lcc_engine* lcc_engine_create(const lcc_model_config* cfg, const lcc_engine_limi
 
 /* Second model family: decoders given as a list of layers.  The engine object, its buffers, slots, lcc_llm_prefill / lcc_llm_decode, the samplers
  * and the slot calls are the same; there is no vision tower and prefill takes no positions (pos3 may be NULL).  A slot's arena holds one
- * [max_kv_len][kv_rank_pad] bf16 block per layer that owns a latent.  Sizes named *_pad are the stored ones (zero rows / columns). */
+ * [max_kv_len][kv_rank_pad] bf16 block per layer that owns a latent; K / V blocks and the fp32 recurrent state of the other mixers (the state belongs
+ * to the slot's length: lcc_slot_set_length does not roll it back).  Sizes named *_pad are the stored ones (zero rows / columns). */
 enum { LCC_FAMILY_QWEN2VL = 0, LCC_FAMILY_DECODER = 1 };
-enum { LCC_MIXER_LATENT = 1 };
+enum { LCC_MIXER_LATENT = 1,
+       LCC_MIXER_PARALLEL = 2,                  /* grouped-query softmax attention with a distance bias beside linear attention with a fixed decay */
+       LCC_MIXER_SSD = 3 };                     /* state-space duality: short convolution, decay and step size from the input */
+/* LCC_BLOCK_PARALLEL: mixer and feed-forward in parallel behind one Dynamic-Tanh norm (latent mixer); LCC_BLOCK_SANDWICH: one after the other,
+ * an RMS norm (weight stored around zero) before and after each (the other mixers) */
+enum { LCC_BLOCK_PARALLEL = 0, LCC_BLOCK_SANDWICH = 1 };
 typedef struct {
   int mixer;                                    /* LCC_MIXER_* */
   int heads, q_rank, kv_rank;                   /* the model's: norms divide by the real ranks */
@@ -373,10 +379,20 @@ typedef struct {
   int kv_from;                                  /* -1: the layer has a latent of its own; else the earlier layer whose cache it reads */
   float scale;                                  /* of the scores */
   int ff_pad;                                   /* 0: no feed-forward */
+  /* softmax half of LCC_MIXER_PARALLEL: heads, dim_pad, vdim_pad, scale above, and */
+  int kv_heads, dim;                            /* dim: the real head size (norms divide by it) */
+  float q_temp_coef; int q_temp_every;          /* queries times 1 + coef ln(floor((p + 1) / every) + 1) */
+  /* recurrent part of LCC_MIXER_PARALLEL / LCC_MIXER_SSD */
+  int rec_heads, rec_groups, rec_key_pad, rec_vdim, rec_vdim_pad, rec_conv_taps, rec_norm_groups;
 } lcc_decoder_layer;
 typedef struct {
   int vocab_size, vocab_pad, width_pad, n_layers;
   float norm_eps, logit_softcap;                /* logit_softcap <= 0: none */
+  int block;                                    /* LCC_BLOCK_* */
+  int width;                                    /* real width (LCC_BLOCK_SANDWICH) */
+  float logit_scale;
+  int bigram_buckets;                           /* 0: none; else a second embedding, row (previous * mul_prev + current * mul_cur) mod buckets */
+  long long bigram_mul_prev, bigram_mul_cur;
 } lcc_decoder_config;
 /* 1 (default): decode steps of up to 16 streams run the fused launches (input + gate/up projections in one; query norm, up-projection, cache
  * append and gates in one for up to 8 streams; output projection + residual + next norm in one); 0: separate launches.  Returns the old value */

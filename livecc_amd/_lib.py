@@ -52,14 +52,18 @@ class Sampling(C.Structure):
 
 class DecoderLayer(C.Structure):
     _fields_ = [(n, C.c_int) for n in ("mixer", "heads", "q_rank", "kv_rank", "dim_pad", "vdim_pad", "q_rank_pad", "kv_rank_pad", "kv_from")] + \
-               [("scale", C.c_float), ("ff_pad", C.c_int)]
+               [("scale", C.c_float), ("ff_pad", C.c_int), ("kv_heads", C.c_int), ("dim", C.c_int), ("q_temp_coef", C.c_float), ("q_temp_every", C.c_int)] + \
+               [(n, C.c_int) for n in ("rec_heads", "rec_groups", "rec_key_pad", "rec_vdim", "rec_vdim_pad", "rec_conv_taps", "rec_norm_groups")]
 
 
 class DecoderConfigC(C.Structure):
-    _fields_ = [(n, C.c_int) for n in ("vocab_size", "vocab_pad", "width_pad", "n_layers")] + [("norm_eps", C.c_float), ("logit_softcap", C.c_float)]
+    _fields_ = [(n, C.c_int) for n in ("vocab_size", "vocab_pad", "width_pad", "n_layers")] + [("norm_eps", C.c_float), ("logit_softcap", C.c_float)] + \
+               [("block", C.c_int), ("width", C.c_int), ("logit_scale", C.c_float), ("bigram_buckets", C.c_int), ("bigram_mul_prev", C.c_longlong),
+                ("bigram_mul_cur", C.c_longlong)]
 
 
-MIXER_LATENT = 1            # LCC_MIXER_LATENT
+MIXER_LATENT, MIXER_PARALLEL, MIXER_SSD = 1, 2, 3            # LCC_MIXER_*
+BLOCK_PARALLEL, BLOCK_SANDWICH = 0, 1                        # LCC_BLOCK_*
 
 
 def declared_symbols() -> List[str]:

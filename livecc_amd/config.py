@@ -11,7 +11,7 @@ from __future__ import annotations
 import dataclasses
 import json
 import os
-from typing import List, Optional
+from typing import Any, List, Optional
 
 
 @dataclasses.dataclass
@@ -261,7 +261,7 @@ class LatentMixerSpec:
 
 @dataclasses.dataclass
 class DecoderLayerSpec:
-    mixer: LatentMixerSpec
+    mixer: Any                    # LatentMixerSpec, ParallelMixerSpec or SsdMixerSpec
     ff: int = 0                   # width of the gated feed-forward; 0: none
 
     @property
@@ -382,12 +382,282 @@ def debunex_7b() -> DebunexConfig:
     return _debunex(3584, 152064, 28, 18944, 28, 128, 128, 1536, 512, 2, "debunex-7b")
 
 
+# ---- layer-list decoders with pre- and post-norms around every sublayer: attention beside linear attention, state-space layers ----
+MAX_REC_KEY = 256             # channels of a recurrent state's key side the scan kernels are built for (after padding)
+MAX_SOFTMAX_HEAD = 256        # head sizes of the grouped-query decode attention with a distance bias (after padding)
+MAX_CONV_TAPS = 16
+MAX_ROW_WIDTH = 8192          # widest row of the row-norm kernels
+
+
+@dataclasses.dataclass
+class SoftmaxMixerSpec:
+    """Grouped-query softmax attention: per-head query / key norms, a query temperature, a linear distance bias per head, no rotation."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    q_temp_coef: float
+    q_temp_every: int
+
+    @property
+    def dim_pad(self) -> int:
+        return pad_head_dim(self.dim)
+
+    @property
+    def vdim_pad(self) -> int:
+        return pad_head_dim(self.vdim)
+
+    def slopes(self) -> List[float]:
+        """Score taken off per token of distance."""
+        return [2.0 ** (-8.0 * (h + 1) / self.heads) for h in range(self.heads)]
+
+
+@dataclasses.dataclass
+class LightningMixerSpec:
+    """Linear attention with a fixed decay per head."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: List[float]
+    groups = property(lambda self: self.heads)        # every head has keys and queries of its own
+    norm_groups = 1
+    conv_taps = 0
+
+    @property
+    def key_pad(self) -> int:
+        return _up(self.dim)
+
+    @property
+    def vdim_pad(self) -> int:
+        return _up(self.vdim)
+
+
+@dataclasses.dataclass
+class ParallelMixerSpec:
+    """Two mixers side by side over the same input; their normed outputs are averaged."""
+    left: SoftmaxMixerSpec
+    right: LightningMixerSpec
+
+    @property
+    def recurrent(self) -> LightningMixerSpec:
+        return self.right
+
+    @property
+    def in_rows(self) -> int:
+        """Rows of the fused input projection: left q | k | v | right q | k | v | gate."""
+        l, r = self.left, self.right
+        return (l.heads + l.kv_heads) * l.dim_pad + l.kv_heads * l.vdim_pad + 2 * r.heads * (r.key_pad + r.vdim_pad)
+
+    @property
+    def kv_bytes_per_token(self) -> int:
+        return 2 * self.left.kv_heads * (self.left.dim_pad + self.left.vdim_pad)
+
+
+@dataclasses.dataclass
+class SsdMixerSpec:
+    """State-space duality (Mamba-2): a short causal convolution, decays and step sizes from the input, a gated group norm."""
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    conv_taps: int
+    norm_groups: int
+
+    @property
+    def recurrent(self) -> "SsdMixerSpec":
+        return self
+
+    @property
+    def key_pad(self) -> int:
+        return _up(self.state)
+
+    @property
+    def vdim_pad(self) -> int:
+        return _up(self.vdim)
+
+    @property
+    def conv_channels(self) -> int:
+        """Stored channels of the convolution: x | B | C."""
+        return self.heads * self.vdim_pad + 2 * self.groups * self.key_pad
+
+    @property
+    def in_rows(self) -> int:
+        """Rows of the input projection: z | x | B | C | dt."""
+        return self.heads * self.vdim_pad + self.conv_channels + _up(self.heads)
+
+    kv_bytes_per_token = 0
+
+
+@dataclasses.dataclass
+class BemuzenConfig:
+    """A decoder-only language model given as a list of layers: mixer and feed-forward one after the other, a norm before and after each; a hashed
+    bigram embedding beside the token's own."""
+    vocab_size: int
+    hidden_size: int
+    layers: List[DecoderLayerSpec]
+    bigram_buckets: int
+    bigram_mul_prev: int
+    bigram_mul_cur: int
+    norm_eps: float = 1e-5
+    logit_scale: float = 1.0
+    max_position_embeddings: int = 32768          # default KV capacity of a stream
+    eos_token_id: Optional[int] = None
+    name: str = "bemuzen"
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def width_pad(self) -> int:
+        return _up(self.hidden_size)
+
+    @property
+    def vocab_pad(self) -> int:
+        return _up(self.vocab_size)
+
+    @property
+    def kv_bytes_per_token(self) -> int:
+        return sum(l.mixer.kv_bytes_per_token for l in self.layers)
+
+    @property
+    def state_bytes(self) -> int:
+        """Recurrent state of one stream (fp32)."""
+        n = 0
+        for l in self.layers:
+            r = l.mixer.recurrent
+            n += 4 * r.heads * r.key_pad * r.vdim_pad + (4 * r.conv_taps * r.conv_channels if r.conv_taps else 0)
+        return n
+
+    def decode_weight_bytes(self) -> int:
+        """bf16 weight bytes one decode step reads (stored sizes)."""
+        n = self.vocab_pad * self.width_pad
+        for l in self.layers:
+            m, r = l.mixer, l.mixer.recurrent
+            n += self.width_pad * (m.in_rows + _up(r.heads * r.vdim) + 3 * l.ff_pad)
+            if isinstance(m, ParallelMixerSpec):
+                n += self.width_pad * m.left.heads * m.left.vdim_pad
+        return 2 * n
+
+    def validate(self) -> None:
+        if not self.layers:
+            raise ValueError("a decoder needs at least one layer")
+        if min(self.vocab_size, self.hidden_size, self.bigram_buckets) < 1:
+            raise ValueError("vocabulary, width and bigram buckets must be positive")
+        if self.width_pad > MAX_ROW_WIDTH:
+            raise ValueError(f"widths above {MAX_ROW_WIDTH} are not supported")
+        if min(self.bigram_mul_prev, self.bigram_mul_cur) < 0:
+            raise ValueError("bigram multipliers must not be negative")
+        for i, l in enumerate(self.layers):
+            m, r = l.mixer, l.mixer.recurrent
+            if l.ff < 0 or min(r.heads, r.vdim, r.groups, r.norm_groups) < 1:
+                raise ValueError(f"layer {i}: sizes must be positive")
+            if isinstance(m, ParallelMixerSpec):
+                a = m.left
+                if min(a.heads, a.kv_heads, a.dim, a.vdim, a.q_temp_every, r.dim) < 1:
+                    raise ValueError(f"layer {i}: sizes must be positive")
+                if a.heads % a.kv_heads:
+                    raise ValueError(f"layer {i}: {a.heads} heads over {a.kv_heads} key/value heads")
+                if max(a.dim_pad, a.vdim_pad) > MAX_SOFTMAX_HEAD:
+                    raise ValueError(f"layer {i}: head sizes above {MAX_SOFTMAX_HEAD} are not supported")
+                if len(r.decay) != r.heads or min(r.decay) < 0.0 or max(r.decay) > 1.0:
+                    raise ValueError(f"layer {i}: one decay in [0, 1] per head")
+            else:
+                if min(m.state, m.conv_taps) < 1 or m.conv_taps > MAX_CONV_TAPS:
+                    raise ValueError(f"layer {i}: state must be positive, convolution taps in 1..{MAX_CONV_TAPS}")
+                if m.heads % m.groups or (m.heads * m.vdim) % m.norm_groups:
+                    raise ValueError(f"layer {i}: {m.heads} heads in {m.groups} groups, {m.heads * m.vdim} channels in {m.norm_groups} norm groups")
+            if r.key_pad > MAX_REC_KEY:
+                raise ValueError(f"layer {i}: recurrent key sizes above {MAX_REC_KEY} are not supported")
+
+    @classmethod
+    def from_dict(cls, raw: dict, name: str = "bemuzen") -> "BemuzenConfig":
+        layers = []
+        for i, e in enumerate(raw["layers"]):
+            m, mlp = e["mixer"], e.get("mlp")
+            if mlp is not None and mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward {mlp['kind']!r}")
+            if e["type"] == "parallel":
+                l, r = m["left"], m["right"]
+                spec = ParallelMixerSpec(
+                    SoftmaxMixerSpec(int(l["heads"]), int(l["kv_heads"]), int(l["dim"]), int(l["vdim"]), float(l["scale"]), float(l["q_temp"]["coef"]),
+                                     int(l["q_temp"]["every"])),
+                    LightningMixerSpec(int(r["heads"]), int(r["dim"]), int(r["vdim"]), [float(x) for x in r["decay"]]))
+            elif e["type"] == "mamba2":
+                spec = SsdMixerSpec(int(m["heads"]), int(m["vdim"]), int(m["state"]), int(m["groups"]), int(m["conv"]), int(m["norm_groups"]))
+            else:
+                raise ValueError(f"layer {i}: unknown layer type {e['type']!r}")
+            layers.append(DecoderLayerSpec(spec, 0 if mlp is None else int(mlp["ff"])))
+        b, eos = raw["embedding"]["bigram"], raw.get("eos_token_id")
+        cfg = cls(vocab_size=int(raw["vocab"]), hidden_size=int(raw["width"]), layers=layers, bigram_buckets=int(b["buckets"]),
+                  bigram_mul_prev=int(b["mul_prev"]), bigram_mul_cur=int(b["mul_cur"]), norm_eps=float(raw["norm"]["eps"]),
+                  logit_scale=float(raw["logit_scale"]), eos_token_id=None if eos is None else int(eos), name=name)
+        cfg.validate()
+        return cfg
+
+    def to_dict(self) -> dict:
+        """The config.json form."""
+        out = {"architecture": "Bemuzen", "vocab": self.vocab_size, "width": self.hidden_size, "norm": {"eps": self.norm_eps},
+               "logit_scale": self.logit_scale, "layers": [],
+               "embedding": {"bigram": {"buckets": self.bigram_buckets, "mul_prev": self.bigram_mul_prev, "mul_cur": self.bigram_mul_cur}}}
+        if self.eos_token_id is not None:
+            out["eos_token_id"] = self.eos_token_id
+        for l in self.layers:
+            m = l.mixer
+            if isinstance(m, ParallelMixerSpec):
+                a, r = m.left, m.right
+                kind, mix = "parallel", {
+                    "left": {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim, "vdim": a.vdim, "scale": a.scale,
+                             "q_temp": {"coef": a.q_temp_coef, "every": a.q_temp_every}},
+                    "right": {"heads": r.heads, "dim": r.dim, "vdim": r.vdim, "decay": list(r.decay)}}
+            else:
+                kind, mix = "mamba2", {"heads": m.heads, "vdim": m.vdim, "state": m.state, "groups": m.groups, "conv": m.conv_taps, "norm_groups": m.norm_groups}
+            out["layers"].append({"type": kind, "mixer": mix, "mlp": {"kind": "dense", "ff": l.ff} if l.ff else None})
+        return out
+
+    @classmethod
+    def from_pretrained(cls, path: str) -> "BemuzenConfig":
+        with open(os.path.join(path, "config.json")) as f:
+            return cls.from_dict(json.load(f), name=os.path.basename(os.path.normpath(path)))
+
+
+def _bemuzen(width, vocab, n_layers, ff, left, right, ssd, every, name) -> BemuzenConfig:
+    """Every `every`-th layer is a state-space layer, the others run attention beside linear attention."""
+    layers = [DecoderLayerSpec(dataclasses.replace(ssd) if i % every == every - 1 else ParallelMixerSpec(dataclasses.replace(left), dataclasses.replace(right)), ff)
+              for i in range(n_layers)]
+    return BemuzenConfig(vocab, width, layers, 65521, 8191, 131, name=name)
+
+
+def _decays(heads: int) -> List[float]:
+    return [1.0 - 2.0 ** (-2.0 - 6.0 * h / max(heads - 1, 1)) for h in range(heads)]
+
+
+def bemuzen_tiny() -> BemuzenConfig:
+    return _bemuzen(192, 320, 3, 224, SoftmaxMixerSpec(6, 2, 24, 40, 0.2, 0.25, 48), LightningMixerSpec(3, 40, 24, _decays(3)), SsdMixerSpec(6, 24, 40, 2, 3, 3),
+                    3, "bemuzen-tiny")
+
+
+def bemuzen_2b() -> BemuzenConfig:
+    """Qwen2-VL-2B's width, feed-forward, attention heads, depth and vocabulary."""
+    return _bemuzen(1536, 151936, 28, 8960, SoftmaxMixerSpec(12, 2, 128, 128, 128 ** -0.5, 0.1, 4096), LightningMixerSpec(12, 128, 128, _decays(12)),
+                    SsdMixerSpec(48, 64, 128, 1, 4, 1), 4, "bemuzen-2b")
+
+
+def bemuzen_7b() -> BemuzenConfig:
+    """LiveCC-7B's width, feed-forward, attention heads, depth and vocabulary."""
+    return _bemuzen(3584, 152064, 28, 18944, SoftmaxMixerSpec(28, 4, 128, 128, 128 ** -0.5, 0.1, 4096), LightningMixerSpec(28, 128, 128, _decays(28)),
+                    SsdMixerSpec(112, 64, 128, 1, 4, 1), 4, "bemuzen-7b")
+
+
 # config.json "architecture" -> configuration class; checkpoints without the key are Qwen2-VL ones
-ARCHITECTURES = {"Debunex": DebunexConfig}
+ARCHITECTURES = {"Debunex": DebunexConfig, "Bemuzen": BemuzenConfig}
+DECODER_CONFIGS = tuple(ARCHITECTURES.values())          # layer lists: served by the engine's decoder family
 
 
 PRESETS = {"livecc-7b": livecc_7b, "qwen2vl-2b": qwen2vl_2b, "qwen2vl-2b-untied": qwen2vl_2b_untied, "qwen2vl-72b": qwen2vl_72b,
-           "tiny": tiny, "small": small, "debunex-tiny": debunex_tiny, "debunex-2b": debunex_2b, "debunex-7b": debunex_7b}
+           "tiny": tiny, "small": small, "debunex-tiny": debunex_tiny, "debunex-2b": debunex_2b, "debunex-7b": debunex_7b,
+           "bemuzen-tiny": bemuzen_tiny, "bemuzen-2b": bemuzen_2b, "bemuzen-7b": bemuzen_7b}
 
 
 def architecture_of(path: str) -> Optional[str]:

@@ -86,10 +86,11 @@ __device__ unsigned int lcc_attn32_ones_page[256] = {[0 ... 255] = 0x3F803F80u};
 // LM (round 6, the tower kernel only): the softmax denominator comes out of the P . V MFMAs -- the V^T rows 80..95 of the third d-tile do not
 // exist at d = 80 and are fed with ONES, so O^T rows 80..95 accumulate sum_k bf16(P) under the same lazy rescale as O -- instead of 16 v_add +
 // the l_run update per region.  l then sums the ROUNDED probabilities the numerator uses (fp32 accumulation either way).
-// D = channels of q / k, DV = channels of v.
-template <int D, int DV, int PW, bool LM, class Issue>
-LCC_DEVICE void attn32_key_loop(const u32x4* alds, Issue issue, const u32x4 (&qf)[D / 16], int tb, int te, int mlim, int lim, float scale_log2e,
-                                bool active, int lane, int hh, f32x16 (&o)[(DV + 31) / 32], float& m_run, float& l_run) {
+// D = channels of q / k, DV = channels of v.  BIAS: slope (pos - key) is taken off the scaled scores (slope in units of log2), pos = this lane's query.
+template <int D, int DV, int PW, bool LM, bool BIAS = false, class Issue>
+LCC_DEVICE void attn32_key_loop(const u32x4* alds, Issue issue, const u32x4 (&qf)[D / 16], int tb, int te, int mlim, int lim, float scale_raw,
+                                bool active, int lane, int hh, f32x16 (&o)[(DV + 31) / 32], float& m_run, float& l_run, float slope = 0.f, int pos = 0) {
+  const float scale_log2e = BIAS ? 1.f : scale_raw;     // with a bias the scores are brought to log2 units before the maximum
   constexpr int KP = D / 16, DT = (DV + 31) / 32, VP = 2 * DT, NP = KP + VP, NSTAGE = 10;
   auto stage_of = [&](int t) { return alds + ((t - tb) % NSTAGE) * (NP * 64); };
   bf16x8 p_prev[2];                                     // P of the previous tile, its P . V still pending
@@ -114,6 +115,11 @@ LCC_DEVICE void attn32_key_loop(const u32x4* alds, Issue issue, const u32x4 (&qf
     for (int ks = 0; ks < KP; ++ks) sc_nxt = mfma32(as_bf16x8(kn[ks * 64 + lane]), as_bf16x8(qf[ks]), sc_nxt);
     // vector pipe: softmax of tile t
     const int kb = t * 32;
+    if (BIAS) {
+      const float base = slope * (float)(kb + 8 * hh - pos);
+#pragma unroll
+      for (int r = 0; r < 16; ++r) sc_cur[r] = fmaf(sc_cur[r], scale_raw, fmaf(slope, (float)(16 * (r >> 3) + (r & 7)), base));
+    }
     if (MASKED) {
 #pragma unroll
       for (int r = 0; r < 16; ++r) sc_cur[r] = (kb + 16 * (r >> 3) + 8 * hh + (r & 7)) < lim ? sc_cur[r] : -INFINITY;
@@ -152,7 +158,7 @@ LCC_DEVICE void attn32_key_loop(const u32x4* alds, Issue issue, const u32x4 (&qf
     for (int i = 0; i < NP; ++i) {
       __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);
       if (i < NP - 3) __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
-      __builtin_amdgcn_sched_group_barrier(0x002, ((MASKED ? 7 : 5) - (LM ? 1 : 0)) * 16 / NP, 0);
+      __builtin_amdgcn_sched_group_barrier(0x002, ((MASKED ? 7 : 5) - (LM ? 1 : 0) + (BIAS ? 2 : 0)) * 16 / NP, 0);
     }
     // region boundary: the accumulators now hold tiles <= t-1 at the OLD maximum; bring them to the new one before tile t's P.V.
     // Lazy: once the running maximum has settled alpha is exactly 1.0 in every lane and the multiplies are skipped (x * 1.0f is
@@ -537,7 +543,8 @@ int attn_prefill32_launch(const bf16_t* q, bf16_t* out, const int32_t* tile_stre
 // dealt to the XCDs in contiguous chunks, groups fastest (and from the back: the long ones first), so the groups that read the same keys share
 // an L2.  The per-head output factor `gate` is applied before the one rounding to bf16.
 // ------------------------------------------------------------------------------------------------------------------------------
-template <int DK, int DV>
+// SLOTS: keys and values out of the slots' arenas, shared by the query heads of a KV head, and a distance bias per head (kernels.h: MhaArgs).
+template <int DK, int DV, bool SLOTS>
 __global__ __launch_bounds__(512, 2) void attn_mha32_kernel(MhaArgs a) {
   constexpr int NWAVE = 8, KP = DK / 16, DT = DV / 32, VP = 2 * DT, NP = KP + VP, NSTAGE = 10, PW = (NP + NWAVE - 1) / NWAVE;
   extern __shared__ __attribute__((aligned(16))) u32x4 alds[];
@@ -547,14 +554,23 @@ __global__ __launch_bounds__(512, 2) void attn_mha32_kernel(MhaArgs a) {
   const int item = (int)(blockIdx.x & 7) * ((n_items + 7) >> 3) + (int)(blockIdx.x >> 3);
   if ((int)(blockIdx.x >> 3) >= ((n_items + 7) >> 3) || item >= n_items) return;      // the whole block leaves before any barrier
   const int h = item / a.n_groups, grp = a.n_groups - 1 - (item - h * a.n_groups);
-  const int q0 = a.grp_q0[grp], nq = a.grp_nq[grp], pos0 = a.grp_pos0[grp], key0 = a.grp_key0[grp];
+  const int q0 = a.grp_q0[grp], nq = a.grp_nq[grp], pos0 = a.grp_pos0[grp], key0 = SLOTS ? 0 : a.grp_key0[grp];
   const int ldq = a.heads * DK;
   const bool active = wave * 32 < nq;
   const int qr = min(wave * 32 + col, nq - 1);           // clamped: surplus columns compute a valid row and are not stored
   const bool valid = wave * 32 + col < nq;
   const int ntile = (pos0 + nq + 31) / 32;               // the keys are stored in whole 32-key tiles (zero-filled)
-  const bf16_t* kbase = a.k + (size_t)key0 * ldq + h * DK;
-  const bf16_t* vbase = a.vt + (size_t)h * DV * a.ldv + key0;
+  const int ldk = SLOTS ? DK : ldq, ldv = SLOTS ? 32 : a.ldv;
+  const bf16_t *kbase, *vbase;
+  if (SLOTS) {
+    const bf16_t* arena = a.kv_base[a.grp_slot[grp]];
+    const int kvh = h / (a.heads / a.kv_heads);
+    kbase = arena + a.k_off + (size_t)kvh * a.lmax * DK;
+    vbase = arena + a.v_off + (size_t)kvh * a.lmax * DV;
+  } else {
+    kbase = a.k + (size_t)key0 * ldq + h * DK;
+    vbase = a.vt + (size_t)h * DV * a.ldv + key0;
+  }
 
   u32x4 qf[KP];
   {
@@ -570,12 +586,12 @@ __global__ __launch_bounds__(512, 2) void attn_mha32_kernel(MhaArgs a) {
   for (int j = 0; j < PW; ++j) {
     const int p = min(j * NWAVE + wave, NP - 1);         // surplus slots re-fetch the last piece (same bytes, same place)
     if (p < KP) {
-      pbase[j] = kbase + (size_t)swap23(col) * ldq + p * 16 + hh * 8;
-      pstride[j] = (size_t)32 * ldq;
+      pbase[j] = kbase + (size_t)swap23(col) * ldk + p * 16 + hh * 8;
+      pstride[j] = (size_t)32 * ldk;
     } else {
       const int dt = (p - KP) >> 1, s = (p - KP) & 1;
-      pbase[j] = vbase + (size_t)(dt * 32 + col) * a.ldv + s * 16 + hh * 8;
-      pstride[j] = 32;
+      pbase[j] = vbase + (size_t)(dt * 32 + col) * ldv + s * 16 + hh * 8;
+      pstride[j] = SLOTS ? (size_t)DV * 32 : 32;
     }
   }
   int tb = 0;
@@ -595,7 +611,8 @@ __global__ __launch_bounds__(512, 2) void attn_mha32_kernel(MhaArgs a) {
   const int key_limit = pos0 + qr + 1;
   int min_limit = pos0 + min(wave * 32, nq - 1) + 1;            // of the wave's first row
   asm volatile("" : "+v"(min_limit));
-  attn32_key_loop<DK, DV, PW, false>(alds, issue, qf, tb, ntile, min_limit, key_limit, a.scale_log2e, active, lane, hh, o, m_run, l_run);
+  const float slope = SLOTS && a.slope ? a.slope[h] : 0.f;
+  attn32_key_loop<DK, DV, PW, false, SLOTS>(alds, issue, qf, tb, ntile, min_limit, key_limit, a.scale_log2e, active, lane, hh, o, m_run, l_run, slope, pos0 + qr);
   if (!active) return;
   const float l = xor32_sum(l_run);
   if (valid) {
@@ -608,21 +625,23 @@ __global__ __launch_bounds__(512, 2) void attn_mha32_kernel(MhaArgs a) {
         st8(op + dt * 32 + 8 * r4 + 4 * hh, (u32x2){pack2(o[dt][4 * r4] * f, o[dt][4 * r4 + 1] * f), pack2(o[dt][4 * r4 + 2] * f, o[dt][4 * r4 + 3] * f)});
   }
 }
-template <int DK, int DV>
+template <int DK, int DV, bool SLOTS>
 static void mha32_go(const MhaArgs& a, hipStream_t st) {
   constexpr size_t lds = (size_t)10 * (DK / 16 + 2 * (DV / 32)) * 1024;
   static DeviceOnce once;   // per instantiation
-  if (once.first()) (void)hipFuncSetAttribute((const void*)attn_mha32_kernel<DK, DV>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+  if (once.first()) (void)hipFuncSetAttribute((const void*)attn_mha32_kernel<DK, DV, SLOTS>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
   const long n_items = (long)a.n_groups * a.heads;
-  attn_mha32_kernel<DK, DV><<<dim3((unsigned)((n_items + 7) / 8 * 8)), dim3(512), lds, st>>>(a);
+  attn_mha32_kernel<DK, DV, SLOTS><<<dim3((unsigned)((n_items + 7) / 8 * 8)), dim3(512), lds, st>>>(a);
 }
-int attn_mha32_launch(const MhaArgs& a, hipStream_t st) {
-  if (a.dim == 128 && a.vdim == 128) mha32_go<128, 128>(a, st);
-  else if (a.dim == 64 && a.vdim == 64) mha32_go<64, 64>(a, st);
-  else if (a.dim == 64 && a.vdim == 128) mha32_go<64, 128>(a, st);
-  else if (a.dim == 128 && a.vdim == 64) mha32_go<128, 64>(a, st);
+template <bool SLOTS>
+static int mha32_pick(const MhaArgs& a, hipStream_t st) {
+  if (a.dim == 128 && a.vdim == 128) mha32_go<128, 128, SLOTS>(a, st);
+  else if (a.dim == 64 && a.vdim == 64) mha32_go<64, 64, SLOTS>(a, st);
+  else if (a.dim == 64 && a.vdim == 128) mha32_go<64, 128, SLOTS>(a, st);
+  else if (a.dim == 128 && a.vdim == 64) mha32_go<128, 64, SLOTS>(a, st);
   else return LCC_ERR_SHAPE;
   return 0;
 }
+int attn_mha32_launch(const MhaArgs& a, hipStream_t st) { return a.grp_slot ? mha32_pick<true>(a, st) : mha32_pick<false>(a, st); }
 
 }  // namespace lcc

@@ -435,6 +435,14 @@ __global__ __launch_bounds__(256, 4) void dgemv_in_swiglu_kernel(DgArgs in, DgAr
   if ((int)blockIdx.x < nb_in) dgemv_body<1, DG_PRO_PLAIN, DG_EPI_F32, 4, 2, 2, DG_CHAIN_NONE>(in, none, blockIdx.x, reinterpret_cast<f32x4(*)[1][64]>(red), nullptr);
   else dgemv_body<2, DG_PRO_PLAIN, DG_EPI_SWIGLU, 4, 1, 2, DG_CHAIN_NONE>(sw, none, (int)blockIdx.x - nb_in, red, nullptr);
 }
+// two independent products of the same rows' inputs in ONE launch (fp32 out): each fills the chip only half by itself
+template <int NW, int UNR>
+__global__ __launch_bounds__(NW * 64) void dgemv_f32_pair_kernel(DgArgs a, DgArgs b, int nb_a) {
+  __shared__ f32x4 red[NW - 1][1][64];
+  const DgChain none{nullptr, 0u, nullptr, 0};
+  if ((int)blockIdx.x < nb_a) dgemv_body<1, DG_PRO_PLAIN, DG_EPI_F32, NW, UNR, 2, DG_CHAIN_NONE>(a, none, blockIdx.x, red, nullptr);
+  else dgemv_body<1, DG_PRO_PLAIN, DG_EPI_F32, NW, UNR, 2, DG_CHAIN_NONE>(b, none, (int)blockIdx.x - nb_a, red, nullptr);
+}
 // query up-projection of the normed query latent (norm as prologue, fp32 out); the M blocks behind it append the rows' cache latents and gates
 __global__ __launch_bounds__(512, 2) void dgemv_latent_q_kernel(DgArgs a, LatentInArgs row, int nb) {
   __shared__ f32x4 red[7][1][64];
@@ -507,6 +515,32 @@ int dgemv_in_swiglu(const DgArgs& in, const DgArgs& sw, hipStream_t st) {
     return LCC_ERR_SHAPE;
   if (!in.W || !in.X || !in.C32 || in.wscale || (sw.N > 0 && (!sw.W || !sw.X || !sw.C || sw.wscale))) return LCC_ERR_ARG;
   dgemv_in_swiglu_kernel<<<dim3(in.N / 16 + sw.N / 32), dim3(256), 0, st>>>(in, sw, in.N / 16);
+  return 0;
+}
+static int dg_f32_check(const DgArgs& a) {
+  g_launch_counts[LC_DGEMV_V2]++;
+  if (a.M < 1 || a.M > 16 || a.N < 16 || (a.N & 15) || (a.K & 31) || a.K < 32 || (a.ldx & 7) || (a.ldc & 3)) return LCC_ERR_SHAPE;
+  return !a.W || !a.X || !a.C32 || a.wscale ? LCC_ERR_ARG : 0;
+}
+int dgemv_f32(const DgArgs& a, hipStream_t st) {
+  if (int rc = dg_f32_check(a)) return rc;
+  if (a.K >= 8192) dgemv_kernel<1, DG_PRO_PLAIN, DG_EPI_F32, 16, 3><<<dim3(a.N / 16), dim3(1024), 0, st>>>(a);
+  else if (a.N >= 8192) dgemv_kernel<1, DG_PRO_PLAIN, DG_EPI_F32, 4, 2><<<dim3(a.N / 16), dim3(256), 0, st>>>(a);
+  else dgemv_kernel<1, DG_PRO_PLAIN, DG_EPI_F32, 8, 4><<<dim3(a.N / 16), dim3(512), 0, st>>>(a);
+  return 0;
+}
+int dgemv_f32_pair(const DgArgs& a, const DgArgs& b, hipStream_t st) {
+  if (int rc = dg_f32_check(a)) return rc;
+  if (int rc = dg_f32_check(b)) return rc;
+  if (a.M != b.M) return LCC_ERR_SHAPE;
+  dgemv_f32_pair_kernel<8, 4><<<dim3(a.N / 16 + b.N / 16), dim3(512), 0, st>>>(a, b, a.N / 16);
+  return 0;
+}
+// gate/up Linear [SwiGLU] of rows that are normed already
+int dgemv_swiglu(const DgArgs& a, hipStream_t st) {
+  if (int rc = dg_check(a, DG_PRO_PLAIN, DG_EPI_SWIGLU)) return rc;
+  if (a.wscale) return LCC_ERR_ARG;
+  dgemv_kernel<2, DG_PRO_PLAIN, DG_EPI_SWIGLU, 4, 1, 2><<<dim3(a.N / 32), dim3(256), 0, st>>>(a);
   return 0;
 }
 bool dgemv_latent_q_ok(int M, int K) { return M >= 1 && M <= 8 && K <= 2048 && (K & 31) == 0; }

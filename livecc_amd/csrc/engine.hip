@@ -162,7 +162,7 @@ extern "C" size_t lcc_engine_workspace_bytes(const lcc_engine* e) {
 }
 extern "C" size_t lcc_engine_state_bytes(const lcc_engine* e) {
   const size_t B = e->lim.max_slots;
-  return align_up(B * 4) * 6 + 256 + align_up(B * 8) + align_up(B * (size_t)e->lim.max_history * 4) + align_up(B * (size_t)e->words * 4) + 4096 + 1024 + 1024;
+  return align_up(B * 4) * 7 + 256 + align_up(B * 8) + align_up(B * (size_t)e->lim.max_history * 4) + align_up(B * (size_t)e->words * 4) + 4096 + 1024 + 1024;
 }
 extern "C" size_t lcc_engine_kv_bytes_per_slot(const lcc_engine* e) { return (e->family == LCC_FAMILY_DECODER ? e->dec_kv_total : e->lay.total()) * 2; }
 extern "C" size_t lcc_engine_meta_bytes(const lcc_engine* e) {
@@ -190,6 +190,7 @@ extern "C" int lcc_engine_bind_buffers(lcc_engine* e, void* workspace_dev, size_
   e->d_cur_tok = cv.take<int32_t>(B); e->d_done = cv.take<int32_t>(B); e->d_rng_ctr = cv.take<uint32_t>(B); e->d_counter = cv.take<int32_t>(16); e->d_attn_cnt = cv.take<int32_t>(256); e->d_chain = cv.take<unsigned>(160); e->d_kv_base = cv.take<bf16_t*>(B);
   e->d_history = cv.take<int32_t>(B * (size_t)e->lim.max_history);
   e->d_seen = cv.take<uint32_t>(B * (size_t)e->words);
+  e->d_prev_tok = cv.take<int32_t>(B);
   HIP_TRY(hipMemset(e->state, 0, state_bytes));
   std::fill(e->chain_epoch.begin(), e->chain_epoch.end(), 0u);   // the device hand-off counters were just zeroed: host mirror follows
   for (int i = 0; i < META_RING; ++i) if (!e->meta_ev[i]) HIP_TRY(hipEventCreateWithFlags(&e->meta_ev[i], hipEventDisableTiming));

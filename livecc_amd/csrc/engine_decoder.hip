@@ -13,15 +13,10 @@
 //   ff      silu(Wgate h) * (Wup h)       one GEMM, SwiGLU epilogue; lands beside the attention output
 //   out     [Wo | Wdown] [attention | ff] one GEMM over the concatenated K: the sum of the parallel sublayers is its accumulator
 //           residual += slabs; h = next norm                  (resid_dyt)
-#include "engine_internal.h"
+#include "engine_decoder.h"
 
 namespace {
 
-struct DecBuffers {
-  float *x, *part, *gate, *ws_o, *ws_ml, *logits;
-  bf16_t *h, *cq, *q, *cat, *kmat, *vmat, *crow, *cfrag, *lat_q, *last;
-  size_t part_cap;     // floats
-};
 struct DecDims {       // maxima over the layers
   int W, in_n = 0, qp = 0, qd = 0, vd = 0, rp = 0, cat = 0, heads = 0; size_t hr = 0;
 };
@@ -41,7 +36,9 @@ DecDims dims_of(const lcc_engine* e) {
 }
 // rows of freshly formed keys one attention launch can hold: any single stream, or a whole call of fresh streams (each rounded up to 32)
 size_t key_rows(const lcc_engine* e) { return std::max<size_t>(e->lim.max_kv_len, (size_t)e->lim.max_new_rows + 32 * (size_t)std::min(e->lim.max_slots, e->lim.max_new_rows)); }
-int logit_rows_max(const lcc_engine* e) { return std::max(std::min(256, e->lim.max_new_rows), std::min(e->lim.max_slots, LCC_MAX_DECODE_BATCH)); }
+}  // namespace
+int decoder_logit_rows_max(const lcc_engine* e) { return std::max(std::min(256, e->lim.max_new_rows), std::min(e->lim.max_slots, LCC_MAX_DECODE_BATCH)); }
+namespace {
 // key splits of the decode attention for `rows` rows: two or more 64-key tiles per block once the chip is full
 int decode_splits(const lcc_engine* e, int rows, int max_len) {
   static const int forced = [] { const char* v = getenv("LCC_LATENT_SPLITS"); return v ? atoi(v) : 0; }();
@@ -57,8 +54,13 @@ size_t decode_slots(const lcc_engine* e) {     // (row, split) pairs of one deco
   return n;
 }
 size_t carve(const lcc_engine* e, DecBuffers* b, char* base) {
+  if (e->dc.block == LCC_BLOCK_SANDWICH) {
+    Carver cv; cv.base = base;
+    carve_mixers(e, b, cv);
+    return cv.off + 4096;
+  }
   const DecDims d = dims_of(e);
-  const size_t S = std::max(e->lim.max_new_rows, std::min(e->lim.max_slots, LCC_MAX_DECODE_BATCH)), T = key_rows(e), V = e->c.vocab_size, LR = logit_rows_max(e);
+  const size_t S = std::max(e->lim.max_new_rows, std::min(e->lim.max_slots, LCC_MAX_DECODE_BATCH)), T = key_rows(e), V = e->c.vocab_size, LR = decoder_logit_rows_max(e);
   Carver cv; cv.base = base;
   b->x = cv.take<float>(S * d.W); b->h = cv.take<bf16_t>(S * d.W);
   const size_t nmax = std::max(std::max(d.in_n, d.qd), d.W);
@@ -80,39 +82,10 @@ int carve_bound(lcc_engine* e, DecBuffers* b) {
   return 0;
 }
 
-// fp32 slab product into b.part; the split count is the one the tiles or the weight-streaming kernels want, bounded by the slab buffer
-int slab_gemm(const DecBuffers& b, const bf16_t* A, int lda, const bf16_t* W, int M, int N, int K, int* nsplit, hipStream_t st) {
-  int s = gemm_routes_skinny(M, K, false) ? gemv_num_splits(N, K) : gemm_tiled_num_splits(M, N, K, true);
-  s = std::min(std::min(s, 8), (K + 63) / 64);
-  while (s > 1 && (size_t)s * M * N > b.part_cap) --s;
-  if ((size_t)s * M * N > b.part_cap) return fail(LCC_ERR_STATE, "slab buffer too small for %d x %d", M, N);
-  GemmArgs g; g.A = A; g.lda = lda; g.W = W; g.ldw = K; g.w_packed = 1; g.M = M; g.N = N; g.K = K; g.partial = b.part; g.nsplit = s;
-  *nsplit = s;
-  return gemm_bf16(g, st);
-}
-int plain_gemm(const bf16_t* A, int lda, const bf16_t* W, bf16_t* C, int ldc, int M, int N, int K, int epilogue, hipStream_t st) {
-  GemmArgs g; g.A = A; g.lda = lda; g.W = W; g.ldw = K; g.w_packed = 1; g.C = C; g.ldc = ldc; g.M = M; g.N = N; g.K = K; g.epilogue = epilogue;
-  return gemm_bf16(g, st);
-}
-
-struct KeyGroup {       // streams whose keys are formed together
-  int tile0, n_tiles, grp0, n_grps, row0, n_rows;
-};
-struct PrefillTables {
-  const int32_t *tok_stream, *tok_pos, *tile_slot, *tile_key0, *tile_nkeys, *grp_q0, *grp_nq, *grp_pos0, *grp_key0;
-  std::vector<KeyGroup> groups;
-};
-
-int tap(lcc_engine* e, const DecBuffers& b, int index, int S, hipStream_t st) {
-  if (!e->llm_taps) return 0;
-  if (S > e->llm_tap_rows) return fail(LCC_ERR_STATE, "taps bound for %d rows, call has %d", e->llm_tap_rows, S);
-  const size_t W = e->c.hidden_size;
-  HIP_TRY(hipMemcpyAsync((float*)e->llm_taps + (size_t)index * e->llm_tap_rows * W, b.x, (size_t)S * W * 4, hipMemcpyDeviceToDevice, st));
-  return 0;
-}
-
+}  // namespace
 int g_fused_decode = 1;      // lcc_debug_set_decoder_fused: decode steps of up to 16 rows run the fused launches (6 per layer instead of 9)
 
+namespace {
 // S packed rows through every layer; pt null: a decode step over the streams `d_slots`.  On exit b.h holds the final norm of the residual.
 int run_decoder_layers(lcc_engine* e, const DecBuffers& b, int S, const PrefillTables* pt, const int32_t* d_slots, int nsplit_attn, const AttnDirect& direct,
                        hipStream_t st) {
@@ -125,7 +98,7 @@ int run_decoder_layers(lcc_engine* e, const DecBuffers& b, int S, const PrefillT
     const DecLayerW& w = e->dw[l];
     const bool own = L.kv_from < 0;
     const int owner = own ? l : L.kv_from, rp = L.kv_rank_pad, in_n = lcc_engine::dec_in_rows(L), ldcat = L.heads * L.vdim_pad + L.ff_pad;
-    const size_t kv_off = e->dec_kv_off[owner];
+    const size_t kv_off = e->dec_off[owner].kv;
     const float scale_log2e = L.scale * 1.4426950408889634f;
     int ns = 1;
     if (fused) {
@@ -185,16 +158,28 @@ int run_decoder_layers(lcc_engine* e, const DecBuffers& b, int S, const PrefillT
   return 0;
 }
 
+// x and the first norm of the rows' tokens: prefill ids per row, decode (pt null) the slots' current tokens
+int embed_rows(lcc_engine* e, const DecBuffers& b, const int32_t* ids, const int32_t* d_slots, const PrefillTables* pt, int S, hipStream_t st) {
+  if (e->dc.block != LCC_BLOCK_SANDWICH) return embed_dyt(ids, d_slots, e->embed, e->dw[0].norm, b.x, b.h, S, e->c.hidden_size, st);
+  BigramEmbed bg; bg.table = e->dec_bigram; bg.buckets = e->dc.bigram_buckets; bg.mul_prev = e->dc.bigram_mul_prev; bg.mul_cur = e->dc.bigram_mul_cur;
+  return embed_bigram_rms(ids, pt ? pt->tok_stream : d_slots, pt ? pt->tok_pos : nullptr, pt ? pt->tok_row0 : nullptr, e->d_kv_len, e->d_prev_tok, e->embed, bg,
+                          e->dw[0].norm1, e->dc.norm_eps, b.x, b.h, S, e->dc.width, e->c.hidden_size, st);
+}
+int run_layers_of(lcc_engine* e, const DecBuffers& b, int S, const PrefillTables* pt, const int32_t* d_slots, int nsplit_attn, const AttnDirect& direct, hipStream_t st) {
+  return e->dc.block == LCC_BLOCK_SANDWICH ? run_mixer_layers(e, b, S, pt, d_slots, nsplit_attn, direct, st)
+                                           : run_decoder_layers(e, b, S, pt, d_slots, nsplit_attn, direct, st);
+}
+
 // logits of n rows of normed activations; `out` (row pitch = padded vocabulary, -inf beyond it) and / or `dense` (row pitch = vocabulary)
 int decoder_logits(lcc_engine* e, const DecBuffers& b, const bf16_t* rows, int n, float* out, float* dense, hipStream_t st) {
   const int V = e->c.vocab_size;
   int ns = 1;
   LCC_TRY(slab_gemm(b, rows, e->c.hidden_size, e->lm_head, n, V, e->c.hidden_size, &ns, st));
-  return logits_cap(b.part, ns, n, V, e->dc.vocab_size, e->dc.logit_softcap, out, dense, st);
+  return logits_cap(b.part, ns, n, V, e->dc.vocab_size, e->dc.block == LCC_BLOCK_SANDWICH ? e->dc.logit_scale : 1.f, e->dc.logit_softcap, out, dense, st);
 }
 int head_and_sample_decoder(lcc_engine* e, const DecBuffers& b, const bf16_t* rows, int B, const int32_t* d_slots, const lcc_sampling* sp, int step_index,
                             hipStream_t st) {
-  const int LR = logit_rows_max(e);
+  const int LR = decoder_logit_rows_max(e);
   for (int r0 = 0; r0 < B; r0 += LR) {       // (a prefill call may start more streams than one logits block holds)
     const int n = std::min(LR, B - r0);
     float* dense = (sp && sp->logits_out) ? (float*)sp->logits_out + ((size_t)step_index * B + r0) * e->dc.vocab_size : nullptr;
@@ -210,6 +195,7 @@ int head_and_sample_decoder(lcc_engine* e, const DecBuffers& b, const bf16_t* ro
 int lcc_engine::dec_in_rows(const lcc_decoder_layer& L) { return L.q_rank_pad + (L.kv_from < 0 ? L.kv_rank_pad : 0) + (L.heads + 15) / 16 * 16; }
 size_t lcc_decoder_ws_bytes(const lcc_engine* e) { DecBuffers b; return carve(e, &b, nullptr); }
 size_t lcc_decoder_meta_bytes(const lcc_engine* e) {
+  if (e->dc.block == LCC_BLOCK_SANDWICH) return mixers_meta_ints(e) * 4;
   const size_t S = e->lim.max_new_rows, B = e->lim.max_slots;
   const size_t tiles = (S + 32 * B) / 16 + (size_t)std::min<size_t>(B, S) * (e->lim.max_kv_len / 16 + 2);      // new rows plus everything cached
   return (4 * S + 3 * tiles + 4 * (S / MHA_GROUP_ROWS + B + 1) + 4 * B + 256) * 4;
@@ -223,7 +209,8 @@ extern "C" lcc_engine* lcc_engine_create_decoder(const lcc_decoder_config* cfg, 
   if (lim->max_kv_len < 64 || (lim->max_kv_len & 63) || lim->max_slots <= 0 || lim->max_slots > 16 * 1024 || lim->max_new_rows <= 0 || lim->max_history <= 0) {
     fail(LCC_ERR_SHAPE, "decoder: max_kv_len %% 64, max_slots, max_new_rows, max_history"); return nullptr;
   }
-  for (int i = 0; i < cfg->n_layers; ++i) {
+  if (cfg->block != LCC_BLOCK_PARALLEL && cfg->block != LCC_BLOCK_SANDWICH) { fail(LCC_ERR_ARG, "decoder: unknown block form %d", cfg->block); return nullptr; }
+  for (int i = 0; i < cfg->n_layers && cfg->block == LCC_BLOCK_PARALLEL; ++i) {
     const lcc_decoder_layer& L = layers[i];
     if (L.mixer != LCC_MIXER_LATENT) { fail(LCC_ERR_ARG, "decoder layer %d: unknown mixer %d", i, L.mixer); return nullptr; }
     if (L.heads < 1 || L.heads > 65535 || L.q_rank < 1 || L.kv_rank < 1 || L.q_rank_pad < L.q_rank || L.kv_rank_pad < L.kv_rank || (L.q_rank_pad & 63) ||
@@ -243,11 +230,15 @@ extern "C" lcc_engine* lcc_engine_create_decoder(const lcc_decoder_config* cfg, 
   e->c.vocab_size = cfg->vocab_pad; e->c.hidden_size = cfg->width_pad; e->c.n_layers = cfg->n_layers; e->c.rms_eps = cfg->norm_eps;
   e->qd = e->kvd = e->qkvd = e->E = 0; e->vit_hd = 0; e->words = cfg->vocab_pad / 32; e->lay = KvLayout{0, 0, lim->max_kv_len, 0};
   e->dl.assign(layers, layers + cfg->n_layers);
-  e->dw.resize(cfg->n_layers); e->dec_kv_off.assign(cfg->n_layers, 0);
-  size_t off = 0;
-  for (int i = 0; i < cfg->n_layers; ++i)
-    if (layers[i].kv_from < 0) { e->dec_kv_off[i] = off; off += align_up((size_t)lim->max_kv_len * layers[i].kv_rank_pad, 128); }
-  e->dec_kv_total = off;
+  e->dw.resize(cfg->n_layers); e->dec_off.assign(cfg->n_layers, DecOffsets());
+  if (cfg->block == LCC_BLOCK_SANDWICH) {
+    if (mixers_layout(e) != 0) { delete e; return nullptr; }
+  } else {
+    size_t off = 0;
+    for (int i = 0; i < cfg->n_layers; ++i)
+      if (layers[i].kv_from < 0) { e->dec_off[i].kv = off; off += align_up((size_t)lim->max_kv_len * layers[i].kv_rank_pad, 128); }
+    e->dec_kv_total = off;
+  }
   e->chain_epoch.assign(128, 0u);
   { int dev = 0; if (hipGetDevice(&dev) == hipSuccess) (void)hipDeviceGetAttribute(&e->cu_count, hipDeviceAttributeMultiprocessorCount, dev); }
   if (e->cu_count <= 0) e->cu_count = 256;
@@ -256,6 +247,7 @@ extern "C" lcc_engine* lcc_engine_create_decoder(const lcc_decoder_config* cfg, 
 }
 
 int lcc_decoder_resolve_weights(lcc_engine* e, std::string* missing) {
+  if (e->dc.block == LCC_BLOCK_SANDWICH) return mixers_resolve_weights(e, missing);
   auto get = [&](const std::string& n) -> const bf16_t* {
     auto it = e->w.find(n);
     if (it == e->w.end()) { if (missing) { *missing += n; *missing += ' '; } return nullptr; }
@@ -283,11 +275,14 @@ int lcc_decoder_prefill(lcc_engine* e, int n_streams, const int32_t* slots, cons
     if (!sp->prompt_rows || !sp->prompt_logits_out || sp->prompt_rows[i] < 0 || sp->prompt_rows[i] >= S) return fail(LCC_ERR_ARG, "prompt_rows[%d] out of range", i);
   PrefillTables pt;
   std::vector<int32_t> tok_stream(S), tok_pos(S), last_row(n_streams), ts, tk, tn, gq, gn, gp, gk;
-  const size_t cap_tiles = key_rows(e) / 16;
+  const bool mixers = e->dc.block == LCC_BLOCK_SANDWICH;
+  const size_t cap_tiles = mixers ? ~(size_t)0 : key_rows(e) / 16;
+  std::vector<int32_t> row0, rlast, gs, sr, sn, ss, sf, st0, stn;
+  const int seg = mixers ? mixers_segment_rows(e, bf, n_new, n_streams) : 0;
   int row = 0;
   KeyGroup kg{0, 0, 0, 0, 0, 0};
   for (int b = 0; b < n_streams; ++b) {
-    const int past = e->h_kv_len[slots[b]], keys = past + n_new[b], tiles = (keys + 31) / 32 * 2;
+    const int past = e->h_kv_len[slots[b]], keys = past + n_new[b], tiles = mixers ? 0 : (keys + 31) / 32 * 2;
     if (kg.n_rows > 0 && (size_t)(kg.n_tiles + tiles) > cap_tiles) {
       pt.groups.push_back(kg);
       kg = KeyGroup{(int)ts.size(), 0, (int)gq.size(), 0, row, 0};
@@ -297,6 +292,13 @@ int lcc_decoder_prefill(lcc_engine* e, int n_streams, const int32_t* slots, cons
       gq.push_back(row - kg.row0 + q); gn.push_back(std::min(MHA_GROUP_ROWS, n_new[b] - q)); gp.push_back(past + q); gk.push_back(kg.n_tiles * 16);
     }
     for (int t = 0; t < tiles; ++t) { ts.push_back(slots[b]); tk.push_back(t * 16); tn.push_back(keys); }
+    if (mixers) {
+      st0.push_back((int)sr.size());
+      for (int q = 0; q < n_new[b]; q += seg) { sr.push_back(row + q); sn.push_back(std::min(seg, n_new[b] - q)); ss.push_back(slots[b]); sf.push_back(past + q == 0); }
+      stn.push_back((int)sr.size() - st0.back());
+      for (int q = 0; q < n_new[b]; q += MHA_GROUP_ROWS) gs.push_back(slots[b]);
+      for (int i = 0; i < n_new[b]; ++i) { row0.push_back(row); rlast.push_back(row + n_new[b] - 1); }
+    }
     kg.n_tiles += tiles; kg.n_grps = (int)gq.size() - kg.grp0; kg.n_rows += n_new[b];
     row += n_new[b];
     last_row[b] = row - 1;
@@ -307,21 +309,29 @@ int lcc_decoder_prefill(lcc_engine* e, int n_streams, const int32_t* slots, cons
   bool ok = mw.put(ids, S, &d_ids) && mw.put(tok_stream.data(), S, &d_stream) && mw.put(tok_pos.data(), S, &d_pos) && mw.put(last_row.data(), n_streams, &d_last) &&
             mw.put(slots, n_streams, &d_slots) && mw.put(ts.data(), ts.size(), &d_ts) && mw.put(tk.data(), tk.size(), &d_tk) && mw.put(tn.data(), tn.size(), &d_tn) &&
             mw.put(gq.data(), gq.size(), &d_gq) && mw.put(gn.data(), gn.size(), &d_gn) && mw.put(gp.data(), gp.size(), &d_gp) && mw.put(gk.data(), gk.size(), &d_gk);
+  int32_t *d_row0 = nullptr, *d_rlast = nullptr, *d_gs = nullptr, *d_sr = nullptr, *d_sn = nullptr, *d_ss = nullptr, *d_sf = nullptr, *d_st0 = nullptr, *d_stn = nullptr;
+  if (ok && mixers)
+    ok = mw.put(row0.data(), S, &d_row0) && mw.put(rlast.data(), S, &d_rlast) && mw.put(gs.data(), gs.size(), &d_gs) && mw.put(sr.data(), sr.size(), &d_sr) &&
+         mw.put(sn.data(), sn.size(), &d_sn) && mw.put(ss.data(), ss.size(), &d_ss) && mw.put(sf.data(), sf.size(), &d_sf) &&
+         mw.put(st0.data(), st0.size(), &d_st0) && mw.put(stn.data(), stn.size(), &d_stn);
   if (ok && nw > 0) ok = nw <= S && mw.put(sp->prompt_rows, nw, &d_want) != nullptr;
   if (!ok) return fail(LCC_ERR_STATE, "meta ring slot too small");
   LCC_TRY(meta_commit(&mw, st));
   pt.tok_stream = d_stream; pt.tok_pos = d_pos; pt.tile_slot = d_ts; pt.tile_key0 = d_tk; pt.tile_nkeys = d_tn;
   pt.grp_q0 = d_gq; pt.grp_nq = d_gn; pt.grp_pos0 = d_gp; pt.grp_key0 = d_gk;
 
+  pt.tok_row0 = d_row0; pt.tok_last = d_rlast; pt.grp_slot = d_gs; pt.seg_row0 = d_sr; pt.seg_rows = d_sn; pt.seg_slot = d_ss; pt.seg_fresh = d_sf;
+  pt.str_seg0 = d_st0; pt.str_nseg = d_stn; pt.n_grps = (int)gq.size(); pt.n_seg = (int)sr.size(); pt.n_streams = n_streams;
+
   for (int b = 0; b < n_streams; ++b) {      // a new generate call of these slots
     HIP_TRY(hipMemsetAsync(e->d_hist_col + slots[b], 0, 4, st));
     HIP_TRY(hipMemsetAsync(e->d_done + slots[b], 0, 4, st));
   }
   LCC_TRY(seen_set(e->d_seen, e->words, d_ids, d_stream, S, 0, nullptr, st));
-  LCC_TRY(embed_dyt(d_ids, nullptr, e->embed, e->dw[0].norm, bf.x, bf.h, S, e->c.hidden_size, st));
-  LCC_TRY(run_decoder_layers(e, bf, S, &pt, nullptr, 1, AttnDirect(), st));
+  LCC_TRY(embed_rows(e, bf, d_ids, nullptr, &pt, S, st));
+  LCC_TRY(run_layers_of(e, bf, S, &pt, nullptr, 1, AttnDirect(), st));
 
-  const int LR = logit_rows_max(e), W = e->c.hidden_size;
+  const int LR = decoder_logit_rows_max(e), W = e->c.hidden_size;
   for (int r0 = 0; r0 < nw; r0 += LR) {
     const int n = std::min(LR, nw - r0);
     LCC_TRY(gather_rows_bf16(bf.h, d_want + r0, bf.last, n, W, st));
@@ -336,6 +346,7 @@ int lcc_decoder_prefill(lcc_engine* e, int n_streams, const int32_t* slots, cons
   for (int b = 0; b < n_streams; ++b) {
     HIP_TRY(hipMemcpyAsync(e->d_kv_len + slots[b], d_kv + b, 4, hipMemcpyDeviceToDevice, st));
     HIP_TRY(hipMemcpyAsync(e->d_pos + slots[b], d_kv + b, 4, hipMemcpyDeviceToDevice, st));
+    HIP_TRY(hipMemcpyAsync(e->d_prev_tok + slots[b], d_ids + last_row[b], 4, hipMemcpyDeviceToDevice, st));
   }
   // the streams' last rows: gathered in blocks the logits buffer holds
   for (int r0 = 0; r0 < n_streams; r0 += LR) {
@@ -353,19 +364,19 @@ int lcc_decoder_prefill(lcc_engine* e, int n_streams, const int32_t* slots, cons
 // the n_steps loop of lcc_llm_decode (engine_llm.hip) behind its checks
 int lcc_decoder_decode(lcc_engine* e, int n_streams, const int32_t* slots, const int32_t* d_slots, int max_len, int n_steps, int first_step_index, const lcc_sampling* sp, hipStream_t st) {
   DecBuffers bf; LCC_TRY(carve_bound(e, &bf));
-  const int nsplit = decode_splits(e, n_streams, max_len);
+  const int nsplit = e->dc.block == LCC_BLOCK_SANDWICH ? mixers_decode_splits(e, n_streams, max_len) : decode_splits(e, n_streams, max_len);
   for (int step = 0; step < n_steps; ++step) {
     const bool prof_step = e->prof_on && (step & 3) == 0 && 2 * (e->step_n + 1) <= (int)e->step_ev.size();
     if (prof_step) HIP_TRY(hipEventRecord(e->step_ev[2 * e->step_n], st));
     LCC_TRY(seen_set(e->d_seen, e->words, e->d_cur_tok, d_slots, n_streams, 1, e->d_done, st));
-    LCC_TRY(embed_dyt(e->d_cur_tok, d_slots, e->embed, e->dw[0].norm, bf.x, bf.h, n_streams, e->c.hidden_size, st));
+    LCC_TRY(embed_rows(e, bf, e->d_cur_tok, d_slots, nullptr, n_streams, st));
     AttnDirect dir;      // (a stream that EOS froze on the device has fewer keys than the host counts: its step is discarded, and the rows exist)
     if (n_streams <= 4) {
       for (int b = 0; b < n_streams; ++b) { dir.base[b] = (const bf16_t*)e->h_kv_base[slots[b]]; dir.n[b] = e->h_kv_len[slots[b]] + step + 1; }
       dir.used = n_streams;
     }
-    LCC_TRY(run_decoder_layers(e, bf, n_streams, nullptr, d_slots, nsplit, dir, st));
-    LCC_TRY(advance_lengths(d_slots, e->d_kv_len, e->d_pos, n_streams, e->d_done, st));
+    LCC_TRY(run_layers_of(e, bf, n_streams, nullptr, d_slots, nsplit, dir, st));
+    LCC_TRY(advance_lengths(d_slots, e->d_kv_len, e->d_pos, n_streams, e->d_done, st, e->d_cur_tok, e->d_prev_tok));
     LCC_TRY(head_and_sample_decoder(e, bf, bf.h, n_streams, d_slots, sp, first_step_index + step, st));
     if (prof_step) {
       HIP_TRY(hipEventRecord(e->step_ev[2 * e->step_n + 1], st));

@@ -60,7 +60,12 @@ struct DecLayerW {     // a layer of a layer-list decoder (engine_decoder.hip)
   DytNorm norm;
   const bf16_t *in_w = nullptr, *q_norm = nullptr, *kv_norm = nullptr, *uq_w = nullptr, *uk_w = nullptr, *ukt_w = nullptr, *uv_w = nullptr,
                *gate_up_w = nullptr, *out_w = nullptr;
+  // LCC_BLOCK_SANDWICH
+  const bf16_t *norm1 = nullptr, *norm1b = nullptr, *norm2 = nullptr, *norm2b = nullptr, *down_w = nullptr;
+  const bf16_t *k_norm = nullptr, *lo_w = nullptr, *l_out = nullptr, *r_out = nullptr, *ro_w = nullptr, *rec_norm = nullptr, *conv_w = nullptr, *conv_b = nullptr;
+  const float *slope = nullptr, *rec_rate = nullptr, *rec_dt_bias = nullptr, *rec_skip = nullptr;
 };
+struct DecOffsets { size_t kv = 0, v = 0, state = 0, conv = 0; };      // a layer's blocks in a slot's arena, in bf16 elements
 
 struct Carver {  // bump allocator over a caller-provided region
   char* base = nullptr;
@@ -86,7 +91,8 @@ struct lcc_engine {
   std::vector<lcc_decoder_layer> dl;
   std::vector<DecLayerW> dw;
   DytNorm dec_final_norm;
-  std::vector<size_t> dec_kv_off;      // element offset of a layer's latents inside a slot's arena (layers that own one)
+  const bf16_t *dec_final_w = nullptr, *dec_bigram = nullptr;          // LCC_BLOCK_SANDWICH
+  std::vector<DecOffsets> dec_off;     // kv: latents (layers that own them) or K
   size_t dec_kv_total = 0;
   static int dec_in_rows(const lcc_decoder_layer& L);      // output rows of the fused input projection
   int qd, kvd, qkvd, words, E, vit_hd;
@@ -123,6 +129,7 @@ struct lcc_engine {
   int32_t* d_counter = nullptr;   // arrival counter of the fused GEMV tails (zero between launches)
   int32_t* d_attn_cnt = nullptr;  // [16 streams x Hkv] arrival counters of the fused decode attention (zero between launches)
   uint32_t* d_seen = nullptr;
+  int32_t* d_prev_tok = nullptr;  // the last token a slot has consumed (models whose embedding looks at it)
   uint32_t* d_rng_ctr = nullptr;  // per-slot Philox draw counter of the sampling kernel (zero for a fresh stream)
   unsigned* d_chain = nullptr;    // [128] monotonic hand-off counters of the chained decode launches (one per layer) + [128] = error word
   std::vector<unsigned> chain_epoch;   // host mirror: launches issued per counter (the consumer's target = epoch * producer blocks)

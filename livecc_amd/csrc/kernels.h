@@ -186,7 +186,8 @@ struct DeviceOnce {
     return true;
   }
 };
-int advance_lengths(const int32_t* slots, int32_t* kv_len, int32_t* pos, int B, const int32_t* done, hipStream_t st);
+// cur_tok / prev_tok (both or none): the token just consumed becomes the slot's previous token
+int advance_lengths(const int32_t* slots, int32_t* kv_len, int32_t* pos, int B, const int32_t* done, hipStream_t st, const int32_t* cur_tok = nullptr, int32_t* prev_tok = nullptr);
 // teacher forcing (tests): the token just sampled for stream b becomes forced[b] (current token + last history column); the forced stream
 // also decides where a slot ends (`done`: flags from before this step, updated by a forced EOS)
 int force_tokens(const int32_t* slots, const int32_t* forced, int B, int32_t* cur_tok, int32_t* history, int hist_ld, const int32_t* hist_col,
@@ -226,7 +227,22 @@ int dgemv_norm_bf16(const DgArgs& a, hipStream_t st);     // [final RMSNorm] lm_
 // ---- layer-list decoders: row operators (decoder_ops.hip) ----
 int embed_dyt(const int32_t* ids, const int32_t* indirect, const bf16_t* table, const DytNorm& nm, float* x, bf16_t* h, int rows, int dim, hipStream_t st);
 int resid_dyt(float* x, const float* part, int nsplit, const DytNorm& nm, bf16_t* h, int rows, int dim, hipStream_t st);
-int logits_cap(const float* part, int nsplit, int rows, int ld, int vocab, float cap, float* out, float* dense, hipStream_t st);
+int logits_cap(const float* part, int nsplit, int rows, int ld, int vocab, float scale, float cap, float* out, float* dense, hipStream_t st);
+// RMS norms with weights stored around zero (x / rms(x) * (1 + w)); `width` = real channels, `dim` = stored ones (zero beyond width)
+struct BigramEmbed { const bf16_t* table = nullptr; int buckets = 0; int64_t mul_prev = 0, mul_cur = 0; };   // row (prev * mul_prev + cur * mul_cur) mod buckets; first token: row `buckets`
+// x = embed[id] + bigram row, h = norm(x).  Prefill: ids[row], the token before it is ids[row - 1] or -- first row of a stream's portion
+// (tok_row0[row] == row) -- prev_tok[slot]; decode (tok_pos null): ids = current token per slot.  tok_stream = the rows' slots
+int embed_bigram_rms(const int32_t* ids, const int32_t* tok_stream, const int32_t* tok_pos, const int32_t* tok_row0, const int32_t* kv_len, const int32_t* prev_tok,
+                     const bf16_t* table, const BigramEmbed& bg, const bf16_t* norm_w, float eps, float* x, bf16_t* h, int rows, int width, int dim, hipStream_t st);
+// Behind a sublayer's output product(s), fp32 slabs: y = the product, or -- part_b -- the mean of two products, each normed with its plain weight;
+// x += norm(y; post_w); h = norm(x; next_w)
+struct PostNormArgs {
+  const float* part = nullptr; int nsplit = 1; const float* part_b = nullptr; int nsplit_b = 1;
+  const bf16_t* w_a = nullptr; const bf16_t* w_b = nullptr;          // part_b only
+  const bf16_t* post_w = nullptr; const bf16_t* next_w = nullptr;
+  float* x = nullptr; bf16_t* h = nullptr; int rows = 0, width = 0, dim = 0; float eps = 0.f;
+};
+int post_norm_resid(const PostNormArgs& a, hipStream_t st);
 int set_tokens(const int32_t* slots, const int32_t* toks, int n, int32_t* cur_tok, int32_t* done, int32_t* hist_col, hipStream_t st);
 
 // ---- latent attention (latent.hip, attn32.hip) ----
@@ -254,6 +270,10 @@ struct MhaArgs {                 // causal multi-head attention of packed rows o
   // groups of up to MHA_GROUP_ROWS consecutive rows of one stream, rows ascending: first row, rows, position of the first row, first key row of the stream
   const int32_t* grp_q0 = nullptr; const int32_t* grp_nq = nullptr; const int32_t* grp_pos0 = nullptr; const int32_t* grp_key0 = nullptr;
   int n_groups = 0, rows = 0, heads = 0, dim = 0, vdim = 0; float scale_log2e = 0.f;
+  // grp_slot set: keys and values are read from the slots' arenas instead (kv_heads heads, `heads / kv_heads` query heads share one):
+  // k [kv_heads][lmax][dim] at k_off, v blocked-transposed [kv_heads][lmax / 32][vdim][32] at v_off
+  const int32_t* grp_slot = nullptr; bf16_t* const* kv_base = nullptr; size_t k_off = 0, v_off = 0; int lmax = 0, kv_heads = 0;
+  const float* slope = nullptr;  // optional fp32 [heads], in units of log2: slope (i - j) is taken off the score of key j at position i
 };
 constexpr int MHA_GROUP_ROWS = 256;
 int attn_mha(const MhaArgs& a, hipStream_t st);
@@ -269,5 +289,67 @@ struct LatentDecodeArgs {
 };
 int latent_attn_decode(const LatentDecodeArgs& a, hipStream_t st);
 int latent_merge_uv(const LatentDecodeArgs& a, const bf16_t* uv, int vdim, const float* gate, bf16_t* out, int ldo, hipStream_t st);
+
+
+// ---- grouped-query attention with a distance bias over slot arenas (biased_attn.hip) ----
+struct GqaInArgs {               // behind the fused input projection: per-head RMS norms, query temperature, cache append
+  const float* part = nullptr; int nsplit = 1, rows = 0, ldn = 0;    // fp32 slabs; columns [0, heads dim) q | kv_heads dim k | kv_heads vdim v
+  int heads = 0, kv_heads = 0, dim = 0, dim_pad = 0, vdim_pad = 0; float eps = 0.f;
+  const bf16_t* q_norm = nullptr; const bf16_t* k_norm = nullptr;    // plain weights [dim_pad], shared by the heads
+  float temp_coef = 0.f; int temp_every = 1;                         // q *= 1 + coef ln(floor((p + 1) / every) + 1)
+  bf16_t* q = nullptr;                                               // [rows][heads dim_pad]
+  const int32_t* tok_stream = nullptr; const int32_t* tok_pos = nullptr; const int32_t* kv_len = nullptr;   // tok_pos null: kv_len[slot]
+  bf16_t* const* kv_base = nullptr; size_t k_off = 0, v_off = 0; int lmax = 0;
+};
+constexpr int GQA_MAX_SPLIT = 64;
+struct GqaDecodeArgs {
+  const bf16_t* q = nullptr; int rows = 0, heads = 0, kv_heads = 0, dim = 0, vdim = 0, nsplit = 1; float scale_log2e = 0.f;
+  const float* slope = nullptr;
+  const int32_t* slots = nullptr; const int32_t* kv_len = nullptr; bf16_t* const* kv_base = nullptr; size_t k_off = 0, v_off = 0; int lmax = 0;
+  float* ws_o = nullptr; float* ws_ml = nullptr;                     // [rows][heads][nsplit][vdim], [rows][heads][nsplit][2]
+  bf16_t* out = nullptr;                                             // [rows][heads vdim]
+  AttnDirect direct;
+};
+int gqa_decode(const GqaDecodeArgs& a, hipStream_t st);              // the splits; the merge runs with rec_norm (gqa_merge_rec_norm)
+
+// ---- recurrent mixers: S_t = 2^(rate dt_t) S_{t-1} + dt_t k_t v_t^T, o_t = S_t^T q_t (+ skip v_t) per head (recurrent.hip) ----
+struct RecInArgs {               // where the inputs lie in the fused input projection (fp32 slabs [nsplit][rows][ldn]), and the state
+  const float* part = nullptr; int nsplit = 1, rows = 0, ldn = 0;
+  int q_col = 0, k_col = 0, v_col = 0, dt_col = -1;                  // [groups key_pad], [groups key_pad], [heads vdim_pad]; dt_col < 0: dt = 1
+  int heads = 0, groups = 0, np = 0, ep = 0;                         // key and value channels per head, stored
+  int taps = 0, conv_col = 0, conv_ch = 0; const bf16_t* conv_w = nullptr; const bf16_t* conv_b = nullptr;   // taps 0: none; channel c = column conv_col + c
+  const float* rate = nullptr; const float* dt_bias = nullptr; const float* skip = nullptr;
+  const int32_t* tok_stream = nullptr; const int32_t* tok_pos = nullptr;   // tok_pos null: kv_len[slot]
+  const int32_t* tok_row0 = nullptr; const int32_t* tok_last = nullptr;    // prefill: first / last row of the row's stream in this call
+  const int32_t* kv_len = nullptr; const int32_t* done = nullptr;
+  bf16_t* const* kv_base = nullptr; size_t state_off = 0, conv_off = 0;    // fp32 [heads][np][ep]; fp32 [taps][conv_ch], position p at row p % taps
+  bf16_t* q = nullptr; bf16_t* k = nullptr; bf16_t* v = nullptr; float* dt = nullptr;   // prefill: activated inputs, [rows][..]; dt [rows][heads]
+};
+int mixer_prep(const GqaInArgs* left, const RecInArgs* rec, hipStream_t st);              // prefill: either or both, one launch
+int rec_decode(const RecInArgs& rec, const GqaInArgs* left, float* y, hipStream_t st);    // decode: state step (y [rows][heads ep]) + the rows of `left`
+struct RecScanArgs {
+  const bf16_t* q = nullptr; const bf16_t* k = nullptr; const bf16_t* v = nullptr; const float* dt = nullptr;      // dt null: 1
+  const float* rate = nullptr; const float* skip = nullptr; float* y = nullptr;
+  int heads = 0, groups = 0, np = 0, ep = 0;
+  // segments of consecutive rows of one stream: first row, rows, slot, 1 = the stream starts here (state zero); streams: first segment, segments
+  const int32_t* seg_row0 = nullptr; const int32_t* seg_rows = nullptr; const int32_t* seg_slot = nullptr; const int32_t* seg_fresh = nullptr; int n_seg = 0;
+  const int32_t* str_seg0 = nullptr; const int32_t* str_nseg = nullptr; int n_streams = 0;
+  float* seg_state = nullptr; float* seg_decay = nullptr;            // more segments than streams: [n_seg][heads][np][ep], [n_seg][heads]
+  bf16_t* const* kv_base = nullptr; size_t state_off = 0;
+};
+constexpr int REC_CHUNK = 64;
+int rec_scan(const RecScanArgs& a, hipStream_t st);
+struct RecNormArgs {             // y -> gated norm over norm_groups equal parts of the concatenated heads -> bf16 [rows][ld], zero behind the real channels
+  const float* y = nullptr; const float* part = nullptr; int nsplit = 1, rows = 0, ldn = 0, gate_col = 0;
+  int gate_first = 0;            // 1: rms(y silu(gate)) w;  0: rms(y) w sigmoid(gate)
+  int heads = 0, vdim = 0, ep = 0, norm_groups = 1; float eps = 0.f; const bf16_t* w = nullptr; bf16_t* out = nullptr; int ld = 0;
+  const RecInArgs* conv = nullptr;   // prefill of a mixer with a convolution: the last inputs of every stream go to its state (by value in the launch)
+};
+int rec_norm(const RecNormArgs& a, hipStream_t st);
+int gqa_merge_rec_norm(const GqaDecodeArgs& m, const RecNormArgs& a, hipStream_t st);
+// decode GEMVs with fp32 output (decode_v2.hip; M <= 16): one product, two independent products in one launch, gate/up with SwiGLU
+int dgemv_f32(const DgArgs& a, hipStream_t st);
+int dgemv_f32_pair(const DgArgs& a, const DgArgs& b, hipStream_t st);
+int dgemv_swiglu(const DgArgs& a, hipStream_t st);
 
 }  // namespace lcc

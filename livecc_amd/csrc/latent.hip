@@ -76,8 +76,22 @@ __global__ __launch_bounds__(256) void attn_mha_rows_kernel(MhaArgs a) {
   // the group of this row
   int lo = 0, hi = a.n_groups - 1;
   while (lo < hi) { const int mid = (lo + hi + 1) >> 1; if (a.grp_q0[mid] <= row) lo = mid; else hi = mid - 1; }
-  const int nkeys = a.grp_pos0[lo] + (row - a.grp_q0[lo]) + 1, kb = a.grp_key0[lo];
+  const int nkeys = a.grp_pos0[lo] + (row - a.grp_q0[lo]) + 1;
   const int ldq = a.heads * a.dim;
+  const bf16_t *kbase, *vbase;                         // key i: row i of kbase (pitch ldk); value: tile i / 32 (pitch vtile), channel d (pitch ldv)
+  const bool slots = a.grp_slot != nullptr;
+  const int ldk = slots ? a.dim : ldq, ldv = slots ? 32 : a.ldv;
+  const size_t vtile = slots ? (size_t)a.vdim * 32 : 32;
+  if (slots) {
+    const bf16_t* arena = a.kv_base[a.grp_slot[lo]];
+    const int kvh = h / (a.heads / a.kv_heads);
+    kbase = arena + a.k_off + (size_t)kvh * a.lmax * a.dim;
+    vbase = arena + a.v_off + (size_t)kvh * a.lmax * a.vdim;
+  } else {
+    kbase = a.k + (size_t)a.grp_key0[lo] * ldq + h * a.dim;
+    vbase = a.vt + (size_t)h * a.vdim * a.ldv + a.grp_key0[lo];
+  }
+  const float slope = a.slope ? a.slope[h] : 0.f;
   for (int d = tid; d < a.dim; d += 256) s_qf[d] = bf2f(a.q[(size_t)row * ldq + h * a.dim + d]);
   __syncthreads();
   float m = -INFINITY, l = 0.f, o[4] = {0.f, 0.f, 0.f, 0.f};        // vdim <= 1024
@@ -85,14 +99,14 @@ __global__ __launch_bounds__(256) void attn_mha_rows_kernel(MhaArgs a) {
     const int key = k0 + tid;
     float s = -INFINITY;
     if (key < nkeys) {
-      const bf16_t* kp = a.k + (size_t)(kb + key) * ldq + h * a.dim;
+      const bf16_t* kp = kbase + (size_t)key * ldk;
       float acc = 0.f;
       for (int d = 0; d < a.dim; d += 8) {
         const u32x4 v = ld16(kp + d);
 #pragma unroll
         for (int e = 0; e < 4; ++e) acc = fmaf(s_qf[d + 2 * e], lo2f(v[e]), fmaf(s_qf[d + 2 * e + 1], hi2f(v[e]), acc));
       }
-      s = acc * a.scale_log2e;
+      s = fmaf(acc, a.scale_log2e, slope * (float)(key + 1 - nkeys));
     }
     const float wm = wave_max(s);
     if (lane == 0) red[wave] = wm;
@@ -111,9 +125,9 @@ __global__ __launch_bounds__(256) void attn_mha_rows_kernel(MhaArgs a) {
     for (int j = 0; j < 4; ++j) {
       const int d = tid + 256 * j;
       if (d < a.vdim) {
-        const bf16_t* vp = a.vt + (size_t)(h * a.vdim + d) * a.ldv + kb + k0;
+        const bf16_t* vp = vbase + (size_t)(k0 >> 5) * vtile + (size_t)d * ldv;
         float acc = 0.f;
-        for (int i = 0; i < n; ++i) acc = fmaf(s_p[i], bf2f(vp[i]), acc);
+        for (int i = 0; i < n; ++i) acc = fmaf(s_p[i], bf2f(vp[(size_t)(i >> 5) * vtile + (i & 31)]), acc);
         o[j] = o[j] * alpha + acc;
       }
     }
@@ -132,8 +146,11 @@ static int mha_rows(const MhaArgs& a, hipStream_t st) {
 }
 int attn_mha(const MhaArgs& a, hipStream_t st) {
   if (a.rows <= 0 || a.n_groups <= 0) return 0;
-  if (a.heads < 1 || a.dim < 8 || (a.dim & 7) || a.dim > 8192 || a.vdim < 1 || a.vdim > 1024 || (a.ldv & 31) || (a.ldo & 3)) return LCC_ERR_SHAPE;
-  if (!a.q || !a.k || !a.vt || !a.out || !a.grp_q0 || !a.grp_nq || !a.grp_pos0 || !a.grp_key0) return LCC_ERR_ARG;
+  if (a.heads < 1 || a.dim < 8 || (a.dim & 7) || a.dim > 8192 || a.vdim < 1 || a.vdim > 1024 || (!a.grp_slot && (a.ldv & 31)) || (a.ldo & 3)) return LCC_ERR_SHAPE;
+  if (!a.q || !a.out || !a.grp_q0 || !a.grp_nq || !a.grp_pos0) return LCC_ERR_ARG;
+  if (a.grp_slot) {
+    if (!a.kv_base || a.lmax < 32 || (a.lmax & 31) || a.kv_heads < 1 || a.heads % a.kv_heads) return LCC_ERR_SHAPE;
+  } else if (!a.k || !a.vt || !a.grp_key0 || a.slope) return LCC_ERR_ARG;
   if ((a.dim == 64 || a.dim == 128) && (a.vdim == 64 || a.vdim == 128)) return attn_mha32_launch(a, st);
   return mha_rows(a, st);
 }

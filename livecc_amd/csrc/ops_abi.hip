@@ -387,7 +387,7 @@ extern "C" int lcc_resid_dyt(float* x, const float* partial, int nsplit, const v
          "lcc_resid_dyt");
 }
 extern "C" int lcc_logits_cap(const float* partial, int nsplit, int rows, int ld, int vocab, float cap, float* out, float* dense, void* stream) {
-  OP_RET(logits_cap(partial, nsplit, rows, ld, vocab, cap, out, dense, (hipStream_t)stream), "lcc_logits_cap");
+  OP_RET(logits_cap(partial, nsplit, rows, ld, vocab, 1.0f, cap, out, dense, (hipStream_t)stream), "lcc_logits_cap");
 }
 extern "C" int lcc_latent_norm_append(const float* partial, int nsplit, int rows, int ldn, int q_rank, int q_rank_pad, const void* q_norm, int kv_rank,
                                       int kv_rank_pad, const void* kv_norm, int heads, float eps, const int32_t* tok_stream, const int32_t* tok_pos,

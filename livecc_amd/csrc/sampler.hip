@@ -552,11 +552,14 @@ int sample_topk_topp(const void* logits, bool f32, int ld, int B, int V, uint32_
 
 // per-stream device counters advanced at the end of a decode step (kv length, rope position, history column)
 // per-slot device counters of a consumed token (kv length, rope position): frozen once the slot has emitted EOS
-__global__ void advance_kernel(const int32_t* slots, int32_t* kv_len, int32_t* pos, int B, const int32_t* done) {
+__global__ void advance_kernel(const int32_t* slots, int32_t* kv_len, int32_t* pos, int B, const int32_t* done, const int32_t* cur_tok, int32_t* prev_tok) {
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= B) return;
   const int s = slots[i];
-  if (done == nullptr || !done[s]) { kv_len[s] += 1; pos[s] += 1; }
+  if (done == nullptr || !done[s]) {
+    kv_len[s] += 1; pos[s] += 1;
+    if (prev_tok != nullptr) prev_tok[s] = cur_tok[s];
+  }
 }
 // Teacher forcing (test instrument): the forced stream decides everything, including where it ends.  The sampler ran with EOS suppressed
 // (engine_llm.hip: head_and_sample), so `done` still holds the flags from BEFORE this step: a slot whose forced stream has ended stays
@@ -578,9 +581,9 @@ int force_tokens(const int32_t* slots, const int32_t* forced, int B, int32_t* cu
   force_tokens_kernel<<<dim3((B + 63) / 64), dim3(64), 0, st>>>(slots, forced, B, cur_tok, history, hist_ld, hist_col, done, eos, eos2);
   return 0;
 }
-int advance_lengths(const int32_t* slots, int32_t* kv_len, int32_t* pos, int B, const int32_t* done, hipStream_t st) {
+int advance_lengths(const int32_t* slots, int32_t* kv_len, int32_t* pos, int B, const int32_t* done, hipStream_t st, const int32_t* cur_tok, int32_t* prev_tok) {
   if (B <= 0) return 0;
-  advance_kernel<<<dim3((B + 63) / 64), dim3(64), 0, st>>>(slots, kv_len, pos, B, done);
+  advance_kernel<<<dim3((B + 63) / 64), dim3(64), 0, st>>>(slots, kv_len, pos, B, done, cur_tok, prev_tok);
   return 0;
 }
 

@@ -10,7 +10,7 @@ import numpy as np
 import torch
 
 from . import _lib
-from .config import DebunexConfig, LiveCCConfig
+from .config import DECODER_CONFIGS, BemuzenConfig, LiveCCConfig, ParallelMixerSpec
 from .weights import WeightArena
 
 # HF image_processing_backends.py:307-311: mean*(1/rescale_factor), std*(1/rescale_factor) as fp32 tensors
@@ -93,7 +93,8 @@ class Engine:
         if self.device.index is None:
             self.device = torch.device("cuda", torch.cuda.current_device())
         torch.cuda.set_device(self.device)
-        self.is_decoder = isinstance(cfg, DebunexConfig)
+        self.is_decoder = isinstance(cfg, DECODER_CONFIGS)
+        self.has_recurrent_state = isinstance(cfg, BemuzenConfig)
         gran = 64 if self.is_decoder else 32
         max_kv_len = (max_kv_len + gran - 1) // gran * gran
         self.max_slots, self.max_kv_len, self.max_history = max_slots, max_kv_len, max_history
@@ -136,6 +137,12 @@ class Engine:
     def _create(self, cfg, lim):
         if self.is_decoder:
             layers = (_lib.DecoderLayer * cfg.num_hidden_layers)()
+            if isinstance(cfg, BemuzenConfig):
+                for i, l in enumerate(cfg.layers):
+                    layers[i] = self._sandwich_layer(l)
+                dc = _lib.DecoderConfigC(cfg.vocab_size, cfg.vocab_pad, cfg.width_pad, cfg.num_hidden_layers, cfg.norm_eps, 0.0, _lib.BLOCK_SANDWICH,
+                                         cfg.hidden_size, cfg.logit_scale, cfg.bigram_buckets, cfg.bigram_mul_prev, cfg.bigram_mul_cur)
+                return self.lib.lcc_engine_create_decoder(C.byref(dc), layers, C.byref(lim))
             for i, l in enumerate(cfg.layers):
                 m = l.mixer
                 layers[i] = _lib.DecoderLayer(_lib.MIXER_LATENT, m.heads, m.q_rank, m.kv_rank, m.dim_pad, m.vdim_pad, m.q_rank_pad, m.kv_rank_pad,
@@ -148,6 +155,18 @@ class Engine:
                               cfg.vit_embed_dim, cfg.vit_num_heads, cfg.vit_mlp_dim, cfg.patch_dim, cfg.spatial_merge_size,
                               1 if getattr(self.weights, "llm_fp8", False) else 0)
         return self.lib.lcc_engine_create(C.byref(mc), C.byref(lim))
+
+    @staticmethod
+    def _sandwich_layer(l) -> _lib.DecoderLayer:
+        m, r, d = l.mixer, l.mixer.recurrent, _lib.DecoderLayer()
+        d.mixer, d.kv_from, d.ff_pad = (_lib.MIXER_PARALLEL if isinstance(m, ParallelMixerSpec) else _lib.MIXER_SSD), -1, l.ff_pad
+        if isinstance(m, ParallelMixerSpec):
+            a = m.left
+            d.heads, d.kv_heads, d.dim, d.dim_pad, d.vdim_pad, d.scale = a.heads, a.kv_heads, a.dim, a.dim_pad, a.vdim_pad, a.scale
+            d.q_temp_coef, d.q_temp_every = a.q_temp_coef, a.q_temp_every
+        d.rec_heads, d.rec_groups, d.rec_key_pad, d.rec_vdim, d.rec_vdim_pad = r.heads, r.groups, r.key_pad, r.vdim, r.vdim_pad
+        d.rec_conv_taps, d.rec_norm_groups = r.conv_taps, r.norm_groups
+        return d
 
     def _bind_vit(self) -> None:
         lib, h = self.lib, self.h
@@ -188,7 +207,11 @@ class Engine:
         _lib.check(self.lib.lcc_slot_get_length(self.h, slot, C.byref(a), C.byref(b)), "lcc_slot_get_length")
         return a.value, b.value
 
-    def set_slot_length(self, slot: int, kv_len: int, next_pos: int) -> None:
+    def set_slot_length(self, slot: int, kv_len: int, next_pos: int, keep_state: bool = False) -> None:
+        """Roll a slot back (or forth) to `kv_len` cached tokens.  A recurrent state belongs to the slot's present length and cannot follow:
+        models that have one refuse another length unless `keep_state` (timing runs) accepts the mismatch."""
+        if self.has_recurrent_state and not keep_state and kv_len != self.slot_length(slot)[0]:
+            raise _lib.LccError(f"slot {slot}: the recurrent state of this model cannot be rolled back to {kv_len} tokens")
         _lib.check(self.lib.lcc_slot_set_length(self.h, slot, kv_len, next_pos, self._stream()), "lcc_slot_set_length")
 
     def _rope(self, grids) -> Tuple[torch.Tensor, torch.Tensor]:

@@ -36,7 +36,7 @@ import numpy as np
 import torch
 
 from . import protocol
-from .config import DebunexConfig, LiveCCConfig, architecture_of, get_config
+from .config import BemuzenConfig, DebunexConfig, LiveCCConfig, architecture_of, get_config
 from .engine import Engine, Sampling
 from .weights import WeightArena, from_hf_model as _arena_from_hf, from_pretrained as _arena_from_pretrained, make_arena
 
@@ -699,14 +699,15 @@ class LiveCCForConditionalGeneration(EngineModel):
             return self._vit_encode(clips)
 
 
-class DebunexForCausalLM(EngineModel):
-    """Debunex on the engine: `from_pretrained(path)`, `generate(input_ids, past_key_values=...)`, `generate_batch([...])` with the sampling
+class DecoderForCausalLM(EngineModel):
+    """A layer-list decoder on the engine: `from_pretrained(path)`, `generate(input_ids, past_key_values=...)`, `generate_batch([...])` with the sampling
     arguments of the other family (greedy, repetition penalty, temperature / top-k / top-p), `forward_step` for given ids.  Text ids only;
     raw logits are fp32.  bf16 weights and activations; no fp32 mode and no CPU path."""
     main_input_name = "input_ids"
     logits_dtype = torch.float32
+    config_class = None          # of the family
 
-    def __init__(self, cfg: DebunexConfig, weights: WeightArena, device, max_streams: int = 1, max_kv_len: Optional[int] = None,
+    def __init__(self, cfg, weights: WeightArena, device, max_streams: int = 1, max_kv_len: Optional[int] = None,
                  max_new_rows: int = 4096, max_history: int = 512, eos_token_ids: Optional[Sequence[int]] = None):
         ids = [] if cfg.eos_token_id is None else [int(cfg.eos_token_id)]
         ids += [int(t) for t in (eos_token_ids or []) if int(t) not in ids]
@@ -716,8 +717,8 @@ class DebunexForCausalLM(EngineModel):
     def from_pretrained(cls, model_path: str, torch_dtype="auto", device_map=None, **kw):
         device = _check_load_args(torch_dtype, device_map)
         cfg = get_config(model_path)
-        if not isinstance(cfg, DebunexConfig):
-            raise ValueError(f"{model_path} is not a Debunex checkpoint")
+        if not isinstance(cfg, cls.config_class):
+            raise ValueError(f"{model_path} is not a {cls.config_class.__name__.removesuffix('Config')} checkpoint")
         gen_cfg, eos_ids = read_generation_config(model_path)
         if eos_ids is not None and "eos_token_ids" not in kw:
             kw["eos_token_ids"] = eos_ids
@@ -726,7 +727,7 @@ class DebunexForCausalLM(EngineModel):
         return model
 
     @classmethod
-    def from_config(cls, cfg: DebunexConfig, device="cuda", seed: int = 0, **kw):
+    def from_config(cls, cfg, device="cuda", seed: int = 0, **kw):
         return cls(cfg, make_arena(cfg, device).fill_random(seed), device, **kw)
 
     def _scores_width(self) -> int:
@@ -747,8 +748,18 @@ class DebunexForCausalLM(EngineModel):
         return r if return_dict_in_generate else r.sequences
 
 
+class DebunexForCausalLM(DecoderForCausalLM):
+    """Latent attention without positions, parallel sublayers behind a Dynamic-Tanh norm."""
+    config_class = DebunexConfig
+
+
+class BemuzenForCausalLM(DecoderForCausalLM):
+    """Attention with a distance bias beside linear attention, state-space layers, norms on both sides of every sublayer, a bigram embedding."""
+    config_class = BemuzenConfig
+
+
 # config.json "architecture" -> model class (None: a Qwen2-VL checkpoint)
-MODEL_CLASSES = {None: LiveCCForConditionalGeneration, "Debunex": DebunexForCausalLM}
+MODEL_CLASSES = {None: LiveCCForConditionalGeneration, "Debunex": DebunexForCausalLM, "Bemuzen": BemuzenForCausalLM}
 
 
 def load_model(model_path: str, **kw) -> EngineModel:

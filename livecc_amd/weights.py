@@ -24,7 +24,7 @@ from typing import Callable, Dict, Iterable, List, Tuple
 
 import torch
 
-from .config import DebunexConfig, LiveCCConfig
+from .config import BemuzenConfig, DebunexConfig, LiveCCConfig, ParallelMixerSpec
 
 
 def qkv_decode_row_permutation(cfg: LiveCCConfig) -> torch.Tensor:
@@ -427,12 +427,173 @@ class DecoderArena(WeightArena):
         return self.load_state_dict(make)
 
 
+# ---- decoders with pre- and post-norms (Bemuzen) ----
+def as_words(t: torch.Tensor) -> torch.Tensor:
+    """fp32 values as pairs of the arena's 16-bit words (bytes, not numbers)."""
+    return t.to(torch.float32).contiguous().view(torch.bfloat16)
+
+
+def bemuzen_weight_shapes(cfg: BemuzenConfig) -> List[Tuple[str, Tuple[int, ...]]]:
+    """Stored (zero-padded) shapes.  Per layer: the four norms; in_w = the mixer's projections in one product; parallel: lo_w / ro_w = the two output
+    products, out norms; state-space: conv_w [taps, channels], conv_b; rec_* = fp32 tables per recurrent head; rec_norm over the real (unpadded)
+    channels of all heads; gate_up_w interleaved; down_w."""
+    W, V = cfg.width_pad, cfg.vocab_pad
+    out: List[Tuple[str, Tuple[int, ...]]] = [("embed", (cfg.vocab_size, W)), ("bigram", (cfg.bigram_buckets + 1, W))]
+    for i, l in enumerate(cfg.layers):
+        m, r, p = l.mixer, l.mixer.recurrent, f"dec.{i}."
+        rin = (r.heads * r.vdim + 63) // 64 * 64
+        out += [(p + "norm1", (W,)), (p + "norm1b", (W,)), (p + "in_w", (m.in_rows, W)), (p + "rec_norm", (rin,)), (p + "rec_rate", (2 * r.heads,)),
+                (p + "ro_w", (W, rin))]
+        if isinstance(m, ParallelMixerSpec):
+            a = m.left
+            out += [(p + "q_norm", (a.dim_pad,)), (p + "k_norm", (a.dim_pad,)), (p + "slope", (2 * a.heads,)), (p + "lo_w", (W, a.heads * a.vdim_pad)),
+                    (p + "l_out", (W,)), (p + "r_out", (W,))]
+        else:
+            out += [(p + "conv_w", (m.conv_taps, m.conv_channels)), (p + "conv_b", (m.conv_channels,)), (p + "rec_dt_bias", (2 * r.heads,)),
+                    (p + "rec_skip", (2 * r.heads,))]
+        if l.ff:
+            out += [(p + "norm2", (W,)), (p + "norm2b", (W,)), (p + "gate_up_w", (2 * l.ff_pad, W)), (p + "down_w", (W, l.ff_pad))]
+    return out + [("final_norm", (W,)), ("lm_head", (V, W))]
+
+
+def bemuzen_param_shapes(cfg: BemuzenConfig) -> Dict[str, Tuple[int, ...]]:
+    """Tensor names and shapes of a checkpoint."""
+    W = cfg.hidden_size
+    out: Dict[str, Tuple[int, ...]] = {"embed": (cfg.vocab_size, W), "bigram": (cfg.bigram_buckets + 1, W), "head": (cfg.vocab_size, W), "final.norm": (W,)}
+    for i, l in enumerate(cfg.layers):
+        m, p = l.mixer, f"l{i}."
+        out.update({p + "norm1": (W,), p + "norm1b": (W,)})
+        if l.ff:
+            out.update({p + "norm2": (W,), p + "norm2b": (W,), p + "mlp.gate": (l.ff, W), p + "mlp.up": (l.ff, W), p + "mlp.down": (W, l.ff)})
+        p += "mix."
+        if isinstance(m, ParallelMixerSpec):
+            a, r = m.left, m.right
+            out.update({p + "left.q": (a.heads * a.dim, W), p + "left.k": (a.kv_heads * a.dim, W), p + "left.v": (a.kv_heads * a.vdim, W),
+                        p + "left.q.norm": (a.dim,), p + "left.k.norm": (a.dim,), p + "left.o": (W, a.heads * a.vdim),
+                        p + "right.q": (r.heads * r.dim, W), p + "right.k": (r.heads * r.dim, W), p + "right.v": (r.heads * r.vdim, W),
+                        p + "right.g": (r.heads * r.vdim, W), p + "right.o": (W, r.heads * r.vdim), p + "right.norm": (r.heads * r.vdim,),
+                        p + "left.out": (W,), p + "right.out": (W,)})
+        else:
+            inner, bc = m.heads * m.vdim, m.groups * m.state
+            out.update({p + "in": (2 * inner + 2 * bc + m.heads, W), p + "conv": (inner + 2 * bc, m.conv_taps), p + "conv.b": (inner + 2 * bc,),
+                        p + "dt_bias": (m.heads,), p + "A_log": (m.heads,), p + "D": (m.heads,), p + "norm": (inner,), p + "o": (W, inner)})
+    return out
+
+
+class BemuzenArena(WeightArena):
+    """The weights of a decoder with pre- and post-norms in the engine's order; same flat arena, packing and views."""
+
+    def __init__(self, cfg: BemuzenConfig, device):
+        self.cfg, self.device, self.llm_fp8 = cfg, torch.device(device), False
+        self._allocate(bemuzen_weight_shapes(cfg), set())
+        self.row_major = {"embed", "bigram"} | {f"dec.{i}.conv_w" for i in range(cfg.num_hidden_layers)}
+
+    @torch.no_grad()
+    def load_state_dict(self, sd_get: Callable[[str], torch.Tensor]) -> "BemuzenArena":
+        cfg = self.cfg
+        W, D = cfg.width_pad, cfg.hidden_size
+        shapes = bemuzen_param_shapes(cfg)
+
+        def get(name: str) -> torch.Tensor:
+            t = sd_get(name)
+            if tuple(t.shape) != shapes[name]:
+                raise ValueError(f"{name}: checkpoint shape {tuple(t.shape)}, the configuration says {shapes[name]}")
+            return t
+
+        def vec(dst: str, src: str, n: int) -> None:
+            self.store(dst, _pad(get(src), (n,)))
+
+        def words(dst: str, t: torch.Tensor) -> None:
+            self.store(dst, as_words(t.to(self.device)))
+
+        def head_rows(t: torch.Tensor, heads: int, d: int, d_pad: int) -> torch.Tensor:
+            """[heads * d, D] -> [heads * d_pad, W]: every head's rows padded to d_pad."""
+            return _pad(t.reshape(heads, d, D), (heads, d_pad, W)).reshape(heads * d_pad, W)
+
+        self.store("embed", _pad(get("embed"), (cfg.vocab_size, W)))
+        self.store("bigram", _pad(get("bigram"), (cfg.bigram_buckets + 1, W)))
+        for i, l in enumerate(cfg.layers):
+            m, r, p, s = l.mixer, l.mixer.recurrent, f"dec.{i}.", f"l{i}."
+            for n in ("norm1", "norm1b") + (("norm2", "norm2b") if l.ff else ()):
+                vec(p + n, s + n, W)
+            inner = r.heads * r.vdim
+            rin = (inner + 63) // 64 * 64
+            if isinstance(m, ParallelMixerSpec):
+                a, c = m.left, s + "mix."
+                self.store(p + "in_w", torch.cat(
+                    [head_rows(get(c + "left.q"), a.heads, a.dim, a.dim_pad), head_rows(get(c + "left.k"), a.kv_heads, a.dim, a.dim_pad),
+                     head_rows(get(c + "left.v"), a.kv_heads, a.vdim, a.vdim_pad), head_rows(get(c + "right.q"), r.heads, r.dim, r.key_pad),
+                     head_rows(get(c + "right.k"), r.heads, r.dim, r.key_pad), head_rows(get(c + "right.v"), r.heads, r.vdim, r.vdim_pad),
+                     head_rows(get(c + "right.g"), r.heads, r.vdim, r.vdim_pad)]))
+                vec(p + "q_norm", c + "left.q.norm", a.dim_pad)
+                vec(p + "k_norm", c + "left.k.norm", a.dim_pad)
+                words(p + "slope", torch.tensor(a.slopes(), dtype=torch.float64) * 1.4426950408889634)
+                self.store(p + "lo_w", _pad(get(c + "left.o").reshape(D, a.heads, a.vdim), (W, a.heads, a.vdim_pad)).reshape(W, a.heads * a.vdim_pad))
+                vec(p + "l_out", c + "left.out", W)
+                vec(p + "r_out", c + "right.out", W)
+                vec(p + "rec_norm", c + "right.norm", rin)
+                self.store(p + "ro_w", _pad(get(c + "right.o"), (W, rin)))
+                words(p + "rec_rate", torch.log2(torch.tensor(r.decay, dtype=torch.float64).clamp_min(2.0 ** -1000)))      # a decay of 0: 2^-1000
+            else:
+                c, gn = s + "mix.", m.groups * m.state
+                z, x, B, Cc, dt = torch.split(get(c + "in"), [inner, inner, gn, gn, m.heads])
+                self.store(p + "in_w", torch.cat(
+                    [head_rows(z, m.heads, m.vdim, m.vdim_pad), head_rows(x, m.heads, m.vdim, m.vdim_pad), head_rows(B, m.groups, m.state, m.key_pad),
+                     head_rows(Cc, m.groups, m.state, m.key_pad), _pad(dt, ((m.heads + 63) // 64 * 64, W))]))
+
+                def channels(t: torch.Tensor) -> torch.Tensor:
+                    """[x | B | C channels, n] -> [n, stored channels]."""
+                    n = t.shape[1]
+                    parts = torch.split(t, [inner, gn, gn])
+                    pads = [(m.heads, m.vdim, m.vdim_pad), (m.groups, m.state, m.key_pad), (m.groups, m.state, m.key_pad)]
+                    return torch.cat([_pad(q.reshape(h, d, n), (h, dp, n)).reshape(h * dp, n) for q, (h, d, dp) in zip(parts, pads)]).T.contiguous()
+                self.store(p + "conv_w", channels(get(c + "conv")))
+                self.store(p + "conv_b", channels(get(c + "conv.b").reshape(-1, 1)).reshape(-1))
+                words(p + "rec_dt_bias", get(c + "dt_bias"))
+                words(p + "rec_skip", get(c + "D"))
+                words(p + "rec_rate", -torch.exp(get(c + "A_log").double()) * 1.4426950408889634)
+                vec(p + "rec_norm", c + "norm", rin)
+                self.store(p + "ro_w", _pad(get(c + "o"), (W, rin)))
+            if l.ff:
+                self.store(p + "gate_up_w", interleave_gate_up(_pad(get(s + "mlp.gate"), (l.ff_pad, W)), _pad(get(s + "mlp.up"), (l.ff_pad, W))))
+                self.store(p + "down_w", _pad(get(s + "mlp.down"), (W, l.ff_pad)))
+        vec("final_norm", "final.norm", W)
+        self.store("lm_head", _pad(get("head"), (cfg.vocab_pad, W)))
+        return self
+
+    @torch.no_grad()
+    def fill_random(self, seed: int = 0, std: float = 0.02) -> "BemuzenArena":
+        """Random weights of the checkpoint's shapes, generated on the arena's device: N(0, std) matrices, plain norm weights around 1, the ones
+        stored around zero around 0, step sizes and rates of trained state-space layers."""
+        shapes = bemuzen_param_shapes(self.cfg)
+        g = torch.Generator(device=self.device).manual_seed(seed)
+
+        def make(name: str) -> torch.Tensor:
+            x = torch.randn(shapes[name], generator=g, device=self.device, dtype=torch.float32)
+            if name.endswith(".conv"):
+                return x.mul_(0.3).to(torch.bfloat16)
+            if x.dim() >= 2:
+                return x.mul_(std).to(torch.bfloat16)
+            if name.endswith(("norm1", "norm1b", "norm2", "norm2b", "final.norm", ".b")):
+                return x.mul_(0.1).to(torch.bfloat16)
+            if name.endswith("A_log"):
+                return x.mul_(0.5).add_(1.0).to(torch.bfloat16)
+            if name.endswith("dt_bias"):
+                return x.sub_(3.0).to(torch.bfloat16)
+            return x.mul_(0.1).add_(1.0).to(torch.bfloat16)
+        return self.load_state_dict(make)
+
+
 def make_arena(cfg, device, llm_fp8: bool = False) -> WeightArena:
     """The weight arena of a configuration's model family."""
     if isinstance(cfg, DebunexConfig):
         if llm_fp8:
             raise ValueError("fp8 weights are available for the Qwen2-VL family only")
         return DecoderArena(cfg, device)
+    if isinstance(cfg, BemuzenConfig):
+        if llm_fp8:
+            raise ValueError("fp8 weights are available for the Qwen2-VL family only")
+        return BemuzenArena(cfg, device)
     return WeightArena(cfg, device, llm_fp8=llm_fp8)
 
 
