@@ -56,8 +56,9 @@ def parse(argv=None):
                          "KV growing to ~32k; oneshot480 = the OTHER half of configs[3]: the reference's video_qa / MCQ first turn "
                          "(ref demo/infer.py:182-242): all 480 frames in ONE generate call (ViT over 96,000 patches in 240 segments, "
                          "one 24k-row LLM prefill served in pieces, then 32 decode tokens at L ~ 24k); both override "
-                         "--frames/--height/--width/--max-new-tokens; decoder = prefill / decode throughput of the Debunex decoder beside the "
+                         "--frames/--height/--width/--max-new-tokens; decoder = prefill / decode throughput of a layer-list decoder beside the "
                          "Qwen2-VL language model at equal size (tools/bench_decoder.py)")
+    ap.add_argument("--decoder-model", choices=["debunex", "bemuzen"], default="debunex", help="decoder: the family")
     ap.add_argument("--decoder-size", choices=["2b", "7b"], default=None, help="decoder: one size only")
     ap.add_argument("--decoder-layers", type=int, default=28, help="decoder: layers of both models")
     ap.add_argument("--decoder-prefill", default="512,2048,8192", help="decoder: prompt lengths")

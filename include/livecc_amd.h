@@ -335,6 +335,62 @@ int lcc_latent_attn_decode(const void* q_latent, const int32_t* slots, const int
                            int kv_rank_pad, float scale, int nsplit, float* ws_o, float* ws_ml, const void* uv, int vdim, const float* gate, void* out,
                            int ldo, void* stream);
 
+/* ---- layer-list decoders with a norm before and after every sublayer: RMS norms with weights stored around zero (x / rms(x) * (1 + w), `width` real
+ * channels of `dim` stored ones), grouped-query attention with a distance bias, recurrent mixers.  Weights bf16, tables and states fp32. */
+/* x = embedding row + bigram row, h = norm(x).  Row of the bigram table: (previous id * mul_prev + id * mul_cur) mod buckets; `buckets` for a sequence's first
+ * token.  tok_pos given: ids per row, the previous id is ids[row - 1] or -- tok_row0[row] == row -- prev_tok[slot]; tok_pos NULL: ids[slot], kv_len[slot] */
+int lcc_embed_bigram_rms(const int32_t* ids, const int32_t* tok_stream, const int32_t* tok_pos, const int32_t* tok_row0, const int32_t* kv_len,
+                         const int32_t* prev_tok, const void* table, const void* bigram, int buckets, long long mul_prev, long long mul_cur, const void* norm_w,
+                         float eps, float* x, void* h, int rows, int width, int dim, void* stream);
+/* y = sum of the slabs, or -- partial_b -- the mean of two sums, each normed with its plain weight; x += norm(y; post_w); h = bf16(norm(x; next_w)) */
+int lcc_post_norm_resid(const float* partial, int nsplit, const float* partial_b, int nsplit_b, const void* w_a, const void* w_b, const void* post_w,
+                        const void* next_w, float* x, void* h, int rows, int width, int dim, float eps, void* stream);
+/* queries, keys and values of grouped-query attention out of a fused projection (fp32 slabs [nsplit][rows][ldn], columns q heads | k heads | v heads): RMS norms
+ * per head, queries times 1 + temp_coef ln(floor((p + 1) / temp_every) + 1), keys and values appended to the slot: K [kv_heads][lmax][dim_pad] at k_off,
+ * V [kv_heads][lmax / 32][vdim_pad][32] at v_off (bf16 elements from the arena's start).  tok_pos NULL: position kv_len[slot] */
+typedef struct {
+  const float* partial; int nsplit, rows, ldn;
+  int heads, kv_heads, dim, dim_pad, vdim_pad; float eps;
+  const void* q_norm; const void* k_norm; float temp_coef; int temp_every;
+  void* q;
+  const int32_t* tok_stream; const int32_t* tok_pos; const int32_t* kv_len; void* const* kv_base; int64_t k_off, v_off; int lmax;
+} lcc_gqa_input;
+/* S_t = 2^(rate dt_t) S_{t-1} + dt_t k_t v_t^T, o_t = S_t^T q_t + skip v_t per head; q, k, v = silu of the projection's columns or (taps > 0) of the causal
+ * convolution over the columns conv_col .. + conv_ch (weights [taps][conv_ch], last row: the current token); dt = softplus(column + dt_bias), 1 without dt_col.
+ * State fp32 [heads][key_pad][vdim_pad] at state_off, convolution inputs fp32 [taps][conv_ch] at conv_off (position p at row p mod taps).
+ * Prefill (tok_pos, tok_row0, tok_last: position, first and last row of the row's stream): q, k, v [rows][..] bf16 and dt [rows][heads] are outputs. */
+typedef struct {
+  const float* partial; int nsplit, rows, ldn;
+  int q_col, k_col, v_col, dt_col, heads, groups, key_pad, vdim_pad;
+  int taps, conv_col, conv_ch; const void* conv_w; const void* conv_b;
+  const float* rate; const float* dt_bias; const float* skip;
+  const int32_t* tok_stream; const int32_t* tok_pos; const int32_t* tok_row0; const int32_t* tok_last; const int32_t* kv_len; const int32_t* done;
+  void* const* kv_base; int64_t state_off, conv_off;
+  void* q; void* k; void* v; float* dt;
+} lcc_rec_input;
+int lcc_mixer_prep(const lcc_gqa_input* attn, const lcc_rec_input* rec, void* stream);                   /* prefill; either may be NULL */
+int lcc_rec_decode(const lcc_rec_input* rec, const lcc_gqa_input* attn, float* y, void* stream);         /* one token per row; y [rows][heads][vdim_pad] */
+/* prefill recurrence over segments of consecutive rows of one stream (first row, rows, slot, 1 = starts at zero), grouped by stream (first segment, segments);
+ * more segments than streams: scratch seg_state [n_seg][heads][key_pad][vdim_pad], seg_decay [n_seg][heads].  dt NULL: 1, skip NULL: 0 */
+int lcc_rec_scan(const void* q, const void* k, const void* v, const float* dt, const float* rate, const float* skip, float* y, int heads, int groups, int key_pad,
+                 int vdim_pad, const int32_t* seg_row0, const int32_t* seg_rows, const int32_t* seg_slot, const int32_t* seg_fresh, int n_seg,
+                 const int32_t* str_seg0, const int32_t* str_nseg, int n_streams, float* seg_state, float* seg_decay, void* const* kv_base, int64_t state_off,
+                 void* stream);
+/* gated norm over norm_groups equal parts of the concatenated heads (vdim real of vdim_pad channels each): gate_first: rms(y silu(gate)) w, else
+ * rms(y) w sigmoid(gate); gate = columns gate_col .. of the slabs.  out [rows][ld] bf16, heads without padding, zero behind them.
+ * conv (optional, prefill): its streams' last convolution inputs go to their slots */
+int lcc_rec_norm(const float* y, const float* partial, int nsplit, int rows, int ldn, int gate_col, int gate_first, int heads, int vdim, int vdim_pad,
+                 int norm_groups, float eps, const void* w, void* out, int ld, const lcc_rec_input* conv, void* stream);
+/* causal attention over the slots' K / V (layout above) with slope[head] (i - j) taken off the scores (slope in units of log2; NULL: none).
+ * prefill: groups of <= 256 rows of one stream as lcc_attn_mha, with the slot of each group; decode: one token per row, nsplit <= 64 key splits
+ * (scratch ws_o [rows*heads*nsplit*vdim], ws_ml [rows*heads*nsplit*2]); dim, vdim padded to multiples of 64, at most 256 */
+int lcc_gqa_attn_prefill(const void* q, void* out, const int32_t* grp_q0, const int32_t* grp_nq, const int32_t* grp_pos0, const int32_t* grp_slot, int n_groups,
+                         int rows, int heads, int kv_heads, int dim, int vdim, float scale, const float* slope, void* const* kv_base, int64_t k_off, int64_t v_off,
+                         int lmax, void* stream);
+int lcc_gqa_attn_decode(const void* q, const int32_t* slots, const int32_t* kv_len, int rows, int heads, int kv_heads, int dim, int vdim, float scale,
+                        const float* slope, void* const* kv_base, int64_t k_off, int64_t v_off, int lmax, int nsplit, float* ws_o, float* ws_ml, void* out,
+                        void* stream);
+
 /* ------------------------------------------------------------------------------------------------
  * Model level -- what `model.generate(**inputs, past_key_values=...)` (ref:demo/infer.py:165-172) executes:
  * ViT (Q2VL:700-729) -> embed+scatter -> 28x decoder layer -> lm_head -> processors -> sample, with the

@@ -62,6 +62,21 @@ class DecoderConfigC(C.Structure):
                 ("bigram_mul_cur", C.c_longlong)]
 
 
+class GqaInput(C.Structure):
+    _fields_ = [("partial", C.c_void_p)] + [(n, C.c_int) for n in ("nsplit", "rows", "ldn", "heads", "kv_heads", "dim", "dim_pad", "vdim_pad")] + \
+               [("eps", C.c_float), ("q_norm", C.c_void_p), ("k_norm", C.c_void_p), ("temp_coef", C.c_float), ("temp_every", C.c_int)] + \
+               [(n, C.c_void_p) for n in ("q", "tok_stream", "tok_pos", "kv_len", "kv_base")] + \
+               [("k_off", C.c_int64), ("v_off", C.c_int64), ("lmax", C.c_int)]
+
+
+class RecInput(C.Structure):
+    _fields_ = [("partial", C.c_void_p)] + [(n, C.c_int) for n in ("nsplit", "rows", "ldn", "q_col", "k_col", "v_col", "dt_col", "heads", "groups", "key_pad",
+                                                                  "vdim_pad", "taps", "conv_col", "conv_ch")] + \
+               [(n, C.c_void_p) for n in ("conv_w", "conv_b", "rate", "dt_bias", "skip", "tok_stream", "tok_pos", "tok_row0", "tok_last", "kv_len", "done",
+                                          "kv_base")] + \
+               [("state_off", C.c_int64), ("conv_off", C.c_int64)] + [(n, C.c_void_p) for n in ("q", "k", "v", "dt")]
+
+
 MIXER_LATENT, MIXER_PARALLEL, MIXER_SSD = 1, 2, 3            # LCC_MIXER_*
 BLOCK_PARALLEL, BLOCK_SANDWICH = 0, 1                        # LCC_BLOCK_*
 
@@ -159,6 +174,14 @@ def load():
         "lcc_attn_mha": (i32, [vp, vp, vp, i32, vp, vp, i32, vp, vp, vp, vp, i32, i32, i32, i32, i32, f32, vp]),
         "lcc_latent_absorb": (i32, [vp, i32, i32, i32, i32, vp, i32, vp, vp]),
         "lcc_latent_attn_decode": (i32, [vp, vp, vp, vp, i64, i32, i32, i32, f32, i32, vp, vp, vp, i32, vp, vp, i32, vp]),
+        "lcc_embed_bigram_rms": (i32, [vp, vp, vp, vp, vp, vp, vp, vp, i32, i64, i64, vp, f32, vp, vp, i32, i32, i32, vp]),
+        "lcc_post_norm_resid": (i32, [vp, i32, vp, i32, vp, vp, vp, vp, vp, vp, i32, i32, i32, f32, vp]),
+        "lcc_mixer_prep": (i32, [C.POINTER(GqaInput), C.POINTER(RecInput), vp]),
+        "lcc_rec_decode": (i32, [C.POINTER(RecInput), C.POINTER(GqaInput), vp, vp]),
+        "lcc_rec_scan": (i32, [vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, vp, vp, vp, vp, i32, vp, vp, i32, vp, vp, vp, i64, vp]),
+        "lcc_rec_norm": (i32, [vp, vp, i32, i32, i32, i32, i32, i32, i32, i32, i32, f32, vp, vp, i32, C.POINTER(RecInput), vp]),
+        "lcc_gqa_attn_prefill": (i32, [vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, f32, vp, vp, i64, i64, i32, vp]),
+        "lcc_gqa_attn_decode": (i32, [vp, vp, vp, i32, i32, i32, i32, i32, f32, vp, vp, i64, i64, i32, i32, vp, vp, vp, vp]),
         "lcc_engine_create_decoder": (vp, [C.POINTER(DecoderConfigC), C.POINTER(DecoderLayer), C.POINTER(EngineLimits)]),
         "lcc_debug_set_decoder_fused": (i32, [i32]),
         "lcc_slot_set_tokens": (i32, [vp, i32, vp, vp, vp]),

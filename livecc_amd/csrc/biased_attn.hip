@@ -143,6 +143,13 @@ __global__ __launch_bounds__(256) void gqa_merge_rec_norm_kernel(GqaDecodeArgs a
   }
   if (on) st8(a.out + (size_t)item * a.vdim + lane * 4, pack4(o));
 }
+int gqa_merge(const GqaDecodeArgs& m, hipStream_t st) {
+  if (m.rows <= 0) return 0;
+  if (!gqa_ok(m) || m.vdim > 256 || (m.vdim & 63)) return LCC_ERR_SHAPE;
+  if (!m.out) return LCC_ERR_ARG;
+  gqa_merge_rec_norm_kernel<<<dim3((m.rows * m.heads + 3) / 4), dim3(256), 0, st>>>(m, RecNormArgs(), 0);
+  return 0;
+}
 bool rec_norm_ok(const RecNormArgs& a);
 int gqa_merge_rec_norm(const GqaDecodeArgs& m, const RecNormArgs& a, hipStream_t st) {
   if (m.rows <= 0) return 0;

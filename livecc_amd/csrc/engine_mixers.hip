@@ -88,14 +88,20 @@ size_t mixers_meta_ints(const lcc_engine* e) {
 }
 // rows per segment of the recurrence: whole streams while they are short (one launch instead of three), else enough segments to fill the chip
 int mixers_segment_rows(const lcc_engine* e, const DecBuffers& b, const int32_t* n_new, int n_streams) {
-  static const int forced = [] { const char* v = getenv("LCC_REC_SEG_CHUNKS"); return v ? std::max(SEG_CHUNKS, atoi(v)) : 0; }();
   int longest = 0;
-  long chunks = 0;
-  for (int i = 0; i < n_streams; ++i) { longest = std::max(longest, n_new[i]); chunks += (n_new[i] + REC_CHUNK - 1) / REC_CHUNK; }
+  for (int i = 0; i < n_streams; ++i) longest = std::max(longest, n_new[i]);
   if (longest <= 2 * SEG_CHUNKS * REC_CHUNK || b.seg_cap == 0) return std::max(longest, 1);
-  long blocks = 1;                     // (head, 64 value channels) pairs of a layer
+  // time of a segment length = rounds of blocks on the chip (two resident per compute unit) x chunks per block, plus about one chunk per block to
+  // start and to pass a state on; the layer with the most (head, 64 value channels) pairs decides
+  long blocks = 1;
   for (const lcc_decoder_layer& L : e->dl) blocks = std::max(blocks, (long)L.rec_heads * (L.rec_vdim_pad / 64));
-  const long per = forced > 0 ? forced : std::max<long>(SEG_CHUNKS, chunks * blocks / (4 * e->cu_count));
+  long per = SEG_CHUNKS, best = -1;
+  for (long c = SEG_CHUNKS; c <= 64; ++c) {
+    long segs = 0;
+    for (int i = 0; i < n_streams; ++i) segs += (n_new[i] + c * REC_CHUNK - 1) / (c * REC_CHUNK);
+    const long cost = ((segs * blocks + 2 * e->cu_count - 1) / (2 * e->cu_count)) * (c + 1);
+    if (best < 0 || cost < best) { best = cost; per = c; }
+  }
   return (int)std::min<long>(per * REC_CHUNK, std::max(longest, 1));
 }
 

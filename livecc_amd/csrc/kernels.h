@@ -310,7 +310,8 @@ struct GqaDecodeArgs {
   bf16_t* out = nullptr;                                             // [rows][heads vdim]
   AttnDirect direct;
 };
-int gqa_decode(const GqaDecodeArgs& a, hipStream_t st);              // the splits; the merge runs with rec_norm (gqa_merge_rec_norm)
+int gqa_decode(const GqaDecodeArgs& a, hipStream_t st);              // the splits
+int gqa_merge(const GqaDecodeArgs& a, hipStream_t st);               // their merge (beside a recurrent mixer: gqa_merge_rec_norm)
 
 // ---- recurrent mixers: S_t = 2^(rate dt_t) S_{t-1} + dt_t k_t v_t^T, o_t = S_t^T q_t (+ skip v_t) per head (recurrent.hip) ----
 struct RecInArgs {               // where the inputs lie in the fused input projection (fp32 slabs [nsplit][rows][ldn]), and the state

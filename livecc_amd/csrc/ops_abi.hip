@@ -403,6 +403,87 @@ extern "C" int lcc_latent_gather(void* const* kv_base, int64_t kv_offset, int kv
   OP_RET(latent_gather((bf16_t* const*)kv_base, (size_t)kv_offset, kv_rank_pad, tile_slot, tile_key0, tile_nkeys, n_tiles, (bf16_t*)rows_out,
                        (bf16_t*)packed_out, (hipStream_t)stream), "lcc_latent_gather");
 }
+extern "C" int lcc_embed_bigram_rms(const int32_t* ids, const int32_t* tok_stream, const int32_t* tok_pos, const int32_t* tok_row0, const int32_t* kv_len,
+                                    const int32_t* prev_tok, const void* table, const void* bigram, int buckets, long long mul_prev, long long mul_cur,
+                                    const void* norm_w, float eps, float* x, void* h, int rows, int width, int dim, void* stream) {
+  BigramEmbed bg; bg.table = (const bf16_t*)bigram; bg.buckets = buckets; bg.mul_prev = mul_prev; bg.mul_cur = mul_cur;
+  OP_RET(embed_bigram_rms(ids, tok_stream, tok_pos, tok_row0, kv_len, prev_tok, (const bf16_t*)table, bg, (const bf16_t*)norm_w, eps, x, (bf16_t*)h, rows, width, dim,
+                          (hipStream_t)stream), "lcc_embed_bigram_rms");
+}
+extern "C" int lcc_post_norm_resid(const float* partial, int nsplit, const float* partial_b, int nsplit_b, const void* w_a, const void* w_b, const void* post_w,
+                                   const void* next_w, float* x, void* h, int rows, int width, int dim, float eps, void* stream) {
+  PostNormArgs a; a.part = partial; a.nsplit = nsplit; a.part_b = partial_b; a.nsplit_b = nsplit_b; a.w_a = (const bf16_t*)w_a; a.w_b = (const bf16_t*)w_b;
+  a.post_w = (const bf16_t*)post_w; a.next_w = (const bf16_t*)next_w; a.x = x; a.h = (bf16_t*)h; a.rows = rows; a.width = width; a.dim = dim; a.eps = eps;
+  OP_RET(post_norm_resid(a, (hipStream_t)stream), "lcc_post_norm_resid");
+}
+static GqaInArgs gqa_in_of(const lcc_gqa_input& i) {
+  GqaInArgs a; a.part = i.partial; a.nsplit = i.nsplit; a.rows = i.rows; a.ldn = i.ldn; a.heads = i.heads; a.kv_heads = i.kv_heads; a.dim = i.dim;
+  a.dim_pad = i.dim_pad; a.vdim_pad = i.vdim_pad; a.eps = i.eps; a.q_norm = (const bf16_t*)i.q_norm; a.k_norm = (const bf16_t*)i.k_norm;
+  a.temp_coef = i.temp_coef; a.temp_every = i.temp_every; a.q = (bf16_t*)i.q; a.tok_stream = i.tok_stream; a.tok_pos = i.tok_pos; a.kv_len = i.kv_len;
+  a.kv_base = (bf16_t* const*)i.kv_base; a.k_off = (size_t)i.k_off; a.v_off = (size_t)i.v_off; a.lmax = i.lmax;
+  return a;
+}
+static RecInArgs rec_in_of(const lcc_rec_input& i) {
+  RecInArgs a; a.part = i.partial; a.nsplit = i.nsplit; a.rows = i.rows; a.ldn = i.ldn; a.q_col = i.q_col; a.k_col = i.k_col; a.v_col = i.v_col; a.dt_col = i.dt_col;
+  a.heads = i.heads; a.groups = i.groups; a.np = i.key_pad; a.ep = i.vdim_pad; a.taps = i.taps; a.conv_col = i.conv_col; a.conv_ch = i.conv_ch;
+  a.conv_w = (const bf16_t*)i.conv_w; a.conv_b = (const bf16_t*)i.conv_b; a.rate = i.rate; a.dt_bias = i.dt_bias; a.skip = i.skip; a.tok_stream = i.tok_stream;
+  a.tok_pos = i.tok_pos; a.tok_row0 = i.tok_row0; a.tok_last = i.tok_last; a.kv_len = i.kv_len; a.done = i.done; a.kv_base = (bf16_t* const*)i.kv_base;
+  a.state_off = (size_t)i.state_off; a.conv_off = (size_t)i.conv_off; a.q = (bf16_t*)i.q; a.k = (bf16_t*)i.k; a.v = (bf16_t*)i.v; a.dt = i.dt;
+  return a;
+}
+extern "C" int lcc_mixer_prep(const lcc_gqa_input* attn, const lcc_rec_input* rec, void* stream) {
+  GqaInArgs l; RecInArgs r;
+  if (attn) l = gqa_in_of(*attn);
+  if (rec) r = rec_in_of(*rec);
+  OP_RET(mixer_prep(attn ? &l : nullptr, rec ? &r : nullptr, (hipStream_t)stream), "lcc_mixer_prep");
+}
+extern "C" int lcc_rec_decode(const lcc_rec_input* rec, const lcc_gqa_input* attn, float* y, void* stream) {
+  if (!rec) return fail(LCC_ERR_ARG, "lcc_rec_decode: null pointer");
+  GqaInArgs l;
+  if (attn) l = gqa_in_of(*attn);
+  OP_RET(rec_decode(rec_in_of(*rec), attn ? &l : nullptr, y, (hipStream_t)stream), "lcc_rec_decode");
+}
+extern "C" int lcc_rec_scan(const void* q, const void* k, const void* v, const float* dt, const float* rate, const float* skip, float* y, int heads, int groups,
+                            int key_pad, int vdim_pad, const int32_t* seg_row0, const int32_t* seg_rows, const int32_t* seg_slot, const int32_t* seg_fresh, int n_seg,
+                            const int32_t* str_seg0, const int32_t* str_nseg, int n_streams, float* seg_state, float* seg_decay, void* const* kv_base,
+                            int64_t state_off, void* stream) {
+  RecScanArgs a; a.q = (const bf16_t*)q; a.k = (const bf16_t*)k; a.v = (const bf16_t*)v; a.dt = dt; a.rate = rate; a.skip = skip; a.y = y; a.heads = heads;
+  a.groups = groups; a.np = key_pad; a.ep = vdim_pad; a.seg_row0 = seg_row0; a.seg_rows = seg_rows; a.seg_slot = seg_slot; a.seg_fresh = seg_fresh; a.n_seg = n_seg;
+  a.str_seg0 = str_seg0; a.str_nseg = str_nseg; a.n_streams = n_streams; a.seg_state = seg_state; a.seg_decay = seg_decay; a.kv_base = (bf16_t* const*)kv_base;
+  a.state_off = (size_t)state_off;
+  OP_RET(rec_scan(a, (hipStream_t)stream), "lcc_rec_scan");
+}
+static RecNormArgs rec_norm_of(const float* y, const float* partial, int nsplit, int rows, int ldn, int gate_col, int gate_first, int heads, int vdim, int vdim_pad,
+                               int norm_groups, float eps, const void* w, void* out, int ld) {
+  RecNormArgs a; a.y = y; a.part = partial; a.nsplit = nsplit; a.rows = rows; a.ldn = ldn; a.gate_col = gate_col; a.gate_first = gate_first; a.heads = heads;
+  a.vdim = vdim; a.ep = vdim_pad; a.norm_groups = norm_groups; a.eps = eps; a.w = (const bf16_t*)w; a.out = (bf16_t*)out; a.ld = ld;
+  return a;
+}
+extern "C" int lcc_rec_norm(const float* y, const float* partial, int nsplit, int rows, int ldn, int gate_col, int gate_first, int heads, int vdim, int vdim_pad,
+                            int norm_groups, float eps, const void* w, void* out, int ld, const lcc_rec_input* conv, void* stream) {
+  RecNormArgs a = rec_norm_of(y, partial, nsplit, rows, ldn, gate_col, gate_first, heads, vdim, vdim_pad, norm_groups, eps, w, out, ld);
+  RecInArgs r;
+  if (conv) { r = rec_in_of(*conv); a.conv = &r; }
+  OP_RET(rec_norm(a, (hipStream_t)stream), "lcc_rec_norm");
+}
+extern "C" int lcc_gqa_attn_prefill(const void* q, void* out, const int32_t* grp_q0, const int32_t* grp_nq, const int32_t* grp_pos0, const int32_t* grp_slot,
+                                    int n_groups, int rows, int heads, int kv_heads, int dim, int vdim, float scale, const float* slope, void* const* kv_base,
+                                    int64_t k_off, int64_t v_off, int lmax, void* stream) {
+  if (!grp_slot) return fail(LCC_ERR_ARG, "lcc_gqa_attn_prefill: null pointer");
+  MhaArgs a; a.q = (const bf16_t*)q; a.out = (bf16_t*)out; a.ldo = heads * vdim; a.grp_q0 = grp_q0; a.grp_nq = grp_nq; a.grp_pos0 = grp_pos0; a.grp_slot = grp_slot;
+  a.n_groups = n_groups; a.rows = rows; a.heads = heads; a.kv_heads = kv_heads; a.dim = dim; a.vdim = vdim; a.scale_log2e = scale * 1.4426950408889634f;
+  a.slope = slope; a.kv_base = (bf16_t* const*)kv_base; a.k_off = (size_t)k_off; a.v_off = (size_t)v_off; a.lmax = lmax;
+  OP_RET(attn_mha(a, (hipStream_t)stream), "lcc_gqa_attn_prefill");
+}
+extern "C" int lcc_gqa_attn_decode(const void* q, const int32_t* slots, const int32_t* kv_len, int rows, int heads, int kv_heads, int dim, int vdim, float scale,
+                                   const float* slope, void* const* kv_base, int64_t k_off, int64_t v_off, int lmax, int nsplit, float* ws_o, float* ws_ml,
+                                   void* out, void* stream) {
+  GqaDecodeArgs a; a.q = (const bf16_t*)q; a.slots = slots; a.kv_len = kv_len; a.rows = rows; a.heads = heads; a.kv_heads = kv_heads; a.dim = dim; a.vdim = vdim;
+  a.scale_log2e = scale * 1.4426950408889634f; a.slope = slope; a.kv_base = (bf16_t* const*)kv_base; a.k_off = (size_t)k_off; a.v_off = (size_t)v_off; a.lmax = lmax;
+  a.nsplit = nsplit; a.ws_o = ws_o; a.ws_ml = ws_ml; a.out = (bf16_t*)out;
+  if (int r = gqa_decode(a, (hipStream_t)stream)) return fail(r, "lcc_gqa_attn_decode: invalid arguments (%d)", r);
+  OP_RET(gqa_merge(a, (hipStream_t)stream), "lcc_gqa_attn_decode");
+}
 extern "C" int lcc_attn_mha(const void* q, const void* k, const void* vt, int ldv, const float* gate, void* out, int ldo, const int32_t* grp_q0,
                             const int32_t* grp_nq, const int32_t* grp_pos0, const int32_t* grp_key0, int n_groups, int rows, int heads, int dim, int vdim,
                             float scale, void* stream) {

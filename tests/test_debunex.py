@@ -282,8 +282,8 @@ def test_oracle_shared_latents_are_the_owners():
 def test_decoder_bench_counts_both_models_alike():
     sys.path.insert(0, os.path.join(ROOT, "tools"))
     import bench_decoder as B
-    for size, (dec, gqa) in B.SIZES.items():
-        a, b = CFG.get_config(dec), CFG.get_config(gqa)
+    for size, gqa in B.LIKE.items():
+        a, b = CFG.get_config(f"debunex-{size}"), CFG.get_config(gqa)
         assert (a.hidden_size, a.vocab_size, a.num_hidden_layers, a.layers[0].ff, a.layers[0].mixer.heads) == \
                (b.hidden_size, b.vocab_size, b.num_hidden_layers, b.intermediate_size, b.num_attention_heads)
         assert 0.8 < B.flops_of(a, 2048) / B.flops_of(b, 2048) < 1.25

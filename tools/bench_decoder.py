@@ -1,8 +1,9 @@
 """Prefill and decode throughput of a layer-list decoder beside the Qwen2-VL language model at equal size (random weights, token ids only):
-`python bench.py --workload decoder [--decoder-size 7b] [--decoder-layers 28]`.  One JSON line per model and size.
+`python bench.py --workload decoder [--decoder-model bemuzen] [--decoder-size 7b] [--decoder-layers 28]`.  One JSON line per model and size.
 
-Same width, feed-forward, query heads, head size, depth and vocabulary; the decoder has latent attention (query rank 0.43 width, latent rank
-512, one latent per two layers), the other model grouped-query attention.  `layer_flops` / `step_bytes` are what the model's own
+Same width, feed-forward, query heads, head size, depth and vocabulary; the other model has grouped-query attention.  debunex: latent attention
+(query rank 0.43 width, latent rank 512, one latent per two layers).  bemuzen: grouped-query attention with a distance bias beside linear
+attention of the same heads, every fourth layer a state-space layer instead.  `decoder_layer_flops` / `step_bytes` are what the model's own
 equations need, so tokens/s of both are also given as a fraction of the dense bf16 peak (prefill) and of the HBM rate (decode)."""
 import dataclasses
 import json
@@ -12,7 +13,8 @@ import numpy as np
 import torch
 
 PEAK_FLOPS, PEAK_BYTES = 2.5e15, 8.0e12
-SIZES = {"2b": ("debunex-2b", "qwen2vl-2b"), "7b": ("debunex-7b", "livecc-7b")}
+LIKE = {"2b": "qwen2vl-2b", "7b": "livecc-7b"}
+CHUNK = 64          # tokens the linear-attention products of a prefill are formed over (scores inside a chunk, states between chunks)
 
 
 def cut(cfg, layers: int):
@@ -28,6 +30,18 @@ def decoder_layer_flops(l, width: int, S: int, past: int) -> float:
     """Multiply-adds x 2 of one layer over S new rows behind `past` cached ones (prefill form, real sizes)."""
     m = l.mixer
     keys = past + (S + 1) / 2
+    if hasattr(m, "recurrent"):
+        r = m.recurrent
+        k = r.state if hasattr(r, "state") else r.dim
+        # chunked recurrence per head: half a chunk of scores and values, the state read and updated
+        n = S * r.heads * ((k + r.vdim) * CHUNK / 2 + 2 * k * r.vdim) + S * width * (r.heads * r.vdim + 3 * l.ff)
+        if hasattr(m, "left"):
+            a = m.left
+            n += S * width * (a.heads * a.dim + a.kv_heads * (a.dim + a.vdim) + a.heads * a.vdim + 2 * r.heads * (r.dim + r.vdim))
+            n += S * keys * a.heads * (a.dim + a.vdim)
+        else:
+            n += S * (width * (2 * r.heads * r.vdim + 2 * r.groups * r.state + r.heads) + r.conv_taps * (r.heads * r.vdim + 2 * r.groups * r.state))
+        return 2.0 * n
     lin = width * (m.q_rank + m.heads + (m.kv_rank if m.kv_from is None else 0)) + m.q_rank * m.heads * m.dim + width * (m.heads * m.vdim + 3 * l.ff)
     lin_keys = m.kv_rank * m.heads * (m.dim + m.vdim)
     return 2.0 * (S * lin + (past + S) * lin_keys + S * keys * m.heads * (m.dim + m.vdim))
@@ -48,7 +62,7 @@ def flops_of(cfg, S: int, past: int = 0) -> float:
 
 
 def step_bytes(cfg, B: int, L: int) -> float:
-    return cfg.decode_weight_bytes() + B * L * cfg.kv_bytes_per_token
+    return cfg.decode_weight_bytes() + B * (L * cfg.kv_bytes_per_token + 2 * getattr(cfg, "state_bytes", 0))          # a state is read and written
 
 
 def build(name: str, layers: int, rows: int, kv: int, streams: int):
@@ -98,7 +112,7 @@ def run_model(name: str, layers: int, prefills, decodes, reps: int, say):
 
         def steps():
             for s in range(B):
-                eng.set_slot_length(s, L, L)
+                eng.set_slot_length(s, L, L, keep_state=True)
             eng.decode(list(range(B)), n, 1, sp)
         t = timed(steps, reps, warm=2) / n
         out["decode"].append(dict(streams=B, keys=L, ms_per_step=round(t * 1e3, 4), tokens_per_s=round(B / t, 1),
@@ -110,10 +124,10 @@ def run_model(name: str, layers: int, prefills, decodes, reps: int, say):
 
 
 def main(args) -> None:
-    sizes = [args.decoder_size] if args.decoder_size else list(SIZES)
+    sizes = [args.decoder_size] if args.decoder_size else list(LIKE)
     prefills = [int(x) for x in args.decoder_prefill.split(",") if x]
     decodes = [tuple(int(y) for y in x.split("x")) for x in args.decoder_decode.split(",") if x]
     for size in sizes:
-        for name in SIZES[size] if not args.decoder_only else SIZES[size][:1]:
+        for name in [f"{args.decoder_model}-{size}"] + ([] if args.decoder_only else [LIKE[size]]):
             r = run_model(name, args.decoder_layers, prefills, decodes, max(1, args.steps), lambda m: print(m, flush=True))
             print(json.dumps(dict(metric="decoder_vs_gqa", size=size, dtype="bf16", data="synthetic", **r)), flush=True)
