@@ -82,6 +82,19 @@ __global__ __launch_bounds__(256) void logits_cap_kernel(const float* __restrict
 // ---- RMS norms with weights stored around zero: one block of NW waves per row, two 4-channel pieces per thread ----
 LCC_DEVICE f32x4 bf4(u32x2 q) { return (f32x4){lo2f(q.x), hi2f(q.x), lo2f(q.y), hi2f(q.y)}; }
 LCC_DEVICE float sq4(f32x4 v) { return (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
+// sum of the slabs, four of them in flight
+LCC_DEVICE f32x4 slabs4(const float* part, int nsplit, size_t slab, size_t at) {
+  f32x4 v = *reinterpret_cast<const f32x4*>(part + at);
+  for (int k = 1; k < nsplit; k += 4) {
+    f32x4 u[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) u[j] = *reinterpret_cast<const f32x4*>(part + (size_t)min(k + j, nsplit - 1) * slab + at);
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (k + j < nsplit) v += u[j];
+  }
+  return v;
+}
 LCC_DEVICE float inv_rms(float sum, int n, float eps) { return 1.f / sqrtf(sum / (float)n + eps); }
 
 template <int NW>
@@ -137,11 +150,11 @@ __global__ __launch_bounds__(NW * 64) void post_norm_resid_kernel(PostNormArgs a
     if (c < a.dim) {
       xv[i] = *reinterpret_cast<const f32x4*>(a.x + at + c);
       wp[i] = ld8(a.post_w + c); wn[i] = ld8(a.next_w + c);
-      for (int k = 0; k < a.nsplit; ++k) y[i] += *reinterpret_cast<const f32x4*>(a.part + k * slab + at + c);
+      y[i] = slabs4(a.part, a.nsplit, slab, at + c);
       s += sq4(y[i]);
       if (PAIR) {
         wa[j] = ld8(a.w_a + c); wb[j] = ld8(a.w_b + c);
-        for (int k = 0; k < a.nsplit_b; ++k) yb[j] += *reinterpret_cast<const f32x4*>(a.part_b + k * slab + at + c);
+        yb[j] = slabs4(a.part_b, a.nsplit_b, slab, at + c);
         sb += sq4(yb[j]);
       }
     }

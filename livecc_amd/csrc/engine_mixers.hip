@@ -4,8 +4,8 @@
 //   in      every projection of the mixer                 one product, fp32
 //   prefill prep (norms, temperature, cache append | convolution, activations)      mixer_prep
 //           attention (attn_mha over the slots' arenas), recurrence (rec_scan), gated norm (rec_norm)
-//   decode  recurrence with its input activations, the attention's rows behind it   rec_decode
-//           attention splits (gqa_decode), merge + gated norm in one launch         gqa_merge_rec_norm
+//   decode  recurrence with its input activations and the attention's splits        rec_gqa_decode (other sizes, many rows: rec_decode, gqa_decode)
+//           merge + gated norm in one launch                                        gqa_merge_rec_norm
 //   out     W_o of the attention and of the recurrence    two products (decode: one launch), fp32
 //           norms, residual, next norm                    post_norm_resid
 //   ff      SwiGLU product, down product, post_norm_resid
@@ -212,14 +212,20 @@ int run_mixer_layers(lcc_engine* e, const DecBuffers& b, int S, const PrefillTab
       if (ri.taps) rn.conv = &ri;
       LCC_TRY(rec_norm(rn, st));
     } else {
-      LCC_TRY(rec_decode(ri, has_attn(L) ? &gi : nullptr, b.y, st));
+      ri.direct = gi.direct = direct;
       if (has_attn(L)) {
         GqaDecodeArgs a; a.q = b.q; a.rows = S; a.heads = L.heads; a.kv_heads = L.kv_heads; a.dim = L.dim_pad; a.vdim = L.vdim_pad; a.nsplit = nsplit_attn;
         a.scale_log2e = scale_log2e; a.slope = w.slope; a.slots = d_slots; a.kv_len = e->d_kv_len; a.kv_base = e->d_kv_base; a.k_off = off.kv; a.v_off = off.v;
         a.lmax = e->lim.max_kv_len; a.ws_o = b.ws_o; a.ws_ml = b.ws_ml; a.out = b.att; a.direct = direct;
-        LCC_TRY(gqa_decode(a, st));
+        if (fused && rec_gqa_decode_ok(ri, a)) {
+          LCC_TRY(rec_gqa_decode(ri, gi, a, b.y, st));
+        } else {
+          LCC_TRY(rec_decode(ri, &gi, b.y, st));
+          LCC_TRY(gqa_decode(a, st));
+        }
         LCC_TRY(gqa_merge_rec_norm(a, rn, st));
       } else {
+        LCC_TRY(rec_decode(ri, nullptr, b.y, st));
         LCC_TRY(rec_norm(rn, st));
       }
     }

@@ -300,6 +300,7 @@ struct GqaInArgs {               // behind the fused input projection: per-head 
   bf16_t* q = nullptr;                                               // [rows][heads dim_pad]
   const int32_t* tok_stream = nullptr; const int32_t* tok_pos = nullptr; const int32_t* kv_len = nullptr;   // tok_pos null: kv_len[slot]
   bf16_t* const* kv_base = nullptr; size_t k_off = 0, v_off = 0; int lmax = 0;
+  AttnDirect direct;                                                 // decode of up to 4 rows: arena and key count (position + 1) by value
 };
 constexpr int GQA_MAX_SPLIT = 64;
 struct GqaDecodeArgs {
@@ -325,9 +326,12 @@ struct RecInArgs {               // where the inputs lie in the fused input proj
   const int32_t* kv_len = nullptr; const int32_t* done = nullptr;
   bf16_t* const* kv_base = nullptr; size_t state_off = 0, conv_off = 0;    // fp32 [heads][np][ep]; fp32 [taps][conv_ch], position p at row p % taps
   bf16_t* q = nullptr; bf16_t* k = nullptr; bf16_t* v = nullptr; float* dt = nullptr;   // prefill: activated inputs, [rows][..]; dt [rows][heads]
+  AttnDirect direct;                                                       // decode of up to 4 rows: arena and position + 1 by value
 };
 int mixer_prep(const GqaInArgs* left, const RecInArgs* rec, hipStream_t st);              // prefill: either or both, one launch
 int rec_decode(const RecInArgs& rec, const GqaInArgs* left, float* y, hipStream_t st);    // decode: state step (y [rows][heads ep]) + the rows of `left`
+bool rec_gqa_decode_ok(const RecInArgs& rec, const GqaDecodeArgs& d);                     // the one-launch form serves this (<= 4 rows, one slab, heads of 64 / 128)
+int rec_gqa_decode(const RecInArgs& rec, const GqaInArgs& left, const GqaDecodeArgs& d, float* y, hipStream_t st);      // state step + the attention's splits
 struct RecScanArgs {
   const bf16_t* q = nullptr; const bf16_t* k = nullptr; const bf16_t* v = nullptr; const float* dt = nullptr;      // dt null: 1
   const float* rate = nullptr; const float* skip = nullptr; float* y = nullptr;

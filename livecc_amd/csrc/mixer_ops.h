@@ -27,8 +27,10 @@ template <int NW>
 LCC_DEVICE void gqa_row(const GqaInArgs& a, int row) {
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const size_t slab = (size_t)a.rows * a.ldn, at = (size_t)row * a.ldn;
-  const int slot = a.tok_stream[row], pos = a.tok_pos ? a.tok_pos[row] : a.kv_len[slot];
-  bf16_t* arena = a.kv_base[slot];
+  int pos;
+  bf16_t* arena;
+  if (a.direct.used) { pos = a.direct.n[row & 3] - 1; arena = const_cast<bf16_t*>(a.direct.base[row & 3]); }
+  else { const int slot = a.tok_stream[row]; pos = a.tok_pos ? a.tok_pos[row] : a.kv_len[slot]; arena = a.kv_base[slot]; }
   const float temp = 1.f + a.temp_coef * logf((float)((pos + 1) / a.temp_every) + 1.f);
   for (int h = wave; h < a.heads + a.kv_heads; h += NW) {
     const bool isq = h < a.heads;
@@ -78,38 +80,53 @@ LCC_DEVICE float rec_dt(const RecInArgs& a, int row, int h) {
   for (int s = 1; s < a.nsplit; ++s) z += p[(size_t)s * a.rows * a.ldn];
   return softplus_f(z + a.dt_bias[h]);
 }
-// one (row, norm group) of the gated norm behind the recurrence, by a block of NW waves; red: NW floats of LDS
-template <int NW>
+// one (row, norm group) of the gated norm behind the recurrence, by a block of NW waves; red: NW floats of LDS.  Up to MAXP pieces of 4 channels per
+// thread stay in registers between the statistic and the result.
+template <int NW, int MAXP>
 LCC_DEVICE void rec_norm_row(const RecNormArgs& a, int row, int grp, float* red) {
   const int tid = threadIdx.x, inner = a.heads * a.vdim, gs = inner / a.norm_groups, nt = NW * 64;
   const size_t slab = (size_t)a.rows * a.ldn;
   const float* y = a.y + (size_t)row * a.heads * a.ep;
   const size_t gate = (size_t)row * a.ldn + a.gate_col;
   bf16_t* out = a.out + (size_t)row * a.ld;
-  auto gate1 = [&](int c) {
-    float z = a.part[gate + c];
-    for (int s = 1; s < a.nsplit; ++s) z += a.part[s * slab + gate + c];
-    return z;
-  };
   const int lo = grp * gs, hi = lo + gs;
   float ss = 0.f;
-  if (((a.vdim | gs) & 3) == 0) {                      // pieces of 4 channels stay inside a head and a group
-    for (int r = lo + tid * 4; r < hi; r += nt * 4) {
-      const int h = r / a.vdim, c = h * a.ep + r - h * a.vdim;
-      f32x4 v = *reinterpret_cast<const f32x4*>(y + c);
-      if (a.gate_first) v *= silu4(slab_sum4(a.part, a.nsplit, slab, gate + c));
-      ss += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+  if (((a.vdim | gs) & 3) == 0 && gs <= nt * 4 * MAXP) {      // pieces of 4 channels stay inside a head and a group
+    f32x4 v[MAXP], g[MAXP];
+    u32x2 w[MAXP];
+#pragma unroll
+    for (int i = 0; i < MAXP; ++i) {
+      const int r = lo + (tid + i * nt) * 4;
+      v[i] = g[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+      w[i] = (u32x2){0u, 0u};
+      if (r < hi) {
+        const int h = r / a.vdim, c = h * a.ep + r - h * a.vdim;
+        v[i] = *reinterpret_cast<const f32x4*>(y + c);
+        g[i] = slab_sum4(a.part, a.nsplit, slab, gate + c);
+        w[i] = ld8(a.w + r);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < MAXP; ++i) {
+      if (a.gate_first) v[i] *= silu4(g[i]);
+      ss += (v[i][0] * v[i][0] + v[i][1] * v[i][1]) + (v[i][2] * v[i][2] + v[i][3] * v[i][3]);
     }
     const float inv = 1.f / sqrtf(block_sum<NW>(ss, red) / (float)gs + a.eps);
-    for (int r = lo + tid * 4; r < hi; r += nt * 4) {
-      const int h = r / a.vdim, c = h * a.ep + r - h * a.vdim;
-      f32x4 v = *reinterpret_cast<const f32x4*>(y + c);
-      const f32x4 g = slab_sum4(a.part, a.nsplit, slab, gate + c), w = unpack4(ld8(a.w + r));
-      if (a.gate_first) v = v * silu4(g) * inv * w;
-      else v = v * inv * w * (f32x4){sigmoid_f(g[0]), sigmoid_f(g[1]), sigmoid_f(g[2]), sigmoid_f(g[3])};
-      st8(out + r, pack4(v));
+#pragma unroll
+    for (int i = 0; i < MAXP; ++i) {
+      const int r = lo + (tid + i * nt) * 4;
+      if (r < hi) {
+        f32x4 o = v[i] * inv * unpack4(w[i]);
+        if (!a.gate_first) o *= (f32x4){sigmoid_f(g[i][0]), sigmoid_f(g[i][1]), sigmoid_f(g[i][2]), sigmoid_f(g[i][3])};
+        st8(out + r, pack4(o));
+      }
     }
   } else {
+    auto gate1 = [&](int c) {
+      float z = a.part[gate + c];
+      for (int s = 1; s < a.nsplit; ++s) z += a.part[s * slab + gate + c];
+      return z;
+    };
     for (int r = lo + tid; r < hi; r += nt) {
       const int h = r / a.vdim, c = h * a.ep + r - h * a.vdim;
       const float v = a.gate_first ? y[c] * silu_f(gate1(c)) : y[c];
@@ -132,6 +149,144 @@ LCC_DEVICE void conv_ring_row(const RecInArgs& a, int row) {
   float* ring = reinterpret_cast<float*>(a.kv_base[a.tok_stream[row]] + a.conv_off) + (size_t)(a.tok_pos[row] % a.taps) * a.conv_ch;
   for (int c = threadIdx.x * 4; c < a.conv_ch; c += NW * 256)
     *reinterpret_cast<f32x4*>(ring + c) = slab_sum4(a.part, a.nsplit, (size_t)a.rows * a.ldn, (size_t)row * a.ldn + a.conv_col + c);
+}
+
+// One wave of the decode attention: a key split of one row, KV head and tile of 16 query heads of it; partial (O, m, l) to the workspace.  A 32-key tile
+// is two 16-key MFMA row tiles whose rows are dealt so that the probabilities a lane ends up with are the 8 consecutive keys its operand of
+// the P.V product needs.  NEW: queries, the new key and the new value come straight from the input projection (one slab), the last split
+// puts the new token into its operands and the cache.
+template <int DK, int DV, bool NEW>
+LCC_DEVICE void gqa_decode_wave(const GqaDecodeArgs& a, const GqaInArgs& in, int split, int kvh, int tile, int b) {
+  constexpr int KS = DK / 32, DT = DV / 16;
+  const int lane = threadIdx.x & 63, li = lane & 15, g = lane >> 4;
+  const int G = a.heads / a.kv_heads, j = tile * 16 + li;
+  const int head = kvh * G + min(j, G - 1);
+  int n;
+  const bf16_t* arena;
+  if (a.direct.used) { n = a.direct.n[b & 3]; arena = a.direct.base[b & 3]; }
+  else { const int slot = a.slots[b]; n = a.kv_len[slot] + 1; arena = a.kv_base[slot]; }
+  const int ntile = (n + 31) >> 5, per = (ntile + a.nsplit - 1) / a.nsplit, t0 = split * per, t1 = min(ntile, t0 + per);
+  if (t0 >= t1) return;                                              // the merge knows which splits exist
+  const bf16_t* kb = arena + a.k_off + (size_t)kvh * a.lmax * DK;
+  const bf16_t* vb = arena + a.v_off + (size_t)kvh * a.lmax * DV;
+  const float slope = a.slope ? a.slope[head] : 0.f;
+  u32x4 qf[KS], knew[NEW ? KS : 1];
+  bf16_t vnew[NEW ? DT : 1];
+  const bool owner = NEW && t1 == ntile;                             // of the new token's key and value
+  if (NEW) {
+    // fragments straight from the projection: lane (head li, g) holds channels 32 k + 8 g .. of its head, the four g of a head share its norm
+    const float* row = in.part + (size_t)b * in.ldn;
+    const float temp = 1.f + in.temp_coef * logf((float)(n / in.temp_every) + 1.f);      // position n - 1
+    auto normed = [&](const float* src, const bf16_t* w, float f, u32x4* dst) {
+      f32x4 x[2 * KS];
+      u32x4 wv[KS];
+      float ss = 0.f;
+#pragma unroll
+      for (int k = 0; k < KS; ++k) {
+        x[2 * k] = *reinterpret_cast<const f32x4*>(src + k * 32 + g * 8);
+        x[2 * k + 1] = *reinterpret_cast<const f32x4*>(src + k * 32 + g * 8 + 4);
+        wv[k] = ld16(w + k * 32 + g * 8);
+      }
+#pragma unroll
+      for (int k = 0; k < 2 * KS; ++k) ss += (x[k][0] * x[k][0] + x[k][1] * x[k][1]) + (x[k][2] * x[k][2] + x[k][3] * x[k][3]);
+      ss += __shfl_xor(ss, 16, 64);
+      ss += __shfl_xor(ss, 32, 64);
+      const float r = f / sqrtf(ss / (float)in.dim + in.eps);
+#pragma unroll
+      for (int k = 0; k < KS; ++k) {
+        const u32x2 lo = pack4(x[2 * k] * r * unpack4((u32x2){wv[k][0], wv[k][1]})), hi = pack4(x[2 * k + 1] * r * unpack4((u32x2){wv[k][2], wv[k][3]}));
+        dst[k] = (u32x4){lo.x, lo.y, hi.x, hi.y};
+      }
+    };
+    normed(row + (size_t)head * DK, in.q_norm, temp, qf);
+    if (owner) {
+      normed(row + (size_t)(a.heads + kvh) * DK, in.k_norm, 1.f, knew);
+#pragma unroll
+      for (int d = 0; d < DT; ++d) vnew[NEW ? d : 0] = f2bf(row[(size_t)(a.heads + a.kv_heads) * DK + kvh * DV + d * 16 + li]);
+    }
+  } else {
+#pragma unroll
+    for (int k = 0; k < KS; ++k) qf[k] = ld16(a.q + ((size_t)b * a.heads + head) * DK + k * 32 + g * 8);
+  }
+  const int krow = (li >> 2) * 8 + (li & 3);                         // row li of key tile u holds key (li / 4) 8 + 4 u + li % 4
+  u32x4 kf[2][KS], vf[DT];
+  auto load_k = [&](int t) {
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+      for (int k = 0; k < KS; ++k) kf[u][k] = ld16(kb + (size_t)(t * 32 + krow + 4 * u) * DK + k * 32 + g * 8);      // whole tiles of the arena are readable
+  };
+  auto load_v = [&](int t) {
+#pragma unroll
+    for (int d = 0; d < DT; ++d) vf[d] = ld16(vb + ((size_t)t * DV + d * 16 + li) * 32 + g * 8);
+  };
+  f32x4 o[DT];
+#pragma unroll
+  for (int d = 0; d < DT; ++d) o[d] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+  load_k(t0);
+  load_v(t0);
+  for (int t = t0; t < t1; ++t) {
+    if (NEW && owner && t == ntile - 1) {                            // the new token: into the operands, and -- one wave per KV head -- into the cache
+      const int at = (n - 1) & 31;
+#pragma unroll
+      for (int u = 0; u < 2; ++u)
+        if (krow + 4 * u == at) {
+#pragma unroll
+          for (int k = 0; k < KS; ++k) {
+            kf[u][k] = knew[NEW ? k : 0];
+            if (tile == 0) st16(const_cast<bf16_t*>(kb) + (size_t)(n - 1) * DK + k * 32 + g * 8, knew[NEW ? k : 0]);
+          }
+        }
+      if (at >> 3 == g) {
+        const int e = at & 7, half = (e & 1) * 16;
+#pragma unroll
+        for (int d = 0; d < DT; ++d) {
+          const unsigned keep = ~(0xffffu << half), put = (unsigned)vnew[NEW ? d : 0] << half;
+#pragma unroll
+          for (int q = 0; q < 4; ++q)
+            if (e >> 1 == q) vf[d][q] = (vf[d][q] & keep) | put;
+          if (tile == 0) const_cast<bf16_t*>(vb)[((size_t)t * DV + d * 16 + li) * 32 + at] = vnew[NEW ? d : 0];
+        }
+      }
+    }
+    f32x4 s[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      s[u] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int k = 0; k < KS; ++k) s[u] = mfma16(as_bf16x8(kf[u][k]), as_bf16x8(qf[k]), s[u]);
+    }
+    if (t + 1 < t1) load_k(t + 1);
+    float mx = -INFINITY;
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int key = t * 32 + g * 8 + u * 4 + r;
+        s[u][r] = key < n ? fmaf(s[u][r], a.scale_log2e, slope * (float)(key + 1 - n)) : -INFINITY;
+        mx = fmaxf(mx, s[u][r]);
+      }
+    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    const float mn = fmaxf(m, mx), alpha = __builtin_amdgcn_exp2f(m - mn);      // finite: a tile has at least one key
+    m = mn;
+    float p[8], sum = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) { p[e] = __builtin_amdgcn_exp2f(s[e >> 2][e & 3] - mn); sum += p[e]; }
+    l = l * alpha + sum;
+    const bf16x8 pf = as_bf16x8((u32x4){pack2(p[0], p[1]), pack2(p[2], p[3]), pack2(p[4], p[5]), pack2(p[6], p[7])});
+#pragma unroll
+    for (int d = 0; d < DT; ++d) { o[d] *= alpha; o[d] = mfma16(as_bf16x8(vf[d]), pf, o[d]); }
+    if (t + 1 < t1) load_v(t + 1);
+  }
+  l += __shfl_xor(l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  if (j >= G) return;
+  const size_t at = ((size_t)b * a.heads + head) * a.nsplit + split;
+#pragma unroll
+  for (int d = 0; d < DT; ++d) *reinterpret_cast<f32x4*>(a.ws_o + at * DV + d * 16 + g * 4) = o[d];
+  if (g == 0) { a.ws_ml[at * 2] = m; a.ws_ml[at * 2 + 1] = l; }
 }
 
 }  // namespace lcc

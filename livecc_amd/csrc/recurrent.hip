@@ -17,20 +17,66 @@ namespace lcc {
 // ------------------------------------------------------------------------------------------------------------------------------
 // Prefill, in front of the scan and the attention: one block per row.
 // ------------------------------------------------------------------------------------------------------------------------------
+// TAPS > 0: REC alone, PREP_ROWS rows per block -- a thread reads its columns of every row once and keeps the window in registers
+constexpr int PREP_ROWS = 4;
+template <int TAPS>
+__global__ __launch_bounds__(256) void conv_prep_kernel(RecInArgs a) {
+  constexpr int WIN = PREP_ROWS + TAPS - 1;
+  const int row0 = blockIdx.x * PREP_ROWS, n = min(PREP_ROWS, a.rows - row0), tid = threadIdx.x, gk = a.groups * a.np, hv = a.heads * a.ep;
+  const size_t slab = (size_t)a.rows * a.ldn;
+  int pos[PREP_ROWS], r0[PREP_ROWS];
+  const float* ring[PREP_ROWS];
+#pragma unroll
+  for (int i = 0; i < PREP_ROWS; ++i) {
+    const int r = min(row0 + i, a.rows - 1);
+    pos[i] = a.tok_pos[r]; r0[i] = a.tok_row0[r];
+    ring[i] = reinterpret_cast<const float*>(a.kv_base[a.tok_stream[r]] + a.conv_off);
+  }
+  for (int p = ((int)blockIdx.y * 256 + tid) * 4; p < 2 * gk + hv; p += (int)gridDim.y * 1024) {
+    const int col = p < gk ? a.q_col + p : p < 2 * gk ? a.k_col + p - gk : a.v_col + p - 2 * gk, ch = col - a.conv_col;
+    f32x4 u[WIN], w[TAPS];
+#pragma unroll
+    for (int i = 0; i < WIN; ++i)
+      u[i] = slab_sum4(a.part, a.nsplit, slab, (size_t)min(max(row0 + i - (TAPS - 1), 0), a.rows - 1) * a.ldn + col);
+#pragma unroll
+    for (int t = 0; t < TAPS; ++t) w[t] = unpack4(ld8(a.conv_w + (size_t)t * a.conv_ch + ch));
+    const f32x4 bias = unpack4(ld8(a.conv_b + ch));
+#pragma unroll
+    for (int i = 0; i < PREP_ROWS; ++i) {
+      if (i >= n) break;
+      f32x4 acc = bias + w[TAPS - 1] * u[i + TAPS - 1];
+#pragma unroll
+      for (int back = 1; back < TAPS; ++back) {
+        f32x4 x = u[i + TAPS - 1 - back];
+        if (row0 + i - back < r0[i])                   // before this portion: out of the slot's ring, zero before the start
+          x = back <= pos[i] ? *reinterpret_cast<const f32x4*>(ring[i] + (size_t)((pos[i] - back) % TAPS) * a.conv_ch + ch) : (f32x4){0.f, 0.f, 0.f, 0.f};
+        acc += w[TAPS - 1 - back] * x;
+      }
+      const u32x2 o = pack4(silu4(acc));
+      const size_t row = (size_t)(row0 + i);
+      if (p < gk) st8(a.q + row * gk + p, o);
+      else if (p < 2 * gk) st8(a.k + row * gk + p - gk, o);
+      else st8(a.v + row * hv + p - 2 * gk, o);
+    }
+  }
+  if (a.dt_col >= 0 && blockIdx.y == 0)
+    for (int i = tid; i < n * a.heads; i += 256) a.dt[(size_t)row0 * a.heads + i] = rec_dt(a, row0 + i / a.heads, i % a.heads);
+}
 template <bool LEFT, bool REC>
 __global__ __launch_bounds__(256) void mixer_prep_kernel(GqaInArgs l, RecInArgs a) {
-  const int row = blockIdx.x, tid = threadIdx.x;
-  if (LEFT) gqa_row<4>(l, row);
-  if (!REC) return;
+  // blockIdx.y: few rows are spread over several blocks -- the attention's part, then shares of the recurrence's columns
+  const int row = blockIdx.x, tid = threadIdx.x, part = LEFT && gridDim.y > 1 ? (int)blockIdx.y - 1 : (int)blockIdx.y, parts = LEFT && gridDim.y > 1 ? gridDim.y - 1 : gridDim.y;
+  if (LEFT && blockIdx.y == 0) gqa_row<4>(l, row);
+  if (!REC || part < 0) return;
   const int pos = a.tok_pos[row], r0 = a.tok_row0[row], gk = a.groups * a.np, hv = a.heads * a.ep;
   const float* ring = a.taps ? reinterpret_cast<const float*>(a.kv_base[a.tok_stream[row]] + a.conv_off) : nullptr;
-  for (int p = tid * 4; p < 2 * gk + hv; p += 1024) {
+  for (int p = (part * 256 + tid) * 4; p < 2 * gk + hv; p += parts * 1024) {
     f32x4 raw;
     if (p < gk) st8(a.q + (size_t)row * gk + p, pack4(rec_in4(a, row, r0, pos, ring, a.q_col + p, &raw)));
     else if (p < 2 * gk) st8(a.k + (size_t)row * gk + p - gk, pack4(rec_in4(a, row, r0, pos, ring, a.k_col + p - gk, &raw)));
     else st8(a.v + (size_t)row * hv + p - 2 * gk, pack4(rec_in4(a, row, r0, pos, ring, a.v_col + p - 2 * gk, &raw)));
   }
-  if (a.dt_col >= 0)
+  if (a.dt_col >= 0 && part == 0)
     for (int h = tid; h < a.heads; h += 256) a.dt[(size_t)row * a.heads + h] = rec_dt(a, row, h);
 }
 static bool gqa_in_ok(const GqaInArgs& a) {
@@ -53,27 +99,31 @@ int mixer_prep(const GqaInArgs* left, const RecInArgs* rec, hipStream_t st) {
   if (rec && (!rec->tok_pos || !rec->tok_row0 || !rec->q || !rec->k || !rec->v || (rec->dt_col >= 0 && !rec->dt))) return LCC_ERR_ARG;
   const GqaInArgs l = left ? *left : GqaInArgs();
   const RecInArgs r = rec ? *rec : RecInArgs();
-  if (left && rec) mixer_prep_kernel<true, true><<<dim3(rows), dim3(256), 0, st>>>(l, r);
+  const int cols = rec ? 2 * r.groups * r.np + r.heads * r.ep : 0, share = std::max(1, std::min((cols + 1023) / 1024, 2048 / rows));
+  if (left && rec) mixer_prep_kernel<true, true><<<dim3(rows, share > 1 ? share + 1 : 1), dim3(256), 0, st>>>(l, r);
   else if (left) mixer_prep_kernel<true, false><<<dim3(rows), dim3(256), 0, st>>>(l, r);
-  else mixer_prep_kernel<false, true><<<dim3(rows), dim3(256), 0, st>>>(l, r);
+  else if (r.taps == 4 && rows >= 64) conv_prep_kernel<4><<<dim3((rows + PREP_ROWS - 1) / PREP_ROWS, std::min((cols + 1023) / 1024, share * PREP_ROWS)), dim3(256), 0, st>>>(r);
+  else mixer_prep_kernel<false, true><<<dim3(rows, share), dim3(256), 0, st>>>(l, r);
   return 0;
 }
 
 // ------------------------------------------------------------------------------------------------------------------------------
 // Decode: block = (row, head, 64 value channels); thread t owns value channels 4 (t & 15) .. of the state rows t / 16, t / 16 + 16, ..
-// The blocks behind them run the rows of the attention beside it (queries, keys, values).
+// The blocks behind them run the attention beside it (rec_gqa_decode_kernel), or only its rows: queries, keys, values (rec_decode_kernel).
 // ------------------------------------------------------------------------------------------------------------------------------
 template <int NT>
-__global__ __launch_bounds__(256) void rec_decode_kernel(RecInArgs a, GqaInArgs l, float* __restrict__ y, int n_rec) {
-  if ((int)blockIdx.x >= n_rec) { gqa_row<4>(l, (int)blockIdx.x - n_rec); return; }
+LCC_DEVICE void rec_decode_block(const RecInArgs& a, float* __restrict__ y) {
   constexpr int NP = NT * 64, NR = NP / 16;
   __shared__ float s_q[NP], s_k[NP];
   __shared__ __attribute__((aligned(16))) float s_v[64];
   __shared__ f32x4 s_o[4][16];
   const int vt = a.ep / 64, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int row = blockIdx.x / (a.heads * vt), rem = blockIdx.x - row * (a.heads * vt), h = rem / vt, v0 = (rem - h * vt) * 64;
-  const int slot = a.tok_stream[row], pos = a.kv_len[slot], grp = h / (a.heads / a.groups);
-  bf16_t* arena = a.kv_base[slot];
+  const int slot = a.tok_stream[row], grp = h / (a.heads / a.groups);
+  int pos;
+  bf16_t* arena;
+  if (a.direct.used) { pos = a.direct.n[row & 3] - 1; arena = const_cast<bf16_t*>(a.direct.base[row & 3]); }
+  else { pos = a.kv_len[slot]; arena = a.kv_base[slot]; }
   float* S = reinterpret_cast<float*>(arena + a.state_off) + (size_t)h * NP * a.ep + v0 + (tid & 15) * 4;
   const int n0 = tid >> 4;
   f32x4 st[NR];
@@ -86,7 +136,7 @@ __global__ __launch_bounds__(256) void rec_decode_kernel(RecInArgs a, GqaInArgs 
     f32x4 raw;
     const f32x4 v = rec_in4(a, row, row, pos, ring, col, &raw);
     // position p replaces position p - taps, which no reader of this step needs; blocks that share a channel write the same value
-    if (ring) *reinterpret_cast<f32x4*>(ring + (size_t)(pos % a.taps) * a.conv_ch + col - a.conv_col) = raw;
+    if (ring && !frozen) *reinterpret_cast<f32x4*>(ring + (size_t)(pos % a.taps) * a.conv_ch + col - a.conv_col) = raw;
     float* dst = p < NP ? s_q + p : p < 2 * NP ? s_k + p - NP : s_v + p - 2 * NP;
 #pragma unroll
     for (int e = 0; e < 4; ++e) dst[e] = v[e];
@@ -114,6 +164,45 @@ __global__ __launch_bounds__(256) void rec_decode_kernel(RecInArgs a, GqaInArgs 
     if (a.skip) r += v * a.skip[h];
     *reinterpret_cast<f32x4*>(y + ((size_t)row * a.heads + h) * a.ep + v0 + tid * 4) = r;
   }
+}
+template <int NT>
+__global__ __launch_bounds__(256) void rec_decode_kernel(RecInArgs a, GqaInArgs l, float* __restrict__ y, int n_rec) {
+  if ((int)blockIdx.x >= n_rec) gqa_row<4>(l, (int)blockIdx.x - n_rec);
+  else rec_decode_block<NT>(a, y);
+}
+// the attention beside it in the same launch: behind the n_rec blocks, four (split, KV head, head tile, row) items per block, splits fastest
+template <int NT, int DK, int DV>
+__global__ __launch_bounds__(256, 2) void rec_gqa_decode_kernel(RecInArgs a, GqaInArgs l, GqaDecodeArgs d, float* __restrict__ y, int n_rec) {
+  if ((int)blockIdx.x < n_rec) { rec_decode_block<NT>(a, y); return; }
+  const int ht = (d.heads / d.kv_heads + 15) / 16, per_row = d.nsplit * d.kv_heads * ht;
+  const int item = __builtin_amdgcn_readfirstlane(((int)blockIdx.x - n_rec) * 4 + (int)(threadIdx.x >> 6));
+  if (item >= d.rows * per_row) return;
+  const int b = item / per_row, r = item - b * per_row, split = r % d.nsplit, hh = r / d.nsplit;
+  gqa_decode_wave<DK, DV, true>(d, l, split, hh / ht, hh % ht, b);
+}
+bool rec_gqa_decode_ok(const RecInArgs& rec, const GqaDecodeArgs& d) {
+  // up to 4 rows: the launch saved; from 8 rows on the two kernels' own occupancies are worth more (8 streams x 4096 keys: 25.7 against 28.6 us)
+  return rec.rows <= 4 && rec.nsplit == 1 && rec.np <= 128 && (d.dim == 64 || d.dim == 128) && (d.vdim == 64 || d.vdim == 128);
+}
+int rec_gqa_decode(const RecInArgs& rec, const GqaInArgs& left, const GqaDecodeArgs& d, float* y, hipStream_t st) {
+  if (rec.rows <= 0) return 0;
+  if (!rec_in_ok(rec) || !gqa_in_ok(left) || !rec_gqa_decode_ok(rec, d) || left.rows != rec.rows || d.rows != rec.rows || left.nsplit != 1 || left.dim_pad != d.dim ||
+      left.vdim_pad != d.vdim || left.heads != d.heads || left.kv_heads != d.kv_heads || d.nsplit < 1 || d.nsplit > GQA_MAX_SPLIT || d.lmax != left.lmax ||
+      (d.direct.used && d.rows > 4))
+    return LCC_ERR_SHAPE;
+  if (!rec.kv_len || !y || !d.slots || !d.kv_len || !d.kv_base || !d.ws_o || !d.ws_ml) return LCC_ERR_ARG;
+  const int n = rec.rows * rec.heads * (rec.ep / 64), items = d.rows * d.nsplit * d.kv_heads * ((d.heads / d.kv_heads + 15) / 16);
+  const dim3 grid(n + (items + 3) / 4);
+#define LCC_GO(NT)                                                                                                          \
+  do {                                                                                                                      \
+    if (d.dim == 64 && d.vdim == 64) rec_gqa_decode_kernel<NT, 64, 64><<<grid, dim3(256), 0, st>>>(rec, left, d, y, n);          \
+    else if (d.dim == 64) rec_gqa_decode_kernel<NT, 64, 128><<<grid, dim3(256), 0, st>>>(rec, left, d, y, n);                    \
+    else if (d.vdim == 64) rec_gqa_decode_kernel<NT, 128, 64><<<grid, dim3(256), 0, st>>>(rec, left, d, y, n);                   \
+    else rec_gqa_decode_kernel<NT, 128, 128><<<grid, dim3(256), 0, st>>>(rec, left, d, y, n);                                    \
+  } while (0)
+  if (rec.np == 64) LCC_GO(1); else LCC_GO(2);
+#undef LCC_GO
+  return 0;
 }
 int rec_decode(const RecInArgs& rec, const GqaInArgs* left, float* y, hipStream_t st) {
   if (rec.rows <= 0) return 0;
@@ -360,11 +449,11 @@ int rec_scan(const RecScanArgs& a, hipStream_t st) {
 // ------------------------------------------------------------------------------------------------------------------------------
 // Behind the recurrence: gated norm, grid (row, norm group); RING: the inputs the convolution of the stream's next call needs
 // ------------------------------------------------------------------------------------------------------------------------------
-template <bool RING>
-__global__ __launch_bounds__(256) void rec_norm_kernel(RecNormArgs a, RecInArgs in) {
-  __shared__ float red[4];
-  if (RING && blockIdx.y == 0) conv_ring_row<4>(in, blockIdx.x);
-  rec_norm_row<4>(a, blockIdx.x, blockIdx.y, red);
+template <bool RING, int NW, int MAXP>
+__global__ __launch_bounds__(NW * 64) void rec_norm_kernel(RecNormArgs a, RecInArgs in) {
+  __shared__ float red[NW];
+  if (RING && blockIdx.y == 0) conv_ring_row<NW>(in, blockIdx.x);
+  rec_norm_row<NW, MAXP>(a, blockIdx.x, blockIdx.y, red);
 }
 bool rec_norm_ok(const RecNormArgs& a) {
   return a.y && a.part && a.nsplit >= 1 && a.w && a.out && a.heads >= 1 && a.vdim >= 1 && a.vdim <= a.ep && !(a.ep & 3) && a.norm_groups >= 1 && a.norm_groups <= 65535 &&
@@ -375,8 +464,19 @@ int rec_norm(const RecNormArgs& a, hipStream_t st) {
   if (a.rows <= 0) return 0;
   if (!rec_norm_ok(a)) return LCC_ERR_SHAPE;
   if (a.conv && (a.conv->taps < 1 || !a.conv->tok_last || !a.conv->tok_pos || !a.conv->tok_stream || !a.conv->kv_base || a.conv->rows != a.rows)) return LCC_ERR_ARG;
-  if (a.conv) rec_norm_kernel<true><<<dim3(a.rows, a.norm_groups), dim3(256), 0, st>>>(a, *a.conv);
-  else rec_norm_kernel<false><<<dim3(a.rows, a.norm_groups), dim3(256), 0, st>>>(a, RecInArgs());
+  const dim3 grid(a.rows, a.norm_groups);
+  const int gs = a.heads * a.vdim / a.norm_groups;
+#define LCC_GO(NW, MAXP)                                                                                \
+  do {                                                                                                  \
+    if (a.conv) rec_norm_kernel<true, NW, MAXP><<<grid, dim3(NW * 64), 0, st>>>(a, *a.conv);            \
+    else rec_norm_kernel<false, NW, MAXP><<<grid, dim3(NW * 64), 0, st>>>(a, RecInArgs());              \
+  } while (0)
+  if (gs <= 1024) LCC_GO(4, 1);
+  else if (a.rows <= 64) LCC_GO(16, 2);                // few rows: latency
+  else if (gs <= 2048) LCC_GO(4, 2);
+  else if (gs <= 4096) LCC_GO(8, 2);
+  else LCC_GO(16, 2);
+#undef LCC_GO
   return 0;
 }
 
