@@ -435,7 +435,7 @@ class LightningMixerSpec:
 
 @dataclasses.dataclass
 class ParallelMixerSpec:
-    """Two mixers side by side over the same input; their normed outputs are averaged."""
+    """Softmax attention and linear attention over one input; their normed outputs are averaged."""
     left: SoftmaxMixerSpec
     right: LightningMixerSpec
 

@@ -90,14 +90,14 @@ def lightning_mixer(h: torch.Tensor, W: Dict[str, torch.Tensor], m: dict, eps: f
 
 
 def parallel_mixer(h: torch.Tensor, W: Dict[str, torch.Tensor], m: dict, eps: float) -> torch.Tensor:
-    """Both mixers read h; each output is normed over the model width, the result is their mean."""
+    """Mean of the two outputs, each brought to unit rms over the width and weighted."""
     sub = lambda side: {n[len(side) + 1:]: w for n, w in W.items() if n.startswith(side + ".")}
     left, right = softmax_mixer(h, sub("left"), m["left"], eps), lightning_mixer(h, sub("right"), m["right"], eps)
     return 0.5 * (over_rms(left, eps) * W["left.out"] + over_rms(right, eps) * W["right.out"])
 
 
 def causal_conv(u: torch.Tensor, w: torch.Tensor, b: torch.Tensor) -> torch.Tensor:
-    """u [T, channels], w [channels, taps] (last column: the current token), zeros before the start."""
+    """u [T, channels], w [channels, taps]: out_t = b + sum_j w_j u_(t - taps + 1 + j), terms with a negative index left out."""
     T, taps = u.shape[0], w.shape[1]
     out = torch.zeros_like(u) + b
     for t in range(T):

@@ -17,12 +17,12 @@ def configs():
         "mixed": BemuzenConfig(331, 200, [L(P(A(6, 2, 24, 40, 0.31, 0.4, 37), Lin(3, 40, 24, [0.5, 0.97, 1.0])), 150), L(S(6, 20, 24, 3, 4, 4), 0),
                                           L(P(A(4, 4, 72, 88, 0.17, 0.2, 64), Lin(2, 72, 100, [0.9, 0.0])), 0), L(S(5, 24, 40, 1, 2, 1), 90)],
                                97, 31, 5, 1e-5, 1.7, name="mixed"),
-        "even": BemuzenConfig(256, 128, [L(P(A(4, 1, 64, 64, 0.2, 0.3, 100), Lin(2, 64, 64, [0.8, 0.995])), 256), L(S(2, 64, 64, 2, 4, 2), 256)], 1021, 17, 3, 1e-6, 1.0,
+        "even": BemuzenConfig(256, 128, [L(P(A(4, 1, 64, 64, 0.2, 0.3, 100), Lin(2, 64, 64, [0.8, 0.995])), 256), L(S(2, 64, 64, 2, 4, 2), 256)], 769, 17, 3, 1e-6, 1.0,
                               name="even"),
         "wide-heads": BemuzenConfig(100, 96, [L(P(A(2, 1, 136, 200, 0.1, 0.1, 16), Lin(2, 200, 130, [0.99, 0.6])), 64), L(S(3, 70, 150, 1, 1, 5), 40),
                                               L(P(A(1, 1, 8, 8, 0.5, 0.0, 1), Lin(3, 8, 24, [0.93, 0.5, 0.99])), 24)], 1, 3, 2, 1e-3, 0.6, name="wide-heads"),
-        "many-heads": BemuzenConfig(513, 320, [L(S(9, 128, 128, 3, 7, 9), 100), L(P(A(34, 2, 128, 33, 0.12, 0.3, 128), Lin(7, 128, 128, [0.9 + 0.014 * h for h in range(7)])), 320),
-                                               L(P(A(3, 3, 100, 128, 0.1, 0.2, 50), Lin(5, 16, 40, [0.75, 0.99, 0.999, 0.3, 0.95])), 64)], 4099, 127, 7, 1e-5, 2.5,
+        "many-heads": BemuzenConfig(513, 320, [L(S(9, 128, 128, 3, 7, 9), 100), L(P(A(34, 2, 128, 33, 0.12, 0.4, 90), Lin(7, 128, 128, [0.9 + 0.014 * h for h in range(7)])), 320),
+                                               L(P(A(3, 3, 100, 128, 0.1, 0.2, 50), Lin(5, 16, 40, [0.75, 0.99, 0.999, 0.3, 0.95])), 64)], 4099, 211, 13, 1e-5, 2.5,
                                     name="many-heads"),
     }
 

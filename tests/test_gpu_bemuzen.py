@@ -196,7 +196,7 @@ def test_biased_attention_of_packed_streams(dev, lib, dim, vdim, heads, kv, new,
         row += n
 
 
-@pytest.mark.parametrize("dim,vdim,heads,kv,lens,ns", [(64, 64, 8, 1, [1, 2, 31, 32, 33, 64, 65], 2), (128, 128, 12, 2, [700], 11), (128, 64, 34, 2, [64] * 18, 1),
+@pytest.mark.parametrize("dim,vdim,heads,kv,lens,ns", [(64, 64, 6, 1, [1, 2, 31, 32, 33, 64, 65], 2), (128, 128, 12, 2, [700], 11), (128, 64, 34, 2, [64] * 18, 1),
                                                        (192, 256, 3, 3, [200, 10], 4), (256, 128, 2, 1, [65], 64), (256, 256, 4, 2, [500, 1, 63], 3), (64, 192, 5, 5, [97], 3)])
 def test_biased_decode_attention(dev, lib, dim, vdim, heads, kv, lens, ns):
     g = torch.Generator().manual_seed(dim * 3 + vdim)
